@@ -27,6 +27,8 @@ class KVCacheSpec:
     head_dim: int
     window: Optional[int] = None
     values_in_keys: bool = False
+    # beside the window the first ``keep_first`` positions of a request are read for good: their pages stay
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -50,7 +52,9 @@ class CacheLayout:
         self.states = states            # key -> StateSpec
 
     @classmethod
-    def from_blocks(cls, blocks, schedule) -> "CacheLayout":
+    def from_blocks(cls, blocks, schedule, beside: dict | None = None) -> "CacheLayout":
+        """``beside``: {key: StateSpec} of what the model keeps for a request beside its layers (a transform of the
+        stream that looks back, say); the keys are names, no layer's index."""
         # A run of a layer either owns its cache or reads the one another run has written earlier in the
         # same pass.  What a run owns is kept under a key: the layer's index, or the key the schedule gives
         # the run (a layer that runs several times with the same weights then has pages and state for every
@@ -94,6 +98,7 @@ class CacheLayout:
                     layer_group[key] = len(groups) - 1
             if state is not None:
                 states[key] = state
+        states.update(beside or {})
         return cls(groups, layer_group, states)
 
     def bytes_per_token(self, element_size: int) -> int:

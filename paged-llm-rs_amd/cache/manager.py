@@ -62,6 +62,7 @@ class GroupGeometry:
     block_size: int
     num_blocks: int
     window: int = 0   # 0: all keys
+    keep: int = 0     # first keys of a request that are read beside the window
 
 
 class CacheManager:
@@ -74,7 +75,7 @@ class CacheManager:
         arr = ctypes.c_int * max(n, 1)
         self._h = self._lib.plh_cache_create(
             n, arr(*[g.block_size for g in groups]), arr(*[g.num_blocks for g in groups]),
-            arr(*[g.window for g in groups]), state_slots)
+            arr(*[g.window for g in groups]), arr(*[g.keep for g in groups]), state_slots)
         if not self._h:
             raise ConfigError(native.last_error())
 

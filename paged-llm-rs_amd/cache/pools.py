@@ -38,7 +38,8 @@ class PagedCache:
         self.dtype = dtype
         self.device = torch.device(device)
         self.max_seqs = max_seqs
-        geometry = [GroupGeometry(block_size, num_blocks, int(g.spec.window or 0)) for g in layout.groups]
+        geometry = [GroupGeometry(block_size, num_blocks, int(g.spec.window or 0), int(g.spec.keep_first) if g.spec.window else 0)
+                    for g in layout.groups]
         self.manager = CacheManager(geometry, state_slots=max_seqs if layout.states else 0)
         self._pools: dict = {}
         for g in layout.groups:
@@ -67,7 +68,7 @@ class PagedCache:
     def layer_pools(self, layer: int):
         return self._pools[layer]
 
-    def layer_state(self, layer: int) -> torch.Tensor:
+    def layer_state(self, layer) -> torch.Tensor:
         if layer not in self._states:
             raise ConfigError(f"layer {layer} keeps no state")
         return self._states[layer]

@@ -1,5 +1,6 @@
 from .dimalix import DimalixConfig
 from .generation import GenerationConfig
+from .guzuvik import GuzuvikConfig
 from .lefavik import LefavikConfig
 from .mukenex import MukenexConfig
 from .papivik import PapivikConfig
@@ -9,7 +10,8 @@ from .specs import (AttentionSpec, GatedMlpSpec, LayerSpec, ModelSpec, NormSpec,
                     ScheduleEntry)
 
 __all__ = [
-    "GenerationConfig", "Qwen3Config", "PapivikConfig", "LefavikConfig", "MukenexConfig", "DimalixConfig", "read_json", "architectures", "config_class_for",
+    "GenerationConfig", "Qwen3Config", "PapivikConfig", "LefavikConfig", "MukenexConfig", "DimalixConfig",
+    "GuzuvikConfig", "read_json", "architectures", "config_class_for",
     "load_config", "register_architecture", "AttentionSpec", "GatedMlpSpec", "LayerSpec",
     "ModelSpec", "NormSpec", "PositionSpec", "ScheduleEntry",
 ]

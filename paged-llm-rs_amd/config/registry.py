@@ -10,6 +10,7 @@ from pathlib import Path
 
 from ..errors import ConfigError, UnsupportedError
 from .dimalix import DimalixConfig
+from .guzuvik import GuzuvikConfig
 from .lefavik import LefavikConfig
 from .mukenex import MukenexConfig
 from .papivik import PapivikConfig
@@ -70,3 +71,4 @@ register_architecture("Papivik", PapivikConfig, model_type="papivik")
 register_architecture("Lefavik", LefavikConfig, model_type="lefavik")
 register_architecture("Mukenex", MukenexConfig, model_type="mukenex")
 register_architecture("Dimalix", DimalixConfig, model_type="dimalix")
+register_architecture("Guzuvik", GuzuvikConfig, model_type="guzuvik")

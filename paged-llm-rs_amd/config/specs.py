@@ -14,7 +14,7 @@ from typing import Any, Optional
 
 @dataclass(frozen=True)
 class NormSpec:
-    """A normalisation over the last axis."""
+    """A normalisation over the last axis: ``rms_norm``, or ``layer_norm`` (mean taken off, a bias added)."""
     kind: str = "rms_norm"
     eps: float = 1e-6
     gain_offset: float = 0.0                # the stored gain plus this is the gain (1.0: gains stored around zero)
@@ -146,6 +146,22 @@ class GatedDeltaSpec:
 
 
 @dataclass(frozen=True)
+class StateSpaceSpec:
+    """A state space a head whose decay and step size come from the token (Mamba-2):
+    S = exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x, dt = softplus(projected dt + dt_bias), with x, B and C
+    behind a short convolution with bias and silu; y times silu(z), then an RMS norm over equal parts of all heads together.
+    ``groups``: B and C have so many heads, head h of x reads head h / (num_heads / groups)."""
+    kind: str = "state_space"
+    num_heads: int = 0
+    value_dim: int = 0           # size of x and y a head
+    state_dim: int = 0           # size of B and C a head
+    groups: int = 1
+    conv_taps: int = 4
+    norm_groups: int = 1
+    eps: float = 1e-6
+
+
+@dataclass(frozen=True)
 class ConvAttentionSpec:
     """Grouped-query softmax attention over a paged cache whose q, k and v pass a short causal convolution
     right behind their projections; value heads may have another size than query and key heads."""
@@ -182,10 +198,11 @@ class DenseMlpSpec:
 
 @dataclass(frozen=True)
 class SinkAttentionSpec:
-    """Grouped-query softmax attention over a paged cache whose softmax has one more term in its denominator
-    (a sink: a score without a key or a value), with optional extras: q and k divided by their root mean
+    """Grouped-query softmax attention over a paged cache with optional extras: one more term in the softmax's
+    denominator (a sink: a score without a key or a value), q and k divided by their root mean
     square over a head (no gain), a query temperature that grows with the logarithm of the position, a
-    penalty a head on the distance between query and key, and a window."""
+    penalty a head on the distance between query and key, a window that may keep a request's first tokens in sight,
+    a soft cap on the scores, values mixed with those of an earlier layer, and a gate a head on the read-out."""
     kind: str = "sink_attention"
     num_heads: int = 0
     num_kv_heads: int = 0
@@ -206,6 +223,12 @@ class SinkAttentionSpec:
     mask: str = "window"
     qk_gain: bool = False                   # the unit q and k times a gain over the head (tensors ``q.norm``, ``k.norm``)
     qkv_bias: bool = False                  # q, k and v projections carry a bias each (``q.b``, ``k.b``, ``v.b``)
+    keep_first: int = 0                     # beside a window: the keys 0 .. keep_first - 1, seen by every later query
+    softcap: Optional[float] = None         # a scaled score s becomes cap * tanh(s / cap), before the distance penalty
+    # Values mixed over layers: every layer with ``value_mix`` but the first of them uses (1 - l) v + l v_first, v_first
+    # being the first one's values of the same token and l the layer's tensor ``vmix`` (one number).
+    value_mix: bool = False
+    head_gate: bool = False                 # head h's read-out times sigmoid((g x)_h), x the layer's input (tensor ``g`` [heads, width])
 
 
 @dataclass(frozen=True)
@@ -280,7 +303,10 @@ class RoutedExpertsSpec:
     score plus ``correction`` (a tensor of that name, where ``corrected``); experts form ``groups`` equal groups of
     neighbours, a group counts by its best choice score, and only experts of the best ``groups_kept`` groups can be
     chosen (``groups`` 1: no groups).  A chosen expert weighs its score (without the correction), divided, where
-    ``normalised``, by the chosen scores' sum plus ``weight_eps``."""
+    ``normalised``, by the chosen scores' sum plus ``weight_eps``.  ``biased``: a tensor ``router.b`` is added to the logits.
+    ``score`` "chosen_logits" instead of "softmax": the choice goes by the logits and the weights are the softmax over the chosen
+    logits alone.  ``activation`` "clamped" with its ``limit``: an expert is down(g sigmoid(1.702 g) (u + 1)) with
+    g = min(gate x, limit) and u = clamp(up x, -limit, limit)."""
     kind: str = "routed_experts"
     experts: int = 0
     identity: int = 0
@@ -293,3 +319,5 @@ class RoutedExpertsSpec:
     groups_kept: int = 1
     normalised: bool = True
     weight_eps: float = 1e-20
+    biased: bool = False
+    limit: Optional[float] = None

@@ -200,20 +200,29 @@ __device__ __forceinline__ bool ad_find_row(int slot, const int* __restrict__ q_
 // at all times with nothing else between them in the queue of loads (page numbers come from LDS, so no
 // round waits behind a table lookup).  Queries and the own key are normalised and rotated while the
 // first two rounds are on their way.
-// EX: the launch has sinks or distance slopes; without them the kernel is compiled as if it knew neither, and takes
-// the arguments it always took.
-template <bool EX>
+// EX 1: the launch has sinks or distance slopes; without them (0) the kernel is compiled as if it knew neither, and takes
+// the arguments it always took.  EX 2: it may also have a soft cap on the scores, first keys kept beside the window
+// and a gate a head (PlAttentionMore).
+// Kept keys stand in front of the window's in the numbering that splits and rounds go by: key number i is key
+// i - (first - kept) of the request where i < first, and key i from `first` on.
+template <int EX>
 struct ad_extras_t {
+    const float* sinks;
+    const float* slopes;
+    PlAttentionMore more;
+};
+template <>
+struct ad_extras_t<1> {
     const float* sinks;
     const float* slopes;
 };
 template <>
-struct ad_extras_t<false> {
+struct ad_extras_t<0> {
     static constexpr const float* sinks = nullptr;
     static constexpr const float* slopes = nullptr;
 };
 
-template <int LPK, int GT, int U, int WV, bool EX = false>
+template <int LPK, int GT, int U, int WV, int EX = 0>
 __global__ void __launch_bounds__(64 * WV)
 paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
                               float* __restrict__ part_acc, float* __restrict__ part_ml,
@@ -257,11 +266,14 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
     // the stretch of keys of this split, in whole rounds of the workgroup
     const int first = pl_first_visible(pos, window);
     const int limit = fuse.mode == 2 ? pos : pos + 1;   // the token's own key is not in the cache yet
-    const int total = max(limit - first, 0);
+    int kept = 0;
+    if constexpr (EX == 2) kept = min(extras.more.keep, first);
+    auto key_at = [&](int i) { return EX == 2 && i < first ? i - (first - kept) : i; };
+    const int total = max(limit - (first - kept), 0);
     // ceil(total / splits): the high half of (total + splits - 1) * ceil(2^32 / splits), exact below 2^32 / splits
     const int share = splits == 1 ? total : static_cast<int>(__umulhi(static_cast<uint32_t>(total + splits - 1), splits_magic));
     const int per_split = pl_ceil_div(share, ROUND) * ROUND;
-    const int s_begin = first + split * per_split;
+    const int s_begin = first - kept + split * per_split;
     const int s_end = min(limit, s_begin + per_split);
     const int rounds = s_end > s_begin ? pl_ceil_div(s_end - s_begin, ROUND) : 0;
 
@@ -280,8 +292,17 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
 
     // ---- everything that does not wait for anything but the position, asked for at once ----
     int unused;
-    const int page_first = rounds > 0 ? page_of(s_begin, unused) : 0;
-    const int page_count = rounds > 0 ? page_of(s_end - 1, unused) - page_first + 1 : 0;
+    // (the pages of the stretch: those of its kept keys, then those of its keys in the window; without kept keys the latter alone)
+    int kept_first = 0, kept_pages = 0;
+    if constexpr (EX == 2) {
+        if (rounds > 0 && s_begin < first) {
+            kept_first = page_of(key_at(s_begin), unused);
+            kept_pages = page_of(key_at(min(s_end, first) - 1), unused) - kept_first + 1;
+        }
+    }
+    const bool in_window = rounds > 0 && (EX != 2 || s_end > first);
+    const int page_first = in_window ? page_of(EX == 2 ? max(s_begin, first) : s_begin, unused) : 0;
+    const int page_count = (in_window ? page_of(s_end - 1, unused) - page_first + 1 : 0) + kept_pages;
     const bool pages_in_lds = page_count <= AD_PAGES_LDS;
     int page_got[AD_PAGES_LDS / (64 * WV) > 0 ? AD_PAGES_LDS / (64 * WV) : 1];
     constexpr int PAGE_TURNS = AD_PAGES_LDS / (64 * WV) > 0 ? AD_PAGES_LDS / (64 * WV) : 1;
@@ -289,7 +310,8 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
 #pragma unroll
         for (int i = 0; i < PAGE_TURNS; ++i) {
             const int e = static_cast<int>(threadIdx.x) + i * 64 * WV;
-            page_got[i] = table[page_first + min(e, max(page_count - 1, 0))];
+            const int ee = min(e, max(page_count - 1, 0));
+            page_got[i] = table[EX == 2 && ee < kept_pages ? kept_first + ee : page_first + ee - kept_pages];
         }
     }
     u32x4 qraw[GT];
@@ -332,8 +354,9 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
             const int j = base + u * KPW + sub;
             const bool in = j < s_end;
             int w;
-            const int bi = page_of(in ? j : s_begin, w);                // a key that exists in any case
-            const int page = pages_in_lds ? pages_lds[bi - page_first] : table[bi];
+            const int i = in ? j : s_begin;                             // a key that exists in any case
+            const int bi = page_of(key_at(i), w);
+            const int page = pages_in_lds ? pages_lds[EX == 2 && i < first ? bi - kept_first : bi - page_first + kept_pages] : table[bi];
             ok[u] = in && page >= 0;
             const size_t off = (static_cast<size_t>(max(page, 0)) * block_size + w) * row_stride + head_off;
             kk[u] = *reinterpret_cast<const u32x4*>(k_pool + off);
@@ -371,7 +394,15 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
     const bool tilted = EX && slopes != nullptr;
     float tilt[EX ? GT : 1];
     int round_now = 0;            // (EX) the round that `consume` is given, for the distance of its keys
-    if constexpr (EX) {
+    // a soft cap, in the exponent's unit: c tanh(s / c) = c (1 - 2 / (2^(2 log2(e) s / c) + 1))
+    float cap_in = 0.f, cap_out = 0.f;
+    if constexpr (EX == 2) {
+        if (extras.more.cap > 0.f) {
+            cap_in = 2.f / extras.more.cap;
+            cap_out = extras.more.cap * 1.4426950408889634f;
+        }
+    }
+    if constexpr (EX != 0) {
 #pragma unroll
         for (int hq = 0; hq < GT; ++hq) tilt[hq] = tilted ? slopes[h0 + min(hq, heads - 1)] * 1.4426950408889634f : 0.f;
     }
@@ -433,9 +464,12 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
 #pragma unroll
                 for (int w = 0; w < 4; ++w) dot = ad_dot2(qp[hq].v[w], kraw[u].v[w], dot);
                 dot = key_sum<LPK>(dot) * scale_log2e;
-                if constexpr (EX) {
+                if constexpr (EX == 2) {
+                    if (cap_out > 0.f) dot = cap_out - 2.f * cap_out * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(dot * cap_in) + 1.f);
+                }
+                if constexpr (EX != 0) {
                     if (tilted)
-                        dot = fmaf(-tilt[hq], static_cast<float>(pos - (s_begin + round_now * ROUND + wave * KPW * U + u * KPW + sub)), dot);
+                        dot = fmaf(-tilt[hq], static_cast<float>(pos - key_at(s_begin + round_now * ROUND + wave * KPW * U + u * KPW + sub)), dot);
                 }
                 s[u][hq] = ok[u] ? dot : -INFINITY;
             }
@@ -481,11 +515,11 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
         }
     };
     for (int r = 0; r < rounds; r += 2) {
-        if constexpr (EX) round_now = r;
+        if constexpr (EX != 0) round_now = r;
         consume(ka, va, oka);
         if (r + 2 < rounds) ask(r + 2, ka, va, oka);
         if (r + 1 < rounds) {
-            if constexpr (EX) round_now = r + 1;
+            if constexpr (EX != 0) round_now = r + 1;
             consume(kb, vb, okb);
             if (r + 3 < rounds) ask(r + 3, kb, vb, okb);
         }
@@ -536,7 +570,11 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
         }
         const int h = h0 + hq;
         if (splits == 1) {
-            if constexpr (EX) {
+            float opened = 1.f;
+            if constexpr (EX == 2) {
+                if (extras.more.gate != nullptr) opened = pl_head_gate(extras.more, t, h);
+            }
+            if constexpr (EX != 0) {
                 if (sinks != nullptr) {
                     // a sink: one more term of the denominator, unscaled, with no value behind it
                     const float sk = sinks[h] * 1.4426950408889634f;
@@ -546,7 +584,7 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
                     a *= keep;
                 }
             }
-            out[(static_cast<size_t>(t) * nq + h) * d + dd] = from_float<bf16_t>(sum > 0.f ? a / sum : 0.f);
+            out[(static_cast<size_t>(t) * nq + h) * d + dd] = from_float<bf16_t>(sum > 0.f ? a / sum * opened : 0.f);
         } else {
             const size_t pi = (static_cast<size_t>(t) * nq + h) * splits + split;
             part_acc[pi * d + dd] = a;
@@ -569,7 +607,8 @@ __global__ void __launch_bounds__(256)
 paged_attention_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
                              bf16_t* __restrict__ out, const int* __restrict__ positions,
                              const int* __restrict__ seq_of, const int* __restrict__ q_len, int short_limit,
-                             int nq, int d, int splits, int n, int num_seqs, const float* __restrict__ sinks) {
+                             int nq, int d, int splits, int n, int num_seqs, const float* __restrict__ sinks,
+                             PlAttentionMore more) {
     const int per_token = nq * d;
     int t, rest;
     bool inside;
@@ -616,6 +655,7 @@ paged_attention_merge_kernel(const float* __restrict__ part_acc, const float* __
         sum = sum * keep + exp2f(sk - top);
         a *= keep;
     }
+    if (EX && more.gate != nullptr) a *= pl_head_gate(more, t, h);
     out[(static_cast<size_t>(t) * nq + h) * d + dd] = from_float<bf16_t>(sum > 0.f ? a / sum : 0.f);
 }
 
@@ -626,18 +666,19 @@ static int launch_decode_keys(const void* q, int q_stride, void* out, float* par
                               const int* positions, const int* seq_of, const int* q_len, int short_limit, int num_seqs,
                               int short_rows, const int* block_table, int max_blocks, int block_size, void* k_pool,
                               void* v_pool, int n, int nq, int nkv, int d, float scale, int window, int splits,
-                              const ad_fuse_t& fuse, const float* sinks, const float* slopes, hipStream_t stream) {
+                              const ad_fuse_t& fuse, const float* sinks, const float* slopes,
+                              const PlAttentionMore& more, hipStream_t stream) {
     constexpr int WV = AD_WAVES;
     const int g = nq / nkv;
     const int tiles = pl_ceil_div(g, GT);
     const size_t lds_bytes = (AD_PAGES_LDS + static_cast<size_t>(WV) * GT * 2 + static_cast<size_t>(WV) * GT * d) * sizeof(float);
     PL_REQUIRE(lds_bytes <= 160 * 1024, "decode attention: %zu bytes of LDS for head size %d", lds_bytes, d);
-    const bool extras = sinks != nullptr || slopes != nullptr;
+    const int extras = pl_has_more(more) ? 2 : (sinks != nullptr || slopes != nullptr ? 1 : 0);
     if (lds_bytes > 48 * 1024) {
-        hipError_t e = extras ? hipFuncSetAttribute(reinterpret_cast<const void*>(&paged_attention_decode_kernel<LPK, GT, U, WV, true>),
-                                                    hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds_bytes))
-                              : hipFuncSetAttribute(reinterpret_cast<const void*>(&paged_attention_decode_kernel<LPK, GT, U, WV, false>),
-                                                    hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds_bytes));
+        const void* kernel = extras == 2 ? reinterpret_cast<const void*>(&paged_attention_decode_kernel<LPK, GT, U, WV, 2>)
+                             : extras == 1 ? reinterpret_cast<const void*>(&paged_attention_decode_kernel<LPK, GT, U, WV, 1>)
+                                           : reinterpret_cast<const void*>(&paged_attention_decode_kernel<LPK, GT, U, WV, 0>);
+        hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds_bytes));
         PL_REQUIRE(e == hipSuccess, "decode attention: %zu bytes of LDS refused: %s", lds_bytes, hipGetErrorString(e));
     }
     // rows of the grid: the step's rows, or, where fewer, the tokens that the short requests can bring
@@ -649,13 +690,16 @@ static int launch_decode_keys(const void* q, int q_stride, void* out, float* par
         static_cast<const bf16_t*>(q), q_stride, static_cast<bf16_t*>(out), part_acc, part_ml, positions, seq_of,      \
         q_len, short_limit, compact ? num_seqs : 0, block_table, max_blocks, block_size, static_cast<bf16_t*>(k_pool), \
         static_cast<bf16_t*>(v_pool), nq, nkv, d, scale * 1.4426950408889634f, window, splits, tiles, g,              \
-        static_cast<uint32_t>((0x100000000ull + splits - 1) / static_cast<unsigned>(splits)), fuse, more)
-    if (extras) {
-        const ad_extras_t<true> more{sinks, slopes};
-        AD_LAUNCH(true);
+        static_cast<uint32_t>((0x100000000ull + splits - 1) / static_cast<unsigned>(splits)), fuse, with)
+    if (extras == 2) {
+        const ad_extras_t<2> with{sinks, slopes, more};
+        AD_LAUNCH(2);
+    } else if (extras == 1) {
+        const ad_extras_t<1> with{sinks, slopes};
+        AD_LAUNCH(1);
     } else {
-        const ad_extras_t<false> more{};
-        AD_LAUNCH(false);
+        const ad_extras_t<0> with{};
+        AD_LAUNCH(0);
     }
 #undef AD_LAUNCH
     PL_CHECK_LAUNCH("paged_attention_decode");
@@ -663,14 +707,14 @@ static int launch_decode_keys(const void* q, int q_stride, void* out, float* par
         const dim3 mgrid = dim3(pl_ceil_div(nq * d, 256), compact ? short_rows : n);
 #define AD_MERGE(SP)                                                                                              \
     do {                                                                                                          \
-        if (sinks != nullptr)                                                                                     \
+        if (sinks != nullptr || more.gate != nullptr)                                                             \
             paged_attention_merge_kernel<SP, true><<<mgrid, 256, 0, stream>>>(                                    \
                 part_acc, part_ml, static_cast<bf16_t*>(out), positions, seq_of, q_len, short_limit, nq, d,       \
-                splits, n, compact ? num_seqs : 0, sinks);                                                        \
+                splits, n, compact ? num_seqs : 0, sinks, more);                                                     \
         else                                                                                                      \
             paged_attention_merge_kernel<SP, false><<<mgrid, 256, 0, stream>>>(                                   \
                 part_acc, part_ml, static_cast<bf16_t*>(out), positions, seq_of, q_len, short_limit, nq, d,       \
-                splits, n, compact ? num_seqs : 0, nullptr);                                                      \
+                splits, n, compact ? num_seqs : 0, nullptr, more);                                                     \
     } while (0)
         if (splits <= 4) AD_MERGE(4);
         else if (splits <= 8) AD_MERGE(8);
@@ -694,12 +738,13 @@ static int launch_decode(const void* q, int q_stride, void* out, float* part_acc
                          const int* positions, const int* seq_of, const int* q_len, int short_limit, int num_seqs,
                          int short_rows, const int* block_table, int max_blocks, int block_size, void* k_pool,
                          void* v_pool, int n, int nq, int nkv, int d, float scale, int window, int splits,
-                         const ad_fuse_t& fuse, const float* sinks, const float* slopes, hipStream_t stream) {
+                         const ad_fuse_t& fuse, const float* sinks, const float* slopes,
+                              const PlAttentionMore& more, hipStream_t stream) {
     const long long workgroups = static_cast<long long>(nkv) * pl_ceil_div(nq / nkv, GT) * n * splits;
 #define AD_KEYS_CALL(U)                                                                                            \
     return launch_decode_keys<LPK, GT, U>(q, q_stride, out, part_acc, part_ml, positions, seq_of, q_len,          \
                                           short_limit, num_seqs, short_rows, block_table, max_blocks, block_size,  \
-                                          k_pool, v_pool, n, nq, nkv, d, scale, window, splits, fuse, sinks, slopes, stream)
+                                          k_pool, v_pool, n, nq, nkv, d, scale, window, splits, fuse, sinks, slopes, more, stream)
     if constexpr (GT <= 2) {
         if (workgroups <= pl_compute_units()) AD_KEYS_CALL(8);
         AD_KEYS_CALL(4);
@@ -714,11 +759,12 @@ static int dispatch_gt(int gt, const void* q, int q_stride, void* out, float* pa
                        const int* positions, const int* seq_of, const int* q_len, int short_limit, int num_seqs,
                        int short_rows, const int* block_table, int max_blocks, int block_size, void* k_pool,
                        void* v_pool, int n, int nq, int nkv, int d, float scale, int window, int splits,
-                       const ad_fuse_t& fuse, const float* sinks, const float* slopes, hipStream_t stream) {
+                       const ad_fuse_t& fuse, const float* sinks, const float* slopes,
+                              const PlAttentionMore& more, hipStream_t stream) {
 #define AD_CALL(G)                                                                                              \
     return launch_decode<LPK, G>(q, q_stride, out, part_acc, part_ml, positions, seq_of, q_len, short_limit,   \
                                  num_seqs, short_rows, block_table, max_blocks, block_size, k_pool, v_pool, n, nq, nkv, d, scale,    \
-                                 window, splits, fuse, sinks, slopes, stream)
+                                 window, splits, fuse, sinks, slopes, more, stream)
     switch (gt) {
         case 1: AD_CALL(1);
         case 2: AD_CALL(2);
@@ -744,7 +790,13 @@ extern "C" int pl_paged_attention_decode(const void* q, int q_stride, void* out,
                                          void* v_pool, int n, int nq, int nkv, int d, float scale, int window,
                                          int splits, int fuse_mode, const void* q_gain, const void* k_gain,
                                          int gain_dtype, float eps, const float* cos_table, const float* sin_table,
-                                         int rot, const float* sinks, const float* slopes, hipStream_t stream) {
+                                         int rot, const float* sinks, const float* slopes, float cap, int keep,
+                                         const float* gate, int gate_stride, hipStream_t stream) {
+    const PlAttentionMore more{cap, keep, gate, gate_stride};
+    PL_REQUIRE(cap >= 0.f && keep >= 0 && (gate == nullptr || gate_stride >= nq) && (keep == 0 || window >= 0),
+               "decode attention: a cap of %g, %d first keys kept beside a window of %d, gates in rows of %d",
+               static_cast<double>(cap), keep, window, gate_stride);
+    PL_REQUIRE(fuse_mode == 0 || !pl_has_more(more), "decode attention: caps, kept keys and gates go with prepared queries");
     PL_REQUIRE(d > 0 && d <= 256 && d % 16 == 0, "decode attention: head size %d, which has to be a multiple of 16 up to 256", d);
     PL_REQUIRE(nq > 0 && nkv > 0 && nq % nkv == 0, "decode attention: %d query heads over %d key heads", nq, nkv);
     PL_REQUIRE(block_size > 0 && max_blocks > 0 && q_stride >= nq * d && q_stride % 8 == 0 && splits >= 1 && splits <= AD_MAX_SPLITS,
@@ -768,7 +820,7 @@ extern "C" int pl_paged_attention_decode(const void* q, int q_stride, void* out,
 #define AD_LPK(L)                                                                                                  \
     return dispatch_gt<L>(gt, q, q_stride, out, part_acc, part_ml, positions, seq_of, q_len, short_limit,        \
                           num_seqs, short_rows, block_table, max_blocks, block_size, k_pool, v_pool, n, nq, nkv, d, scale, window,      \
-                          splits, fuse, sinks, slopes, stream)
+                          splits, fuse, sinks, slopes, more, stream)
     if (chunks <= 2) AD_LPK(2);
     if (chunks <= 4) AD_LPK(4);
     if (chunks <= 8) AD_LPK(8);

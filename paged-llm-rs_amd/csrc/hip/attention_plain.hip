@@ -12,7 +12,8 @@
 //
 // Two optional extras, a number a query head each: `slopes` (slope_h * (i - j) is taken off the score of key
 // j for the query at position i) and `sinks` (exp(sink_h) joins the softmax's denominator once: a score
-// that is not scaled and has no key and no value).  Key and value pool may be one and the same tensor.
+// that is not scaled and has no key and no value).  `more` (PlAttentionMore): a soft cap on the scores, first keys
+// that every later query sees beside its window, and a gate a head on the read-out.  Key and value pool may be one and the same tensor.
 #include "common.hpp"
 
 #define PL_MAX_HEAD_DIM 1024
@@ -25,7 +26,7 @@ paged_attention_plain_kernel(const T* __restrict__ q, int q_stride, T* __restric
                              const int* __restrict__ block_table, int max_blocks, int block_size,
                              const T* k_pool, const T* v_pool, int nq,
                              int nkv, int d, float scale, int window, const float* __restrict__ sinks,
-                             const float* __restrict__ slopes) {
+                             const float* __restrict__ slopes, PlAttentionMore more) {
     __shared__ float qs[REGS * PL_WAVE];
     const int t = blockIdx.x;
     const int h = blockIdx.y;
@@ -47,18 +48,25 @@ paged_attention_plain_kernel(const T* __restrict__ q, int q_stride, T* __restric
 #pragma unroll
     for (int r = 0; r < REGS; ++r) acc[r] = 0.f;
 
-    for (int j0 = first; j0 <= pos; j0 += PL_WAVE) {
+    // first the kept keys in front of the window, then the window's
+    const int kept = min(more.keep, first);
+    for (int j0 = kept > 0 ? 0 : first, next; j0 <= pos; j0 = next) {
+        const bool front = j0 < kept;
+        const int stop = front ? kept - 1 : pos;           // the last key of this stretch
+        next = front && j0 + PL_WAVE >= kept ? first : j0 + PL_WAVE;
         const int j = j0 + lane;
         float s = -INFINITY;
         int slot = -1;
-        if (j <= pos) {
+        if (j <= stop) {
             const int blk = table[j / block_size];
             if (blk >= 0) {
                 slot = blk * block_size + j % block_size;
                 const T* krow = k_pool + (static_cast<size_t>(slot) * nkv + kvh) * d;
                 float dot = 0.f;
                 for (int i = 0; i < d; ++i) dot = fmaf(qs[i], to_float(krow[i]), dot);
-                s = dot * scale - slope * static_cast<float>(pos - j);
+                s = dot * scale;
+                if (more.cap > 0.f) s = more.cap * tanhf(s / more.cap);
+                s -= slope * static_cast<float>(pos - j);
             }
         }
         const float tile_max = wave_max(s);
@@ -69,7 +77,7 @@ paged_attention_plain_kernel(const T* __restrict__ q, int q_stride, T* __restric
         l = l * corr + wave_sum(p);
 #pragma unroll
         for (int r = 0; r < REGS; ++r) acc[r] *= corr;
-        const int count = min(PL_WAVE, pos - j0 + 1);
+        const int count = min(PL_WAVE, stop - j0 + 1);
         for (int jj = 0; jj < count; ++jj) {
             const float pj = __shfl(p, jj, PL_WAVE);
             const int sj = __shfl(slot, jj, PL_WAVE);
@@ -92,11 +100,12 @@ paged_attention_plain_kernel(const T* __restrict__ q, int q_stride, T* __restric
 #pragma unroll
         for (int r = 0; r < REGS; ++r) acc[r] *= corr;
     }
+    const float opened = more.gate != nullptr ? pl_head_gate(more, t, h) : 1.f;
     T* orow = out + (static_cast<size_t>(t) * nq + h) * d;
 #pragma unroll
     for (int r = 0; r < REGS; ++r) {
         const int i = lane + r * PL_WAVE;
-        if (i < d) orow[i] = from_float<T>(l > 0.f ? acc[r] / l : 0.f);
+        if (i < d) orow[i] = from_float<T>(l > 0.f ? acc[r] / l * opened : 0.f);
     }
 }
 
@@ -104,7 +113,12 @@ extern "C" int pl_paged_attention_plain(const void* q, int q_stride, void* out, 
                                         const int* seq_of, const int* block_table, int max_blocks,
                                         int block_size, const void* k_pool, const void* v_pool, int n,
                                         int nq, int nkv, int d, float scale, int window, int dtype,
-                                        const float* sinks, const float* slopes, hipStream_t stream) {
+                                        const float* sinks, const float* slopes, float cap, int keep,
+                                        const float* gate, int gate_stride, hipStream_t stream) {
+    PL_REQUIRE(cap >= 0.f && keep >= 0 && (gate == nullptr || gate_stride >= nq), "attention: a cap of %g, %d first keys kept, gates in rows of %d",
+               static_cast<double>(cap), keep, gate_stride);
+    PL_REQUIRE(keep == 0 || window >= 0, "attention: first keys kept beside blocks of positions");
+    const PlAttentionMore more{cap, keep, gate, gate_stride};
     PL_REQUIRE(d > 0 && d <= PL_MAX_HEAD_DIM, "attention: head size %d, which has to be between 1 and %d", d, PL_MAX_HEAD_DIM);
     PL_REQUIRE(nq > 0 && nkv > 0 && nq % nkv == 0, "attention: %d query heads over %d key heads", nq, nkv);
     PL_REQUIRE(block_size > 0 && max_blocks > 0 && q_stride >= nq * d,
@@ -116,7 +130,7 @@ extern "C" int pl_paged_attention_plain(const void* q, int q_stride, void* out, 
     paged_attention_plain_kernel<T, REGS><<<grid, PL_WAVE, 0, stream>>>(                                                \
         static_cast<const T*>(q), q_stride, static_cast<T*>(out), positions, seq_of, block_table, max_blocks,          \
         block_size, static_cast<const T*>(k_pool), static_cast<const T*>(v_pool), nq, nkv, d, scale, window, sinks,    \
-        slopes)
+        slopes, more)
     if (dtype == PL_DTYPE_F32) {
         if (d <= 256) PL_PLAIN_LAUNCH(float, 4);
         else PL_PLAIN_LAUNCH(float, 16);

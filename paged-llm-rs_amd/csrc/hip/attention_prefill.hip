@@ -168,7 +168,17 @@ __device__ __forceinline__ bool ap_find_tile(int slot, const int* __restrict__ q
     return false;
 }
 
-template <int DT, int NW, int KS, int FEED, bool GR = false>
+// MORE: the launch may have a soft cap on the scores, first keys kept beside the window and a gate a head
+// (PlAttentionMore); without it the kernel is compiled as if it knew none of them.  The tiles of keys of a token tile are then those of
+// the kept keys, where these end before the window's first tile, and the window's behind them.
+template <bool MORE>
+struct ap_more_t {
+    PlAttentionMore more;
+};
+template <>
+struct ap_more_t<false> {};
+
+template <int DT, int NW, int KS, int FEED, bool GR, bool MORE>
 __global__ void __launch_bounds__(64 * NW * KS, DT <= 4 ? AP_OCC : 1)
 paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
                                const int* __restrict__ q_start, const int* __restrict__ q_len,
@@ -178,7 +188,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
                                const bf16_t* __restrict__ v_pool, int nq, int nkv, int d, float scale_log2e,
                                int window, int total_work, int splits, float* __restrict__ part_acc,
                                float* __restrict__ part_ml, int compact, const float* __restrict__ sinks,
-                               const float* __restrict__ slopes) {
+                               const float* __restrict__ slopes, ap_more_t<MORE> with) {
     constexpr int DP = 32 * DT;
     constexpr int BM = 32 * NW;
     constexpr int NT = 64 * NW * KS;
@@ -280,6 +290,19 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
 
     const int last_pos = GR ? start + q0 : start + min(q0 + BM, count) - 1;   // the last key any query of the tile sees
     const int first_pos = pl_first_visible(start + q0, window);
+    int keep_first = 0, kept = 0;             // keys kept for good, and those of them in front of the first query's window
+    float cap_in = 0.f, cap_out = 0.f;
+    if constexpr (MORE) {
+        keep_first = with.more.keep;
+        kept = min(keep_first, first_pos);
+        // c tanh(s / c) = c (1 - 2 / (2^(2 log2(e) s / c) + 1)), in the unit of the raw scores
+        if (with.more.cap > 0.f) {
+            cap_in = 2.f * scale_log2e / with.more.cap;
+            cap_out = with.more.cap * 1.4426950408889634f / scale_log2e;
+        }
+    }
+    // a key that no query of the tile sees and whose page may have been given back
+    auto gone = [&](int j) { return j < first_pos && (!MORE || j >= kept); };
     const int* table = block_table + static_cast<size_t>(seq) * max_blocks;
     const size_t row_stride = static_cast<size_t>(nkv) * d;
     const size_t head_off = static_cast<size_t>(kvh) * d;
@@ -374,7 +397,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
                 size_t vat = base + lane_place;
                 if (kj0[i] + 64 / CP - 1 > last_pos || kj0[i] < first_pos) {   // (the same for the wave)
                     const int j = kj0[i] + lane / CP;
-                    vat = (j > last_pos || j < first_pos) ? last_base + lane_piece : vat;
+                    vat = (j > last_pos || gone(j)) ? last_base + lane_piece : vat;
                 }
                 vreg[i] = *reinterpret_cast<const ap_vec4*>(reinterpret_cast<const char*>(v_pool) + vat);
             } else {
@@ -406,11 +429,27 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
     };
 
     // this workgroup's share of the key tiles
-    const int k_lowest = (first_pos / AP_BN) * AP_BN;
-    const int key_tiles = (last_pos - k_lowest) / AP_BN + 1;
+    int k_lowest = (first_pos / AP_BN) * AP_BN, kept_tiles = 0;
+    if constexpr (MORE) {
+        kept_tiles = (kept + AP_BN - 1) / AP_BN;
+        if (kept_tiles * AP_BN >= k_lowest) {         // (one run of tiles, or nothing kept)
+            if (kept_tiles > 0) k_lowest = 0;
+            kept_tiles = 0;
+        }
+    }
+    const int key_tiles = kept_tiles + (last_pos - k_lowest) / AP_BN + 1;
     const int tiles_a_split = (key_tiles + splits - 1) / splits;
-    const int k_first = k_lowest + split * tiles_a_split * AP_BN;
-    const int k_end = min(k_lowest + key_tiles * AP_BN, k_first + tiles_a_split * AP_BN);
+    const int tile_first_no = split * tiles_a_split, tile_end_no = min(key_tiles, tile_first_no + tiles_a_split);
+    // the first key of tile n of this workgroup's share
+    const int k_share = k_lowest + (tile_first_no - kept_tiles) * AP_BN;
+    auto key_of = [&](int n) {
+        if constexpr (MORE) {
+            if (tile_first_no + n < kept_tiles) return (tile_first_no + n) * AP_BN;
+        }
+        return k_share + n * AP_BN;
+    };
+    const int k_first = key_of(0);
+    const int k_end = tile_first_no < tile_end_no ? key_of(tile_end_no - 1 - tile_first_no) + AP_BN : k_first;
     if (k_first >= k_end) {          // more splits than key tiles: nothing to add
         if (kt0 == 0 && q_ok) {
             float* ml = part_ml + ((static_cast<size_t>(row0 + wq) * nq + q_head) * splits + split) * 2;
@@ -447,7 +486,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
     const uint32_t page_bytes = static_cast<uint32_t>(block_size) * row_bytes;
     auto ask = [&]() {               // pages from kblk/kwithin, looked up before
         if constexpr (DIRECT) {
-            const int tile_first = k_first + asked * AP_BN;
+            const int tile_first = key_of(asked);
             const bool at_an_edge = tile_first + AP_BN - 1 > last_pos || tile_first < first_pos;
 #pragma unroll
             for (int i = 0; i < KI; ++i) {
@@ -458,7 +497,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
                 const char* gv = reinterpret_cast<const char*>(v_pool) + base + place_v[ROWS_ALTERNATE ? i & 1 : 0];
                 if (at_an_edge && (kj0[i] + 64 / CP - 1 > last_pos || kj0[i] < first_pos)) {   // (the same for the wave)
                     const int j = kj0[i] + lane / CP;
-                    if (j > last_pos || j < first_pos)
+                    if (j > last_pos || gone(j))
                         gv = reinterpret_cast<const char*>(v_pool) + last_base + piece_v[ROWS_ALTERNATE ? i & 1 : 0];
                 }
                 uint16_t* lk = Kbase + asked_k * KTILE + first_row * KROW;
@@ -483,20 +522,20 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
         lookup(k_first);
         ask();
         if constexpr (AHEAD == 2) {
-            lookup(k_first + AP_BN);
+            lookup(key_of(1));
             ask();
         }
-        lookup(k_first + AHEAD * AP_BN);         // for the first round's asking
+        lookup(key_of(AHEAD));         // for the first round's asking
         __builtin_amdgcn_s_waitcnt(0x0F70);      // vmcnt(0): the first tiles have landed
         __builtin_amdgcn_s_barrier();
         asm volatile("" ::: "memory");
     } else {
         lookup(k_first);
         fetch();
-        lookup(k_first + AP_BN);
+        lookup(key_of(1));
         stash(0, 0);
         fetch();                         // the second tile, all zeros past the last key
-        lookup(k_first + 2 * AP_BN);
+        lookup(key_of(2));
         __syncthreads();
     }
     // The registers hold tile `staged`: it goes into buffers that nobody reads now, the tile after it
@@ -508,7 +547,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
             if constexpr (UP) {
                 take_pages();
             } else {
-                lookup(k_first + (staged + 2) * AP_BN);
+                lookup(key_of(staged + 2));
             }
             ++staged;
             staged_v = staged_v + 1 == NVB ? 0 : staged_v + 1;
@@ -619,6 +658,15 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
         // (and c > reach - seen, seen the keys from the first one the query sees to its own); it stands
         // reach - c positions before the query.
         const int reach = q_pos - k0 - 32 * kt0 - 4 * h;
+        if constexpr (MORE) {
+            if (cap_out != 0.f) {
+#pragma unroll
+                for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+                    for (int r = 0; r < 16; ++r)
+                        s[kt][r] = fmaf(-2.f * cap_out, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[kt][r] * cap_in) + 1.f), cap_out);
+            }
+        }
         if (tilted) {
             const float from = -tilt * static_cast<float>(reach);
 #pragma unroll
@@ -628,13 +676,14 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
                     s[kt][r] += fmaf(tilt, static_cast<float>(32 * kt + 8 * (r >> 2) + (r & 3)), from);
         }
         if (masked) {
+            const int kept_below = keep_first - k0 - 32 * kt0 - 4 * h;
             const int behind = window != 0 ? reach - (q_pos - pl_first_visible(q_pos, window) + 1) : -(1 << 30);
 #pragma unroll
             for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int c = 32 * kt + 8 * (r >> 2) + (r & 3);
-                    s[kt][r] = (c <= reach && c > behind) ? s[kt][r] : -INFINITY;
+                    s[kt][r] = (c <= reach && (c > behind || (MORE && c < kept_below))) ? s[kt][r] : -INFINITY;
                 }
         }
 #pragma unroll
@@ -696,11 +745,11 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
     auto feed_before = [&]() {
         if constexpr (DIRECT) {
             ask();
-            look_ahead(k_first + asked * AP_BN);
+            look_ahead(key_of(asked));
         }
     };
     if (behind_group) {              // half a round in which the later group only moves a tile
-        look_ahead(k_first + (staged + 2) * AP_BN);
+        look_ahead(key_of(staged + 2));
         advance();
         if (ask_late) feed_before();
         half_done();
@@ -735,7 +784,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
     // few tiles around the diagonal, where keys are hidden and waves of early tokens are done.
     // A tile that left no probabilities (the one before the first, one a wave sat out) left zeros:
     // the values are multiplied in every round.
-    int k0 = k_first, kbuf = 0, vbuf_before = 0;   // vbuf_before: where the values of the tile before lie
+    int k0 = k_first, tile_now = 0, kbuf = 0, vbuf_before = 0;   // vbuf_before: where the values of the tile before lie
     auto no_weights = [&]() {
 #pragma unroll
         for (int kt = 0; kt < KT; ++kt)
@@ -748,7 +797,8 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
     const int open_end = window != 0 ? k_first : ((start + q0 + 1) / AP_BN) * AP_BN;   // keys below it are seen by all
     auto next_tile = [&]() {
         if (k0 != k_first) vbuf_before = vbuf_before + 1 == NVB ? 0 : vbuf_before + 1;
-        k0 += AP_BN;
+        ++tile_now;
+        k0 = MORE ? key_of(tile_now) : k0 + AP_BN;
         kbuf = kbuf + 1 == NKB ? 0 : kbuf + 1;
     };
     const int open_stop = min(open_end, k_end);
@@ -757,7 +807,7 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
         multiply(kbuf, vbuf_before, true);
         feed_after();
         half_done();
-        if constexpr (!DIRECT) look_ahead(k_first + (staged + 2) * AP_BN);
+        if constexpr (!DIRECT) look_ahead(key_of(staged + 2));
         if (ask_late) feed_before();
         soften(k0, false);
         advance();
@@ -767,12 +817,13 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
     for (; k0 < k_end; next_tile()) {
         // a wave whose queries all stand before this tile, or that has no queries, has nothing to add
         const bool idle = !wave_active || k0 + 32 * kt0 > wave_last ||
-                          (window != 0 && k0 + 32 * (kt0 + KT) - 1 < pl_first_visible(wave_first, window));
+                          (window != 0 && k0 + 32 * (kt0 + KT) - 1 < pl_first_visible(wave_first, window) &&
+                           !(MORE && k0 + 32 * kt0 < keep_first));
         if (!ask_late) feed_before();
         multiply(kbuf, vbuf_before, !idle);
         feed_after();
         half_done();
-        if constexpr (!DIRECT) look_ahead(k_first + (staged + 2) * AP_BN);
+        if constexpr (!DIRECT) look_ahead(key_of(staged + 2));
         if (ask_late) feed_before();
         if (!idle) soften(k0, true);
         else no_weights();
@@ -836,7 +887,10 @@ paged_attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_
         stays = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m * scale_log2e - top);
         total = lsum * stays + __builtin_amdgcn_exp2f(sk - top);
     }
-    const float inv = total > 0.f ? stays / total : 0.f;
+    float inv = total > 0.f ? stays / total : 0.f;
+    if constexpr (MORE) {
+        if (with.more.gate != nullptr) inv *= pl_head_gate(with.more, row0 + wq, q_head);
+    }
     bf16_t* orow = out + (static_cast<size_t>(row0 + wq) * nq + q_head) * d;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
@@ -865,7 +919,7 @@ paged_attention_prefill_merge_kernel(const float* __restrict__ part_acc, const f
                                           bf16_t* __restrict__ out, const int* __restrict__ q_start,
                                           const int* __restrict__ q_len, const int* __restrict__ ctx_len,
                                           int short_limit, int num_seqs, int nq, int d, int splits, int total_rows,
-                                          int grouped, const float* __restrict__ sinks) {
+                                          int grouped, const float* __restrict__ sinks, PlAttentionMore more) {
     const int quads = d / 4, rows = blockDim.x / quads;
     const int r = blockIdx.x * rows + threadIdx.x / quads;
     const int head = blockIdx.y;
@@ -924,7 +978,8 @@ paged_attention_prefill_merge_kernel(const float* __restrict__ part_acc, const f
         keep = big == -INFINITY ? 0.f : exp2f(big - top);
         sum = sum * keep + exp2f(sk - top);
     }
-    const float inv = sum > 0.f ? keep / sum : 0.f;
+    float inv = sum > 0.f ? keep / sum : 0.f;
+    if (more.gate != nullptr) inv *= pl_head_gate(more, r, head);
     ap_u32x2 w;
     w.v[0] = ap_pack2(a[0] * inv, a[1] * inv);
     w.v[1] = ap_pack2(a[2] * inv, a[3] * inv);
@@ -936,7 +991,8 @@ static int launch_prefill(const void* q, int q_stride, void* out, const int* q_s
                           const int* ctx_len, int short_limit, int num_seqs, int max_q_len, const int* block_table,
                           int max_blocks, int block_size, const void* k_pool, const void* v_pool, int nq, int nkv,
                           int d, float scale, int window, int splits, float* part_acc, float* part_ml,
-                          int total_rows, int short_rows, const float* sinks, const float* slopes, hipStream_t stream) {
+                          int total_rows, int short_rows, const float* sinks, const float* slopes,
+                          const PlAttentionMore& more, hipStream_t stream) {
     constexpr int DP = 32 * DT;
     constexpr int BM = 32 * NW;
     const size_t tile_bytes = FEED == 2 ? (2 * ap_direct_ahead(GR) + 3) * static_cast<size_t>(AP_BN) * DP * 2
@@ -945,8 +1001,9 @@ static int launch_prefill(const void* q, int q_stride, void* out, const int* q_s
     const size_t hand_bytes = KS == 2 ? static_cast<size_t>(NW) * (16 * DT + 2) * PL_WAVE * sizeof(float) : 0;
     const size_t lds_bytes = tile_bytes > hand_bytes ? tile_bytes : hand_bytes;
     if (lds_bytes > 48 * 1024) {
-        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&paged_attention_prefill_kernel<DT, NW, KS, FEED, GR>),
-                                           hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds_bytes));
+        const void* kernel = pl_has_more(more) ? reinterpret_cast<const void*>(&paged_attention_prefill_kernel<DT, NW, KS, FEED, GR, true>)
+                                               : reinterpret_cast<const void*>(&paged_attention_prefill_kernel<DT, NW, KS, FEED, GR, false>);
+        hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds_bytes));
         PL_REQUIRE(e == hipSuccess, "prefill attention: %zu bytes of LDS refused: %s", lds_bytes, hipGetErrorString(e));
     }
     const int tiles = GR ? max_q_len : pl_ceil_div(max_q_len, BM);
@@ -968,18 +1025,22 @@ static int launch_prefill(const void* q, int q_stride, void* out, const int* q_s
     }
     const long long total = whole * splits;
     PL_REQUIRE(total > 0 && total < (1ll << 30), "prefill attention: %lld workgroups", total);
-    paged_attention_prefill_kernel<DT, NW, KS, FEED, GR><<<static_cast<int>(total), 64 * NW * KS, lds_bytes, stream>>>(
-        static_cast<const bf16_t*>(q), q_stride, static_cast<bf16_t*>(out), q_start, q_len, ctx_len, short_limit, tiles,
-        num_seqs, block_table, max_blocks, block_size, static_cast<const bf16_t*>(k_pool),
-        static_cast<const bf16_t*>(v_pool), nq, nkv, d, scale * 1.4426950408889634f, window, static_cast<int>(total),
-        splits, part_acc, part_ml, compact, sinks, slopes);
+#define AP_KERNEL(MORE, WITH)                                                                                            \
+    paged_attention_prefill_kernel<DT, NW, KS, FEED, GR, MORE><<<static_cast<int>(total), 64 * NW * KS, lds_bytes, stream>>>( \
+        static_cast<const bf16_t*>(q), q_stride, static_cast<bf16_t*>(out), q_start, q_len, ctx_len, short_limit, tiles,   \
+        num_seqs, block_table, max_blocks, block_size, static_cast<const bf16_t*>(k_pool),                                 \
+        static_cast<const bf16_t*>(v_pool), nq, nkv, d, scale * 1.4426950408889634f, window, static_cast<int>(total),      \
+        splits, part_acc, part_ml, compact, sinks, slopes, WITH)
+    if (pl_has_more(more)) AP_KERNEL(true, ap_more_t<true>{more});
+    else AP_KERNEL(false, ap_more_t<false>{});
+#undef AP_KERNEL
     PL_CHECK_LAUNCH("paged_attention_prefill");
     if (splits > 1) {
         const int rows = 256 / (d / 4);
 #define AP_MERGE(SP)                                                                                               \
     paged_attention_prefill_merge_kernel<SP><<<dim3(pl_ceil_div(total_rows, rows), nq), 256, 0, stream>>>(         \
         part_acc, part_ml, static_cast<bf16_t*>(out), q_start, q_len, ctx_len, short_limit, num_seqs, nq, d, splits, \
-        total_rows, GR ? 1 : 0, sinks)
+        total_rows, GR ? 1 : 0, sinks, more)
         if (splits <= 2) AP_MERGE(2);
         else if (splits <= 4) AP_MERGE(4);
         else if (splits <= 8) AP_MERGE(8);
@@ -995,11 +1056,11 @@ static int ap_dispatch(bool small, bool uniform_pages, const void* q, int q_stri
                        const int* q_len, const int* ctx_len, int short_limit, int num_seqs, int max_q_len,
                        const int* block_table, int max_blocks, int block_size, const void* k_pool, const void* v_pool,
                        int nq, int nkv, int d, float scale, int window, int splits, float* part_acc, float* part_ml,
-                       int total_rows, const float* sinks, const float* slopes, hipStream_t stream) {
+                       int total_rows, const float* sinks, const float* slopes, const PlAttentionMore& more, hipStream_t stream) {
 #define AP_LAUNCH(NW, KS, FEED)                                                                                    \
     launch_prefill<D, NW, KS, FEED>(q, q_stride, out, q_start, q_len, ctx_len, short_limit, num_seqs, max_q_len,    \
                                     block_table, max_blocks, block_size, k_pool, v_pool, nq, nkv, d, scale, window, \
-                                    splits, part_acc, part_ml, total_rows, 0, sinks, slopes, stream)
+                                    splits, part_acc, part_ml, total_rows, 0, sinks, slopes, more, stream)
     constexpr bool can_fit = 64 % (4 * D) == 0;
     constexpr int BEST = (D == 2 || D == 4) && AP_KS == 2 && AP_SMALL_KS == 2 ? AP_FEED : 1;   // the feed with uniform pages
     if constexpr (D <= 4) {
@@ -1022,6 +1083,11 @@ static int ap_dispatch(bool small, bool uniform_pages, const void* q, int q_stri
 #undef AP_LAUNCH
 }
 
+static bool ap_more_fits(const PlAttentionMore& more, int nq, int window, float scale) {
+    return more.cap >= 0.f && more.keep >= 0 && (more.gate == nullptr || more.gate_stride >= nq) && (more.keep == 0 || window >= 0) &&
+           (more.cap == 0.f || scale != 0.f);
+}
+
 // bfloat16 only.  q rows begin with the nq*d rotated query values; request s brings the rows
 // q_start[s] .. q_start[s] + q_len[s] - 1, which stand at the positions ctx_len[s] - q_len[s] .. ctx_len[s] - 1.
 // Requests with q_len < short_limit are skipped.  max_q_len bounds q_len over the requests.
@@ -1039,7 +1105,11 @@ extern "C" int pl_paged_attention_prefill(const void* q, int q_stride, void* out
                                           int max_q_len, const int* block_table, int max_blocks, int block_size,
                                           const void* k_pool, const void* v_pool, int nq, int nkv, int d,
                                           float scale, int window, int splits, float* part_acc, float* part_ml,
-                                          int total_rows, const float* sinks, const float* slopes, hipStream_t stream) {
+                                          int total_rows, const float* sinks, const float* slopes, float cap, int keep,
+                                          const float* gate, int gate_stride, hipStream_t stream) {
+    const PlAttentionMore more{cap, keep, gate, gate_stride};
+    PL_REQUIRE(ap_more_fits(more, nq, window, scale), "prefill attention: a cap of %g, %d first keys kept beside a window of %d, gates in rows of %d",
+               static_cast<double>(cap), keep, window, gate_stride);
     PL_REQUIRE(splits >= 1 && splits <= AP_MERGE_MAX && (splits == 1 || (part_acc && part_ml)),
                "prefill attention: %d splits%s", splits, splits > 1 ? " without a workspace" : "");
     PL_REQUIRE(d > 0 && d <= 256 && d % 16 == 0, "prefill attention: head size %d, which has to be a multiple of 16 up to 256", d);
@@ -1066,7 +1136,7 @@ extern "C" int pl_paged_attention_prefill(const void* q, int q_stride, void* out
 #define AP_CALL(D)                                                                                                 \
     return ap_dispatch<D>(small, pages_fit, q, q_stride, out, q_start, q_len, ctx_len, short_limit, num_seqs, max_q_len, \
                           block_table, max_blocks, block_size, k_pool, v_pool, nq, nkv, d, scale, window, splits,   \
-                          part_acc, part_ml, total_rows, sinks, slopes, stream)
+                          part_acc, part_ml, total_rows, sinks, slopes, more, stream)
     switch (dt) {
         case 1: AP_CALL(1);
         case 2: AP_CALL(2);
@@ -1107,11 +1177,11 @@ static int ap_dispatch_grouped(bool uniform_pages, const void* q, int q_stride, 
                                const int* block_table, int max_blocks, int block_size, const void* k_pool,
                                const void* v_pool, int nq, int nkv, int d, float scale, int window, int splits,
                                float* part_acc, float* part_ml, int total_rows, int short_rows, const float* sinks,
-                               const float* slopes, hipStream_t stream) {
+                               const float* slopes, const PlAttentionMore& more, hipStream_t stream) {
 #define AP_GROUPED(FEED)                                                                                           \
     launch_prefill<D, 4, 1, FEED, true>(q, q_stride, out, q_start, q_len, ctx_len, short_limit, num_seqs, max_q_len, \
                                         block_table, max_blocks, block_size, k_pool, v_pool, nq, nkv, d, scale,    \
-                                        window, splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, stream)
+                                        window, splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, more, stream)
     constexpr bool can_fit = 64 % (4 * D) == 0;
     if constexpr (can_fit) {
         if (uniform_pages) return AP_GROUPED(1);
@@ -1126,7 +1196,10 @@ extern "C" int pl_paged_attention_grouped(const void* q, int q_stride, void* out
                                           const void* k_pool, const void* v_pool, int nq, int nkv, int d,
                                           float scale, int window, int splits, float* part_acc, float* part_ml,
                                           int total_rows, int short_rows, const float* sinks, const float* slopes,
-                                          hipStream_t stream) {
+                                          float cap, int keep, const float* gate, int gate_stride, hipStream_t stream) {
+    const PlAttentionMore more{cap, keep, gate, gate_stride};
+    PL_REQUIRE(ap_more_fits(more, nq, window, scale), "grouped attention: a cap of %g, %d first keys kept beside a window of %d, gates in rows of %d",
+               static_cast<double>(cap), keep, window, gate_stride);
     PL_REQUIRE(pl_paged_attention_grouped_applies(nq, nkv, d, block_size),
                "grouped attention: %d query heads over %d key heads of %d, pages of %d", nq, nkv, d, block_size);
     PL_REQUIRE(splits >= 1 && splits <= AP_MERGE_MAX && (splits == 1 || (part_acc && part_ml)),
@@ -1145,7 +1218,7 @@ extern "C" int pl_paged_attention_grouped(const void* q, int q_stride, void* out
 #define AP_CALL(D)                                                                                                 \
     return ap_dispatch_grouped<D>(pages_fit, q, q_stride, out, q_start, q_len, ctx_len, short_limit, num_seqs, max_q_len, \
                                   block_table, max_blocks, block_size, k_pool, v_pool, nq, nkv, d, scale, window,  \
-                                  splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, stream)
+                                  splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, more, stream)
         switch (dt) {
             case 1: AP_CALL(1);
             case 2: AP_CALL(2);
@@ -1161,8 +1234,8 @@ extern "C" int pl_paged_attention_grouped(const void* q, int q_stride, void* out
     if (d == 64)
         return launch_prefill<2, 1, 2, 2, true>(q, q_stride, out, q_start, q_len, ctx_len, short_limit, num_seqs, max_q_len,
                                                 block_table, max_blocks, block_size, k_pool, v_pool, nq, nkv, d, scale,
-                                                window, splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, stream);
+                                                window, splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, more, stream);
     return launch_prefill<4, 1, 2, 2, true>(q, q_stride, out, q_start, q_len, ctx_len, short_limit, num_seqs, max_q_len,
                                             block_table, max_blocks, block_size, k_pool, v_pool, nq, nkv, d, scale,
-                                            window, splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, stream);
+                                            window, splits, part_acc, part_ml, total_rows, short_rows, sinks, slopes, more, stream);
 }

@@ -76,6 +76,10 @@ __device__ __forceinline__ float block_sum(float v, float* scratch /* >= 16 floa
 #define PL_ACT_SILU 0
 #define PL_ACT_GELU_TANH 1
 #define PL_ACT_GELU 2
+#define PL_ACT_RELU2 3        // max(x, 0)^2
+// What a gated feed-forward may do to gate and up together instead of act(gate) * up (pl_gate_pair alone takes it):
+// with g = min(gate, limit) and u = max(min(up, limit), -limit), g sigmoid(1.702 g) (u + 1).
+#define PL_ACT_CLAMPED 4
 
 // EXACT: the library's exponential (what the 32-bit path needs); otherwise the hardware's.  `act` is the
 // same for a whole launch.
@@ -83,7 +87,22 @@ template <bool EXACT>
 __device__ __forceinline__ float pl_activate(float g, int act) {
     if (act == PL_ACT_SILU) return g / (1.f + (EXACT ? expf(-g) : __expf(-g)));
     if (act == PL_ACT_GELU_TANH) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+    if (act == PL_ACT_RELU2) {
+        const float r = fmaxf(g, 0.f);
+        return r * r;
+    }
     return 0.5f * g * (1.f + erff(g * 0.7071067811865476f));
+}
+
+// What stands between the products of a gated feed-forward: act(gate) * up, or the clamped pair of PL_ACT_CLAMPED.
+template <bool EXACT>
+__device__ __forceinline__ float pl_gate_pair(float gate, float up, int act, float limit) {
+    if (act == PL_ACT_CLAMPED) {
+        const float g = fminf(gate, limit), u = fmaxf(fminf(up, limit), -limit);
+        const float e = EXACT ? expf(-1.702f * g) : __expf(-1.702f * g);
+        return g / (1.f + e) * (u + 1.f);
+    }
+    return pl_activate<EXACT>(gate, act) * up;
 }
 
 // ---- the error channel -------------------------------------------------------
@@ -119,4 +138,18 @@ __host__ __device__ static inline int pl_first_visible(int pos, int window) {
     if (window > 0) return pos + 1 > window ? pos + 1 - window : 0;
     if (window < 0) return pos - pos % (-window);
     return 0;
+}
+
+// What an attention layer may have beside its mask, its sinks and its distance slopes; all off by default.
+struct PlAttentionMore {
+    float cap;            // > 0: a scaled score s becomes cap * tanh(s / cap), before the distance penalty
+    int keep;             // the keys 0 .. keep - 1 of a request are seen by every later query, whatever the window
+    const float* gate;    // [rows, gate_stride]: head h's read-out of row t times sigmoid(gate[t, h]); null: none
+    int gate_stride;
+};
+
+static inline bool pl_has_more(const PlAttentionMore& m) { return m.cap > 0.f || m.keep > 0 || m.gate != nullptr; }
+
+__device__ __forceinline__ float pl_head_gate(const PlAttentionMore& m, int row, int head) {
+    return 1.f / (1.f + expf(-m.gate[static_cast<size_t>(row) * m.gate_stride + head]));
 }

@@ -393,7 +393,7 @@ extern "C" int pl_delta_chunked(const float* qkv, int qkv_stride, int q_off, int
     PL_REQUIRE(Kn != nullptr && Qn != nullptr && Tm != nullptr && Aq != nullptr && scal != nullptr, "delta_chunked: no room for the chunks");
     PL_REQUIRE(seqs >= 0 && seqs <= 65535 && H <= 65535, "delta_chunked: %d requests, %d heads", seqs, H);
     if (seqs == 0 || max_q_len < from) return 0;
-    DeltaArgs da{{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, a_log, dt_bias, 0.f, state,
+    DeltaArgs da{{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, a_log, dt_bias, nullptr, 0.f, state,
                   state_stride, 0, 0, 0, out, q_start, q_len, state_slots, H, G, D, V, from},
                  Kn, Qn, Tm, Aq, scal};
     return D <= 128 ? launch_delta<64>(da, seqs, max_q_len, stream) : launch_delta<32>(da, seqs, max_q_len, stream);

@@ -684,7 +684,7 @@ swiglu_wide_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t 
 
 extern "C" int pl_swiglu(const void* gu, void* out, int n, int I, int dtype, int act, hipStream_t stream) {
     PL_REQUIRE(n >= 0 && I > 0, "swiglu: rows %d, width %d", n, I);
-    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_GELU, "swiglu: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_RELU2, "swiglu: activation code %d", act);
     const size_t count = static_cast<size_t>(n) * I;
     if (count == 0) return 0;
     if (I % 8 == 0 && (dtype == PL_DTYPE_F32 || dtype == PL_DTYPE_BF16)) {

@@ -27,7 +27,7 @@ extern "C" int pl_gemm_skinny(const void* x, const void* w, void* y, const float
     PL_REQUIRE(gain || !rows, "skinny product: a row list without a norm");
     PL_REQUIRE(epilogue != EPI_SWIGLU || !out_f32, "skinny product: the activation is stored in bfloat16");
     PL_REQUIRE(!(gain && epilogue == EPI_ADD), "skinny product: a product that reads the residual stream cannot add into it");
-    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_GELU, "skinny product: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_RELU2, "skinny product: activation code %d", act);
     if (n == 0) return 0;
     PL_REQUIRE(!strips || sk_strips_apply(n, N_out, K),
                "skinny product: %d rows, %d columns, width %d are not read from weights in strips", n, N_out, K);
@@ -56,7 +56,7 @@ extern "C" int pl_gemm_skinny_hand(const void* x, const void* w, void* y, int n,
     PL_REQUIRE(epilogue >= EPI_STORE && epilogue <= EPI_ADD, "skinny product: epilogue code %d", epilogue);
     PL_REQUIRE(epilogue != EPI_ADD || out_f32, "skinny product: the residual stream is 32-bit");
     PL_REQUIRE(epilogue != EPI_SWIGLU || !out_f32, "skinny product: the activation is stored in bfloat16");
-    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_GELU, "skinny product: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_RELU2, "skinny product: activation code %d", act);
     PL_REQUIRE(!ssq_parts || (parts > 0 && sk_hand_applies(n, N_out, K, epilogue, true)),
                "skinny product: %d rows, %d columns, width %d take no handed norm (%d sums a row)", n, N_out, K, parts);
     PL_REQUIRE((hand_x != nullptr) == (hand_ssq != nullptr) && (hand_x != nullptr) == (hand_gain != nullptr),

@@ -366,7 +366,7 @@ extern "C" int pl_gemm_stream(const void* x, const void* w, void* y, float* ws, 
     PL_REQUIRE(epilogue >= 0 && epilogue <= 2, "streamed product: epilogue %d", epilogue);
     PL_REQUIRE(splits >= 1 && splits <= GS_MAX_SPLITS && (splits == 1 || ws != nullptr),
                "streamed product: %d stretches of K (%d at most), which need a workspace", splits, GS_MAX_SPLITS);
-    PL_REQUIRE(act == PL_ACT_SILU || act == PL_ACT_GELU_TANH || act == PL_ACT_GELU, "streamed product: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_RELU2, "streamed product: activation code %d", act);
     PL_REQUIRE(static_cast<long long>(N_out) * (epilogue == 1 ? 2 : 1) <= 0x7fffffffLL / 2, "streamed product: %d columns", N_out);
     const int mode = epilogue == 1 ? GS_SWIGLU : (epilogue == 2 ? GS_ADD : (out_f32 ? GS_STORE_F32 : GS_STORE_BF16));
     const bf16_t* xb = static_cast<const bf16_t*>(x);
@@ -388,7 +388,7 @@ extern "C" int pl_gemm_finish(const float* ws, void* y, long long n, int N_out, 
     PL_REQUIRE(n > 0 && N_out > 0 && splits >= 1 && splits <= 64 && ws != nullptr && y != nullptr,
                "sum of partial products: %lld rows, %d columns, %d parts", n, N_out, splits);
     PL_REQUIRE(epilogue >= 0 && epilogue <= 2, "sum of partial products: epilogue %d", epilogue);
-    PL_REQUIRE(act == PL_ACT_SILU || act == PL_ACT_GELU_TANH || act == PL_ACT_GELU, "sum of partial products: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_RELU2, "sum of partial products: activation code %d", act);
     PL_REQUIRE(n * N_out < (1ll << 31) * 256 && n <= 0x7fffffff, "sum of partial products: %lld x %d results", n, N_out);
     const int Nw = epilogue == 1 ? 2 * N_out : N_out;
     const int mode = epilogue == 1 ? GS_SWIGLU : (epilogue == 2 ? GS_ADD : (out_f32 ? GS_STORE_F32 : GS_STORE_BF16));

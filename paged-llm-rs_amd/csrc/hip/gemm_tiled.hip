@@ -45,6 +45,7 @@ struct GtGroups {
     // of y (`y_split_stride` elements apart); whoever reads y adds the copies in their order.
     int splits;
     long long y_split_stride;
+    float limit;               // of the clamped gate (PL_ACT_CLAMPED)
 };
 
 // 16 bytes a lane from global memory straight into LDS (see attention_prefill.hip: assembly, so that
@@ -229,7 +230,8 @@ gemm_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, vo
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const float g = acc[0][mb][4 * j + i];
-                    v[i] = pl_activate<false>(g, act) * acc[1][mb][4 * j + i];
+                    if constexpr (GROUPED) v[i] = pl_gate_pair<false>(g, acc[1][mb][4 * j + i], act, groups.limit);
+                    else v[i] = pl_activate<false>(g, act) * acc[1][mb][4 * j + i];
                 }
                 uint2 packed;
                 packed.x = gt_pack2(v[0], v[1]);
@@ -304,7 +306,7 @@ static int gt_launch(const void* x, const void* w, void* y, int M, int N, int K,
     }
     gemm_tiled_kernel<EPI><<<static_cast<int>(total), 256, lds_bytes, stream>>>(
         static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), y, M, N, K, row_tiles, static_cast<int>(total), act,
-        GtGroups{nullptr, nullptr, 0, 1, 0});
+        GtGroups{nullptr, nullptr, 0, 1, 0, 0.f});
     PL_CHECK_LAUNCH("gemm_tiled");
     return 0;
 }
@@ -341,14 +343,14 @@ static int gt_launch_grouped(const void* x, const void* w, void* y, int row_tile
 // splits > 1 (epilogue 3 only): y has that many copies, [splits][row_tiles * 128, N], a stretch of K each.
 extern "C" int pl_gemm_tiled_grouped(const void* x, const void* w, void* y, const int* tile_group, const int* gather,
                                      long long w_stride, int row_tiles, int x_rows, int N, int K, int epilogue, int act,
-                                     int splits, hipStream_t stream) {
+                                     int splits, float limit, hipStream_t stream) {
     PL_REQUIRE(splits >= 1 && splits <= K / GT_BK && (splits == 1 || epilogue == GT_STORE32),
                "grouped tiled product: %d stretches of an inner width of %d, epilogue %d", splits, K, epilogue);
-    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_GELU, "grouped tiled product: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_CLAMPED, "grouped tiled product: activation code %d", act);
     PL_REQUIRE(row_tiles > 0 && x_rows > 0 && N > 0 && K > 0 && K % GT_BK == 0 && N % 8 == 0 && (epilogue != GT_SWIGLU || N % (GT_BN / 2) == 0),
                "grouped tiled product: %d tiles of rows, %d columns, inner width %d, epilogue %d", row_tiles, N, K, epilogue);
     PL_REQUIRE(tile_group != nullptr && (gather != nullptr || x_rows >= row_tiles * GT_BM), "grouped tiled product: %d rows for %d tiles", x_rows, row_tiles);
-    const GtGroups groups{tile_group, gather, w_stride, splits, static_cast<long long>(row_tiles) * GT_BM * N};
+    const GtGroups groups{tile_group, gather, w_stride, splits, static_cast<long long>(row_tiles) * GT_BM * N, limit};
     if (epilogue == GT_SWIGLU) return gt_launch_grouped<GT_SWIGLU>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
     if (epilogue == GT_STORE32) return gt_launch_grouped<GT_STORE32>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
     if (epilogue == GT_STORE) return gt_launch_grouped<GT_STORE>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
@@ -366,7 +368,7 @@ extern "C" int pl_gemm_tiled_applies(int M, int N, int K, int epilogue) {
 // x: bfloat16 [M, K].  w: bfloat16 [N, K], or [2 N, K] with the gate rows first for epilogue 1.
 // epilogue 0: y (bfloat16 [M, N]) = result.  1: y = act(gate) * up (act: PL_ACT_*).  2: y (32-bit [M, N]) += result.
 extern "C" int pl_gemm_tiled(const void* x, const void* w, void* y, int M, int N, int K, int epilogue, int act, hipStream_t stream) {
-    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_GELU, "tiled product: activation code %d", act);
+    PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_RELU2, "tiled product: activation code %d", act);
     PL_REQUIRE(pl_gemm_tiled_applies(M, N, K, epilogue), "tiled product: %d rows, %d columns, inner width %d, epilogue %d", M, N,
                K, epilogue);
     if (epilogue == GT_SWIGLU) return gt_launch<GT_SWIGLU>(x, w, y, M, N, K, act, stream);

@@ -4,7 +4,8 @@
 // where they have any): q and k divided by
 // their root mean square over the head (optional, with an optional gain), the rotation of a stretch of the
 // head (optional: value 2i with value 2i + 1, from tables of cosines and sines), q times a temperature that
-// grows with the logarithm of the position (optional), then q into the query buffer and k and v into the
+// grows with the logarithm of the position (optional), v mixed with an earlier layer's values of the same token
+// (optional), then q into the query buffer and k and v into the
 // request's pages.  Heads are stored in rows of Dp values with zeros behind a head's own size, so that query,
 // key and value heads of different sizes share the attention kernels' one head size.
 //
@@ -39,6 +40,11 @@ struct HeadPrepareArgs {
     void* k_pool;             // [pages * block_size, G * Dp]
     void* v_pool;
     int H, G, D, V, Dp;
+    // values mixed with those of an earlier layer: v <- (1 - mix) v + mix (first + first_bias)
+    const float* first;       // [n, first_stride]: the earlier layer's projected values from its first column on, or null
+    int first_stride;
+    const float* first_bias;  // [G V] or null
+    float mix;
 };
 
 // A wave a token and head (a query head, a key head or a value head).
@@ -59,7 +65,13 @@ __global__ __launch_bounds__(64) void head_prepare_kernel(HeadPrepareArgs a) {
 
     float ss = 0.f;
     for (int e = lane; e < width; e += 64) {
-        const float x = bias != nullptr ? src[e] + bias[e] : src[e];
+        float x = bias != nullptr ? src[e] + bias[e] : src[e];
+        if (kind == 2 && a.first != nullptr) {
+            const int c = index * V + e;
+            float other = a.first[static_cast<size_t>(t) * a.first_stride + c];
+            if (a.first_bias != nullptr) other += a.first_bias[c];
+            x = (1.f - a.mix) * x + a.mix * other;
+        }
         head[e] = x;
         ss += x * x;
     }
@@ -110,7 +122,8 @@ extern "C" int pl_head_prepare(const float* rows, const float* bias, int stride,
                                int table_rows, int tempered, float temp_coef, int temp_every, const int* positions,
                                const int* seq_of, const int* block_table, int max_blocks, int block_size, int write_kv,
                                void* q_out, void* k_pool, void* v_pool, int dtype, int n, int H, int G, int D, int V,
-                               int Dp, hipStream_t stream) {
+                               int Dp, const float* first, int first_stride, const float* first_bias, float mix, hipStream_t stream) {
+    PL_REQUIRE(first == nullptr || first_stride >= G * V, "head_prepare: values of %d to mix with, from rows of %d", G * V, first_stride);
     PL_REQUIRE(n >= 0 && H > 0 && G > 0 && H % G == 0 && H + 2 * G <= 65535, "head_prepare: rows %d, %d query heads over %d key heads", n, H, G);
     PL_REQUIRE(D > 0 && V > 0 && Dp >= D && Dp >= V && Dp <= 1024, "head_prepare: heads of %d and %d in rows of %d (up to 1024)", D, V, Dp);
     PL_REQUIRE(rot >= 0 && rot % 2 == 0 && rot_off >= 0 && rot_off + rot <= D && (rot == 0 || (cos != nullptr && sin != nullptr && table_rows > 0)),
@@ -120,7 +133,7 @@ extern "C" int pl_head_prepare(const float* rows, const float* bias, int stride,
     if (n == 0) return 0;
     HeadPrepareArgs a{rows, bias, stride, off, unit, eps, q_gain, k_gain, cos, sin, rot_off, rot, table_rows, tempered, temp_coef,
                       temp_every, positions, seq_of, block_table, max_blocks, block_size, write_kv, q_out, k_pool, v_pool,
-                      H, G, D, V, Dp};
+                      H, G, D, V, Dp, first, first_stride, first_bias, mix};
     const dim3 grid(n, H + 2 * G);
     if (dtype == PL_DTYPE_F32) head_prepare_kernel<float><<<grid, 64, 0, stream>>>(a);
     else if (dtype == PL_DTYPE_BF16) head_prepare_kernel<bf16_t><<<grid, 64, 0, stream>>>(a);

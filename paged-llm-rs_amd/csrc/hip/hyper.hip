@@ -242,6 +242,7 @@ struct MoeArgs {
     const int* choice;
     const float* weight;
     int identity;
+    float limit;           // of the clamped gate (PL_ACT_CLAMPED)
 };
 
 // The expert of pair (t, c), or -1: the router's choice, or the table's row of the token's id.
@@ -270,7 +271,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
     for (int f = blockIdx.y * waves + wave; f < F; f += gridDim.y * waves) {
         const float g = moe_dot<T>(gate + static_cast<size_t>(f) * W, moe_x, W, lane);
         const float u = moe_dot<T>(up + static_cast<size_t>(f) * W, moe_x, W, lane);
-        if (lane == 0) h[f] = from_float<T>(pl_activate<true>(g, a.act) * u);
+        if (lane == 0) h[f] = from_float<T>(pl_gate_pair<true>(g, u, a.act, a.limit));
     }
 }
 
@@ -311,8 +312,8 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
 extern "C" int pl_moe_rows(const void* x, const int* ids, const int* src, const int* fed, const int* positions,
                            const int* table, const void* w_gu, const void* w_down, void* h, float* out, int dtype,
                            int n, int W, int F, int E, int top, int vocab, int act, const int* choice, const float* weight,
-                           int identity, hipStream_t stream) {
-    PL_REQUIRE(n >= 0 && W > 0 && F > 0 && E > 0 && top > 0 && top <= E + identity && identity >= 0 && vocab > 0 && act >= 0 && act <= 2,
+                           int identity, float limit, hipStream_t stream) {
+    PL_REQUIRE(n >= 0 && W > 0 && F > 0 && E > 0 && top > 0 && top <= E + identity && identity >= 0 && vocab > 0 && act >= 0 && act <= PL_ACT_CLAMPED,
                "moe_rows: %d rows of %d, %d experts of %d, %d a row", n, W, E, F, top);
     PL_REQUIRE((choice != nullptr) != (table != nullptr) && (weight == nullptr || choice != nullptr),
                "moe_rows: the experts of a row are a table's or a router's");
@@ -320,7 +321,7 @@ extern "C" int pl_moe_rows(const void* x, const int* ids, const int* src, const 
     PL_REQUIRE(W <= 16384 && static_cast<long long>(top) * F <= 16384, "moe_rows: rows of %d, %d experts of %d a row", W, top, F);
     PL_REQUIRE(static_cast<long long>(n) * top < (1ll << 31), "moe_rows: %d rows", n);
     if (n == 0) return 0;
-    MoeArgs a{x, ids, src, fed, positions, table, w_gu, w_down, h, out, n, W, F, E, top, vocab, act, choice, weight, identity};
+    MoeArgs a{x, ids, src, fed, positions, table, w_gu, w_down, h, out, n, W, F, E, top, vocab, act, choice, weight, identity, limit};
     // few rows: deal an expert's rows of weights to several workgroups, so that the chip has work
     const int cu = pl_compute_units();
     int up_parts = 1, down_parts = 1;
@@ -522,7 +523,10 @@ __device__ __forceinline__ void router_dots(const T* __restrict__ w, const float
     for (int j = 0; j < 4; ++j) out[j] = wave_sum(acc[j]);
 }
 
-// A workgroup a row; its first wave chooses.  z [n, stride] are the router's 32-bit logits over `total` outputs.
+// A workgroup a row; its first wave chooses.  z [n, stride] are the router's 32-bit logits over `total` outputs; `bias`
+// [total], where there is one, is added to them first.
+// `of_chosen`: the choice goes by the logits themselves and the weights are the softmax over the chosen logits alone
+// (`correction`, `normalised` and `weight_eps` then do not enter).  Otherwise
 // s = softmax(z); the choice goes
 // by s + correction; outputs form `groups` equal groups of neighbours, a group counts by its largest choice score and
 // only members of the `kept` best groups can be chosen (the others count as minus infinity); the `top` largest are
@@ -537,7 +541,8 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
                                                             const int* __restrict__ positions, int total_all, int top, int groups_all,
                                                             int kept, int normalised, float weight_eps, int* __restrict__ choice,
                                                             float* __restrict__ weight, const T* __restrict__ x,
-                                                            const T* __restrict__ w, int W) {
+                                                            const T* __restrict__ w, int W, const float* __restrict__ bias,
+                                                            int of_chosen) {
     extern __shared__ float router_lds[];             // score [total], choice score [total], group score [groups], kept or not [groups]
     float* score = router_lds;                        // (and behind them, where the logits are worked out here: logits [total], the row [W])
     float* pick = router_lds + total_all;
@@ -573,19 +578,26 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     // (a wave that does not choose sees no outputs and no groups)
     const int total = chooser ? total_all : 0, groups = chooser ? groups_all : 0;
     float largest = -INFINITY;
-    for (int e = lane; e < total; e += PL_WAVE) largest = fmaxf(largest, row[e]);
-    largest = wave_max(largest);
-    float sum = 0.f;
     for (int e = lane; e < total; e += PL_WAVE) {
-        const float v = expf(row[e] - largest);
+        const float v = bias != nullptr ? row[e] + bias[e] : row[e];
         score[e] = v;
-        sum += v;
+        pick[e] = v;
+        largest = fmaxf(largest, v);
     }
-    sum = wave_sum(sum);
-    for (int e = lane; e < total; e += PL_WAVE) {
-        const float s = score[e] / sum;
-        score[e] = s;
-        pick[e] = correction != nullptr ? s + correction[e] : s;
+    if (!of_chosen) {
+        largest = wave_max(largest);
+        float sum = 0.f;
+        for (int e = lane; e < total; e += PL_WAVE) {
+            const float v = expf(score[e] - largest);
+            score[e] = v;
+            sum += v;
+        }
+        sum = wave_sum(sum);
+        for (int e = lane; e < total; e += PL_WAVE) {
+            const float s = score[e] / sum;
+            score[e] = s;
+            pick[e] = correction != nullptr ? s + correction[e] : s;
+        }
     }
     __syncthreads();
     if (groups_all > 1) {
@@ -616,7 +628,7 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
             if (stays[e / size] == 0.f) pick[e] = -INFINITY;
         __syncthreads();
     }
-    float chosen_sum = 0.f;
+    float chosen_sum = 0.f, first_logit = 0.f;
     for (int c = 0; c < top; ++c) {
         float v = -INFINITY;
         int at = 0x7fffffff;
@@ -629,7 +641,11 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
         }
         wave_best(v, at);
         if (at == 0x7fffffff) at = -1;               // (nothing left to choose from)
-        const float s = (chooser && at >= 0) ? score[at] : 0.f;
+        float s = (chooser && at >= 0) ? score[at] : 0.f;
+        if (of_chosen) {                             // (the first chosen logit is the largest)
+            if (c == 0) first_logit = s;
+            s = at >= 0 ? expf(s - first_logit) : 0.f;
+        }
         chosen_sum += s;
         if (chooser && lane == 0) {
             chosen[c] = at;
@@ -638,7 +654,9 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
         }
         __syncthreads();
     }
-    if (normalised && chooser) {
+    if (of_chosen && chooser) {
+        for (int c = lane; c < top; c += PL_WAVE) counts[c] = counts[c] / chosen_sum;
+    } else if (normalised && chooser) {
         for (int c = lane; c < top; c += PL_WAVE) counts[c] = counts[c] / (chosen_sum + weight_eps);
     }
 }
@@ -646,7 +664,9 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
 // z [n, stride] holds the logits, or, where it is null, x [n, W] and w [total, W] of type `dtype` give them.
 extern "C" int pl_router_select(const float* z, int stride, const float* correction, const int* positions, int n, int total,
                                 int top, int groups, int kept, int normalised, float weight_eps, int* choice, float* weight,
-                                const void* x, const void* w, int W, int dtype, hipStream_t stream) {
+                                const void* x, const void* w, int W, int dtype, const float* bias, int of_chosen,
+                                hipStream_t stream) {
+    PL_REQUIRE(!of_chosen || correction == nullptr, "router_select: a correction of scores where the logits themselves choose");
     PL_REQUIRE(n >= 0 && total > 0 && total <= 8192 && top > 0 && top <= total && (z == nullptr || stride >= total),
                "router_select: %d rows, %d of %d outputs in rows of %d", n, top, total, stride);
     PL_REQUIRE((z != nullptr) != (x != nullptr) && (x == nullptr || (w != nullptr && W > 0 && W <= 8192 && total <= 1024)),
@@ -657,17 +677,17 @@ extern "C" int pl_router_select(const float* z, int stride, const float* correct
     size_t lds = 2 * (static_cast<size_t>(total) + groups) * sizeof(float);
     if (x == nullptr) {
         router_select_kernel<float><<<n, 64, lds, stream>>>(z, stride, correction, positions, total, top, groups, kept, normalised,
-                                                            weight_eps, choice, weight, nullptr, nullptr, 0);
+                                                            weight_eps, choice, weight, nullptr, nullptr, 0, bias, of_chosen);
     } else {
         lds += (static_cast<size_t>(total) + W) * sizeof(float);
         if (dtype == PL_DTYPE_F32)
             router_select_kernel<float><<<n, 256, lds, stream>>>(nullptr, 0, correction, positions, total, top, groups, kept, normalised,
                                                                 weight_eps, choice, weight, static_cast<const float*>(x),
-                                                                static_cast<const float*>(w), W);
+                                                                static_cast<const float*>(w), W, bias, of_chosen);
         else if (dtype == PL_DTYPE_BF16)
             router_select_kernel<bf16_t><<<n, 256, lds, stream>>>(nullptr, 0, correction, positions, total, top, groups, kept, normalised,
                                                                  weight_eps, choice, weight, static_cast<const bf16_t*>(x),
-                                                                 static_cast<const bf16_t*>(w), W);
+                                                                 static_cast<const bf16_t*>(w), W, bias, of_chosen);
         else
             PL_REQUIRE(false, "router_select: dtype code %d", dtype);
     }

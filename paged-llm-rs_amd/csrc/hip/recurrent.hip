@@ -1,6 +1,7 @@
 // Mixers that carry a matrix of state from token to token instead of keys and values in pages:
-// linear attention with a fixed decay a head, the matrix memory with exponential gates, and the gated
-// delta rule; the short causal convolution with its carried history; and the norm over groups of the
+// linear attention with a fixed decay a head, the matrix memory with exponential gates, the gated
+// delta rule, and the state space whose decay and step size a token brings itself (ssd: q, k and v are its
+// C, B and x; S = e^(-e^A_log dt) S + dt k v^T, o = S^T q + D v, dt = softplus(x1 + dt_bias)); the short causal convolution with its carried history; and the norm over groups of the
 // read-out, multiplied by a gate.  States, gates, decays and read-outs are 32-bit whatever the model's
 // type is; the rows these kernels read are the 32-bit sums of the projections.
 //
@@ -65,7 +66,8 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
     }
     float decay = 0.f, a_rate = 0.f, dt_bias = 0.f, bias_i = 0.f, bias_f = 0.f;
     if (KIND == PL_SCAN_LIGHTNING) decay = a.p1[h];
-    if (KIND == PL_SCAN_DELTA) { a_rate = expf(a.p1[h]); dt_bias = a.p2[h]; }
+    if (KIND == PL_SCAN_DELTA || KIND == PL_SCAN_SSD) { a_rate = expf(a.p1[h]); dt_bias = a.p2[h]; }
+    const float skip = KIND == PL_SCAN_SSD ? a.p3[h] : 0.f;
     if (KIND == PL_SCAN_MLSTM) { bias_i = a.p1[h]; bias_f = a.p2[h]; }
     const float q_scale = 1.f / sqrtf(static_cast<float>(D));
     const int HV = H * V;
@@ -95,8 +97,12 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
         }
         if (KIND != PL_SCAN_LIGHTNING && lane < count) {
             const float* row = a.gates + static_cast<size_t>(start + c0 + lane) * a.gates_stride;
-            const float x1 = row[a.g1_off + h], x2 = row[a.g2_off + h];
-            if (KIND == PL_SCAN_MLSTM) {
+            const float x1 = row[a.g1_off + h], x2 = KIND == PL_SCAN_SSD ? 0.f : row[a.g2_off + h];
+            if (KIND == PL_SCAN_SSD) {
+                const float dt = softplus_f(x1 + dt_bias);
+                g1[lane] = dt;
+                g2[lane] = expf(-a_rate * dt);
+            } else if (KIND == PL_SCAN_MLSTM) {
                 g1[lane] = a.cap * tanhf((x1 + bias_i) / a.cap);
                 g2[lane] = logsigmoid_f(a.cap * tanhf((x2 + bias_f) / a.cap));
             } else {
@@ -151,6 +157,13 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
                         o += S[i] * q[i];
                     }
                 o = o / (fmaxf(fabsf(nq), expf(-m_new)) + 1e-6f);
+            } else if (KIND == PL_SCAN_SSD) {
+                const float keep = g2[t], dv = g1[t] * v;
+                PL_ROWS_OF_S {
+                        S[i] = keep * S[i] + k[i] * dv;
+                        o += S[i] * q[i];
+                    }
+                o += skip * v;
             } else {
                 const float beta = g1[t], gd = g2[t];
                 float mem = 0.f;
@@ -197,11 +210,12 @@ static int launch_scan(const ScanArgs& a, int seqs, hipStream_t stream) {
 
 extern "C" int pl_recurrent_scan(int kind, const float* qkv, int qkv_stride, int q_off, int k_off, int v_off,
                                  const float* gates, int gates_stride, int g1_off, int g2_off,
-                                 const float* p1, const float* p2, float cap,
+                                 const float* p1, const float* p2, const float* p3, float cap,
                                  float* state, long state_stride, int s_off, int n_off, int m_off,
                                  float* out, const int* q_start, const int* q_len, const int* state_slots,
                                  int seqs, int H, int G, int D, int V, int below, hipStream_t stream) {
-    PL_REQUIRE(kind >= 0 && kind <= 2, "recurrent_scan: kind %d", kind);
+    PL_REQUIRE(kind >= 0 && kind <= PL_SCAN_SSD, "recurrent_scan: kind %d", kind);
+    PL_REQUIRE(kind != PL_SCAN_SSD || p3 != nullptr, "recurrent_scan: what v counts in its own read-out is missing");
     PL_REQUIRE(H > 0 && G > 0 && H % G == 0, "recurrent_scan: %d heads over %d heads of q and k", H, G);
     PL_REQUIRE(D > 0 && D <= 256 && V > 0, "recurrent_scan: a state of %d by %d a head (q and k up to 256)", D, V);
     PL_REQUIRE(seqs >= 0 && seqs <= 65535 && H <= 65535, "recurrent_scan: %d requests, %d heads", seqs, H);
@@ -210,10 +224,11 @@ extern "C" int pl_recurrent_scan(int kind, const float* qkv, int qkv_stride, int
     PL_REQUIRE(kind != PL_SCAN_LIGHTNING || p1 != nullptr, "recurrent_scan: the decays are missing");
     PL_REQUIRE(kind != PL_SCAN_MLSTM || cap > 0.f, "recurrent_scan: a gate cap of %g", cap);
     if (seqs == 0) return 0;
-    ScanArgs a{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, p1, p2, cap,
+    ScanArgs a{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, p1, p2, p3, cap,
                state, state_stride, s_off, n_off, m_off, out, q_start, q_len, state_slots, H, G, D, V, below};
     if (kind == PL_SCAN_LIGHTNING) return launch_scan<PL_SCAN_LIGHTNING>(a, seqs, stream);
     if (kind == PL_SCAN_MLSTM) return launch_scan<PL_SCAN_MLSTM>(a, seqs, stream);
+    if (kind == PL_SCAN_SSD) return launch_scan<PL_SCAN_SSD>(a, seqs, stream);
     return launch_scan<PL_SCAN_DELTA>(a, seqs, stream);
 }
 
@@ -241,7 +256,8 @@ __global__ void short_conv_kernel(const float* __restrict__ rows, int stride, in
                                   const float* __restrict__ w, int taps, const float* __restrict__ state,
                                   long state_stride, int hist_off, const int* __restrict__ positions,
                                   const int* __restrict__ seq_of, const int* __restrict__ q_start,
-                                  const int* __restrict__ state_slots, float* __restrict__ out, int act) {
+                                  const int* __restrict__ state_slots, float* __restrict__ out, int act,
+                                  const float* __restrict__ bias) {
     const int t = blockIdx.x;
     const int c = blockIdx.y * blockDim.x + threadIdx.x;
     if (c >= C || positions[t] < 0) return;
@@ -249,18 +265,63 @@ __global__ void short_conv_kernel(const float* __restrict__ rows, int stride, in
     const int slot = state_slots[s];
     if (slot < 0) return;
     const float* hist = state + static_cast<size_t>(slot) * state_stride + hist_off;
-    const float y = conv_at(rows, stride, off, C, w, taps, hist, t, t - q_start[s], c);
+    float y = conv_at(rows, stride, off, C, w, taps, hist, t, t - q_start[s], c);
+    if (bias != nullptr) y += bias[c];
     out[static_cast<size_t>(t) * C + c] = act ? silu_f(y) : y;
 }
 
+// A step of one token a request: the thread that convolves a channel of a request is the only one that reads that
+// channel's history, and moves it on as well.  TAPS: the filter's length when it is known, 0 when not.
+template <int TAPS>
+__global__ void short_conv_single_kernel(const float* __restrict__ rows, int stride, int off, int C,
+                                         const float* __restrict__ w, int taps_given, float* __restrict__ state,
+                                         long state_stride, int hist_off, const int* __restrict__ positions,
+                                         const int* __restrict__ seq_of, const int* __restrict__ state_slots,
+                                         float* __restrict__ out, int act, const float* __restrict__ bias) {
+    const int taps = TAPS > 0 ? TAPS : taps_given;
+    constexpr int MOST = TAPS > 0 ? TAPS : 16;
+    const int t = blockIdx.x;
+    const int c = blockIdx.y * blockDim.x + threadIdx.x;
+    if (c >= C || positions[t] < 0) return;
+    const int slot = state_slots[seq_of[t]];
+    if (slot < 0) return;
+    float* hist = state + static_cast<size_t>(slot) * state_stride + hist_off;
+    float u[MOST], f[MOST];
+#pragma unroll
+    for (int j = 0; j < MOST; ++j)
+        if (j < taps) {
+            u[j] = j < taps - 1 ? hist[static_cast<size_t>(j) * C + c] : rows[static_cast<size_t>(t) * stride + off + c];
+            f[j] = w[j * C + c];
+        }
+    float y = 0.f;
+#pragma unroll
+    for (int j = 0; j < MOST; ++j)
+        if (j < taps) y += f[j] * u[j];
+    if (bias != nullptr) y += bias[c];
+    out[static_cast<size_t>(t) * C + c] = act ? silu_f(y) : y;
+#pragma unroll
+    for (int j = 0; j + 1 < MOST; ++j)
+        if (j < taps - 1) hist[static_cast<size_t>(j) * C + c] = u[j + 1];
+}
+
+// bias [C] or null: added before the activation.  single: every request of the step brings one token, and the history
+// moves on in the same launch (conv_history is then not called).
 extern "C" int pl_short_conv(const float* rows, int stride, int off, int C, const float* w, int taps,
-                             const float* state, long state_stride, int hist_off, const int* positions,
+                             float* state, long state_stride, int hist_off, const int* positions,
                              const int* seq_of, const int* q_start, const int* state_slots, float* out, int act,
-                             int n, hipStream_t stream) {
+                             const float* bias, int single, int n, hipStream_t stream) {
     PL_REQUIRE(C > 0 && taps >= 1 && taps <= 16 && n >= 0, "short_conv: %d channels, %d taps, %d rows", C, taps, n);
     if (n == 0) return 0;
-    short_conv_kernel<<<dim3(n, pl_ceil_div(C, 256)), 256, 0, stream>>>(rows, stride, off, C, w, taps, state, state_stride,
-                                                                      hist_off, positions, seq_of, q_start, state_slots, out, act);
+    const dim3 grid(n, pl_ceil_div(C, 256));
+    if (!single)
+        short_conv_kernel<<<grid, 256, 0, stream>>>(rows, stride, off, C, w, taps, state, state_stride, hist_off, positions,
+                                                    seq_of, q_start, state_slots, out, act, bias);
+    else if (taps == 4)
+        short_conv_single_kernel<4><<<grid, 256, 0, stream>>>(rows, stride, off, C, w, taps, state, state_stride, hist_off,
+                                                              positions, seq_of, state_slots, out, act, bias);
+    else
+        short_conv_single_kernel<0><<<grid, 256, 0, stream>>>(rows, stride, off, C, w, taps, state, state_stride, hist_off,
+                                                              positions, seq_of, state_slots, out, act, bias);
     PL_CHECK_LAUNCH("short_conv");
     return 0;
 }
@@ -301,15 +362,22 @@ extern "C" int pl_conv_history(const float* rows, int stride, int off, int C, in
 // ---------------------------------------------------------------------------
 // out[t, c] = x[t, c] / sqrt(mean over c's group of x^2 + eps) * gain[c mod gain_len] * act(gate[t, c])
 // Groups are runs of `group` columns (a head, or the whole row).  One wave a row and group.
-// act: 0 sigmoid, 1 silu, -1 no gate.
+// act: 0 sigmoid, 1 silu, -1 no gate.  FIRST: the gate multiplies x before the statistic is taken, and not the result:
+//   u = x * act(gate);  out = u / sqrt(mean over the group of u^2 + eps) * gain
 // ---------------------------------------------------------------------------
-template <typename T>
+template <typename T, bool FIRST>
 __global__ __launch_bounds__(64) void gated_group_norm_kernel(const float* __restrict__ x, int width, int group,
                                                               const float* __restrict__ gain, int gain_len, float eps,
                                                               const float* __restrict__ gate, int gate_stride,
                                                               int gate_off, int act, T* __restrict__ out) {
     const int t = blockIdx.x, first = blockIdx.y * group;
     const float* row = x + static_cast<size_t>(t) * width + first;
+    const float* g = gate != nullptr ? gate + static_cast<size_t>(t) * gate_stride + gate_off + first : nullptr;
+    auto value = [&](int e) {
+        float u = row[e];
+        if (FIRST && act >= 0) u *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
+        return u;
+    };
     // a lane keeps up to eight of its values between the sum and the output (groups up to 512 are read once)
     constexpr int KEEP = 8;
     float kept[KEEP];
@@ -317,33 +385,35 @@ __global__ __launch_bounds__(64) void gated_group_norm_kernel(const float* __res
 #pragma unroll
     for (int k = 0; k < KEEP; ++k) {
         const int e = threadIdx.x + 64 * k;
-        kept[k] = e < group ? row[e] : 0.f;
+        kept[k] = e < group ? value(e) : 0.f;
         ss += kept[k] * kept[k];
     }
-    for (int e = threadIdx.x + 64 * KEEP; e < group; e += 64) ss += row[e] * row[e];
+    for (int e = threadIdx.x + 64 * KEEP; e < group; e += 64) {
+        const float u = value(e);
+        ss += u * u;
+    }
     ss = wave_sum(ss);
     const float inv = 1.f / sqrtf(ss / static_cast<float>(group) + eps);
-    const float* g = gate != nullptr ? gate + static_cast<size_t>(t) * gate_stride + gate_off + first : nullptr;
     T* o = out + static_cast<size_t>(t) * width + first;
 #pragma unroll
     for (int k = 0; k < KEEP; ++k) {
         const int e = threadIdx.x + 64 * k;
         if (e < group) {
             float y = kept[k] * inv * gain[(first + e) % gain_len];
-            if (act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
+            if (!FIRST && act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
             o[e] = from_float<T>(y);
         }
     }
     for (int e = threadIdx.x + 64 * KEEP; e < group; e += 64) {
-        float y = row[e] * inv * gain[(first + e) % gain_len];
-        if (act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
+        float y = value(e) * inv * gain[(first + e) % gain_len];
+        if (!FIRST && act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
         o[e] = from_float<T>(y);
     }
 }
 
 // The same for groups of more than 512 columns (all heads normalised together): a workgroup of four waves a row and
 // group, so that a group of up to 2,048 is read once, every load asked for at once.
-template <typename T>
+template <typename T, bool FIRST>
 __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float* __restrict__ x, int width, int group,
                                                                     const float* __restrict__ gain, int gain_len, float eps,
                                                                     const float* __restrict__ gate, int gate_stride,
@@ -353,6 +423,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
     const float* row = x + static_cast<size_t>(t) * width + first;
     const float* g = gate != nullptr ? gate + static_cast<size_t>(t) * gate_stride + gate_off + first : nullptr;
     const float* gains = gain + (gain_len == width ? first : 0);     // (gain_len is the row's width or the group's)
+    auto opened = [&](float gv) { return act == 0 ? sigmoid_f(gv) : silu_f(gv); };
     constexpr int KEEP = 8;
     float kept[KEEP], gates[KEEP], scale[KEEP];
     float ss = 0.f;
@@ -362,9 +433,13 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
         kept[k] = e < group ? row[e] : 0.f;
         gates[k] = (e < group && act >= 0) ? g[e] : 0.f;
         scale[k] = e < group ? gains[e] : 0.f;
+        if (FIRST && act >= 0) kept[k] *= opened(gates[k]);
         ss += kept[k] * kept[k];
     }
-    for (int e = threadIdx.x + 256 * KEEP; e < group; e += 256) ss += row[e] * row[e];
+    for (int e = threadIdx.x + 256 * KEEP; e < group; e += 256) {
+        const float u = FIRST && act >= 0 ? row[e] * opened(g[e]) : row[e];
+        ss += u * u;
+    }
     ss = block_sum(ss, scratch);
     const float inv = 1.f / sqrtf(ss / static_cast<float>(group) + eps);
     T* o = out + static_cast<size_t>(t) * width + first;
@@ -373,20 +448,20 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
         const int e = threadIdx.x + 256 * k;
         if (e < group) {
             float y = kept[k] * inv * scale[k];
-            if (act >= 0) y *= act == 0 ? sigmoid_f(gates[k]) : silu_f(gates[k]);
+            if (!FIRST && act >= 0) y *= opened(gates[k]);
             o[e] = from_float<T>(y);
         }
     }
     for (int e = threadIdx.x + 256 * KEEP; e < group; e += 256) {
         float y = row[e] * inv * gains[e];
-        if (act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
+        if (act >= 0) y *= opened(g[e]);
         o[e] = from_float<T>(y);
     }
 }
 
 extern "C" int pl_gated_group_norm(const float* x, int n, int width, int group, const float* gain, int gain_len,
-                                   float eps, const float* gate, int gate_stride, int gate_off, int act, void* out,
-                                   int dtype, hipStream_t stream) {
+                                   float eps, const float* gate, int gate_stride, int gate_off, int act, int gate_first,
+                                   void* out, int dtype, hipStream_t stream) {
     PL_REQUIRE(n >= 0 && width > 0 && group > 0 && width % group == 0, "gated_group_norm: rows %d, width %d, groups of %d", n, width, group);
     PL_REQUIRE(gain_len > 0 && width % gain_len == 0 && (gain_len == width || gain_len == group),
                "gated_group_norm: %d gains for rows of %d in groups of %d", gain_len, width, group);
@@ -394,20 +469,24 @@ extern "C" int pl_gated_group_norm(const float* x, int n, int width, int group, 
     if (n == 0) return 0;
     PL_REQUIRE(width / group <= 65535, "gated_group_norm: %d groups a row", width / group);
     const dim3 grid(n, width / group);
-    if (group > 512 && (dtype == PL_DTYPE_F32 || dtype == PL_DTYPE_BF16)) {
-        if (dtype == PL_DTYPE_F32)
-            gated_group_norm_wide_kernel<float><<<grid, 256, 0, stream>>>(x, width, group, gain, gain_len, eps, gate, gate_stride, gate_off, act, static_cast<float*>(out));
-        else
-            gated_group_norm_wide_kernel<bf16_t><<<grid, 256, 0, stream>>>(x, width, group, gain, gain_len, eps, gate, gate_stride, gate_off, act, static_cast<bf16_t*>(out));
-        PL_CHECK_LAUNCH("gated_group_norm");
-        return 0;
-    }
-    if (dtype == PL_DTYPE_F32)
-        gated_group_norm_kernel<float><<<grid, 64, 0, stream>>>(x, width, group, gain, gain_len, eps, gate, gate_stride, gate_off, act, static_cast<float*>(out));
-    else if (dtype == PL_DTYPE_BF16)
-        gated_group_norm_kernel<bf16_t><<<grid, 64, 0, stream>>>(x, width, group, gain, gain_len, eps, gate, gate_stride, gate_off, act, static_cast<bf16_t*>(out));
-    else
-        PL_REQUIRE(false, "gated_group_norm: dtype code %d", dtype);
+#define PL_GROUP_NORM(KERNEL, T, FIRST, THREADS)                                                                          \
+    KERNEL<T, FIRST><<<grid, THREADS, 0, stream>>>(x, width, group, gain, gain_len, eps, gate, gate_stride, gate_off, act, \
+                                                   static_cast<T*>(out))
+#define PL_GROUP_NORM_OF(T)                                                                  \
+    do {                                                                                     \
+        if (group > 512) {                                                                   \
+            if (gate_first) PL_GROUP_NORM(gated_group_norm_wide_kernel, T, true, 256);       \
+            else PL_GROUP_NORM(gated_group_norm_wide_kernel, T, false, 256);                 \
+        } else {                                                                             \
+            if (gate_first) PL_GROUP_NORM(gated_group_norm_kernel, T, true, 64);             \
+            else PL_GROUP_NORM(gated_group_norm_kernel, T, false, 64);                       \
+        }                                                                                    \
+    } while (0)
+    if (dtype == PL_DTYPE_F32) PL_GROUP_NORM_OF(float);
+    else if (dtype == PL_DTYPE_BF16) PL_GROUP_NORM_OF(bf16_t);
+    else PL_REQUIRE(false, "gated_group_norm: dtype code %d", dtype);
+#undef PL_GROUP_NORM_OF
+#undef PL_GROUP_NORM
     PL_CHECK_LAUNCH("gated_group_norm");
     return 0;
 }

@@ -85,7 +85,7 @@ __global__ void activation_kernel(const T* __restrict__ x, T* __restrict__ out, 
 }
 
 extern "C" int pl_activation(const void* x, void* out, int dtype, int act, long count, hipStream_t stream) {
-    PL_REQUIRE(count >= 0 && act >= 0 && act <= 2, "activation: %ld values, code %d", count, act);
+    PL_REQUIRE(count >= 0 && act >= 0 && act <= PL_ACT_RELU2, "activation: %ld values, code %d", count, act);
     if (count == 0) return 0;
     const bool eights = count % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0;
     const size_t items = eights ? count / 8 : count;

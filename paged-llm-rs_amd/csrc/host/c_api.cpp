@@ -60,10 +60,10 @@ static uint64_t pool_counter(const BlockPool& pool, int which) {
 uint64_t plh_pool_counter(void* p, int which) { return pool_counter(*static_cast<BlockPool*>(p), which); }
 
 // ---- the cache manager ------------------------------------------------------
-void* plh_cache_create(int groups, const int* block_size, const int* num_blocks, const int* window, int state_slots) {
+void* plh_cache_create(int groups, const int* block_size, const int* num_blocks, const int* window, const int* keep, int state_slots) {
     try {
         std::vector<GroupSpec> specs;
-        for (int g = 0; g < groups; ++g) specs.push_back(GroupSpec{block_size[g], num_blocks[g], window[g]});
+        for (int g = 0; g < groups; ++g) specs.push_back(GroupSpec{block_size[g], num_blocks[g], window[g], keep[g]});
         return new CacheManager(std::move(specs), state_slots);
     } catch (const std::exception& e) {
         g_error = e.what();

@@ -117,6 +117,7 @@ CacheManager::CacheManager(std::vector<GroupSpec> groups, int state_slots)
         if (g.block_size < 1) throw Error("block size " + std::to_string(g.block_size) + ", which has to be at least one");
         if (g.num_blocks < 1) throw Error("a pool of " + std::to_string(g.num_blocks) + " pages");
         if (g.window < 0) throw Error("window " + std::to_string(g.window));
+        if (g.keep < 0) throw Error("a window that keeps the first " + std::to_string(g.keep) + " keys");
         pools_.emplace_back(static_cast<size_t>(g.num_blocks));
     }
     if (state_slots_ < 0) state_slots_ = 0;
@@ -240,7 +241,8 @@ void CacheManager::release_passed(SequenceTable& t) {
         const size_t first_needed = t.tokens - window + 1;
         const size_t bs = static_cast<size_t>(groups_[g].block_size);
         const size_t dead = std::min(first_needed / bs, t.blocks[g].size());
-        for (size_t b = 0; b < dead; ++b) {
+        const size_t kept = (static_cast<size_t>(groups_[g].keep) + bs - 1) / bs;
+        for (size_t b = kept; b < dead; ++b) {
             if (t.blocks[g][b] == kNoBlock) continue;
             pools_[g].release(t.blocks[g][b]);
             t.blocks[g][b] = kNoBlock;
@@ -332,8 +334,9 @@ bool CacheManager::fits_in_total(size_t length, size_t budget) const {
         const size_t bs = static_cast<size_t>(groups_[g].block_size);
         size_t pages = (length + bs - 1) / bs;
         if (groups_[g].window > 0) {
-            // A windowed group holds at most the window plus one step's tokens at a time.
-            const size_t live = (static_cast<size_t>(groups_[g].window) + budget + bs - 1) / bs + 1;
+            // A windowed group holds at most the window plus one step's tokens at a time, and its kept first keys.
+            const size_t live = (static_cast<size_t>(groups_[g].window) + budget + bs - 1) / bs + 1 +
+                                (static_cast<size_t>(groups_[g].keep) + bs - 1) / bs;
             pages = std::min(pages, live);
         }
         if (pages > pools_[g].total()) return false;

@@ -80,7 +80,8 @@ private:
 struct GroupSpec {
     int block_size;  // tokens a page
     int num_blocks;  // pages in this group's pool
-    int window;      // 0: every key is kept; w > 0: only the last w keys are read
+    int window;      // 0: every key is kept; w > 0: only the last w keys are read ...
+    int keep = 0;    // ... and, beside them, the first `keep` keys of a request, whose pages stay
 };
 
 // Where one request's tokens live: per group a list of pages in logical order
@@ -131,7 +132,7 @@ public:
     // how many tokens now fit (at most count).
     size_t reserve_up_to(uint64_t id, size_t count);
     // Record that `count` tokens were written.  Refused past the capacity.  A
-    // windowed group then gives back the pages the window has passed.
+    // windowed group then gives back the pages the window has passed (but not those of kept first keys).
     void advance(uint64_t id, size_t count);
     // Slot of a position in a group's pool, or -1 (blocks.rs:411-414).
     long slot_of(uint64_t id, size_t group, size_t position) const;

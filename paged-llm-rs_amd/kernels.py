@@ -35,9 +35,10 @@ def _signatures(lib) -> None:
         "pl_qk_norm_rope_kv_write": [p, p, p, i, f, p, p, i, p, p, p, i, i, p, p, i, i, i, i, i, i, i, p],
         "pl_swiglu": [p, p, i, i, i, i, p],
         "pl_gemm_plain": [p, p, p, i, i, i, i, i, i, i, p],
-        "pl_paged_attention_plain": [p, i, p, p, p, p, i, i, p, p, i, i, i, i, f, i, i, p, p, p],
+        "pl_paged_attention_plain": [p, i, p, p, p, p, i, i, p, p, i, i, i, i, f, i, i, p, p, f, i, p, i, p],
         "pl_gemm_heads": [p, p, p, i, i, i, i, i, ctypes.c_long, i, ctypes.c_long, i, i, p],
-        "pl_head_prepare": [p, p, i, i, i, f, p, p, p, p, i, i, i, i, f, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, i, p],
+        "pl_head_prepare": [p, p, i, i, i, f, p, p, p, p, i, i, i, i, f, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, i,
+                            p, i, p, f, p],
         "pl_latent_prepare": [p, i, i, i, p, f, p, p, i, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, i, p],
         "pl_head_gate": [p, i, p, i, i, p, i, i, i, i, p],
         "pl_add_position_rows": [p, p, i, p, i, i, i, p],
@@ -54,20 +55,20 @@ def _signatures(lib) -> None:
         "pl_gemm_stream_splits": [i, i, i, i],
         "pl_gemm_finish": [p, p, ctypes.c_longlong, i, i, i, i, i, p],
         "pl_paged_attention_decode": [p, i, p, p, p, p, p, p, i, i, i, p, i, i, p, p, i, i, i, i, f, i, i,
-                                      i, p, p, i, f, p, p, i, p, p, p],
-        "pl_paged_attention_prefill": [p, i, p, p, p, p, i, i, i, p, i, i, p, p, i, i, i, f, i, i, p, p, i, p, p, p],
-        "pl_paged_attention_grouped": [p, i, p, p, p, p, i, i, i, p, i, i, p, p, i, i, i, f, i, i, p, p, i, i, p, p, p],
+                                      i, p, p, i, f, p, p, i, p, p, f, i, p, i, p],
+        "pl_paged_attention_prefill": [p, i, p, p, p, p, i, i, i, p, i, i, p, p, i, i, i, f, i, i, p, p, i, p, p, f, i, p, i, p],
+        "pl_paged_attention_grouped": [p, i, p, p, p, p, i, i, i, p, i, i, p, p, i, i, i, f, i, i, p, p, i, i, p, p, f, i, p, i, p],
         "pl_paged_attention_grouped_applies": [i, i, i, i],
-        "pl_recurrent_scan": [i, p, i, i, i, i, p, i, i, i, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
+        "pl_recurrent_scan": [i, p, i, i, i, i, p, i, i, i, p, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
                               i, i, i, i, i, i, p],
-        "pl_recurrent_chunked": [i, p, i, i, i, i, p, i, i, i, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
-                                 i, i, i, i, i, i, p, p, p, p, p, p],
+        "pl_recurrent_chunked": [i, p, i, i, i, i, p, i, i, i, p, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
+                                 i, i, i, i, i, i, i, p, p, p, p, p, p],
         "pl_recurrent_chunk_tokens": [i],
         "pl_delta_chunked": [p, i, i, i, i, p, i, i, i, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, i,
                              p, p, p, p, p, p],
-        "pl_short_conv": [p, i, i, i, p, i, p, ctypes.c_long, i, p, p, p, p, p, i, i, p],
+        "pl_short_conv": [p, i, i, i, p, i, p, ctypes.c_long, i, p, p, p, p, p, i, p, i, i, p],
         "pl_conv_history": [p, i, i, i, i, p, ctypes.c_long, i, p, p, p, i, p],
-        "pl_gated_group_norm": [p, i, i, i, p, i, f, p, i, i, i, p, i, p],
+        "pl_gated_group_norm": [p, i, i, i, p, i, f, p, i, i, i, i, p, i, p],
         "pl_conv_qk_prepare": [p, i, i, p, i, p, ctypes.c_long, i, p, p, f, p, i, p, p, p, p, p, i, i, p, p, p, i,
                                i, i, i, i, i, i, p],
         "pl_rmsnorm_onto": [p, p, p, f, p, i, i, i, p],
@@ -78,13 +79,15 @@ def _signatures(lib) -> None:
         "pl_hc_step": [p, p, p, p, p, p, f, p, i, p, i, i, i, p],
         "pl_stream_copies": [p, p, i, i, i, p],
         "pl_softcap": [p, f, ctypes.c_long, p],
-        "pl_moe_rows": [p, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, p, p, i, p],
+        "pl_moe_rows": [p, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, p, p, i, f, p],
         "pl_moe_sort": [p, p, p, p, p, p, i, i, i, i, i, i, p, p, p, p],
         "pl_moe_combine": [p, p, p, i, i, i, i, ctypes.c_longlong, p, p, p, i, i, p, p],
-        "pl_router_select": [p, i, p, p, i, i, i, i, i, i, f, p, p, p, p, i, i, p],
+        "pl_router_select": [p, i, p, p, i, i, i, i, i, i, f, p, p, p, p, i, i, p, i, p],
         "pl_wide_prepare": [p, p, i, i, i, f, p, p, p, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, p],
         "pl_parallel_step": [p, p, p, p, p, p, p, p, f, p, p, i, p, i, i, p],
-        "pl_gemm_tiled_grouped": [p, p, p, p, p, ctypes.c_longlong, i, i, i, i, i, i, i, p],
+        "pl_gemm_tiled_grouped": [p, p, p, p, p, ctypes.c_longlong, i, i, i, i, i, i, i, f, p],
+        "pl_sandwich_step": [p, p, p, p, f, p, p, f, p, i, p, i, i, i, p],
+        "pl_bigram_add": [p, p, p, p, p, p, p, p, p, p, p, i, ctypes.c_longlong, ctypes.c_longlong, ctypes.c_longlong, i, i, p],
     }
     for name, argtypes in table.items():
         fn = getattr(lib, name)
@@ -240,14 +243,28 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, q_gain, k_gain, eps: float, cos, si
         _code(qkv, "fused q/k/v projection"), 1 if neighbours else 0, _stream()))
 
 
-# The activations of a gated feed-forward's gate branch, by the names config.json gives them.
-ACTIVATIONS = {"silu": 0, "swish": 0, "gelu_pytorch_tanh": 1, "gelu_tanh": 1, "gelu_new": 1, "gelu": 2}
+# The activations of a feed-forward (of the gate branch where it is gated), by the names config.json gives them.
+ACTIVATIONS = {"silu": 0, "swish": 0, "gelu_pytorch_tanh": 1, "gelu_tanh": 1, "gelu_new": 1, "gelu": 2, "relu2": 3}
+# What experts may do to gate and up together instead of act(gate) * up: with g = min(gate, limit) and
+# u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+CLAMPED_GATE = "clamped"
 
 
 def activation_code(name: str) -> int:
     if name not in ACTIVATIONS:
         raise TensorError(f"activation {name!r}, the kernels know {', '.join(sorted(ACTIVATIONS))}")
     return ACTIVATIONS[name]
+
+
+def _gate_code(name: str, limit) -> tuple:
+    """(code, limit) of what stands between the two products of an expert."""
+    if name == CLAMPED_GATE:
+        if limit is None or not limit > 0:
+            raise TensorError(f"a clamped gate with a limit of {limit}")
+        return 4, float(limit)
+    if limit is not None:
+        raise TensorError(f"a limit for the activation {name!r}, which has none")
+    return activation_code(name), 0.0
 
 
 def swiglu(gate_up: torch.Tensor, out: torch.Tensor | None = None, activation: str = "silu") -> torch.Tensor:
@@ -290,16 +307,42 @@ def _head_numbers(t, what: str, heads: int):
     return _need(t, what, (heads,), torch.float32)
 
 
+class AttentionMore:
+    """What an attention layer may have beside its mask, its sinks and its distance slopes.  ``cap``: a scaled score s
+    becomes cap * tanh(s / cap), before the distance penalty.  ``keep``: the first so many keys of a request are seen
+    by every later query, whatever the window.  ``gate`` (32-bit rows, from column ``gate_off``): head h's read-out of
+    row t is multiplied by sigmoid(gate[t, gate_off + h])."""
+
+    __slots__ = ("cap", "keep", "gate", "gate_off")
+
+    def __init__(self, cap=None, keep: int = 0, gate: torch.Tensor | None = None, gate_off: int = 0):
+        self.cap, self.keep, self.gate, self.gate_off = float(cap or 0.0), int(keep), gate, int(gate_off)
+        if self.cap < 0 or self.keep < 0:
+            raise TensorError(f"a cap of {cap} on the scores, {keep} first keys kept")
+
+
+def _more_args(more, nq: int, rows: int) -> tuple:
+    """(cap, keep, gates, values between two rows of the gates) as the attention kernels take them."""
+    if more is None:
+        return 0.0, 0, 0, 0
+    if more.gate is None:
+        return more.cap, more.keep, 0, 0
+    _need(more.gate, "gate rows", None, torch.float32)
+    if more.gate.dim() != 2 or more.gate.shape[0] != rows or not 0 <= more.gate_off <= more.gate.shape[1] - nq:
+        raise TensorError(f"gate rows of shape {tuple(more.gate.shape)} for {rows} tokens and {nq} heads from column {more.gate_off}")
+    return more.cap, more.keep, more.gate.data_ptr() + 4 * more.gate_off, more.gate.shape[1]
+
+
 def paged_attention_plain(q: torch.Tensor, q_row_stride: int, out: torch.Tensor, positions: torch.Tensor,
                           seq_of: torch.Tensor, block_table: torch.Tensor, block_size: int,
                           k_pool: torch.Tensor, v_pool: torch.Tensor, nq: int, nkv: int, d: int,
                           scale: float, window: int = 0, sinks: torch.Tensor | None = None,
-                          slopes: torch.Tensor | None = None) -> torch.Tensor:
+                          slopes: torch.Tensor | None = None, more: AttentionMore | None = None) -> torch.Tensor:
     """Attention of every token over the keys 0..position of its request, read
     through the block table.  ``q`` is the fused projection buffer whose rows begin
     with the nq*d query values.  ``slopes`` [nq]: slope_h * (i - j) is taken off the score of key j for
     the query at position i.  ``sinks`` [nq]: exp(sink_h) joins the softmax's denominator, once, unscaled
-    and without a value.  Key and value pool may be the same tensor."""
+    and without a value.  ``more``: see ``AttentionMore``.  Key and value pool may be the same tensor."""
     n = positions.numel()
     _need(q, "query buffer")
     if q.dim() != 2 or q.shape[0] != n or q.shape[1] != q_row_stride or q_row_stride < nq * d:
@@ -316,7 +359,8 @@ def paged_attention_plain(q: torch.Tensor, q_row_stride: int, out: torch.Tensor,
     _check(library().pl_paged_attention_plain(
         q.data_ptr(), q_row_stride, out.data_ptr(), positions.data_ptr(), seq_of.data_ptr(),
         block_table.data_ptr(), block_table.shape[1], block_size, k_pool.data_ptr(), v_pool.data_ptr(),
-        n, nq, nkv, d, float(scale), int(window or 0), _code(q, "query buffer"), _ptr(sinks), _ptr(slopes), _stream()))
+        n, nq, nkv, d, float(scale), int(window or 0), _code(q, "query buffer"), _ptr(sinks), _ptr(slopes),
+        *_more_args(more, nq, n), _stream()))
     return out
 
 
@@ -423,14 +467,14 @@ def paged_attention_decode(q: torch.Tensor, q_row_stride: int, out: torch.Tensor
                            window: int = 0, splits: int = 1, q_len: torch.Tensor | None = None,
                            short_limit: int = 0, fuse: "QkFusion | None" = None, live_seqs: int | None = None,
                            short_rows: int = 0, sinks: torch.Tensor | None = None,
-                           slopes: torch.Tensor | None = None) -> torch.Tensor:
+                           slopes: torch.Tensor | None = None, more: AttentionMore | None = None) -> torch.Tensor:
     """bfloat16 attention of single tokens over their requests' pages, split along the context.
     With ``q_len`` the tokens of requests with ``short_limit`` tokens or more are left out; ``short_rows``
     then bounds the tokens that the other requests bring (0: not known) and ``live_seqs`` says how many
     requests, the first ones, bring tokens, so that the launch has workgroups for those tokens only.
     With ``fuse`` the rows of ``q`` are the raw projection [q | k | v]: queries (and, when it says so, each
     token's key) are normalised and rotated inside the kernel, and key and value are written into the pages.
-    ``sinks`` and ``slopes``: as in ``paged_attention_plain``."""
+    ``sinks``, ``slopes`` and ``more``: as in ``paged_attention_plain``."""
     n = positions.numel()
     sinks, slopes = _head_numbers(sinks, "sinks", nq), _head_numbers(slopes, "distance slopes", nq)
     _need(q, "query buffer", None, torch.bfloat16)
@@ -474,7 +518,7 @@ def paged_attention_decode(q: torch.Tensor, q_row_stride: int, out: torch.Tensor
         block_table.data_ptr(), block_table.shape[1], block_size,
         k_pool.data_ptr(), v_pool.data_ptr(), n, nq, nkv, d, float(scale), int(window or 0), int(splits),
         mode, _ptr(q_gain), _ptr(k_gain), gain_code, float(eps), _ptr(cos), _ptr(sin), int(rot), _ptr(sinks),
-        _ptr(slopes), _stream()))
+        _ptr(slopes), *_more_args(more, nq, n), _stream()))
     return out
 
 
@@ -495,7 +539,8 @@ def paged_attention_prefill(q: torch.Tensor, q_row_stride: int, out: torch.Tenso
                             block_size: int, k_pool: torch.Tensor, v_pool: torch.Tensor, nq: int, nkv: int, d: int,
                             scale: float, window: int = 0, short_limit: int = 0, max_ctx: int | None = None,
                             splits: int | None = None, live_seqs: int | None = None,
-                            sinks: torch.Tensor | None = None, slopes: torch.Tensor | None = None) -> torch.Tensor:
+                            sinks: torch.Tensor | None = None, slopes: torch.Tensor | None = None,
+                            more: AttentionMore | None = None) -> torch.Tensor:
     """bfloat16 attention of prompt portions on the matrix cores.  Request s brings the rows
     q_start[s] .. q_start[s]+q_len[s]-1 at the positions ctx_len[s]-q_len[s] .. ctx_len[s]-1;
     requests with fewer than ``short_limit`` tokens are skipped.  ``max_ctx`` (the longest context
@@ -532,7 +577,8 @@ def paged_attention_prefill(q: torch.Tensor, q_row_stride: int, out: torch.Tenso
         int(short_limit), live, int(max_q_len), block_table.data_ptr(), block_table.shape[1], block_size,
         k_pool.data_ptr(), v_pool.data_ptr(), nq, nkv, d, float(scale), int(window or 0), int(splits),
         part_acc.data_ptr() if splits > 1 else None, part_ml.data_ptr() if splits > 1 else None, n,
-        _ptr(_head_numbers(sinks, "sinks", nq)), _ptr(_head_numbers(slopes, "distance slopes", nq)), _stream()))
+        _ptr(_head_numbers(sinks, "sinks", nq)), _ptr(_head_numbers(slopes, "distance slopes", nq)),
+        *_more_args(more, nq, n), _stream()))
     return out
 
 
@@ -574,7 +620,7 @@ def paged_attention_grouped(q: torch.Tensor, q_row_stride: int, out: torch.Tenso
                             scale: float, window: int = 0, short_limit: int = 0, max_ctx: int | None = None,
                             splits: int | None = None, live_seqs: int | None = None,
                             tokens: int | None = None, sinks: torch.Tensor | None = None,
-                            slopes: torch.Tensor | None = None) -> torch.Tensor:
+                            slopes: torch.Tensor | None = None, more: AttentionMore | None = None) -> torch.Tensor:
     """bfloat16 attention for single tokens and the tokens of short portions, the query heads of a
     key-head group as the rows of a tile of the tiled kernel.  Arguments as for
     ``paged_attention_prefill``, but requests with ``short_limit`` tokens or more are the ones skipped
@@ -610,7 +656,8 @@ def paged_attention_grouped(q: torch.Tensor, q_row_stride: int, out: torch.Tenso
         int(short_limit), live, int(max_q_len), block_table.data_ptr(), block_table.shape[1], block_size,
         k_pool.data_ptr(), v_pool.data_ptr(), nq, nkv, d, float(scale), int(window or 0), int(splits),
         part_acc.data_ptr() if splits > 1 else None, part_ml.data_ptr() if splits > 1 else None, n, int(tokens or 0),
-        _ptr(_head_numbers(sinks, "sinks", nq)), _ptr(_head_numbers(slopes, "distance slopes", nq)), _stream()))
+        _ptr(_head_numbers(sinks, "sinks", nq)), _ptr(_head_numbers(slopes, "distance slopes", nq)),
+        *_more_args(more, nq, n), _stream()))
     return out
 
 
@@ -670,7 +717,7 @@ TILED_TAKES_SHORT_WORKGROUPS = 512
 
 def paged_attention(qkv: torch.Tensor, out: torch.Tensor, batch, kv, nq: int, nkv: int, d: int,
                     scale: float, window: int = 0, sinks: torch.Tensor | None = None,
-                    slopes: torch.Tensor | None = None) -> torch.Tensor:
+                    slopes: torch.Tensor | None = None, more: AttentionMore | None = None) -> torch.Tensor:
     """Attention for every token of a step.  ``qkv`` rows begin with the rotated queries.
     In bfloat16 the long portions go to the tiled kernel and the tokens of short ones
     (decoded tokens among them) to the kernel for single tokens, or, where many query heads share a key
@@ -678,7 +725,7 @@ def paged_attention(qkv: torch.Tensor, out: torch.Tensor, batch, kv, nq: int, nk
     if qkv.dtype != torch.bfloat16 or _attention_mode != "kernel" or d % 16 or d > 256:
         return paged_attention_plain(qkv, qkv.shape[1], out, batch.positions, batch.seq_of, kv.block_table,
                                      kv.block_size, kv.k_pool, kv.v_pool, nq, nkv, d, scale, window,
-                                     sinks=sinks, slopes=slopes)
+                                     sinks=sinks, slopes=slopes, more=more)
     stride = qkv.shape[1]
     short_tokens = batch.tokens_of_short_requests(SHORT_PORTION)
     if batch.max_q_len >= SHORT_PORTION:
@@ -690,24 +737,26 @@ def paged_attention(qkv: torch.Tensor, out: torch.Tensor, batch, kv, nq: int, nk
         paged_attention_prefill(qkv, stride, out, batch.q_start, batch.q_len, batch.ctx_len, batch.max_q_len,
                                 kv.block_table, kv.block_size, kv.k_pool, kv.v_pool, nq, nkv, d, scale, window,
                                 short_limit=0 if all_tiled else SHORT_PORTION, max_ctx=batch.max_ctx_len,
-                                live_seqs=getattr(batch, "live_seqs", None), sinks=sinks, slopes=slopes)
+                                live_seqs=getattr(batch, "live_seqs", None), sinks=sinks, slopes=slopes, more=more)
         if short_tokens == 0 or all_tiled:
             return out
     mixed = batch.max_q_len >= SHORT_PORTION
+    # the most keys a single token reads: a window's and the kept first ones, where there is a window
+    reach = min(batch.max_ctx_len, window + more.keep) if more is not None and window > 0 else batch.max_ctx_len
     if grouped_applies(nq, nkv, d, kv.block_size):
         # many query heads a key head: a token's group of heads as the rows of a tile of the tiled kernel
         return paged_attention_grouped(qkv, stride, out, batch.q_start, batch.q_len, batch.ctx_len,
                                        min(batch.max_q_len, SHORT_PORTION - 1), kv.block_table, kv.block_size,
                                        kv.k_pool, kv.v_pool, nq, nkv, d, scale, window,
-                                       short_limit=SHORT_PORTION if mixed else 0, max_ctx=batch.max_ctx_len,
+                                       short_limit=SHORT_PORTION if mixed else 0, max_ctx=reach,
                                        live_seqs=getattr(batch, "live_seqs", None), tokens=short_tokens,
-                                       sinks=sinks, slopes=slopes)
-    splits = decode_splits(short_tokens, nq, nkv, batch.max_ctx_len, d)
+                                       sinks=sinks, slopes=slopes, more=more)
+    splits = decode_splits(short_tokens, nq, nkv, reach, d)
     return paged_attention_decode(qkv, stride, out, batch.positions, batch.seq_of, kv.block_table,
                                   kv.block_size, kv.k_pool, kv.v_pool, nq, nkv, d, scale, window, splits,
                                   q_len=batch.q_len if mixed else None, short_limit=SHORT_PORTION if mixed else 0,
                                   live_seqs=getattr(batch, "live_seqs", None), short_rows=short_tokens,
-                                  sinks=sinks, slopes=slopes)
+                                  sinks=sinks, slopes=slopes, more=more)
 
 
 class HandedNorm:
@@ -1088,7 +1137,7 @@ def linear_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype,
 # ---------------------------------------------------------------------------
 # Mixers with a carried state, short convolutions, and the layer that normalises a sublayer's output
 
-SCAN_KINDS = {"lightning": 0, "mlstm": 1, "delta": 2}
+SCAN_KINDS = {"lightning": 0, "mlstm": 1, "delta": 2, "ssd": 3}
 SCAN_MAX_DIM = 256
 # A request that brings at least this many tokens to a step goes through the chunked kernels, where its mixer has
 # them (64 tokens at once instead of one after the other); the others, single tokens among them, go token by token.
@@ -1121,7 +1170,8 @@ def scan_state_floats(kind: str, heads: int, dim: int, vdim: int) -> int:
 def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor,
                    batch, heads: int, qk_heads: int, dim: int, vdim: int, *, gates: torch.Tensor | None = None,
                    g1_off: int = 0, g2_off: int = 0, p1: torch.Tensor | None = None, p2: torch.Tensor | None = None,
-                   cap: float = 0.0, out: torch.Tensor | None = None, chunked: bool = False) -> torch.Tensor:
+                   p3: torch.Tensor | None = None, cap: float = 0.0, out: torch.Tensor | None = None,
+                   chunked: bool = False) -> torch.Tensor:
     """The read-out [rows, heads * vdim] (32-bit) of a mixer that carries a [dim, vdim] matrix a head from
     token to token, over the tokens of a step, request by request, from and into the requests' state slots.
 
@@ -1131,6 +1181,9 @@ def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: 
     slot is laid out as ``scan_state_floats`` says.
     ``delta``: ``qkv`` holds convolved and activated rows; q and k become unit vectors, beta = sigmoid(x1),
     decay = exp(-exp(A_log) softplus(x2 + dt_bias)); ``p1`` = A_log, ``p2`` = dt_bias.
+    ``ssd``: ``qkv`` holds convolved and activated rows, q, k and v being a state space's C, B and x; with
+    dt = softplus(x1 + dt_bias), S = exp(-exp(A_log) dt) S + dt k v^T, o = S^T q + D v; ``p1`` = A_log, ``p2`` = dt_bias,
+    ``p3`` = D; one gate column a head, from ``g1_off``.
     q and k have ``qk_heads`` heads (head h of v reads head h / (heads / qk_heads)).
     ``chunked`` (lightning only with decays above zero): requests that bring ``SCAN_CHUNKED_FROM`` tokens or more
     are computed in chunks of tokens, the same sums in another order."""
@@ -1154,6 +1207,9 @@ def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: 
     _step_rows(batch, n)
     if kind != "lightning":
         _need(gates, "rows of the gates", None, torch.float32)
+        if kind == "ssd":
+            g2_off = g1_off
+            _need(p3, "what v counts in its own read-out", (heads,), torch.float32)
         if gates.dim() != 2 or gates.shape[0] != n or not (0 <= g1_off and g1_off + heads <= gates.shape[1]
                                                          and 0 <= g2_off and g2_off + heads <= gates.shape[1]):
             raise TensorError(f"gates at columns {g1_off}, {g2_off} of rows of shape {tuple(gates.shape)}")
@@ -1165,7 +1221,7 @@ def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: 
     hdv = heads * dim * vdim
     chunked = bool(chunked) and batch.max_q_len >= SCAN_CHUNKED_FROM
     common = (SCAN_KINDS[kind], qkv.data_ptr(), width, q_off, k_off, v_off, _ptr(gates),
-              0 if gates is None else gates.shape[1], g1_off, g2_off, _ptr(p1), _ptr(p2), float(cap),
+              0 if gates is None else gates.shape[1], g1_off, g2_off, _ptr(p1), _ptr(p2), _ptr(p3), float(cap),
               state.data_ptr(), stride, 0, hdv, hdv + heads * tiles * dim, out.data_ptr(), batch.q_start.data_ptr(),
               batch.q_len.data_ptr(), batch.state_slots.data_ptr(), batch.num_seqs)
     _check(library().pl_recurrent_scan(*common, heads, qk_heads, dim, vdim, SCAN_CHUNKED_FROM if chunked else 0, _stream()))
@@ -1190,7 +1246,7 @@ def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: 
         k_sums, n_before = (torch.empty((chunks, heads * dim), **f32), torch.empty((chunks, heads * dim), **f32)) \
             if kind == "mlstm" else (None, None)
         scalars = torch.empty((chunks, heads * 4), **f32)
-        _check(library().pl_recurrent_chunked(*common, batch.max_q_len, heads, dim, vdim, SCAN_CHUNKED_FROM,
+        _check(library().pl_recurrent_chunked(*common, batch.max_q_len, heads, qk_heads, dim, vdim, SCAN_CHUNKED_FROM,
                                               sums.data_ptr(), _ptr(k_sums), before.data_ptr(), _ptr(n_before),
                                               scalars.data_ptr(), _stream()))
     return out
@@ -1213,19 +1269,27 @@ def _conv_args(rows, off, weight, history, batch):
 
 
 def short_conv(rows: torch.Tensor, off: int, weight: torch.Tensor, history: torch.Tensor, batch,
-               silu: bool = False, out: torch.Tensor | None = None) -> torch.Tensor:
+               silu: bool = False, out: torch.Tensor | None = None, bias: torch.Tensor | None = None,
+               move_history: bool = False) -> torch.Tensor:
     """y[t, c] = sum_j weight[j, c] * u[t - taps + 1 + j, c] over the columns [off, off + channels) of
     ``rows`` (``weight`` is [taps, channels]: a checkpoint's [channels, taps] transposed, so that neighbouring
     channels' values of a tap are neighbours in memory); the rows before a request's first of this step come from ``history`` [slots, (taps-1) * channels]
-    (newest last, zeros at a request's start), which is left as it is: ``conv_history`` moves it afterwards."""
+    (newest last, zeros at a request's start), which is left as it is: ``conv_history`` moves it afterwards.  ``bias``
+    (32-bit, one a channel) is added before the activation.  ``move_history``: the history is moved on here as well (in
+    the same launch where every request of the step brings one token)."""
     n, channels, taps, history, stride = _conv_args(rows, off, weight, history, batch)
     if out is None:
         out = torch.empty((n, channels), dtype=torch.float32, device=rows.device)
     _need(out, "convolved rows", (n, channels), torch.float32)
+    if bias is not None:
+        _need(bias, "biases of the convolution", (channels,), torch.float32)
+    single = move_history and batch.max_q_len == 1
     _check(library().pl_short_conv(rows.data_ptr(), rows.shape[1], off, channels, weight.data_ptr(), taps,
                                    history.data_ptr(), stride, 0, batch.positions.data_ptr(), batch.seq_of.data_ptr(),
                                    batch.q_start.data_ptr(), batch.state_slots.data_ptr(), out.data_ptr(),
-                                   1 if silu else 0, n, _stream()))
+                                   1 if silu else 0, _ptr(bias), 1 if single else 0, n, _stream()))
+    if move_history and not single:
+        conv_history(rows, off, weight, history, batch)
     return out
 
 
@@ -1241,9 +1305,11 @@ GATES = {None: -1, "sigmoid": 0, "silu": 1}
 
 
 def gated_group_norm(x: torch.Tensor, group: int, gain: torch.Tensor, eps: float, out_dtype: torch.dtype,
-                     gate: torch.Tensor | None = None, gate_off: int = 0, gate_act: str | None = None) -> torch.Tensor:
+                     gate: torch.Tensor | None = None, gate_off: int = 0, gate_act: str | None = None,
+                     gate_first: bool = False) -> torch.Tensor:
     """x / sqrt(mean over each run of ``group`` columns of x^2 + eps) * gain * act(gate); ``gain`` has a value a
-    column or a value a column of a group; ``gate`` are the columns from ``gate_off`` of 32-bit rows."""
+    column or a value a column of a group; ``gate`` are the columns from ``gate_off`` of 32-bit rows.  ``gate_first``:
+    x * act(gate) takes the place of x, statistic included, and the result is not gated."""
     n, width = x.shape
     _need(x, "read-out", None, torch.float32)
     _need(gain, "gain of the grouped norm", None, torch.float32)
@@ -1258,7 +1324,7 @@ def gated_group_norm(x: torch.Tensor, group: int, gain: torch.Tensor, eps: float
     out = torch.empty((n, width), dtype=out_dtype, device=x.device)
     _check(library().pl_gated_group_norm(x.data_ptr(), n, width, group, gain.data_ptr(), gain.numel(), float(eps),
                                          _ptr(gate), 0 if gate is None else gate.shape[1], gate_off, GATES[gate_act],
-                                         out.data_ptr(), _code(out, "normalised read-out"), _stream()))
+                                         1 if gate_first else 0, out.data_ptr(), _code(out, "normalised read-out"), _stream()))
     return out
 
 
@@ -1371,13 +1437,15 @@ GEMM_HEADS_PLAIN_ROWS = 0
 def head_prepare(rows: torch.Tensor, off: int, batch, kv, q_out: torch.Tensor, H: int, G: int, D: int, V: int,
                  padded: int, unit_eps: float | None = None, q_gain=None, k_gain=None, cos=None, sin=None,
                  rot_off: int = 0, rot: int = 0, temperature: tuple | None = None, write_kv: bool = True,
-                 bias: torch.Tensor | None = None) -> None:
+                 bias: torch.Tensor | None = None, mix: tuple | None = None) -> None:
     """Between an attention layer's projections and the attention kernels: ``rows`` [n, >= off + H D + G D + G V]
     (32-bit) holds q | k | v from column ``off``.  q and k are divided by their root mean square over a head
     (``unit_eps``; times a gain where one is given), ``rot`` values from ``rot_off`` on turn in pairs (2i, 2i + 1)
     by the tables' angles, q is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1) (``temperature`` =
     (coef, every)); q goes to ``q_out`` [n, H * padded], k and v into the pages, every head in ``padded`` values.
-    ``bias`` (32-bit, [H D + G D + G V]): the projections' biases, added to q | k | v before anything else."""
+    ``bias`` (32-bit, [H D + G D + G V]): the projections' biases, added to q | k | v before anything else.
+    ``mix`` = (first, first_off, first_bias, share): v becomes (1 - share) v + share (first + first_bias), ``first`` being
+    the columns from ``first_off`` of an earlier layer's 32-bit projected rows, ``first_bias`` [G V] or None."""
     n = rows.shape[0]
     _need(rows, "projected rows", None, torch.float32)
     if rows.dim() != 2:
@@ -1400,13 +1468,24 @@ def head_prepare(rows: torch.Tensor, off: int, batch, kv, q_out: torch.Tensor, H
     coef, every = temperature if temperature is not None else (0.0, 1)
     if bias is not None:
         _need(bias, "biases of q, k and v", (H * D + G * D + G * V,), torch.float32)
+    first_at = first_stride = 0
+    first_bias, share = None, 0.0
+    if mix is not None:
+        first, first_off, first_bias, share = mix
+        _need(first, "rows of the values to mix with", None, torch.float32)
+        if first.dim() != 2 or first.shape[0] != n or not 0 <= first_off <= first.shape[1] - G * V:
+            raise TensorError(f"values of {G * V} from column {first_off} of rows of shape {tuple(first.shape)}")
+        if first_bias is not None:
+            _need(first_bias, "bias of the values to mix with", (G * V,), torch.float32)
+        first_at, first_stride = first.data_ptr() + 4 * int(first_off), first.shape[1]
     _check(library().pl_head_prepare(
         rows.data_ptr(), _ptr(bias), rows.shape[1], int(off), 1 if unit_eps is not None else 0, float(unit_eps or 0.0),
         _ptr(q_gain), _ptr(k_gain), _ptr(cos) if rot else 0, _ptr(sin) if rot else 0, int(rot_off), int(rot), table_rows,
         1 if temperature is not None else 0, float(coef), int(every), batch.positions.data_ptr(),
         batch.seq_of.data_ptr(), kv.block_table.data_ptr(), kv.block_table.shape[1], kv.block_size,
         1 if write_kv else 0, q_out.data_ptr(), kv.k_pool.data_ptr(), kv.v_pool.data_ptr(),
-        _code(q_out, "query buffer"), n, H, G, D, V, padded, _stream()))
+        _code(q_out, "query buffer"), n, H, G, D, V, padded, first_at, first_stride, _ptr(first_bias), float(share),
+        _stream()))
 
 
 def latent_prepare(rows: torch.Tensor, q_off: int, kv_off: int, gain, eps: float, cos, sin, turned: int, batch, kv,
@@ -1474,11 +1553,12 @@ def add_position_rows_(x: torch.Tensor, table: torch.Tensor, positions: torch.Te
 
 
 def sink_attention(q: torch.Tensor, out: torch.Tensor, batch, kv, nq: int, nkv: int, d: int, scale: float,
-                   window: int = 0, sinks: torch.Tensor | None = None, slopes: torch.Tensor | None = None) -> torch.Tensor:
+                   window: int = 0, sinks: torch.Tensor | None = None, slopes: torch.Tensor | None = None,
+                   more: AttentionMore | None = None) -> torch.Tensor:
     """Attention for every token of a step with a sink a head in the softmax's denominator and a penalty a
     head on the distance; ``q`` [n, nq * d] holds the prepared queries.  In bfloat16 the matrix-core kernel for
     portions and the kernels for single tokens, for head sizes they take; the plain kernel otherwise."""
-    return paged_attention(q, out, batch, kv, nq, nkv, d, scale, window, sinks=sinks, slopes=slopes)
+    return paged_attention(q, out, batch, kv, nq, nkv, d, scale, window, sinks=sinks, slopes=slopes, more=more)
 
 
 # ---- several copies of the stream; experts chosen by a table over token ids ------------------------------------
@@ -1547,14 +1627,14 @@ def _routed(n: int, E: int, choice, weight, identity: int) -> int:
 
 
 def moe_rows(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: torch.Tensor,
-             activation: str = "silu", choice=None, weight=None, identity: int = 0) -> torch.Tensor:
+             activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None) -> torch.Tensor:
     """Experts chosen by a table over token ids, a row at a time: 32-bit [n, W], row t the mean over the experts e
     that ``table[id of t]`` names of down_e (act(gate_e x_t) * (up_e x_t)).  ``w_gate_up`` [E, 2 F, W] (an expert's
     gate rows, then its up rows), ``w_down`` [E, W, F], of ``x``'s type; ``table`` [vocabulary, top] int32.  A row's
     id is the batch's, or the one an earlier step left on the device; padding rows give zeros.
     With ``choice`` and ``weight`` ([n, top]; no table) a router has chosen: pair (t, c) runs expert choice[t, c] and
     counts weight[t, c]; a choice of E .. E + ``identity`` - 1 is an identity expert, whose output is the row itself;
-    -1 is none."""
+    -1 is none.  ``activation`` "clamped" (with its ``limit``): see ``CLAMPED_GATE``."""
     n, W = x.shape
     _need(x, "rows")
     E, F2, _ = w_gate_up.shape
@@ -1566,6 +1646,7 @@ def moe_rows(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: tor
     else:
         _need(table, "table of experts", None, torch.int32)
         vocab, top = table.shape
+    act, bound = _gate_code(activation, limit)
     fed = getattr(batch, "fed_tokens", None)
     src = batch.token_src if fed is not None else None
     h = torch.empty((n, top, F), dtype=x.dtype, device=x.device)
@@ -1573,7 +1654,7 @@ def moe_rows(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: tor
     _check(library().pl_moe_rows(x.data_ptr(), batch.token_ids.data_ptr(), _ptr(src), _ptr(fed),
                                  batch.positions.data_ptr(), _ptr(table), w_gate_up.data_ptr(), w_down.data_ptr(),
                                  h.data_ptr(), out.data_ptr(), _code(x, "rows"), n, W, F, E, top, vocab,
-                                 activation_code(activation), _ptr(choice), _ptr(weight), int(identity), _stream()))
+                                 act, _ptr(choice), _ptr(weight), int(identity), bound, _stream()))
     return out
 
 
@@ -1597,7 +1678,7 @@ def moe_down_splits(tiles: int, width: int, ff: int) -> int:
 
 
 def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: torch.Tensor,
-                activation: str = "silu", choice=None, weight=None, identity: int = 0) -> torch.Tensor:
+                activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None) -> torch.Tensor:
     """What ``moe_rows`` computes, with the step's (row, choice) pairs dealt to their experts first: an expert's
     pairs fill tiles of 128 rows, and two grouped products on the matrix cores (gate and up with the activation
     behind them; down with 32-bit sums out) read an expert's weights once a tile.  A last pass adds a row's
@@ -1614,6 +1695,7 @@ def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: 
     else:
         _need(table, "table of experts", None, torch.int32)
         vocab, top = table.shape
+    act, bound = _gate_code(activation, limit)
     out = torch.empty((n, W), dtype=torch.float32, device=x.device)
     if n == 0:
         return out
@@ -1631,11 +1713,11 @@ def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: 
                            tile_group.data_ptr(), stream))
     hidden = torch.empty((slots, F), dtype=torch.bfloat16, device=x.device)
     _check(lib.pl_gemm_tiled_grouped(x.data_ptr(), w_gate_up.data_ptr(), hidden.data_ptr(), tile_group.data_ptr(),
-                                     gather.data_ptr(), 2 * F * W, tiles, n, F, W, 1, activation_code(activation), 1, stream))
+                                     gather.data_ptr(), 2 * F * W, tiles, n, F, W, 1, act, 1, bound, stream))
     splits = moe_down_splits(tiles, W, F)
     y = torch.empty((splits, slots, W), dtype=torch.float32, device=x.device)
     _check(lib.pl_gemm_tiled_grouped(hidden.data_ptr(), w_down.data_ptr(), y.data_ptr(), tile_group.data_ptr(), 0,
-                                     W * F, tiles, slots, W, F, 3, 0, splits, stream))
+                                     W * F, tiles, slots, W, F, 3, 0, splits, 0.0, stream))
     _check(lib.pl_moe_combine(y.data_ptr(), slot_of.data_ptr(), out.data_ptr(), n, top, W, splits, slots * W,
                               _ptr(weight), _ptr(choice), x.data_ptr(), _code(x, "rows"), E, batch.positions.data_ptr(), stream))
     return out
@@ -1652,14 +1734,17 @@ def router_fuses(rows: int, total: int, width: int) -> bool:
 
 
 def router_select(logits, correction, positions, top: int, groups: int = 1, kept: int = 1,
-                  normalised: bool = True, weight_eps: float = 1e-20, x=None, w=None):
+                  normalised: bool = True, weight_eps: float = 1e-20, x=None, w=None, bias=None,
+                  of_chosen: bool = False):
     """A router's choice for every row of its 32-bit ``logits`` [n, outputs]: (chosen [n, top] int32, weights [n, top]
     32-bit).  Scores are the softmax over all outputs; the choice goes by score plus ``correction`` ([outputs] 32-bit, or
     None); outputs form ``groups`` equal groups of neighbours, a group counts by its best choice score, and only members
     of the best ``kept`` groups can be chosen; the ``top`` largest are chosen, the lower index among equals; a chosen
     output weighs its score, divided (``normalised``) by the chosen scores' sum plus ``weight_eps``.  Rows at
     position -1 choose nothing (-1).  With ``logits`` None the kernel works them out itself from the rows ``x`` [n, W]
-    and the router's matrix ``w`` [outputs, W] (one type; 32-bit sums)."""
+    and the router's matrix ``w`` [outputs, W] (one type; 32-bit sums).  ``bias`` ([outputs] 32-bit) is added to the logits
+    first.  ``of_chosen``: the choice goes by the logits themselves and the weights are the softmax over the chosen
+    logits alone (no correction; ``normalised`` and ``weight_eps`` do not enter)."""
     if logits is not None:
         _need(logits, "router logits", None, torch.float32)
         if logits.dim() != 2:
@@ -1674,6 +1759,8 @@ def router_select(logits, correction, positions, top: int, groups: int = 1, kept
         (n, width), total, code, device = x.shape, w.shape[0], _code(x, "rows"), x.device
     if correction is not None:
         _need(correction, "correction of the choice", (total,), torch.float32)
+    if bias is not None:
+        _need(bias, "bias of the router", (total,), torch.float32)
     if positions is not None:
         _need(positions, "positions", (n,), torch.int32)
     choice = torch.empty((n, top), dtype=torch.int32, device=device)
@@ -1681,7 +1768,8 @@ def router_select(logits, correction, positions, top: int, groups: int = 1, kept
     _check(library().pl_router_select(_ptr(logits), total, _ptr(correction), _ptr(positions), n, total, int(top),
                                       int(groups), int(kept), 1 if normalised else 0, float(weight_eps),
                                       choice.data_ptr(), weight.data_ptr(), _ptr(x) if logits is None else 0,
-                                      _ptr(w) if logits is None else 0, int(width), code, _stream()))
+                                      _ptr(w) if logits is None else 0, int(width), code, _ptr(bias),
+                                      1 if of_chosen else 0, _stream()))
     return choice, weight
 
 
@@ -1751,3 +1839,62 @@ def parallel_step(resid: torch.Tensor, a=None, ls1=None, b=None, ls2=None, more=
                                       _ptr(gain2), float(eps), _ptr(out1), _ptr(out2), _CODES[out_dtype], _ptr(rows),
                                       count, W, _stream()))
     return out1, out2
+
+
+# ---- sublayers between two norms; an embedding that looks at the token before ------------------------------------
+
+SANDWICH_MAX_WIDTH = 16384
+
+
+def sandwich_step(resid: torch.Tensor, y=None, norm_y: tuple | None = None, norm_x: tuple | None = None,
+                  out_dtype: torch.dtype = torch.float32, rows=None, centred: bool = True):
+    """One pass over the rows of the 32-bit stream, either half optional.  ``y`` [n, W] (32-bit) joins the stream through
+    the norm ``norm_y``, resid += norm(y), in place; the norm ``norm_x`` of the updated rows comes back in ``out_dtype``
+    (None without it).  A norm is (gain, bias or None, eps), 32-bit, layer norms with ``centred``, RMS norms without.
+    ``rows``: the rows to norm (then nothing joins the stream)."""
+    _need(resid, "residual stream", None, torch.float32)
+    if resid.dim() != 2 or resid.shape[1] > SANDWICH_MAX_WIDTH:
+        raise TensorError(f"a stream of shape {tuple(resid.shape)} (rows of up to {SANDWICH_MAX_WIDTH})")
+    n, W = resid.shape
+    if (y is None) != (norm_y is None) or (y is not None and rows is not None):
+        raise TensorError("what joins the stream needs its norm, and no list of rows")
+    if y is not None:
+        _need(y, "sublayer output", (n, W), torch.float32)
+    for norm, what in ((norm_y, "norm behind a sublayer"), (norm_x, "norm before a sublayer")):
+        if norm is not None:
+            _need(norm[0], f"gain of the {what}", (W,), torch.float32)
+            if norm[1] is not None:
+                _need(norm[1], f"bias of the {what}", (W,), torch.float32)
+    count = n
+    if rows is not None:
+        _need(rows, "rows to norm", None, torch.int32)
+        count = rows.numel()
+    out = torch.empty((count, W), dtype=out_dtype, device=resid.device) if norm_x is not None else None
+    if y is None and norm_x is None:
+        return None
+    gy, by, ey = norm_y if norm_y is not None else (None, None, 0.0)
+    gx, bx, ex = norm_x if norm_x is not None else (None, None, 0.0)
+    _check(library().pl_sandwich_step(resid.data_ptr(), _ptr(y), _ptr(gy), _ptr(by), float(ey), _ptr(gx), _ptr(bx), float(ex),
+                                      _ptr(out), _CODES[out_dtype], _ptr(rows), 1 if centred else 0, count, W, _stream()))
+    return out
+
+
+def bigram_add_(x: torch.Tensor, batch, table: torch.Tensor, last: torch.Tensor, mul_prev: int, mul_cur: int) -> torch.Tensor:
+    """x[t] += table[(token before t * mul_prev + token of t * mul_cur) mod buckets] on the 32-bit stream, ``table``
+    [buckets + 1, W]; a request's first token takes the last row.  ``last`` [slots, 1] (int32) holds a request's last token
+    between steps and is moved on.  Tokens are the batch's, or those an earlier step left on the device."""
+    n, W = x.shape
+    _need(x, "stream", None, torch.float32)
+    _need(table, "table of pairs of tokens")
+    if table.dim() != 2 or table.shape[1] != W or table.shape[0] < 2:
+        raise TensorError(f"a table of pairs of tokens of shape {tuple(table.shape)} for a stream of width {W}")
+    _need(last, "last tokens", None, torch.int32)
+    _step_rows(batch, n)
+    _need(batch.token_ids, "token ids", (n,), torch.int32)
+    fed = getattr(batch, "fed_tokens", None)
+    src = batch.token_src if fed is not None else None
+    _check(library().pl_bigram_add(x.data_ptr(), batch.token_ids.data_ptr(), _ptr(src), _ptr(fed), batch.positions.data_ptr(),
+                                   batch.seq_of.data_ptr(), batch.q_start.data_ptr(), batch.q_len.data_ptr(),
+                                   batch.state_slots.data_ptr(), last.data_ptr(), table.data_ptr(), _code(table, "table of pairs of tokens"),
+                                   int(mul_prev), int(mul_cur), table.shape[0] - 1, n, W, _stream()))
+    return x

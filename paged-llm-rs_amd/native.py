@@ -22,7 +22,7 @@ def _signatures(lib) -> None:
         "plh_pool_allocate": ([vp], i32), "plh_pool_acquire_cached": ([vp, u64], i32),
         "plh_pool_publish": ([vp, i32, u64], None), "plh_pool_release": ([vp, i32], lg),
         "plh_pool_clear_cache": ([vp], None), "plh_pool_counter": ([vp, i32], u64),
-        "plh_cache_create": ([i32, P(i32), P(i32), P(i32), i32], vp), "plh_cache_destroy": ([vp], None),
+        "plh_cache_create": ([i32, P(i32), P(i32), P(i32), P(i32), i32], vp), "plh_cache_destroy": ([vp], None),
         "plh_cache_add_sequence": ([vp, u64], lg), "plh_cache_free_sequence": ([vp, u64], None),
         "plh_cache_has": ([vp, u64], i32), "plh_cache_tokens": ([vp, u64], lg),
         "plh_cache_capacity": ([vp, u64], lg), "plh_cache_blocks_needed": ([vp, u64, sz], lg),

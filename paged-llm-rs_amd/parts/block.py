@@ -15,7 +15,7 @@ import torch
 
 from .. import kernels
 from ..errors import ConfigError
-from .norm import PendingNorm
+from .norm import PendingNorm, bare_decls, bare_params
 from .registry import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, lookup, prefixed, register_block, scoped)
 
 
@@ -542,3 +542,118 @@ class ParallelBlock:
 
 
 register_block("parallel", ParallelBlock)
+
+
+class PendingJoin:
+    """A sublayer's 32-bit output that has not joined the stream yet, and the norm it joins through.  The layer behind
+    adds it in the pass that norms its own rows."""
+
+    __slots__ = ("y", "norm")
+    filled = True            # (what a layer hands to the next is looked at only when it says it holds something)
+
+    def __init__(self, y, norm):
+        self.y, self.norm = y, norm
+
+
+class SandwichBlock:
+    """The arrangement with a norm in front of and behind each sublayer: x <- x + norm1b(mixer(norm1(x))), then
+    x <- x + norm2b(feed_forward(norm2(x))).  A layer whose spec has no feed-forward has the first sublayer only
+    (``norm2`` and ``norm2b``, if a checkpoint carries them, are not used).
+
+    The stream, every norm and every sum into the stream are 32-bit; sublayers hand back 32-bit rows.  One kernel adds
+    a sublayer's output through the norm behind it and norms the next sublayer's rows in the same pass
+    (``kernels.sandwich_step``), also from one layer to the next: a layer that is followed by another of this arrangement
+    leaves its last sum to that layer's first pass (``PendingJoin``), so a layer is two passes over the stream.
+    Tensor names: the norms' gains under the norms' own names, a bias with ``.b`` behind."""
+
+    NAMES = {"norm1": "norm1", "mixer": "mix", "norm1b": "norm1b", "norm2": "norm2", "feed_forward": "mlp", "norm2b": "norm2b"}
+
+    @classmethod
+    def names_of(cls, layer) -> dict:
+        given = getattr(layer, "names", None) or {}
+        unknown = sorted(set(given) - set(cls.NAMES))
+        if unknown:
+            raise ConfigError(f"a layer names members that this arrangement does not have: {unknown}")
+        return {**cls.NAMES, **given}
+
+    @classmethod
+    def declare(cls, layer, hidden: int) -> list:
+        n = cls.names_of(layer)
+        norm = lookup(NORMS, layer.norm.kind, "norm")
+        mixer = lookup(MIXERS, layer.mixer.kind, "mixer")
+        has_ffn = layer.feed_forward is not None
+        decls = []
+        for which in ("norm1", "norm1b", "norm2", "norm2b"):
+            decls += bare_decls(norm, layer.norm, hidden, n[which], optional=which.startswith("norm2") and not has_ffn)
+        decls += prefixed(mixer.declare(layer.mixer, hidden), n["mixer"])
+        if has_ffn:
+            ffn = lookup(FEED_FORWARDS, layer.feed_forward.kind, "feed-forward")
+            decls += prefixed(ffn.declare(layer.feed_forward, hidden), n["feed_forward"])
+        return decls
+
+    def __init__(self, layer, hidden: int, params: dict, dtype, device, shared: dict):
+        n = self.names = self.names_of(layer)
+        norm = lookup(NORMS, layer.norm.kind, "norm")
+        if not hasattr(norm, "sandwich"):
+            raise ConfigError(f"norm {layer.norm.kind!r} cannot run inside the pass over the stream of a layer whose "
+                              "sublayers stand between two norms")
+
+        def norm_of(which):
+            return norm(layer.norm, hidden, bare_params(norm, layer.norm, hidden, n[which], params), dtype, device)
+
+        self.dtype, self.hidden = dtype, hidden
+        self.norm1, self.norm1b = norm_of("norm1"), norm_of("norm1b")
+        self.norm1.takes_pending_join = True       # (how the layer before learns that its last sum can wait)
+        self.mixer = lookup(MIXERS, layer.mixer.kind, "mixer")(
+            layer.mixer, hidden, scoped(params, n["mixer"]), dtype, device, shared)
+        self.norm2 = self.norm2b = self.feed_forward = None
+        if layer.feed_forward is not None:
+            self.norm2, self.norm2b = norm_of("norm2"), norm_of("norm2b")
+            self.feed_forward = lookup(FEED_FORWARDS, layer.feed_forward.kind, "feed-forward")(
+                layer.feed_forward, hidden, scoped(params, n["feed_forward"]), dtype, device, shared)
+
+    @property
+    def graph_safe(self) -> bool:
+        return getattr(self.mixer, "graph_safe", True) and getattr(self.feed_forward, "graph_safe", True)
+
+    @property
+    def first_norm(self):
+        return self.norm1
+
+    @staticmethod
+    def _wide(out):
+        return out if out.dtype == torch.float32 else out.float()
+
+    def _pass(self, resid, y, behind, before):
+        """``y`` joins the stream through the norm ``behind`` it (either may be None); the rows of the norm ``before`` the next sublayer."""
+        centred = (before or behind).centred
+        if behind is not None and before is not None and behind.centred != before.centred:
+            kernels.sandwich_step(resid, y=y, norm_y=behind.sandwich, centred=behind.centred)
+            y = behind = None
+        return kernels.sandwich_step(resid, y=y, norm_y=behind.sandwich if behind is not None else None,
+                                     norm_x=before.sandwich if before is not None else None,
+                                     out_dtype=self.dtype, centred=centred)
+
+    def forward(self, resid, delta, ctx):
+        if delta is not None:
+            kernels.residual_add(resid, delta)
+        pending = getattr(ctx, "handed", None)
+        if isinstance(pending, PendingJoin):
+            rows = self._pass(resid, pending.y, pending.norm, self.norm1)
+        else:
+            rows = self._pass(resid, None, None, self.norm1)
+        y, behind = self._wide(self.mixer.forward(rows, ctx)), self.norm1b
+        if self.feed_forward is not None:
+            rows = self._pass(resid, y, behind, self.norm2)
+            ffn = self.feed_forward
+            out = ffn.forward(rows, batch=ctx.batch) if getattr(ffn, "takes_batch", False) else ffn.forward(rows)
+            y, behind = self._wide(out), self.norm2b
+        after = getattr(ctx, "norm_after", None)
+        if ctx.trace is None and after is not None and getattr(after, "takes_pending_join", False):
+            ctx.handed_out = PendingJoin(y, behind)
+        else:
+            self._pass(resid, y, behind, None)
+        return None
+
+
+register_block("sandwich_norm", SandwichBlock)

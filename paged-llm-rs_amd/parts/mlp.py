@@ -154,7 +154,7 @@ class RoutedExperts:
     do: dealt to their experts and multiplied as grouped products on the matrix cores, or a pair at a time.  Nothing
     depends on the other rows of the step.  The result comes back in 32-bit.
     Tensors: ``e<i>.gate``, ``e<i>.up`` [ff, width], ``e<i>.down`` [width, ff]; ``router`` [experts + identity, width];
-    ``correction`` [experts + identity]."""
+    ``router.b`` and ``correction`` [experts + identity], where the spec has them."""
 
     # forward needs the step (padding rows choose nothing)
     takes_batch = True
@@ -169,15 +169,23 @@ class RoutedExperts:
                       ParamDecl(f"e{e}.down", (hidden, spec.intermediate_size))]
         total = spec.experts + spec.identity
         decls.append(ParamDecl("router", (total, hidden), "router"))
+        if spec.biased:
+            decls.append(ParamDecl("router.b", (total,), "bias"))
         if spec.corrected:
             decls.append(ParamDecl("correction", (total,), "bias"))
         return decls
 
     def __init__(self, spec, hidden: int, params: dict, dtype, device, shared: dict):
-        if spec.activation not in kernels.ACTIVATIONS:
-            raise UnsupportedError(f"activation {spec.activation!r}, the kernels know {', '.join(sorted(kernels.ACTIVATIONS))}")
-        if spec.score != "softmax":
-            raise UnsupportedError(f"router scores of kind {spec.score!r} (softmax)")
+        if spec.activation == kernels.CLAMPED_GATE:
+            if spec.limit is None or not spec.limit > 0:
+                raise UnsupportedError(f"a clamped gate with a limit of {spec.limit}")
+        elif spec.activation not in kernels.ACTIVATIONS or spec.limit is not None:
+            raise UnsupportedError(f"activation {spec.activation!r} (limit {spec.limit}), the kernels know "
+                                   f"{', '.join(sorted(kernels.ACTIVATIONS))} without a limit and {kernels.CLAMPED_GATE} with one")
+        if spec.score not in ("softmax", "chosen_logits"):
+            raise UnsupportedError(f"router scores of kind {spec.score!r} (softmax or chosen_logits)")
+        if spec.score == "chosen_logits" and spec.corrected:
+            raise UnsupportedError("a correction of the scores where the logits themselves choose")
         E, total = spec.experts, spec.experts + spec.identity
         if E < 1 or spec.identity < 0 or not 1 <= spec.top <= total:
             raise UnsupportedError(f"{spec.top} of {E} + {spec.identity} experts a token")
@@ -190,21 +198,22 @@ class RoutedExperts:
         self.w_gate_up = torch.stack([torch.cat([params[f"e{e}.gate"], params[f"e{e}.up"]], 0) for e in range(E)]).contiguous()
         self.w_down = torch.stack([params[f"e{e}.down"] for e in range(E)]).contiguous()
         self.router = Linear(params["router"])
+        self.bias = params["router.b"].to(torch.float32).contiguous() if spec.biased else None
         self.correction = params["correction"].to(torch.float32).contiguous() if spec.corrected else None
 
     def forward(self, x, batch):
         spec = self.spec
+        how = dict(bias=self.bias, of_chosen=spec.score == "chosen_logits")
         if kernels.router_fuses(x.shape[0], self.router.out_features, x.shape[1]):
             # (few rows: the kernel that chooses works the logits out itself)
-            choice, weight = kernels.router_select(None, self.correction, batch.positions, spec.top, spec.groups, spec.groups_kept,
-                                                   spec.normalised, spec.weight_eps, x=x, w=self.router.weight)
+            logits, how["x"], how["w"] = None, x, self.router.weight
         else:
             logits = self.router.forward(x, out_dtype=torch.float32)
-            choice, weight = kernels.router_select(logits, self.correction, batch.positions, spec.top, spec.groups,
-                                                   spec.groups_kept, spec.normalised, spec.weight_eps)
+        choice, weight = kernels.router_select(logits, self.correction, batch.positions, spec.top, spec.groups,
+                                               spec.groups_kept, spec.normalised, spec.weight_eps, **how)
         run = kernels.moe_grouped if kernels.moe_grouped_applies(x, x.shape[1], spec.intermediate_size) else kernels.moe_rows
         return run(x, batch, None, self.w_gate_up, self.w_down, self.activation, choice=choice, weight=weight,
-                   identity=spec.identity)
+                   identity=spec.identity, limit=spec.limit)
 
 
 register_feed_forward("routed_experts", RoutedExperts)

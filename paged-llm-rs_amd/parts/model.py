@@ -19,7 +19,7 @@ from ..weights.loader import ParamDecl, load_weights
 from . import (attention, block, conv_attention, latent_attention, mlp, norm, parallel, recurrent, sink_attention,  # noqa: F401
                tied_attention, transforms)                       # (register the built-in parts)
 from .linear import Linear, linears_of
-from .norm import PendingNorm
+from .norm import PendingNorm, bare_decls, bare_params
 from .registry import BLOCKS, EMBED_TRANSFORMS, FINAL_TRANSFORMS, LOGIT_TRANSFORMS, NORMS, lookup, prefixed, scoped
 from .trace import ActivationTrace
 
@@ -40,6 +40,22 @@ class TransformChain:
         return x
 
 
+class EmbedTransforms(TransformChain):
+    """The transforms of the stream behind the embedding, where one of them keeps something for every request between steps
+    (``state_spec``): it is handed its state of the cache, which keeps it under the transform's place in the chain."""
+
+    def states(self) -> dict:
+        return {("embed_transform", i): m.state_spec() for i, m in enumerate(self.members) if hasattr(m, "state_spec")}
+
+    def __call__(self, x, batch, cache):
+        for i, member in enumerate(self.members):
+            if hasattr(member, "state_spec"):
+                x = member(x, batch, cache.layer_state(("embed_transform", i)))
+            else:
+                x = member(x, batch)
+        return x
+
+
 def _transforms(spec) -> list:
     """(attribute, classes) of the transforms the spec names: of the stream behind the embedding, of the stream
     before the final norm and of the logits.  A spec names one transform or a list of them, applied in that order."""
@@ -56,18 +72,15 @@ def _transforms(spec) -> list:
 
 def _final_norm_decls(spec, final) -> list:
     """The final norm's tensors: under the stem of ``final_norm_name``, or, where the spec says that a norm's
-    gain is stored under the norm's own name (``extra["bare_norm_names"]``), the one tensor of that name."""
+    gain is stored under the norm's own name (``extra["bare_norm_names"]``), under that (a bias with ``.b`` behind)."""
     if (spec.extra or {}).get("bare_norm_names"):
-        decls = final.declare(spec.final_norm, spec.hidden_size)
-        if len(decls) != 1:
-            raise ConfigError(f"a norm of {len(decls)} tensors cannot be stored under its own name alone")
-        return [ParamDecl(spec.final_norm_name, decls[0].shape, decls[0].role, decls[0].optional)]
+        return bare_decls(final, spec.final_norm, spec.hidden_size, spec.final_norm_name)
     return prefixed(final.declare(spec.final_norm, spec.hidden_size), spec.final_norm_name.rsplit(".", 1)[0])
 
 
 def _final_norm_params(spec, final, params: dict) -> dict:
     if (spec.extra or {}).get("bare_norm_names"):
-        return {final.declare(spec.final_norm, spec.hidden_size)[0].name: params[spec.final_norm_name]}
+        return bare_params(final, spec.final_norm, spec.hidden_size, spec.final_norm_name, params)
     return scoped(params, spec.final_norm_name.rsplit(".", 1)[0])
 
 
@@ -93,7 +106,7 @@ class LayerContext:
     the pages of the layer it reads from) and its state slots."""
 
     __slots__ = ("batch", "cache", "layer", "cache_layer", "writes_cache", "residual", "trace", "hand", "handed",
-                 "norm_after", "handed_out", "stream_rows", "stream_addend")
+                 "norm_after", "handed_out", "stream_rows", "stream_addend", "carried")
 
     def __init__(self, batch, cache, layer: int, cache_layer: int, writes_cache: bool):
         # ``layer`` and ``cache_layer`` are the keys under which the cache keeps this run's state and the pages it
@@ -123,6 +136,9 @@ class LayerContext:
         # schedule says so), for a block that takes them into its own first pass (``takes_stream_addend``) and
         # clears this; for any other block the decoder has added them already and this is None.
         self.stream_addend = None
+        # What one layer of a pass leaves for later layers of the same pass, by name (the values that later layers mix
+        # into theirs, say): one dict for all runs of a pass, empty at its start.
+        self.carried: dict = {}
 
     def kv(self):
         return self.cache.layer_view(self.cache_layer, self.batch)
@@ -161,13 +177,17 @@ class DecoderModel:
         self.embed_transform = self.final_transform = self.logit_transform = None
         for key, classes in _transforms(spec):
             members = [cls(spec, params, dtype, self.device) for cls in classes]
-            setattr(self, key, members[0] if len(members) == 1 else TransformChain(members))
+            if key == "embed_transform" and any(hasattr(m, "state_spec") for m in members):
+                self.embed_transform = EmbedTransforms(members)
+            else:
+                setattr(self, key, members[0] if len(members) == 1 else TransformChain(members))
         for entry in spec.schedule:
             if not 0 <= entry.layer < len(self.blocks):
                 raise ConfigError(f"the schedule names layer {entry.layer} of {len(self.blocks)}")
             if entry.cache_from is not None and entry.cache_key is not None:
                 raise ConfigError(f"a run of layer {entry.layer} both keeps a cache of its own and reads another's")
-        self.cache_layout = CacheLayout.from_blocks(self.blocks, spec.schedule)
+        self.cache_layout = CacheLayout.from_blocks(self.blocks, spec.schedule,
+                                                    self.embed_transform.states() if self._embedding_keeps_state else None)
         self.graph_safe = (all(getattr(b, "graph_safe", True) for b in self.blocks)
                            and getattr(self.embed_transform, "graph_safe", True)
                            and getattr(self.final_transform, "graph_safe", True)
@@ -177,6 +197,10 @@ class DecoderModel:
         self.portion_limits = tuple(sorted({int(limit) for b in self.blocks
                                             for limit in [getattr(getattr(b, "mixer", None), "short_portion", None)]
                                             if limit}))
+
+    @property
+    def _embedding_keeps_state(self) -> bool:
+        return isinstance(self.embed_transform, EmbedTransforms)
 
     def matrix_bytes(self) -> tuple:
         """(bytes of the weight matrices as stored, bytes of their second copies in strips)."""
@@ -212,12 +236,14 @@ class DecoderModel:
         resid = kernels.embed(batch.token_ids, self.embed_tokens,
                               src=batch.token_src if fed is not None else None, fed=fed)
         if self.embed_transform is not None:
-            resid = self.embed_transform(resid, batch)
+            resid = (self.embed_transform(resid, batch, cache) if self._embedding_keeps_state
+                     else self.embed_transform(resid, batch))
         if top is not None:
             top.record(self.spec.embed_name.rsplit(".", 1)[0] + ".out", resid)
         delta = None
         handed = None
         stream_rows = None
+        carried: dict = {}
         schedule = self.spec.schedule
         # (kept only where a run of the schedule adds it to the stream again)
         began_with = resid.clone() if any(e.add_embedding for e in schedule) else None
@@ -231,6 +257,7 @@ class DecoderModel:
                 prefix = self.spec.layers[entry.layer].weight_prefix
                 ctx.trace = top.child(prefix if again == 0 else f"{prefix}.run{again}")
             ctx.handed = handed
+            ctx.carried = carried
             ctx.stream_rows = stream_rows
             if entry.add_embedding:
                 if getattr(self.blocks[entry.layer], "takes_stream_addend", False):

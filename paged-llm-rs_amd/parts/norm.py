@@ -1,10 +1,11 @@
-"""RMSNorm fused with the residual add (reference: model/layers.rs:40-65)."""
+"""RMSNorm fused with the residual add (reference: model/layers.rs:40-65), and the layer norm with a bias."""
 
 from __future__ import annotations
 
 import torch
 
 from .. import kernels
+from ..errors import ConfigError
 from ..weights.loader import ParamDecl
 from .registry import register_norm
 
@@ -36,6 +37,26 @@ class PendingNorm:
         return self.norm.apply(self.resid, None, self.out_dtype, rows=self.rows)
 
 
+def bare_names(norm, spec, width: int, stem: str) -> list:
+    """[(a norm's local tensor name, its name under ``stem``)] where a gain is stored under the norm's own name: the one
+    tensor of an RMS norm is ``stem``; a bias beside the gain is ``stem.b``."""
+    names = [d.name for d in norm.declare(spec, width)]
+    known = {"weight": stem, "bias": stem + ".b"}
+    if names[0] != "weight" or any(n not in known for n in names):
+        raise ConfigError(f"a norm of the tensors {', '.join(names)} cannot be stored under its own name")
+    return [(n, known[n]) for n in names]
+
+
+def bare_decls(norm, spec, width: int, stem: str, optional: bool = False) -> list:
+    """A norm's tensors under the norm's own name (``bare_names``)."""
+    names = dict(bare_names(norm, spec, width, stem))
+    return [ParamDecl(names[d.name], d.shape, d.role, d.optional or optional) for d in norm.declare(spec, width)]
+
+
+def bare_params(norm, spec, width: int, stem: str, params: dict) -> dict:
+    return {local: params[name] for local, name in bare_names(norm, spec, width, stem)}
+
+
 class RmsNorm:
     """x / sqrt(mean(x^2) + eps) * gain, statistic and product in 32-bit.  A spec with a ``gain_offset`` stores
     its gains as distances from that number (gains around zero for an offset of one): the sum is taken once,
@@ -58,6 +79,14 @@ class RmsNorm:
         # the product kernels that take the norm as their first stage read the gain in 32-bit
         self.gain32 = self.gain if self.gain.dtype == torch.float32 else self.gain.float()
 
+    @property
+    def sandwich(self) -> tuple:
+        """(gain, bias, eps) for the pass over a layer whose sublayers stand between two norms."""
+        return self.gain32, None, self.eps
+
+    # what that pass is told: no mean is taken off
+    centred = False
+
     def handoff(self, rows: int, device):
         """Room for this norm handed forward by a product that adds into the stream (``kernels.HandedNorm``),
         or None where no product would take it: many rows, a wide stream."""
@@ -79,3 +108,34 @@ class RmsNorm:
 
 
 register_norm("rms_norm", RmsNorm)
+
+
+class LayerNorm:
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * gain + bias, all in 32-bit, rounded once at the store."""
+
+    centred = True
+
+    @staticmethod
+    def declare(spec, width: int) -> list:
+        return [ParamDecl("weight", (width,), "gain"), ParamDecl("bias", (width,), "bias")]
+
+    def __init__(self, spec, width: int, params: dict, dtype, device):
+        if width > kernels.SANDWICH_MAX_WIDTH:
+            raise ConfigError(f"a layer norm over rows of {width} (up to {kernels.SANDWICH_MAX_WIDTH})")
+        self.eps, self.width = float(spec.eps), width
+        self.gain = params["weight"].to(torch.float32).contiguous()
+        self.bias = params["bias"].to(torch.float32).contiguous()
+
+    @property
+    def sandwich(self) -> tuple:
+        return self.gain, self.bias, self.eps
+
+    def apply(self, resid: torch.Tensor, delta, out_dtype: torch.dtype, rows=None) -> torch.Tensor:
+        if delta is not None:
+            if rows is not None:
+                raise ConfigError("a sum into the stream beside a list of rows")
+            kernels.residual_add(resid, delta)
+        return kernels.sandwich_step(resid, norm_x=self.sandwich, out_dtype=out_dtype, rows=rows)
+
+
+register_norm("layer_norm", LayerNorm)

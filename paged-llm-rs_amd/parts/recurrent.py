@@ -1,7 +1,8 @@
 """Mixers that keep a matrix of state a head instead of keys and values in pages: linear attention with
-a fixed decay, the matrix memory with exponential gates (mLSTM), and the gated delta rule.
+a fixed decay, the matrix memory with exponential gates (mLSTM), the gated delta rule, and the state space
+whose decay and step size come from the token (Mamba-2).
 
-All three are one product for every projection of the layer's input (32-bit sums out), the scan over
+All of them are one product for every projection of the layer's input (32-bit sums out), the scan over
 the step's tokens request by request (``kernels.recurrent_scan``: state, gates, decays and read-out in
 32-bit, from and into the request's state slot), a norm over groups of the read-out times a gate, and
 the output projection.  A request's state is one run of 32-bit floats in its slot; what a step's result
@@ -25,7 +26,7 @@ def _f32(t: torch.Tensor) -> torch.Tensor:
 
 
 class _ScanMixer:
-    """What the three have in common: the fused projection and where its pieces lie in a row."""
+    """What they have in common: the fused projection and where its pieces lie in a row."""
 
     graph_safe = True
 
@@ -166,6 +167,61 @@ class GatedDelta(_ScanMixer):
         return self.o_proj.forward(normed, out_dtype=torch.float32)
 
 
+class StateSpace(_ScanMixer):
+    """One projection [z | x | B | C | dt]; x, B and C pass a short convolution with bias and silu together (channels of
+    all heads side by side) and are v, k and q of the scan (``kernels.recurrent_scan``, kind ``ssd``).  The read-out is
+    gated by silu(z) first and normed then, in equal parts of all heads' values together.
+    Tensors: ``in``, ``conv`` [channels, taps], ``conv.b``, ``dt_bias``, ``A_log``, ``D`` (one a head), ``norm``, ``o``."""
+
+    @staticmethod
+    def declare(spec, hidden: int) -> list:
+        H, inner = spec.num_heads, spec.num_heads * spec.value_dim
+        channels = inner + 2 * spec.groups * spec.state_dim
+        return [ParamDecl("in", (inner + channels + H, hidden)), ParamDecl("conv", (channels, spec.conv_taps), "filter"),
+                ParamDecl("conv.b", (channels,), "bias"), ParamDecl("dt_bias", (H,), "bias"), ParamDecl("A_log", (H,), "bias"),
+                ParamDecl("D", (H,), "gain"), ParamDecl("norm", (inner,), "gain"), ParamDecl("o", (hidden, inner))]
+
+    def __init__(self, spec, hidden: int, params: dict, dtype, device, shared: dict):
+        H, G, N, V = spec.num_heads, spec.groups, spec.state_dim, spec.value_dim
+        if H < 1 or V < 1 or not 1 <= N <= kernels.SCAN_MAX_DIM:
+            raise UnsupportedError(f"a state space of {H} heads of {N} by {V}: the scan takes states up to {kernels.SCAN_MAX_DIM} rows")
+        if G < 1 or H % G:
+            raise UnsupportedError(f"{H} heads over {G} groups of B and C, which do not group evenly")
+        if not 1 <= spec.conv_taps <= 16:
+            raise UnsupportedError(f"a convolution of {spec.conv_taps} taps (1 to 16)")
+        if spec.norm_groups < 1 or (H * V) % spec.norm_groups:
+            raise UnsupportedError(f"a norm over {H * V} values in {spec.norm_groups} equal parts")
+        self.spec, self.dtype = spec, dtype
+        self.H, self.G, self.N, self.V = H, G, N, V
+        self.inner = H * V
+        self.channels = self.inner + 2 * G * N
+        self.proj = Linear(params["in"])
+        self.conv_w = _f32(params["conv"]).t().contiguous()                # [taps, channels]
+        self.conv_b = _f32(params["conv.b"])
+        self.o_proj = Linear(params["o"])
+        self.gain, self.skip = _f32(params["norm"]), _f32(params["D"])
+        self.a_log, self.dt_bias = _f32(params["A_log"]), _f32(params["dt_bias"])
+        self.matrix = H * N * V
+
+    def state_spec(self):
+        # S [H, N, V], then the convolution's last taps - 1 inputs [taps - 1, channels]
+        return StateSpec((self.matrix + (self.spec.conv_taps - 1) * self.channels,), torch.float32)
+
+    def forward(self, x, ctx):
+        inner, G, N = self.inner, self.G, self.N
+        state = ctx.state()
+        rows = self.proj.forward(x, out_dtype=torch.float32)
+        mixed = kernels.short_conv(rows, inner, self.conv_w, state[:, self.matrix:], ctx.batch, silu=True, bias=self.conv_b,
+                                   move_history=True)
+        read = kernels.recurrent_scan("ssd", mixed, inner + G * N, inner, 0, state[:, :self.matrix], ctx.batch, self.H, G, N,
+                                      self.V, gates=rows, g1_off=inner + self.channels, p1=self.a_log, p2=self.dt_bias,
+                                      p3=self.skip, chunked=True)
+        normed = kernels.gated_group_norm(read, inner // self.spec.norm_groups, self.gain, self.spec.eps, self.dtype,
+                                          gate=rows, gate_off=0, gate_act="silu", gate_first=True)
+        return self.o_proj.forward(normed, out_dtype=torch.float32)
+
+
 register_mixer("lightning_attention", LightningAttention)
 register_mixer("mlstm", Mlstm)
 register_mixer("gated_delta", GatedDelta)
+register_mixer("state_space", StateSpace)

@@ -28,6 +28,8 @@ transform     of the stream behind the embedding (``register_embed_transform``) 
               ``__init__(spec, params, dtype, device)`` (``params``: all tensors by checkpoint name);
               ``__call__(x, batch) -> x``: the 32-bit stream [rows, hidden] (padding rows have
               position -1), or the 32-bit logits [wanted rows, vocabulary]; it may work in place.
+              A transform behind the embedding that keeps something for every request between steps has
+              ``state_spec() -> StateSpec`` and is called with its state, [slots, ...], as a third argument.
               A third kind (``register_final_transform``, ``extra["final_transform"]``) stands between the
               last layer and the final norm: it gets the stream as the layers leave it and gives the rows
               whose logits are wanted, [wanted rows, hidden] in 32-bit (the sum of several copies of the

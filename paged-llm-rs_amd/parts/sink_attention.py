@@ -2,10 +2,13 @@
 denominator, q and k as unit vectors (divided by their root mean square over a head, with or without a
 gain), biases on the projections, a query temperature that grows with the logarithm of the position, a
 penalty a head on the distance between query and key, and a window or a mask of blocks (a query sees the
-keys of its own block of positions, blocks counted from the request's position 0).
+keys of its own block of positions, blocks counted from the request's position 0).  A window may keep the first tokens of a
+request in sight of every later one (their pages stay).  Scores may pass a soft cap, values may be mixed with those of the
+first layer that mixes (handed on through ``LayerContext.carried``: its projected rows, whatever the order of the layers),
+and a head's read-out may be multiplied by a gate worked out from the layer's input.
 
 weights_ij = exp(s_ij) / (exp(sink_h) + sum over the visible j of exp(s_ij)),
-s_ij = scale (q_i . k_j) - slope_h (i - j); a sink has no key and no value, so a row's weights sum to
+s_ij = cap(scale (q_i . k_j)) - slope_h (i - j); a sink has no key and no value, so a row's weights sum to
 less than one.  One kernel stands between the projection and the attention kernel (unit vectors,
 temperature, queries out, keys and values into the pages), all in 32-bit from the projection's 32-bit
 sums, one rounding at the store.  Query/key heads and value heads may differ in size: every head is
@@ -63,6 +66,10 @@ class SinkAttention:
             decls.append(ParamDecl("sink", (H,), "bias"))
         if spec.qk_gain:
             decls += [ParamDecl("q.norm", (D,), "gain"), ParamDecl("k.norm", (D,), "gain")]
+        if spec.head_gate:
+            decls.append(ParamDecl("g", (H, hidden)))
+        if spec.value_mix:
+            decls.append(ParamDecl("vmix", (), "share"))
         if spec.qkv_bias:
             decls += [ParamDecl("q.b", (H * D,), "bias"), ParamDecl("k.b", (G * D,), "bias"), ParamDecl("v.b", (G * V,), "bias")]
         return decls
@@ -71,6 +78,10 @@ class SinkAttention:
         H, G, D, V = spec.num_heads, spec.num_kv_heads, spec.head_dim, spec.value_dim
         if spec.mask not in ("window", "block"):
             raise UnsupportedError(f"a mask of kind {spec.mask!r} (window or block)")
+        if spec.keep_first and (spec.mask != "window" or spec.window is None):
+            raise UnsupportedError(f"{spec.keep_first} first tokens kept in sight where no window would hide them")
+        if spec.softcap is not None and not spec.softcap > 0:
+            raise UnsupportedError(f"a soft cap of {spec.softcap} on the scores")
         if spec.qk_gain and spec.qk_unit_eps is None:
             raise UnsupportedError("a gain on q and k that are not divided by their root mean square")
         if H < 1 or G < 1 or H % G:
@@ -91,7 +102,10 @@ class SinkAttention:
         # keeps what it fuses, and a pass over the rows is saved)
         self.bias = (torch.cat([params["q.b"], params["k.b"], params["v.b"]]).to(torch.float32).contiguous()
                      if spec.qkv_bias else None)
-        self.proj = Linear.fused([params["q"], params["k"], params["v"]])
+        self.proj = Linear.fused([params["q"], params["k"], params["v"]] + ([params["g"]] if spec.head_gate else []))
+        self.v_off, self.gate_off = (H + G) * D, (H + G) * D + G * V
+        self.v_bias = self.bias[self.v_off:] if self.bias is not None else None
+        self.share = float(params["vmix"]) if spec.value_mix else 0.0
         self.q_gain = params["q.norm"].to(torch.float32).contiguous() if spec.qk_gain else None
         self.k_gain = params["k.norm"].to(torch.float32).contiguous() if spec.qk_gain else None
         self.sinks = head_sinks(spec.sink, H, params, device)
@@ -107,10 +121,22 @@ class SinkAttention:
 
     def cache_spec(self):
         # (no key further back than the block's size is ever read: pages behind it come back as behind a window)
-        return KVCacheSpec(self.G, self.padded, self.window or None)
+        return KVCacheSpec(self.G, self.padded, self.window or None, keep_first=int(self.spec.keep_first))
 
     def state_spec(self):
         return None
+
+    def _mix(self, rows, ctx):
+        """What ``kernels.head_prepare`` needs to mix this layer's values: None where they stay as they are."""
+        if not self.spec.value_mix:
+            return None
+        carried = ctx.carried.setdefault("values", (rows, self.v_off, self.v_bias, self.G * self.V))
+        if carried[0] is rows:
+            return None                           # (the first layer that mixes: its values are what the others mix in)
+        first, off, bias, width = carried
+        if width != self.G * self.V:
+            raise UnsupportedError(f"values of {self.G * self.V} mixed with values of {width}")
+        return first, off, bias, self.share
 
     def forward(self, x, ctx):
         """``x``: the normed rows, or a norm still to run.  The output comes back as 32-bit sums, or None where the output projection
@@ -121,10 +147,13 @@ class SinkAttention:
         q = torch.empty((n, self.H * self.padded), dtype=self.dtype, device=rows.device)
         kernels.head_prepare(rows, 0, batch, kv, q, self.H, self.G, self.D, self.V, self.padded,
                              unit_eps=self.spec.qk_unit_eps, q_gain=self.q_gain, k_gain=self.k_gain,
-                             temperature=self.temperature, write_kv=ctx.writes_cache, bias=self.bias)
+                             temperature=self.temperature, write_kv=ctx.writes_cache, bias=self.bias, mix=self._mix(rows, ctx))
+        more = None
+        if self.spec.softcap is not None or self.spec.keep_first or self.spec.head_gate:
+            more = kernels.AttentionMore(self.spec.softcap, self.spec.keep_first, rows if self.spec.head_gate else None, self.gate_off)
         out = torch.empty((n, self.H * self.padded), dtype=self.dtype, device=rows.device)
         kernels.sink_attention(q, out, batch, kv, self.H, self.G, self.padded, self.scale, self.mask,
-                               sinks=self.sinks, slopes=self.slopes)
+                               sinks=self.sinks, slopes=self.slopes, more=more)
         return self.o_proj.forward(out, out_dtype=torch.float32, add_into=getattr(ctx, "residual", None))
 
 

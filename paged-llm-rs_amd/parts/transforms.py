@@ -5,6 +5,7 @@ from __future__ import annotations
 import torch
 
 from .. import kernels
+from ..cache.layout import StateSpec
 from ..errors import ConfigError
 from ..weights.loader import ParamDecl
 from .registry import NORMS, lookup, register_embed_transform, register_final_transform, register_logit_transform
@@ -65,6 +66,33 @@ class StreamNorm:
     def __call__(self, x, batch):
         # (the normalised rows in 32-bit are the stream from here on)
         return self.norm.apply(x, None, torch.float32)
+
+
+class BigramEmbedding:
+    """x[t] <- x[t] + table[(token before t * mul_prev + token of t * mul_cur) mod buckets], a second embedding row chosen by
+    a pair of tokens; a request's first token takes the row behind the buckets.  ``extra["bigram"]`` = (table name,
+    buckets, mul_prev, mul_cur).  The token before a step's first one is state: kept for each request in a slot."""
+
+    graph_safe = True
+
+    @staticmethod
+    def declare(spec) -> list:
+        name, buckets, _, _ = spec.extra["bigram"]
+        return [ParamDecl(name, (buckets + 1, spec.hidden_size), "embedding")]
+
+    def __init__(self, spec, params: dict, dtype, device):
+        name, _, self.mul_prev, self.mul_cur = spec.extra["bigram"]
+        self.table = params[name]
+
+    @staticmethod
+    def state_spec() -> StateSpec:
+        return StateSpec((1,), torch.int32)
+
+    def __call__(self, x, batch, state):
+        return kernels.bigram_add_(x, batch, self.table, state, self.mul_prev, self.mul_cur)
+
+
+register_embed_transform("bigram", BigramEmbedding)
 
 
 class LogitScale:

@@ -45,6 +45,12 @@ def random_tensor(name: str, shape, role: str, seed: int, std: float, gain_std: 
         x = 1.0 + x * gain_std
     elif role == "gain_around_zero":
         x = x * gain_std
+    elif role == "filter":
+        # the taps of a short convolution, [channels, taps]: the current token's leads
+        x = x * 0.3 / shape[-1] ** 0.5
+        x[:, -1] += 0.7
+    elif role == "share":
+        x = torch.sigmoid(x)
     elif role == "copy_in":
         # weights with which the copies of the stream are read: around an even share each
         x = (1.0 + x * gain_std) / shape[0]
