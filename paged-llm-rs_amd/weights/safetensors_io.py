@@ -133,6 +133,6 @@ def write_safetensors(path, tensors, metadata: dict | None = None) -> None:
                 t = make().contiguous()
                 if tuple(t.shape) != tuple(shape) or t.dtype != dtype:
                     raise WeightError(f"{name}: made {tuple(t.shape)} {t.dtype}, declared {shape} {dtype}")
-                f.write(t.view(torch.uint8).numpy().tobytes() if t.numel() else b"")
+                f.write(t.reshape(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b"")
     except OSError as e:
         raise IoError(f"writing {path}: {e}") from e

@@ -1,0 +1,903 @@
+"""The Guzuvik design in the engine against the plain implementation: the new kernels alone (the pass between two norms,
+the embedding row of a pair of tokens, the state space's scan token by token and in chunks, the convolution with bias that
+moves its history on, the norm behind a gate, attention with a cap, kept keys and gates on every kernel, mixed values, the
+router of chosen logits, experts with clamped gates), every mixer and feed-forward alone, whole prompts, tokens decoded
+one by one, portions down to two tokens, mixed batches with pages and slots used again, keys far away under a sharp
+softmax, keys just inside and just outside a window and among the kept first ones (in prompts and while decoding, at page
+borders), caps, mixtures, gates and biases that carry weight, the first tokens of a request, long decoding, other sizes,
+and greedy generation through the engine's own entry point and the command line."""
+
+from __future__ import annotations
+
+import copy
+import json
+import math
+import random
+import subprocess
+import sys
+from pathlib import Path
+
+import numpy as np
+import pytest
+import torch
+
+import guzuvik_util as gu
+import replay_util as ru
+
+pytestmark = pytest.mark.gpu
+
+# Against the plain implementation (64-bit): 32-bit runs are held tightly.  In bfloat16 a run gets a loose bound there
+# and a tight one against the engine's own whole-prompt run of the same requests (the same roundings; what differs
+# between schedules is the cache and the batch: a lost key shows there in full).  All bounds are for a position that
+# amplifies rounding as the median position does, and grow with a position's own amplification.  A position at which a
+# router decides by less than MARGIN of logit is left out: the choice may fall the other way under rounding.
+TOLERANCE = {"float32": 5e-5, "bfloat16": 0.1}
+MARGIN = {"float32": 2e-5, "bfloat16": 5e-2}
+BETWEEN_SCHEDULES = 4e-2
+DTYPES = ["float32", "bfloat16"]
+F = torch.float64
+
+
+def replayer(folder, dtype, prompts, live=4, block_size=16, graphs=True):
+    from paged_llm_rs_amd.engine.replay import Replayer
+
+    return Replayer(folder, dtype, max_tokens=ru.pool_tokens(prompts, live), block_size=block_size, max_live=live,
+                    graphs=graphs)
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    made = {}
+
+    def get(name, dtype):
+        if (name, dtype) not in made:
+            made[name, dtype] = gu.write_model(tmp_path_factory.mktemp(f"guzuvik_{name}_{dtype}"), gu.CONFIGS[name],
+                                               seed=sorted(gu.CONFIGS).index(name) + 1, dtype=dtype)
+        return made[name, dtype]
+    return get
+
+
+_whole: dict = {}
+_factor: dict = {}
+_plain: dict = {}
+_close: dict = {}
+
+
+def check(folder, dtype, prompts, steps, live=4, block_size=16, tolerance=None, between=BETWEEN_SCHEDULES, most_close=0.5):
+    r = replayer(folder, dtype, prompts, live, block_size)
+    got = ru.collect(r, steps)
+    key = (str(folder), repr(sorted(prompts.items())))
+    if key not in _plain:
+        _plain[key] = gu.plain_logits(folder, prompts)
+        _factor[key] = gu.sensitivity(folder, prompts)
+    if (key, dtype) not in _close:
+        _close[key, dtype] = gu.close_calls(folder, prompts, MARGIN[dtype], _factor[key])
+    want, factor, close = _plain[key], _factor[key], _close[key, dtype]
+    compared = {k: row for k, row in got.items() if not bool(close[k[0]][k[1]])}
+    assert len(compared) >= (1 - most_close) * len(got), f"{len(got) - len(compared)} of {len(got)} positions are close calls of a router"
+    scale = max(float(want[n][p].abs().max()) for (n, p) in got)
+    bound = tolerance or TOLERANCE[dtype]
+    worst = {}
+    for (n, p), row in compared.items():
+        ref = want[n][p].numpy()
+        assert row.shape == ref.shape
+        err = float(np.abs(row.astype(np.float64) - ref).max()) / scale
+        if not err <= bound * float(factor[n][p]):
+            worst[n, p] = err / (bound * float(factor[n][p]))
+    # (in bfloat16 another token's close call may reach a position through what layers carry)
+    spare = 0 if dtype == "float32" else max(1, len(got) // 50)
+    assert len(worst) <= spare and all(x <= 4.0 for x in worst.values()), \
+        f"over the bound by {sorted(worst.items(), key=lambda x: -x[1])[:5]} of {len(got)}"
+    assert r.cache.manager.live_sequences == 0, "every request's pages came back"
+    if dtype == "bfloat16":
+        if key not in _whole:
+            _whole[key] = ru.collect(replayer(folder, dtype, prompts, live), ru.whole(prompts))
+        spread = float(np.mean([want[n][p].std() for (n, p) in got]))
+        over = {}
+        for (n, p), row in compared.items():
+            gap = float(np.sqrt(np.mean((row - _whole[key][(n, p)]) ** 2))) / spread
+            if not gap <= between * float(factor[n][p]):
+                over[n, p] = gap / (between * float(factor[n][p]))
+        assert len(over) <= max(1, len(got) // 50) and all(x <= 3.0 for x in over.values()), \
+            f"between this schedule and the whole prompt, over the bound by {sorted(over.items(), key=lambda x: -x[1])[:5]} of {len(got)}"
+    return r, got
+
+
+# --- the new kernels alone --------------------------------------------------------------------------------------------
+
+def dev(t, dtype=torch.float32):
+    return t.to(dtype).cuda().contiguous()
+
+
+class Step:
+    """What a kernel reads of a step of requests that bring ``counts`` tokens, request i from position ``starts[i]`` on."""
+
+    def __init__(self, counts, starts=None, slots=None, ids=None, padding=0):
+        starts = starts or [0] * len(counts)
+        slots = slots if slots is not None else list(range(len(counts)))
+        i32 = lambda x: torch.tensor(x, dtype=torch.int32).cuda()
+        n = sum(counts) + padding
+        positions, seq_of, q_start, at = [], [], [], 0
+        for s, (c, first) in enumerate(zip(counts, starts)):
+            positions += list(range(first, first + c))
+            seq_of += [s] * c
+            q_start.append(at)
+            at += c
+        if padding:
+            positions += [-1] * padding
+            seq_of += [len(counts)] * padding
+            counts, slots, q_start = counts + [padding], slots + [-1], q_start + [at]
+        self.positions, self.seq_of, self.q_start, self.q_len = i32(positions), i32(seq_of), i32(q_start), i32(counts)
+        self.state_slots = i32(slots)
+        self.ctx_len = i32([f + c for f, c in zip(starts, counts)] + ([0] if padding else []))
+        self.num_seqs, self.num_tokens = len(counts), n
+        self.live_seqs = self.num_seqs - (1 if padding else 0)
+        self.max_q_len, self.max_ctx_len = max(counts), max(1024, int(self.ctx_len.max()))
+        self.token_ids = i32(ids if ids is not None else [0] * n)
+        self.token_src = self.fed_tokens = None
+        self.counts = list(counts)[:self.live_seqs]
+
+    def tokens_of_short_requests(self, limit):
+        return sum(c for c in self.counts if c < limit)
+
+
+def close_to(got, want, tol):
+    assert torch.isfinite(got).all()
+    err = float((got.double().cpu() - want).abs().max()) / max(float(want.abs().max()), 1e-30)
+    assert err <= tol, err
+
+
+@pytest.mark.parametrize("centred", [True, False])
+@pytest.mark.parametrize("width", [52, 75, 200, 1024, 4096, 5000, 9001, 12288])
+def test_the_pass_between_two_norms(width, centred):
+    """A sublayer's output joins the stream through its norm and the next norm reads the updated row: together and each
+    alone, with and without biases, for chosen rows, both types of rows out; rows whose mean is far above their spread."""
+    from paged_llm_rs_amd import kernels
+
+    g = torch.Generator().manual_seed(width)
+    n, eps = 21, 1e-5
+    x, y = torch.randn((n, width), generator=g) * 3, torch.randn((n, width), generator=g) * 2
+    x[3], y[4] = x[3] * 0.01 + 50.0, y[4] * 0.01 - 30.0
+    ga, gb = (1 + 0.4 * torch.randn((width,), generator=g) for _ in range(2))
+    ba, bb = (0.5 * torch.randn((width,), generator=g) for _ in range(2))
+
+    def norm(u, gain, bias):
+        u = u.double()
+        if centred:
+            u = u - u.mean(-1, keepdim=True)
+        out = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * gain.double()
+        return out if bias is None else out + bias.double()
+
+    for biased in (True, False):
+        na, nb = (dev(ga), dev(ba) if biased else None, eps), (dev(gb), dev(bb) if biased else None, eps)
+        summed = x.double() + norm(y, ga, ba if biased else None)
+        for dtype, tol in ((torch.float32, 2e-4), (torch.bfloat16, 8e-3)):       # (row 3's spread is a 5000th of its mean)
+            stream = dev(x)
+            rows = kernels.sandwich_step(stream, y=dev(y), norm_y=na, norm_x=nb, out_dtype=dtype, centred=centred)
+            close_to(stream, summed, 2e-5)
+            assert rows.dtype == dtype
+            close_to(rows, norm(stream.cpu(), gb, bb if biased else None), tol)
+        stream = dev(x)
+        close_to(kernels.sandwich_step(stream, norm_x=nb, centred=centred), norm(x, gb, bb if biased else None), 2e-4)
+        assert torch.equal(stream, dev(x)), "a norm alone changes nothing"
+        assert kernels.sandwich_step(stream, y=dev(y), norm_y=na, centred=centred) is None
+        close_to(stream, summed, 2e-5)
+        chosen = torch.tensor([5, 0, 20, 5], dtype=torch.int32).cuda()
+        got = kernels.sandwich_step(stream, norm_x=nb, rows=chosen, centred=centred)
+        close_to(got, norm(stream.cpu(), gb, bb if biased else None)[chosen.cpu().long()], 2e-4)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("buckets,mul_prev,mul_cur,width", [(101, 31, 5, 72), (1, 3, 4, 52), (50021, 2000000011, 999999937, 300), (7, 0, 1, 64)])
+def test_the_row_of_a_pair_of_tokens(dtype, buckets, mul_prev, mul_cur, width):
+    """Whole prompts, portions and single tokens against rows worked out by hand; the last token waits in the request's
+    slot; a token that the step before left on the device; slots used again; rows of padding stay."""
+    from paged_llm_rs_amd import kernels
+
+    g = torch.Generator().manual_seed(buckets)
+    table = torch.randn((buckets + 1, width), generator=g).to(dtype)
+    last = torch.zeros((5, 1), dtype=torch.int32).cuda()
+    rng = random.Random(buckets)
+    tokens = {s: [rng.randrange(200000) for _ in range(40)] for s in range(4)}
+    at = {s: 0 for s in tokens}
+
+    def row(s, p):
+        if p == 0:
+            return buckets
+        return (tokens[s][p - 1] * mul_prev + tokens[s][p] * mul_cur) % buckets
+
+    for step in ([(0, 5), (1, 1)], [(1, 3), (0, 1), (2, 2)], [(0, 1), (1, 1), (2, 1)], [(2, 17), (3, 20), (0, 1)], [(3, 2), (1, 30)]):
+        ids = [t for s, c in step for t in tokens[s][at[s]:at[s] + c]]
+        b = Step([c for _, c in step], [at[s] for s, _ in step], [4 - s for s, _ in step], ids + [0, 0, 0], padding=3)
+        x = torch.randn((b.num_tokens, width), generator=g)
+        want = x.clone()
+        k = 0
+        for s, c in step:
+            for p in range(at[s], at[s] + c):
+                want[k] += table[row(s, p)].float()
+                k += 1
+            at[s] += c
+        got = kernels.bigram_add_(dev(x), b, table.cuda(), last, mul_prev, mul_cur)
+        assert torch.equal(got.cpu(), want)
+        for s, c in step:
+            assert int(last[4 - s, 0]) == tokens[s][at[s] - 1]
+    # a single token known on the device only
+    b = Step([1, 1], [at[0], at[3]], [4, 1], [0, tokens[3][at[3]]])
+    b.token_src = torch.tensor([2, -1], dtype=torch.int32).cuda()
+    b.fed_tokens = torch.tensor([9, 9, tokens[0][at[0]]], dtype=torch.int32).cuda()
+    x = torch.zeros((2, width))
+    got = kernels.bigram_add_(dev(x), b, table.cuda(), last, mul_prev, mul_cur)
+    assert torch.equal(got.cpu(), torch.stack([table[row(0, at[0])], table[row(3, at[3])]]).float())
+    assert int(last[4, 0]) == tokens[0][at[0]]
+
+
+@pytest.mark.parametrize("H,G,N,V", [(6, 3, 20, 12), (4, 2, 128, 64), (5, 1, 8, 24), (2, 1, 150, 70), (1, 1, 1, 17), (3, 3, 64, 1), (8, 1, 64, 96)])
+@pytest.mark.parametrize("kind", ["mild", "wild"])
+def test_the_state_spaces_scan(H, G, N, V, kind):
+    """Requests of many tokens (in chunks) beside short ones and single tokens, from and into their slots, and again in other
+    portions, against the plain recurrence in 64-bit.  Wild: decays that forget everything within a token beside decays
+    near one, in the same chunk."""
+    from paged_llm_rs_amd import kernels
+    import plain_guzuvik as plain
+
+    g = torch.Generator().manual_seed(H * 100 + N)
+    T = [170, 64, 3, 1, 65, 33]
+    inner, off = H * V, 3
+    x, B, C = ([torch.randn((t, w), generator=g) for t in T] for w in (inner, G * N, G * N))
+    raw = [torch.randn((t, H), generator=g) * (1.0 if kind == "mild" else 6.0) - 1.0 for t in T]
+    a_log = torch.randn((H,), generator=g) * (0.7 if kind == "mild" else 2.0)
+    bias, skip = torch.randn((H,), generator=g) * 0.5, torch.randn((H,), generator=g)
+    want = [plain.state_space_scan(x[i].double().view(-1, H, V), B[i].double().view(-1, G, N), C[i].double().view(-1, G, N),
+                                   plain.softplus((raw[i] + bias).double()), a_log.double(), skip.double()).reshape(-1, inner)
+            for i in range(len(T))]
+    scale = max(float(w.abs().max()) for w in want)
+
+    def run(plan, slots):
+        """``plan``: steps of (request, tokens)."""
+        state = torch.full((8, H * N * V + 5), 7.0).cuda()
+        state[:, :H * N * V] = 0
+        at, got = {i: 0 for i in range(len(T))}, {i: [] for i in range(len(T))}
+        for step in plan:
+            b = Step([c for _, c in step], [at[i] for i, _ in step], [slots[i] for i, _ in step], padding=2)
+            rows = torch.zeros((b.num_tokens, off + inner + 2 * G * N))
+            gates = torch.zeros((b.num_tokens, H + 4))
+            k = 0
+            for i, c in step:
+                span = slice(at[i], at[i] + c)
+                rows[k:k + c, off:] = torch.cat([x[i][span], B[i][span], C[i][span]], -1)
+                gates[k:k + c, 4:] = raw[i][span]
+                k += c
+            out = kernels.recurrent_scan("ssd", dev(rows), off + inner + G * N, off + inner, off, state[:, :H * N * V], b, H, G, N, V,
+                                         gates=dev(gates), g1_off=4, p1=dev(a_log), p2=dev(bias), p3=dev(skip), chunked=True).double().cpu()
+            k = 0
+            for i, c in step:
+                got[i].append(out[k:k + c])
+                at[i] += c
+                k += c
+        assert (state[:, H * N * V:] == 7.0).all(), "nothing beside the state is touched"
+        for i, pieces in got.items():
+            err = float((torch.cat(pieces) - want[i]).abs().max()) / scale
+            assert err <= 3e-5, (i, err)
+
+    run([[(i, t) for i, t in enumerate(T)]], [5, 0, 3, 1, 7, 2])
+    run([[(0, 15), (1, 16), (2, 1), (4, 63)], [(0, 64), (2, 1), (1, 48), (5, 2)], [(0, 1), (3, 1), (4, 2), (2, 1)], [(0, 90), (5, 31)]],
+        [0, 1, 2, 3, 4, 5])
+
+
+@pytest.mark.parametrize("taps", [1, 2, 3, 4, 5, 16])
+def test_the_convolution_with_a_bias_that_moves_its_history_on(taps):
+    """Portions, then single tokens (one launch for both the convolution and its history), against whole sequences."""
+    from paged_llm_rs_amd import kernels
+    import plain_guzuvik as plain
+
+    g = torch.Generator().manual_seed(taps)
+    C, off, T = 300, 7, [40, 25, 18]
+    w, bias = torch.randn((C, taps), generator=g), torch.randn((C,), generator=g)
+    u = [torch.randn((t, C), generator=g) for t in T]
+    want = [plain.silu(plain.causal_convolution(x.double(), w.double(), bias.double())) for x in u]
+    history = torch.zeros((6, (taps - 1) * C + 9)).cuda()
+    at, slots = [0, 0, 0], [4, 1, 2]
+    plan = [[(0, 5), (1, 1)], [(0, 1), (2, 2)], [(1, 9), (2, 1), (0, 2)]] + [[(i, 1) for i in range(3)]] * 12 + [[(0, 20), (1, 3), (2, 3)]]
+    for step in plan:
+        b = Step([c for _, c in step], [at[i] for i, _ in step], [slots[i] for i, _ in step])
+        rows = torch.randn((b.num_tokens, off + C + 2), generator=g)
+        rows[:, off:off + C] = torch.cat([u[i][at[i]:at[i] + c] for i, c in step])
+        out = kernels.short_conv(dev(rows), off, dev(w.t()), history[:, 9:], b, silu=True, bias=dev(bias), move_history=True)
+        ref = torch.cat([want[i][at[i]:at[i] + c] for i, c in step])
+        assert (out.double().cpu() - ref).abs().max() <= 2e-5 * ref.abs().max()
+        for i, c in step:
+            at[i] += c
+    assert at == T and (history[:, :9] == 0).all() and (history[0] == 0).all()
+
+
+@pytest.mark.parametrize("width,group", [(72, 36), (120, 30), (1024, 512), (4096, 2048), (2080, 1040), (6000, 6000), (64, 64)])
+def test_the_norm_behind_a_gate(width, group):
+    from paged_llm_rs_amd import kernels
+
+    g = torch.Generator().manual_seed(width)
+    n, off, eps = 19, 5, 1e-5
+    x, gate = torch.randn((n, width), generator=g) * 2, torch.randn((n, off + width + 3), generator=g) * 2
+    gain = 1 + 0.3 * torch.randn((width,), generator=g)
+    z = gate[:, off:off + width].double()
+    u = (x.double() * z * torch.sigmoid(z)).view(n, -1, group)
+    want = (u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps)).reshape(n, width) * gain.double()
+    for dtype, tol in ((torch.float32, 3e-6), (torch.bfloat16, 8e-3)):
+        got = kernels.gated_group_norm(dev(x), group, dev(gain), eps, dtype, gate=dev(gate), gate_off=off, gate_act="silu", gate_first=True)
+        close_to(got, want, tol)
+
+
+def _attend(q, k, v, positions, first_pos, scale, window, keep, cap, slopes, gates):
+    """One request, 64-bit: q [n, H, d] at ``positions``, k and v [T, G, d]."""
+    n, H, d = q.shape
+    T, G = k.shape[:2]
+    i, j = positions[:, None], torch.arange(T)[None, :]
+    seen = j <= i
+    if window:
+        seen = seen & ((i - j < window) | (j < keep))
+    out = torch.zeros((n, H, d), dtype=F)
+    for h in range(H):
+        s = (q[:, h] @ k[:, h // (H // G)].T) * scale
+        if cap:
+            s = cap * torch.tanh(s / cap)
+        s = s - slopes[h] * (i - j)
+        s = s.masked_fill(~seen, -math.inf)
+        out[:, h] = torch.softmax(s, -1) @ v[:, h // (H // G)]
+    return out * torch.sigmoid(gates)[:, :, None]
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,G,d,page", [(4, 4, 64, 16), (4, 2, 128, 16), (8, 2, 96, 16), (8, 1, 64, 16), (16, 1, 128, 8), (16, 2, 48, 16),
+                                        (3, 1, 32, 5), (6, 1, 192, 16)])
+@pytest.mark.parametrize("window,keep", [(0, 0), (37, 5), (64, 64), (70, 200), (1, 1), (150, 17)])
+def test_attention_with_a_cap_kept_keys_and_gates(dtype, H, G, d, page, window, keep):
+    """Every kernel (portions on the matrix cores in one and in several shares, single tokens in one and in several shares, grouped heads, the
+    plain one) through scattered pages, against 64-bit arithmetic.  Pages behind the window that keep no first key are gone from the
+    table, and every row of the pools that is not a key of the request holds NaN: a key that is not to be seen cannot hide.
+    A key in three of the kept ones and one just outside the window are made to stand out for some queries."""
+    from paged_llm_rs_amd import kernels
+    from paged_llm_rs_amd.cache.pools import LayerKV
+
+    g = torch.Generator().manual_seed(H * 1000 + d + window)
+    T, cap, scale = 420, 3.0, 4.0 / d
+    slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)])
+    k, v = torch.randn((T, G, d), generator=g).to(dtype), torch.randn((T, G, d), generator=g).to(dtype)
+    pages = -(-T // page)
+    order = (torch.randperm(pages + 3, generator=g)[:pages]).tolist()
+    pool_k = torch.full(((pages + 3) * page, G * d), math.nan, dtype=dtype)
+    pool_v = pool_k.clone()
+    for j in range(T):
+        at = order[j // page] * page + j % page
+        pool_k[at], pool_v[at] = k[j].reshape(-1), v[j].reshape(-1)
+    tol = 2e-5 if dtype == torch.float32 else 2e-2
+
+    def run(first, count, splits=None):
+        positions = torch.arange(first, first + count)
+        q = torch.randn((count, H, d), generator=g)
+        for t, p in enumerate(positions.tolist()):
+            for target, every in ((min(max(keep - 1, 0), p), 3), (max(keep, p - window), 4), (max(p - max(window, 1) + 1, 0), 5)):
+                if t % every == 0:
+                    q[t] = k[target].float()[:, None, :].expand(G, H // G, d).reshape(H, d) * 3
+        q = q.to(dtype)
+        gates = torch.randn((count, 3 + H + 2), generator=g)
+        b = Step([count], [first])
+        b.max_ctx_len = 1024
+        b.ctx_len = torch.tensor([first + count], dtype=torch.int32).cuda()
+        table = list(order)
+        pk, pv = pool_k.clone(), pool_v.clone()
+        for i in range(pages):                # what a step that starts here has given back, and what it has not written yet
+            dead = window and (i + 1) * page <= first - window + 1 and i >= -(-keep // page)
+            if dead or i * page >= first + count:
+                pk[table[i] * page:(table[i] + 1) * page] = math.nan
+                pv[table[i] * page:(table[i] + 1) * page] = math.nan
+                table[i] = -1
+        for j in range(first + count, T):
+            pk[order[j // page] * page + j % page] = math.nan
+            pv[order[j // page] * page + j % page] = math.nan
+        kv = LayerKV(pk.cuda(), pv.cuda(), torch.tensor([table], dtype=torch.int32).cuda(), page, 0)
+        more = kernels.AttentionMore(cap, keep, dev(gates), 3)
+        want = _attend(q.double(), k.double(), v.double(), positions, first, scale, window, keep, cap, slopes.double(), gates[:, 3:3 + H].double())
+        rows = q.reshape(count, H * d).cuda().contiguous()
+        outs = []
+        if splits is None:
+            out = torch.empty((count, H * d), dtype=dtype, device="cuda")
+            kernels.sink_attention(rows, out, b, kv, H, G, d, scale, window, slopes=dev(slopes), more=more)
+            outs.append(out)
+        else:
+            kind, n = splits
+            out = torch.empty((count, H * d), dtype=dtype, device="cuda")
+            if kind == "decode":
+                kernels.paged_attention_decode(rows, H * d, out, b.positions, b.seq_of, kv.block_table, page, kv.k_pool, kv.v_pool, H, G, d,
+                                               scale, window, n, slopes=dev(slopes), more=more)
+            elif kind == "prefill":
+                kernels.paged_attention_prefill(rows, H * d, out, b.q_start, b.q_len, b.ctx_len, count, kv.block_table, page, kv.k_pool,
+                                                kv.v_pool, H, G, d, scale, window, splits=n, slopes=dev(slopes), more=more)
+            else:
+                kernels.paged_attention_grouped(rows, H * d, out, b.q_start, b.q_len, b.ctx_len, count, kv.block_table, page, kv.k_pool,
+                                                kv.v_pool, H, G, d, scale, window, splits=n, slopes=dev(slopes), more=more)
+            outs.append(out)
+        for out in outs:
+            assert torch.isfinite(out).all(), (first, count, splits)
+            err = float((out.double().cpu().view(count, H, d) - want).abs().max())
+            assert err <= tol * 4, (first, count, splits, err)
+
+    for first, count in ((0, 1), (0, 20), (0, 200), (36, 1), (37, 1), (63, 3), (130, 90), (205, 17), (300, 1), (301, 2), (419, 1), (355, 65)):
+        run(first, count)
+    if dtype == torch.bfloat16:
+        for first, count, splits in ((400, 1, ("decode", 3)), (250, 9, ("decode", 2)), (150, 1, ("decode", 64)), (3, 1, ("decode", 4)),
+                                     (290, 130, ("prefill", 2)), (0, 64, ("prefill", 3)), (200, 150, ("prefill", 6)), (388, 20, ("prefill", 1))):
+            run(first, count, splits)
+        if kernels.library().pl_paged_attention_grouped_applies(H, G, d, page):
+            for first, count, n in ((400, 1, 3), (250, 9, 1), (150, 2, 5), (3, 1, 2)):
+                run(first, count, ("grouped", n))
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,G,D,V,page", [(6, 2, 24, 40, 16), (4, 4, 40, 20, 4), (1, 1, 16, 16, 16)])
+def test_values_mixed_with_an_earlier_layers(dtype, H, G, D, V, page):
+    from paged_llm_rs_amd import kernels
+    from paged_llm_rs_amd.cache.pools import LayerKV
+
+    g = torch.Generator().manual_seed(D)
+    n, off, first_off, eps, share = 20, 3, 7, 1e-5, 0.3
+    padded = max(D, V) if dtype == torch.float32 else (max(D, V) + 15) // 16 * 16
+    rows = torch.randn((n, off + (H + G) * D + G * V + 2), generator=g)
+    first = torch.randn((n, first_off + G * V + 4), generator=g)
+    bias, first_bias = torch.randn(((H + G) * D + G * V,), generator=g), torch.randn((G * V,), generator=g)
+    b = Step([n], [5], padding=0)
+    pages = -(-25 // page)
+    kv = LayerKV(torch.zeros((pages * page, G * padded), dtype=dtype).cuda(), torch.full((pages * page, G * padded), 7.0, dtype=dtype).cuda(),
+                 torch.arange(pages, dtype=torch.int32).view(1, -1).cuda(), page, 0)
+    q = torch.zeros((n, H * padded), dtype=dtype).cuda()
+    for fb in (first_bias, None):
+        kernels.head_prepare(dev(rows), off, b, kv, q, H, G, D, V, padded, unit_eps=eps, bias=dev(bias),
+                             mix=(dev(first), first_off, dev(fb) if fb is not None else None, share))
+        own = (rows[:, off + (H + G) * D:off + (H + G) * D + G * V] + bias[(H + G) * D:]).double()
+        other = first[:, first_off:first_off + G * V].double() + (fb.double() if fb is not None else 0)
+        want = ((1 - share) * own + share * other).view(n, G, V)
+        got = kv.v_pool.double().cpu()[5:25].view(n, G, padded)
+        assert (got[..., :V] - want).abs().max() <= (2e-6 if dtype == torch.float32 else 8e-3) * want.abs().max() and (got[..., V:] == 0).all()
+        u = (rows[:, off:off + H * D] + bias[:H * D]).double().view(n, H, D)
+        u = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps)
+        close_to(q.view(n, H, padded)[..., :D], u, 2e-6 if dtype == torch.float32 else 8e-3)
+
+
+@pytest.mark.parametrize("total,top", [(12, 2), (9, 9), (1, 1), (64, 6), (300, 5), (5, 3)])
+def test_a_router_of_chosen_logits(total, top):
+    from paged_llm_rs_amd import kernels
+
+    g = torch.Generator().manual_seed(total * 31 + top)
+    n, width = 120, 96
+    bias = torch.randn((total,), generator=g) * 2
+    positions = torch.arange(n, dtype=torch.int32)
+    positions[17] = -1
+    rows = [t for t in range(n) if t != 17]
+    z = torch.randn((n, total), generator=g) * 40          # (far apart: a softmax over all of them would be next to nothing for most)
+    chosen, weight = kernels.router_select(dev(z), None, positions.cuda(), top, bias=dev(bias), of_chosen=True)
+    best, at = (z.float() + bias.float()).double().topk(top, -1)
+    assert (chosen.cpu()[17] == -1).all() and (weight.cpu()[17] == 0).all()
+    assert torch.equal(chosen.cpu()[rows].long(), at[rows])
+    assert (weight.cpu().double() - torch.softmax(best, -1))[rows].abs().max() <= 2e-5
+    for dtype in (torch.float32, torch.bfloat16):
+        x, w = torch.randn((n, width), generator=g).to(dtype), (torch.randn((total, width), generator=g) * 0.3).to(dtype)
+        z = x.double() @ w.double().T + bias.double()
+        chosen, weight = kernels.router_select(None, None, positions.cuda(), top, x=x.cuda(), w=w.cuda(), bias=dev(bias), of_chosen=True)
+        best, at = z.topk(top, -1)
+        same = [t for t in rows if torch.equal(chosen.cpu()[t].long(), at[t])]
+        assert len(same) >= n - 3
+        assert (weight.cpu().double() - torch.softmax(best, -1))[same].abs().max() <= 2e-5
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("experts,top,ff,width,rows,limit", [(8, 3, 64, 160, 50, 1.0), (3, 3, 44, 52, 7, 0.6), (1, 1, 24, 100, 9, 7.0),
+                                                             (16, 4, 128, 256, 300, 2.0), (4, 1, 256, 512, 129, 0.8)])
+def test_experts_with_clamped_gates(dtype, experts, top, ff, width, rows, limit):
+    from paged_llm_rs_amd import kernels
+
+    g = torch.Generator().manual_seed(experts * 100 + rows)
+    w_gu = (torch.randn((experts, 2 * ff, width), generator=g) * 2 * width ** -0.5).to(dtype)
+    w_down = (torch.randn((experts, width, ff), generator=g) * ff ** -0.5).to(dtype)
+    x = torch.randn((rows, width), generator=g).to(dtype)
+    choice = torch.rand((rows, experts), generator=g).argsort(1)[:, :top].to(torch.int32)
+    weight = torch.rand((rows, top), generator=g)
+    want = torch.zeros((rows, width), dtype=F)
+    for t in range(rows):
+        for c, e in enumerate(choice[t].tolist()):
+            both = w_gu[e].double() @ x[t].double()
+            a, u = torch.clamp(both[:ff], max=limit), torch.clamp(both[ff:], -limit, limit)
+            hidden = a * torch.sigmoid(1.702 * a) * (u + 1)
+            if dtype == torch.bfloat16:
+                hidden = hidden.to(torch.bfloat16).double()
+            want[t] += (w_down[e].double() @ hidden) * weight[t, c].double()
+    b = Step([rows])
+    args = (x.cuda(), b, None, w_gu.cuda(), w_down.cuda(), "clamped")
+    got = kernels.moe_rows(*args, choice=choice.cuda(), weight=dev(weight), limit=limit)
+    close_to(got, want, 1e-5 if dtype == torch.float32 else 2e-2)
+    if dtype == torch.bfloat16 and kernels.moe_grouped_applies(x.cuda(), width, ff):
+        dealt = kernels.moe_grouped(*args, choice=choice.cuda(), weight=dev(weight), limit=limit)
+        close_to(dealt, got.double().cpu(), 1e-2)
+
+
+def test_the_squared_relu():
+    from paged_llm_rs_amd import kernels
+
+    x = torch.randn((37, 60), generator=torch.Generator().manual_seed(0)) * 3
+    for dtype, tol in ((torch.float32, 1e-7), (torch.bfloat16, 5e-3)):
+        y = x.to(dtype)
+        close_to(kernels.activation(y.cuda(), "relu2"), torch.clamp(y.double(), min=0) ** 2, tol)
+
+
+# --- every mixer and feed-forward alone, in 32-bit, the stream behind the layer against the plain implementation's ----
+
+ALONE = {
+    "attention, everything": [gu.attention(6, 3, 24, 32, 0.6, window=11, keep=3, cap=1.5, mix=True)],
+    "attention, nothing": [gu.attention(2, 1, 40, 40, 0.2)],
+    "attention, a window that keeps more than it sees": [gu.attention(4, 1, 16, 24, 0.3, window=4, keep=19)],
+    "attention, a cap": [gu.attention(2, 2, 16, 16, 1.0, cap=0.7, mix=False)],
+    "mamba2": [gu.mamba(6, 10, 24, groups=3, conv=4, parts=4)],
+    "mamba2, one of everything": [gu.mamba(1, 1, 1, groups=1, conv=1, parts=1)],
+    "mamba2, a large state": [gu.mamba(2, 72, 136, groups=2, conv=6, parts=3)],
+    "dense feed-forward": [gu.mamba(1, 16, 4, mlp=gu.dense(136))],
+    "experts": [gu.mamba(1, 16, 4, mlp=gu.moe(6, 3, 40, 0.8))],
+    "values mixed over three layers": [gu.attention(2, 2, 16, 12, 0.3, mix=True), gu.mamba(2, 8, 8), gu.attention(4, 1, 20, 24, 0.4, mix=True),
+                                       gu.attention(2, 1, 8, 16, 0.4), gu.attention(8, 4, 8, 6, 0.5, mix=True)],
+}
+
+
+@pytest.mark.parametrize("which", sorted(ALONE))
+def test_a_layer_alone_against_its_plain_function(tmp_path, which):
+    """32-bit, the stream behind every layer against the plain implementation's: whole, and again in portions (the later
+    portions read what the earlier ones left in pages and slots)."""
+    layers = ALONE[which]
+    config = gu.model(88, 61, layers, eps=1e-5, bigram=(37, 5, 11))
+    folder = gu.write_model(tmp_path / "m", config, seed=7, std=0.2)
+    tokens = [random.Random(3).randrange(61) for _ in range(45)]
+    cfg, weights = gu.load_plain(folder)
+    want = []
+    gu.plain.forward(cfg, weights, tokens, want)
+    names = [f"l{i}.out" for i in range(len(layers))]
+    r = replayer(folder, "float32", {"a": tokens}, graphs=False)
+    rec = {}
+    r.step([{"id": "a", "tokens": tokens, "want": []}], ["a"], trace=rec)
+    for name, stream in zip(names, want):
+        assert (rec[name].double().cpu() - stream).abs().max() <= 5e-5 * stream.abs().max(), (which, name)
+    pieces, at = {name: [] for name in names}, 0
+    for n in (1, 2, 17, 3, 22):
+        rec = {}
+        r.step([{"id": "b", "tokens": tokens[at:at + n], "want": []}], ["b"] if at + n == 45 else [], trace=rec)
+        for name in names:
+            pieces[name].append(rec[name].double().cpu())
+        at += n
+    for name, stream in zip(names, want):
+        assert (torch.cat(pieces[name]) - stream).abs().max() <= 5e-5 * stream.abs().max(), (which, name, "in portions")
+
+
+# --- whole models of other sizes under every schedule ------------------------------------------------------------------
+
+LENGTHS = [70, 3, 41, 18, 1, 33, 57]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(gu.CONFIGS))
+def test_whole_prompts(folders, name, dtype):
+    prompts = ru.make_prompts(gu.CONFIGS[name]["vocab"], LENGTHS, seed=1)
+    check(folders(name, dtype), dtype, prompts, ru.whole(prompts))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(gu.CONFIGS))
+def test_prefill_then_tokens_one_by_one(folders, name, dtype):
+    prompts = ru.make_prompts(gu.CONFIGS[name]["vocab"], LENGTHS, seed=1)
+    check(folders(name, dtype), dtype, prompts, ru.tail_decoded(prompts, tail=40))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(gu.CONFIGS))
+@pytest.mark.parametrize("block_size", [16, 8])
+def test_portions_down_to_two_tokens(folders, name, dtype, block_size):
+    prompts = ru.make_prompts(gu.CONFIGS[name]["vocab"], LENGTHS, seed=1)
+    check(folders(name, dtype), dtype, prompts, ru.portions(prompts), block_size=block_size)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(gu.CONFIGS))
+@pytest.mark.parametrize("seed", [0, 1])
+def test_unequal_requests_together_with_pages_and_slots_used_again(folders, name, dtype, seed):
+    """Nine requests of unequal length through a pool and slots for four: portions of some beside single tokens of others,
+    requests left out of steps, pages and slots of finished requests taken by the next."""
+    prompts = ru.make_prompts(gu.CONFIGS[name]["vocab"], [70, 3, 41, 18, 1, 33, 57, 64, 22], seed=2 + seed)
+    check(folders(name, dtype), dtype, prompts, ru.mixed(prompts, seed=seed, max_live=4, tail=14))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("seed", range(12))
+def test_drawn_configurations(tmp_path, seed, dtype):
+    """Twelve drawn models (order of layers, sizes, head counts, windows, kept tokens, caps, mixtures, states, taps, experts,
+    constants; `guzuvik_util.drawn_config`) under a mixed schedule and whole, over pages of 16, 8 and 32."""
+    config = gu.drawn_config(100 + seed)
+    folder = gu.write_model(tmp_path / "m", config, seed=seed, dtype=dtype, std=0.1)
+    prompts = ru.make_prompts(config["vocab"], [75, 9, 130, 33, 2], seed=seed)
+    block_size = (16, 8, 32)[seed % 3]
+    check(folder, dtype, prompts, ru.mixed(prompts, seed=seed, max_live=3, tail=20), live=3, block_size=block_size, most_close=0.6)
+    check(folder, dtype, prompts, ru.whole(prompts), live=3, block_size=block_size, most_close=0.6)
+
+
+def test_schedules_agree_with_each_other_in_32_bit(folders):
+    folder = folders("odd", "float32")
+    prompts = ru.make_prompts(gu.ODD["vocab"], LENGTHS, seed=1)
+    close = gu.close_calls(folder, prompts, 1e-4)
+    whole = ru.collect(replayer(folder, "float32", prompts), ru.whole(prompts))
+    scale = max(float(np.abs(row).max()) for row in whole.values())
+    for steps in (ru.tail_decoded(prompts, tail=40), ru.portions(prompts), ru.mixed(prompts, seed=5)):
+        for key, row in ru.collect(replayer(folder, "float32", prompts), steps).items():
+            if not bool(close[key[0]][key[1]]):
+                assert float(np.abs(row - whole[key]).max()) <= 2e-5 * scale, key
+
+
+# --- keys far away, edges of windows, kept first tokens, states that reach far ----------------------------------------------
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_one_key_among_hundreds_under_a_sharp_softmax(tmp_path, dtype):
+    """Scales several times the usual under a high cap make every softmax sharp, and a penalty that is small for the last heads
+    lets its weight lie hundreds of tokens back: a key lost at a page border, at the edge of a tile of keys or between
+    shares of the context moves the logits in full."""
+    config = gu.model(64, 90, [gu.attention(8, 2, 32, 32, 1.2, cap=60.0, mix=True, mlp=gu.dense(64)),
+                               gu.attention(8, 1, 64, 32, 0.5, window=300, keep=70, cap=40.0, mlp=gu.moe(4, 2, 32, 2.0)),
+                               gu.attention(4, 2, 32, 32, 1.0, window=400, keep=20, mix=True)], bigram=(500, 17, 5))
+
+    def edit(tensors):
+        gu.telling(tensors)
+        for name in list(tensors):           # (without the biases a key is its token's own)
+            if name.endswith(("q.b", "k.b")):
+                tensors[name] = tensors[name] * 0.2
+
+    folder = gu.write_model(tmp_path / "m", config, seed=11, dtype=dtype, std=0.15, edit=edit)
+    prompts = ru.make_prompts(90, [700, 333], seed=4)
+    cfg, w = gu.load_plain(folder)
+    # the test's own premise: the first layer's softmaxes are sharp and their heaviest keys lie far back
+    m = cfg["layers"][0]["mixer"]
+    h = gu.plain.layer_norm(gu.plain.embed(cfg, w, torch.tensor(prompts["r0"])), w["l0.norm1"], w["l0.norm1.b"], 1e-6)
+    q = gu.plain.rms((h @ w["l0.mix.q"].T + w["l0.mix.q.b"]).view(700, 8, 32), 1e-6)
+    k = gu.plain.rms((h @ w["l0.mix.k"].T + w["l0.mix.k.b"]).view(700, 2, 32), 1e-6)
+    distance = torch.arange(700)[:, None] - torch.arange(700)[None, :]
+    score = gu.plain.capped(q[:, 7] @ k[:, 1].T * m["scale"], m["softcap"]) - 2.0 ** -8 * distance
+    score = score.masked_fill(distance < 0, -np.inf)
+    far = (torch.arange(700) - score.argmax(-1))[400:]
+    assert (far > 100).double().mean() > 0.3 and torch.softmax(score, -1).max(-1).values[400:].median() > 0.25
+    steps = ru.tail_decoded(prompts, tail=48)
+    for s in steps:            # every seventh position of the long first steps is compared, and every decoded token
+        for e in s["entries"]:
+            e["want"] = list(range(0, len(e["tokens"]), 7)) + ([len(e["tokens"]) - 1] if (len(e["tokens"]) - 1) % 7 else [])
+    loose = 0.5 if dtype == "bfloat16" else 2e-4
+    check(folder, dtype, prompts, steps, live=2, tolerance=loose, between=5 * BETWEEN_SCHEDULES, most_close=0.6)
+    check(folder, dtype, prompts, ru.portions(prompts, sizes=(130, 2, 61, 16, 17, 300, 5)), live=2, tolerance=loose,
+          between=5 * BETWEEN_SCHEDULES, most_close=0.6)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("window,keep", [(1, 1), (2, 0), (16, 3), (17, 16), (33, 17), (15, 32), (64, 15), (20, 1)])
+def test_keys_just_inside_and_just_outside_a_window_and_the_first_ones(tmp_path, dtype, window, keep):
+    """A layer whose scale is small, so that its softmax is flat and every key it sees carries its share of the
+    weight: the engine's logits are the plain implementation's with this size of the window and these kept tokens, and
+    clearly not those with a window one token larger or smaller or one kept token more or fewer, in prompts, in portions and
+    for tokens decoded one by one, with pages of 16 and of 4 tokens (edges at a page's border, before it and behind it).  Slopes are
+    what they are: the last head's is small enough for every key of these prompts."""
+    config = gu.model(48, 70, [gu.attention(8, 2, 16, 24, 0.02, window=window, keep=keep, cap=9.0)])
+
+    def edit(tensors):
+        gu.telling(tensors)
+        for name in list(tensors):
+            if name.endswith((".v.b", "norm1b.b")):
+                tensors[name] = tensors[name] * 0.05
+            elif name == "embed" or name.endswith((".q.b", ".k.b")):
+                tensors[name] = tensors[name] / 12
+            elif name.endswith(".mix.o"):            # (the heads whose penalty lets them see only the nearest keys)
+                tensors[name][:, :5 * 24] = 0
+
+    folder = gu.write_model(tmp_path / "m", config, seed=20 + window, dtype=dtype, std=0.25, edit=edit)
+    prompts = ru.make_prompts(70, [90, 49], seed=6)
+    want = gu.plain_logits(folder, prompts)
+    others = []
+    for change in ({"size": window - 1}, {"size": window + 1}, {"keep_first": keep - 1}, {"keep_first": keep + 1}):
+        if min(change.values()) >= (1 if "size" in change else 0):
+            changed = copy.deepcopy(config)
+            changed["layers"][0]["mixer"]["mask"].update(change)
+            others.append(gu.plain_logits(folder, prompts, changed))
+    for block_size in (16, 4):
+        for steps in (ru.whole(prompts), ru.tail_decoded(prompts, tail=45), ru.portions(prompts, sizes=(18, 2, 15, 33, 3))):
+            got = ru.collect(replayer(folder, dtype, prompts, live=2, block_size=block_size), steps)
+            closer = total = 0
+            for (n, p), row in got.items():
+                err = float(np.sqrt(np.mean((row - want[n][p].numpy()) ** 2)))
+                for o in others:
+                    moved = float(((want[n][p] - o[n][p]) ** 2).mean().sqrt())
+                    if moved < (1e-9 if dtype == "float32" else 2e-2) * float(want[n][p].std()):
+                        continue          # (a position that sees the same keys under both, or whose difference is next to nothing)
+                    total += 1
+                    closer += err < (0.25 if dtype == "float32" else 0.5) * moved
+            assert closer >= (total if dtype == "float32" else 0.9 * total), (block_size, closer, total)
+            assert total > 5 or dtype == "bfloat16", "(in bfloat16 a wide window's edge is told by the kernels' own test)"
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_a_token_that_a_state_remembers(tmp_path, dtype):
+    """Decays near one: changing the first tokens changes the logits hundreds of tokens later, and the engine follows the plain
+    implementation there, whatever the schedule; a state that a slot's last owner left would show."""
+    config = gu.model(64, 60, [gu.mamba(4, 16, 32, groups=2, conv=4, parts=2, mlp=gu.dense(48)), gu.mamba(2, 24, 16, conv=3)])
+
+    def edit(tensors):
+        gu.telling(tensors)
+        for name in list(tensors):
+            if name.endswith(".A_log"):
+                tensors[name] = tensors[name] * 0 - 6.0
+
+    folder = gu.write_model(tmp_path / "m", config, seed=5, dtype=dtype, std=0.15, edit=edit)
+    prompts = ru.make_prompts(60, [400, 150, 31, 260], seed=3)
+    cfg, w = gu.load_plain(folder)
+    base = gu.plain.forward(cfg, w, prompts["r0"])
+    other = gu.plain.forward(cfg, w, [(t + 7) % 60 for t in prompts["r0"][:100]] + prompts["r0"][100:])
+    assert float((base - other)[-1].std() / base[-1].std()) > 0.02
+    check(folder, dtype, prompts, ru.tail_decoded(prompts, tail=60), live=1)
+    check(folder, dtype, prompts, ru.mixed(prompts, seed=3, max_live=2, tail=30), live=2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_caps_gates_mixtures_biases_and_pairs_that_carry_weight(tmp_path, dtype):
+    """The engine agrees with the plain implementation, whose logits move by far more than the engine's error when the
+    cap, the kept tokens, the mixture or the second embedding is taken away, when the step sizes' or the routers' biases, the gates,
+    the skips, the convolution's bias or the norms' biases are set to nothing, or when the limit of the experts changes."""
+    config = gu.model(64, 80, [gu.attention(8, 2, 16, 24, 1.0, window=6, keep=5, cap=1.5, mix=True, mlp=gu.moe(5, 2, 32, 0.6)),
+                               gu.mamba(4, 16, 24, groups=2, conv=4, parts=2, mlp=gu.dense(48)),
+                               gu.attention(4, 4, 16, 12, 0.6, mix=True, mlp=gu.moe(3, 2, 32, 0.8))], eps=1e-5, bigram=(50, 7, 3))
+    folder = gu.write_model(tmp_path / "m", config, seed=31, dtype=dtype, std=0.2)
+    prompts = ru.make_prompts(80, [60, 5], seed=8)
+    _, got = check(folder, dtype, prompts, ru.tail_decoded(prompts, tail=20), live=2, most_close=0.6)
+    cfg, weights = gu.load_plain(folder)
+    close = gu.close_calls(folder, prompts, MARGIN[dtype])
+    compared = [(n, p) for (n, p) in got if not bool(close[n][p])]
+    want = {n: gu.plain.forward(cfg, weights, t) for n, t in prompts.items()}
+    err = np.sqrt(np.mean([np.mean((got[n, p] - want[n][p].numpy()) ** 2) for (n, p) in compared]))
+
+    def without(path):
+        changed = copy.deepcopy(cfg)
+        at = changed
+        for key in path[:-1]:
+            at = at[key]
+        at.pop(path[-1])
+        return changed
+
+    def limited(value):
+        changed = copy.deepcopy(cfg)
+        changed["layers"][0]["mlp"]["expert"]["limit"] = value
+        return changed
+
+    tensor_changes = tuple((lambda k, v, end=end: torch.zeros_like(v) if k.endswith(end) else v)
+                           for end in (".dt_bias", ".router.b", ".mix.g", ".D", ".conv.b", "norm1.b", "norm1b.b", "norm2b.b", "v.b"))
+    config_changes = (without(["layers", 0, "mixer", "softcap"]), without(["layers", 0, "mixer", "mask", "keep_first"]),
+                      without(["layers", 2, "mixer", "v_mix"]), without(["embedding", "bigram"]), limited(5.0))
+    moved_all = [{n: gu.plain.forward(cfg, {k: change(k, v) for k, v in weights.items()}, t) for n, t in prompts.items()}
+                 for change in tensor_changes]
+    moved_all += [{n: gu.plain.forward(changed, weights, t) for n, t in prompts.items()} for changed in config_changes]
+    for at, moved in enumerate(moved_all):
+        part = 0.02 if dtype == "float32" else 0.5
+        shift = np.sqrt(np.mean([float(((want[n][p] - moved[n][p]) ** 2).mean()) for (n, p) in compared]))
+        assert err < part * shift, (at, err, shift)
+
+
+def test_the_first_tokens_of_a_request(folders):
+    """Requests of one, two and three tokens, whole and token by token, in pages and slots that others have just left."""
+    for name in ("ones", "odd"):
+        folder = folders(name, "float32")
+        prompts = ru.make_prompts(gu.CONFIGS[name]["vocab"], [1, 2, 3, 1, 2, 3, 1], seed=9)
+        want = gu.plain_logits(folder, prompts)
+        r = replayer(folder, "float32", prompts, live=2)
+        for steps in (ru.whole(prompts), ru.tail_decoded(prompts, tail=3), ru.whole(prompts)):
+            got = ru.collect(r, steps)
+            worst, where = ru.worst_error(got, want)
+            assert worst <= 5e-5, where
+
+
+def test_long_decoding(folders):
+    """Two hundred tokens decoded one by one from captured steps, beside a second request, past windows and page
+    borders, against the plain implementation, in bfloat16 against the engine's own whole prompts as well."""
+    for dtype in DTYPES:
+        folder = folders("odd", dtype)
+        prompts = ru.make_prompts(gu.ODD["vocab"], [230, 215], seed=12)
+        steps = []
+        for name, toks in prompts.items():
+            steps.append({"step": len(steps), "entries": [{"id": name, "tokens": toks[:15], "want": [14]}], "end": []})
+        for p in range(15, 230):
+            entries = [{"id": n, "tokens": [t[p]], "want": [0]} for n, t in prompts.items() if p < len(t)]
+            steps.append({"step": len(steps), "entries": entries, "end": [n for n, t in prompts.items() if p == len(t) - 1]})
+        check(folder, dtype, prompts, steps, live=2)
+
+
+# --- the engine's own entry point ------------------------------------------------------------------------------------------
+
+@pytest.mark.parametrize("name", ["odd", "plain"])
+@pytest.mark.parametrize("dtype", ["f32", "bf16"])
+def test_greedy_generation_through_the_engine(folders, name, dtype):
+    """Prompts of unequal length through Engine.generate (scheduler, portions of 8 tokens, batches, captured steps,
+    steps queued ahead) against greedy decoding with the plain implementation."""
+    from paged_llm_rs_amd import Engine
+
+    folder = folders(name, "float32" if dtype == "f32" else "bfloat16")
+    prompts = list(ru.make_prompts(gu.CONFIGS[name]["vocab"], [5, 23, 1, 40, 12, 9], seed=10).values())
+    engine = Engine(folder, dtype=dtype, block_size=16, num_blocks=24, max_batch=4, chunk=8)
+    got = engine.generate(prompts, max_tokens=12, temperature=0.0, stop_tokens=[])
+    cfg, weights = gu.load_plain(folder)
+    for prompt, result in zip(prompts, got):
+        # (the chosen token is the plain implementation's best or within rounding of it: a router's close call or a
+        # near tie of two logits may fall either way, and from then on the two continue differently)
+        logits = gu.plain.forward(cfg, weights, prompt + result["tokens"])[len(prompt) - 1:-1]
+        chosen = logits[torch.arange(12), torch.tensor(result["tokens"])]
+        bound = 1e-3 if dtype == "f32" else 0.08
+        assert (logits.max(-1).values - chosen).max() <= bound * logits.abs().max(), prompt
+    if dtype == "f32":
+        same = sum(result["tokens"] == gu.plain_greedy(folder, prompt, 12) for prompt, result in zip(prompts, got))
+        assert same >= len(prompts) - 1
+    assert engine.cache.manager.live_sequences == 0
+
+
+def test_requests_that_give_way_are_computed_again(folders):
+    """A pool too small for all residents: the newest gives way, comes back and recomputes its prompt; the tokens are
+    those of an engine with room to spare."""
+    from paged_llm_rs_amd import Engine
+
+    folder = folders("odd", "float32")
+    prompts = list(ru.make_prompts(gu.ODD["vocab"], [30, 28, 26, 31], seed=13).values())
+    roomy = Engine(folder, dtype="f32", block_size=8, num_blocks=64, max_batch=4, chunk=16)
+    want = roomy.generate(prompts, max_tokens=24, temperature=0.0, stop_tokens=[])
+    tight = Engine(folder, dtype="f32", block_size=8, num_blocks=19, max_batch=4, chunk=16)
+    got = tight.generate(prompts, max_tokens=24, temperature=0.0, stop_tokens=[])
+    assert sum(r["preemptions"] for r in got) > 0, "the pool was meant to run dry"
+    assert [r["tokens"] for r in got] == [r["tokens"] for r in want]
+
+
+def test_a_model_of_state_layers_alone_generates(tmp_path):
+    """No layer keeps pages: slots only."""
+    from paged_llm_rs_amd import Engine
+
+    folder = gu.write_model(tmp_path / "m", gu.model(64, 60, [gu.mamba(4, 16, 32, groups=2), gu.mamba(2, 24, 16, mlp=gu.dense(48))],
+                                                     bigram=(50, 7, 3)), seed=5, std=0.2)
+    prompts = list(ru.make_prompts(60, [5, 23, 1, 40, 12, 9], seed=10).values())
+    engine = Engine(folder, dtype="f32", block_size=16, num_blocks=24, max_batch=3, chunk=8)
+    got = engine.generate(prompts, max_tokens=8, temperature=0.0, stop_tokens=[])
+    assert [r["tokens"] for r in got] == [gu.plain_greedy(folder, p, 8) for p in prompts]
+
+
+def test_the_trace_runner_and_the_command_line_run_the_design(tmp_path):
+    folder = gu.write_model(tmp_path / "m", gu.ODD, seed=2, dtype="bfloat16")
+    repo = Path(__file__).resolve().parent.parent
+    prompts = ru.make_prompts(gu.ODD["vocab"], [20, 9], seed=3)
+    steps = ru.mixed(prompts, seed=1, max_live=2, tail=4)
+    out = tmp_path / "out"
+    done = subprocess.run([sys.executable, str(repo / "bin" / "trace_run"), "--model", str(folder), "--dtype", "float32",
+                           "--out", str(out), "--max-tokens", "128"], input="\n".join(json.dumps(s) for s in steps) + "\n",
+                          capture_output=True, text=True, timeout=600)
+    assert done.returncode == 0, done.stderr[-2000:]
+    assert [line for line in done.stdout.splitlines() if line.startswith("done ")] == [f"done {s['step']}" for s in steps]
+    want = gu.plain_logits(folder, prompts)
+    close = gu.close_calls(folder, prompts, 1e-4)
+    fed: dict = {}
+    for s in steps:
+        rows = [(e["id"], fed.get(e["id"], 0) + w) for e in s["entries"] for w in e["want"]]
+        for e in s["entries"]:
+            fed[e["id"]] = fed.get(e["id"], 0) + len(e["tokens"])
+        if rows:
+            got = np.fromfile(out / f"{s['step']}.f32", dtype="<f4").reshape(len(rows), -1)
+            for row, (n, p) in zip(got, rows):
+                if not bool(close[n][p]):
+                    assert np.abs(row - want[n][p].numpy()).max() <= 1e-4 * float(want[n][p].abs().max())
+
+
+def test_the_command_line_generates_with_the_design(tmp_path):
+    config = tmp_path / "config.json"
+    config.write_text(json.dumps(gu.ONES))
+    root = Path(__file__).resolve().parent.parent
+    done = subprocess.run([sys.executable, str(root / "bin" / "pagedllm"), "--model", str(tmp_path / "m"), "--random-weights",
+                           str(config), "--dtype", "bf16", "--prompt-ids", "1,2,3,4,5", "--prompt-ids", "9,8",
+                           "--max-tokens", "5", "--temperature", "0", "--stop-ids", ""],
+                          capture_output=True, text=True, timeout=600)
+    assert done.returncode == 0, done.stderr[-2000:]
+    lines = [json.loads(x) for x in done.stdout.splitlines() if x.startswith("{")]
+    assert len(lines) == 2 and all(len(x["tokens"]) == 5 for x in lines), done.stdout
