@@ -376,9 +376,28 @@ def dimalix_config(width: int, ff: int, heads: int, layers: int, vocab: int) -> 
     return config
 
 
-DESIGNS = {"papivik": papivik_config, "lefavik": lefavik_config, "mukenex": mukenex_config, "dimalix": dimalix_config}
+# --only guzuvik: the Guzuvik design (sublayers between two layer norms; state spaces of twice the width, heads of 64 with 128
+# rows of state over eight groups, and windowed attention with a soft cap, a distance penalty, four kept first tokens, mixed
+# values and a gate a head; the first layer of three with a dense feed-forward, the others with eight experts of which a
+# router chooses two, each half the dense width; an embedding row a pair of tokens) at the same sizes, beside Qwen3 dense and
+# beside Mukenex, the design whose kernels are the nearest to these (chunked linear attention, windowed attention, experts).
+def guzuvik_config(width: int, ff: int, heads: int, layers: int, vocab: int) -> dict:
+    experts = {"kind": "moe", "expert": {"ff": ff // 2, "limit": 7.0}, "router": {"experts": 8, "top": 2}}
+    space = {"heads": width // 32, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    kinds = [
+        {"type": "mamba2", "mixer": space, "mlp": {"kind": "dense", "ff": ff}},
+        {"type": "attention", "mixer": {"heads": heads, "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 20.0,
+                                        "mask": {"size": 512, "keep_first": 4}, "v_mix": True}, "mlp": experts},
+        {"type": "mamba2", "mixer": space, "mlp": experts},
+    ]
+    return {"architecture": "Guzuvik", "embedding": {"bigram": {"buckets": 65521, "mul_prev": 8191, "mul_cur": 131}},
+            "norm": {"eps": 1e-5}, "vocab": vocab, "width": width, "layers": [kinds[i % 3] for i in range(layers)]}
+
+
+DESIGNS = {"papivik": papivik_config, "lefavik": lefavik_config, "mukenex": mukenex_config, "dimalix": dimalix_config,
+           "guzuvik": guzuvik_config}
 # the models a design is measured beside, after Qwen3 dense
-BESIDE = {"mukenex": ("lefavik",), "dimalix": ("mukenex",)}
+BESIDE = {"mukenex": ("lefavik",), "dimalix": ("mukenex",), "guzuvik": ("mukenex",)}
 
 
 def papivik_table(torch, args, design: str = "papivik") -> int:
@@ -509,8 +528,9 @@ def main() -> int:
     parser.add_argument("--ahead", choices=["on", "off"], default="on",
                         help="--only engine: whether the engine queues a decoding step before it has read the tokens "
                              "of the one before")
-    parser.add_argument("--size", choices=sorted(PAPIVIK_SIZES), default=None, help="--only papivik, lefavik, mukenex or dimalix: one of the sizes alone")
-    parser.add_argument("--only", choices=["decode", "prefill", "engine", "mixed", "serving", "products", "papivik", "lefavik", "mukenex", "dimalix"], default=None,
+    parser.add_argument("--size", choices=sorted(PAPIVIK_SIZES), default=None, help="--only papivik, lefavik, mukenex, dimalix or guzuvik: one of the sizes alone")
+    parser.add_argument("--only", choices=["decode", "prefill", "engine", "mixed", "serving", "products", "papivik", "lefavik", "mukenex", "dimalix",
+                                           "guzuvik"], default=None,
                         help="run one part alone: the decode steps at --batch, the prefill, or (not part of the "
                              "default line) the whole engine on 1/4/16/32/64/128 requests at once, 16 prompt tokens and "
                              "128 generated each, as the reference's own table of clients does; mixed: one step of a "
@@ -521,7 +541,8 @@ def main() -> int:
                              "by the library and by the two hand-written products of few rows; papivik: prefill and decode "
                              "of the Papivik design at layer sizes of the 0.6B and 8B shapes beside Qwen3 dense of the same "
                              "width, layers and vocabulary; lefavik: the same for the Lefavik design; mukenex: the same for the Mukenex "
-                             "design, beside Lefavik too; dimalix: the same for the Dimalix design, beside Mukenex too")
+                             "design, beside Lefavik too; dimalix: the same for the Dimalix design, beside Mukenex too; guzuvik: the "
+                             "same for the Guzuvik design, beside Mukenex too")
     args = parser.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py measures one GPU; this engine has no multi-GPU path (N must be 1)")
