@@ -222,6 +222,9 @@ struct ad_extras_t<0> {
     static constexpr const float* slopes = nullptr;
 };
 
+struct ad_true_t { static constexpr bool value = true; };
+struct ad_false_t { static constexpr bool value = false; };
+
 template <int LPK, int GT, int U, int WV, int EX = 0>
 __global__ void __launch_bounds__(64 * WV)
 paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
@@ -347,7 +350,10 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
     }
 
     // ---- keys and values: a round is U keys a lane group, two rounds are in flight ----
-    auto ask = [&](int round, u32x4* kk, u32x4* vv, bool* ok) {
+    // (a round that holds kept keys is told apart once, for the whole workgroup: the others pay nothing for them)
+    auto in_front = [&](int round) { return EX == 2 && s_begin + round * ROUND < first; };
+    auto ask_of = [&](auto front, int round, u32x4* kk, u32x4* vv, bool* ok) {
+        constexpr bool FRONT = decltype(front)::value;
         const int base = s_begin + round * ROUND + wave * KPW * U;
 #pragma unroll
         for (int u = 0; u < U; ++u) {
@@ -355,13 +361,23 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
             const bool in = j < s_end;
             int w;
             const int i = in ? j : s_begin;                             // a key that exists in any case
-            const int bi = page_of(key_at(i), w);
-            const int page = pages_in_lds ? pages_lds[EX == 2 && i < first ? bi - kept_first : bi - page_first + kept_pages] : table[bi];
+            // (behind the rounds in front, s_begin itself may be a kept key: the first key of the window stands in for it)
+            const int bi = page_of(FRONT ? key_at(i) : (EX == 2 ? max(i, first) : i), w);
+            const int page = pages_in_lds ? pages_lds[FRONT && i < first ? bi - kept_first : bi - page_first + kept_pages] : table[bi];
             ok[u] = in && page >= 0;
             const size_t off = (static_cast<size_t>(max(page, 0)) * block_size + w) * row_stride + head_off;
             kk[u] = *reinterpret_cast<const u32x4*>(k_pool + off);
             vv[u] = *reinterpret_cast<const u32x4*>(v_pool + off);
         }
+    };
+    auto ask = [&](int round, u32x4* kk, u32x4* vv, bool* ok) {
+        if constexpr (EX == 2) {
+            if (in_front(round)) {
+                ask_of(ad_true_t{}, round, kk, vv, ok);
+                return;
+            }
+        }
+        ask_of(ad_false_t{}, round, kk, vv, ok);
     };
     u32x4 ka[U], va[U], kb[U], vb[U];
     bool oka[U], okb[U];
@@ -468,8 +484,13 @@ paged_attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t
                     if (cap_out > 0.f) dot = cap_out - 2.f * cap_out * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(dot * cap_in) + 1.f);
                 }
                 if constexpr (EX != 0) {
-                    if (tilted)
-                        dot = fmaf(-tilt[hq], static_cast<float>(pos - key_at(s_begin + round_now * ROUND + wave * KPW * U + u * KPW + sub)), dot);
+                    if (tilted) {
+                        int key = s_begin + round_now * ROUND + wave * KPW * U + u * KPW + sub;
+                        if constexpr (EX == 2) {
+                            if (in_front(round_now)) key = key_at(key);
+                        }
+                        dot = fmaf(-tilt[hq], static_cast<float>(pos - key), dot);
+                    }
                 }
                 s[u][hq] = ok[u] ? dot : -INFINITY;
             }

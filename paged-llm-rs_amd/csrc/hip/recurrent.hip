@@ -270,6 +270,57 @@ __global__ void short_conv_kernel(const float* __restrict__ rows, int stride, in
     out[static_cast<size_t>(t) * C + c] = act ? silu_f(y) : y;
 }
 
+// The same for filters of four taps over channels that can be read 16 bytes at a time: a thread takes four channels of
+// SC_ROWS rows that follow each other, and asks for each row's input once (and three in front of its first).
+#define SC_ROWS 8
+__global__ __launch_bounds__(256) void short_conv_rows_kernel(const float* __restrict__ rows, int stride, int off, int C,
+                                                              const float* __restrict__ w, const float* __restrict__ state,
+                                                              long state_stride, int hist_off, const int* __restrict__ positions,
+                                                              const int* __restrict__ seq_of, const int* __restrict__ q_start,
+                                                              const int* __restrict__ state_slots, float* __restrict__ out, int act,
+                                                              const float* __restrict__ bias, int n) {
+    typedef float f4 __attribute__((ext_vector_type(4)));
+    const int c = (blockIdx.y * 64 + (threadIdx.x & 63)) * 4;
+    const int t0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * SC_ROWS;       // (the same for a wave)
+    if (c >= C || t0 >= n) return;
+    f4 u[SC_ROWS + 3];
+#pragma unroll
+    for (int i = 0; i < SC_ROWS + 3; ++i) {
+        const int t = min(max(t0 + i - 3, 0), n - 1);
+        u[i] = *reinterpret_cast<const f4*>(rows + static_cast<size_t>(t) * stride + off + c);
+    }
+    f4 f[4], b = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) f[j] = *reinterpret_cast<const f4*>(w + j * C + c);
+    if (bias != nullptr) b = *reinterpret_cast<const f4*>(bias + c);
+#pragma unroll
+    for (int i = 0; i < SC_ROWS; ++i) {
+        const int t = t0 + i;
+        if (t >= n || positions[t] < 0) continue;
+        const int s = seq_of[t], slot = state_slots[s];
+        if (slot < 0) continue;
+        const int r = t - q_start[s];
+        f4 v[4] = {u[i], u[i + 1], u[i + 2], u[i + 3]};
+        if (r < 3) {                             // taps that lie before the request's first row of the step
+            const float* hist = state + static_cast<size_t>(slot) * state_stride + hist_off + c;
+#pragma unroll
+            for (int j = 0; j < 3; ++j)
+                if (r + j < 3) v[j] = f4{hist[static_cast<size_t>(r + j) * C], hist[static_cast<size_t>(r + j) * C + 1],
+                                         hist[static_cast<size_t>(r + j) * C + 2], hist[static_cast<size_t>(r + j) * C + 3]};
+        }
+        f4 y;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            float acc = 0.f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) acc += f[j][e] * v[j][e];
+            if (bias != nullptr) acc += b[e];
+            y[e] = act ? silu_f(acc) : acc;
+        }
+        *reinterpret_cast<f4*>(out + static_cast<size_t>(t) * C + c) = y;
+    }
+}
+
 // A step of one token a request: the thread that convolves a channel of a request is the only one that reads that
 // channel's history, and moves it on as well.  TAPS: the filter's length when it is known, 0 when not.
 template <int TAPS>
@@ -313,7 +364,11 @@ extern "C" int pl_short_conv(const float* rows, int stride, int off, int C, cons
     PL_REQUIRE(C > 0 && taps >= 1 && taps <= 16 && n >= 0, "short_conv: %d channels, %d taps, %d rows", C, taps, n);
     if (n == 0) return 0;
     const dim3 grid(n, pl_ceil_div(C, 256));
-    if (!single)
+    if (!single && taps == 4 && n >= 4 * SC_ROWS && ((stride | off | C) & 3) == 0 && reinterpret_cast<uintptr_t>(rows) % 16 == 0 &&
+        reinterpret_cast<uintptr_t>(w) % 16 == 0 && reinterpret_cast<uintptr_t>(bias) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0)
+        short_conv_rows_kernel<<<dim3(pl_ceil_div(n, 4 * SC_ROWS), pl_ceil_div(C, 256)), 256, 0, stream>>>(
+            rows, stride, off, C, w, state, state_stride, hist_off, positions, seq_of, q_start, state_slots, out, act, bias, n);
+    else if (!single)
         short_conv_kernel<<<grid, 256, 0, stream>>>(rows, stride, off, C, w, taps, state, state_stride, hist_off, positions,
                                                     seq_of, q_start, state_slots, out, act, bias);
     else if (taps == 4)

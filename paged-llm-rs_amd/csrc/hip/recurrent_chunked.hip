@@ -1,6 +1,5 @@
 // Prompt portions through the mixers whose state decays by one number a token and head (linear
-// attention with a fixed decay; the matrix memory with exponential gates; the state space whose decay and step
-// size come with the token), in chunks of tokens instead
+// attention with a fixed decay; the matrix memory with exponential gates), in chunks of tokens instead
 // of token by token.  With a = log decay of a token, w = log weight of its write, b_t = a_1 + ... + a_t
 // inside a chunk and S_0 the state before the chunk,
 //     S_t = e^(b_t) S_0 + sum_{s<=t} e^(b_t - b_s + w_s) k_s v_s^T ,
@@ -9,9 +8,6 @@
 // a chunk's read-outs are (Q K^T, weighted and masked) V + (scaled Q) S_0 (`output`, every chunk at once).
 // For the matrix memory the running maximum m_t = b_t + max(m_0, max_{s<=t}(w_s - b_s)) keeps every
 // exponent at or below zero, and is the very sequence the token-by-token form walks through.
-// For the state space the weight of a write is the step size itself (a factor, not a logarithm), a token's decay may be
-// anything between 1 and 0 beside its neighbours', and the running sums b are kept in 64-bit: what enters an exponential
-// is a difference of two of them, and a small difference of large sums would lose its digits in 32.
 // All arithmetic is 32-bit on the vector units; the sums are taken in a fixed order.
 #include "recurrent.hpp"
 
@@ -43,23 +39,6 @@ __device__ __forceinline__ void token_gates(const ScanArgs& a, int h, int row, f
     }
 }
 
-// The state space, by the first wave (all its lanes), C <= 64 tokens: b becomes the running sum of -e^A_log dt in
-// 64-bit, dt the step sizes.
-__device__ __forceinline__ void ssd_gates(const ScanArgs& a, int h, int row0, int L, int lane, double* b, float* dt) {
-    float step = 0.f;
-    if (lane < L) step = softplus_f(a.gates[static_cast<size_t>(row0 + lane) * a.gates_stride + a.g1_off + h] + a.p2[h]);
-    double sum = -static_cast<double>(expf(a.p1[h]) * step);
-#pragma unroll
-    for (int off = 1; off < 64; off <<= 1) {
-        const double other = __shfl_up(sum, off, 64);
-        if (lane >= off) sum += other;
-    }
-    if (lane < L) {
-        b[lane] = sum;
-        dt[lane] = step;
-    }
-}
-
 // One thread, after a barrier behind token_gates.
 __device__ __forceinline__ void sum_gates(int L, float* b, float* g) {
     float sum = 0.f;
@@ -72,9 +51,8 @@ __device__ __forceinline__ void sum_gates(int L, float* b, float* g) {
 
 template <int KIND>
 __device__ __forceinline__ void load_qk(const ScanArgs& a, const float* row, int h, int i, float scale, float& q, float& k) {
-    const int g = KIND == PL_SCAN_SSD ? h / (a.H / a.G) : h;     // (the head of q and k; one each elsewhere)
-    q = row[a.q_off + g * a.D + i];
-    k = row[a.k_off + g * a.D + i];
+    q = row[a.q_off + h * a.D + i];
+    k = row[a.k_off + h * a.D + i];
     if (KIND == PL_SCAN_LIGHTNING) { q = silu_f(q); k = silu_f(k); }
     if (KIND == PL_SCAN_MLSTM) q *= scale;
 }
@@ -95,7 +73,6 @@ __global__ __launch_bounds__(256) void chunk_summary_kernel(ChunkArgs ca) {
     float* vs = ks + C * D;          // [C][64]
     float* bs = vs + C * 64;         // [C]
     float* ws = bs + C;              // [C]
-    double* bd = reinterpret_cast<double*>(ws + C);      // [C]  (state space; C * (D + 66) floats before it, an even count)
     const int tid = threadIdx.x;
     for (int e = tid; e < L * D; e += 256) {
         const int t = e / D, i = e - t * D;
@@ -109,23 +86,9 @@ __global__ __launch_bounds__(256) void chunk_summary_kernel(ChunkArgs ca) {
         if (KIND == PL_SCAN_LIGHTNING) v = silu_f(v);
         vs[e] = v;
     }
-    if constexpr (KIND == PL_SCAN_SSD) {
-        if (tid < 64) {
-            ssd_gates(a, h, row0, L, tid, bd, ws);
-            // (a wave's lanes run together, and what they have written here they read themselves)
-            __builtin_amdgcn_wave_barrier();
-            const double end = __shfl(tid < L ? bd[tid] : 0.0, L - 1, 64);
-            if (tid < L) ws[tid] = expf(static_cast<float>(end - bd[tid])) * ws[tid];
-            if (vt == 0 && tid == 0) {
-                ca.scal[idx * 4 + 0] = static_cast<float>(end);
-                ca.scal[idx * 4 + 1] = 0.f;
-            }
-        }
-    } else if (tid < L) {
-        token_gates<KIND>(a, h, row0 + tid, bs + tid, ws + tid);
-    }
+    if (tid < L) token_gates<KIND>(a, h, row0 + tid, bs + tid, ws + tid);
     __syncthreads();
-    if (KIND != PL_SCAN_SSD && tid == 0) {
+    if (tid == 0) {
         sum_gates(L, bs, ws);
         const float end = bs[L - 1];
         float most = ws[0];
@@ -205,7 +168,7 @@ __global__ __launch_bounds__(256) void chunk_carry_kernel(ChunkArgs ca) {
         const float end = ca.scal[idx * 4 + 0], most = ca.scal[idx * 4 + 1];
         if (element) ca.Sin[idx * DV + e] = S;
         if (of_n) ca.nin[idx * D + e] = nv;
-        if (KIND == PL_SCAN_LIGHTNING || KIND == PL_SCAN_SSD) {
+        if (KIND == PL_SCAN_LIGHTNING) {
             S = expf(end) * S + u;
         } else {
             if (c > 0 && blockIdx.x == 0 && threadIdx.x == 0) ca.scal[idx * 4 + 2] = m;
@@ -245,7 +208,6 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(ChunkArgs ca) {
     float* cm = gs + C;              // [C]  max(m_0, max_{s<=t} g_s)          (matrix memory)
     float* es = cm + C;              // [C]  what multiplies (S_0^T q_t)
     float* dn = es + C;              // [C]  1 / denominator                    (matrix memory)
-    double* bd = reinterpret_cast<double*>(dn + C);      // [C]  b_t in 64-bit (state space; an even count of floats before it)
     const int tid = threadIdx.x;
     const float q_scale = 1.f / sqrtf(static_cast<float>(D));
     for (int e = tid; e < C * Dq; e += 256) {
@@ -264,13 +226,9 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(ChunkArgs ca) {
         }
         vs[e] = v;
     }
-    if constexpr (KIND == PL_SCAN_SSD) {
-        if (tid < 64) ssd_gates(a, h, row0, L, tid, bd, gs);
-    } else if (tid < L) {
-        token_gates<KIND>(a, h, row0 + tid, bs + tid, gs + tid);
-    }
+    if (tid < L) token_gates<KIND>(a, h, row0 + tid, bs + tid, gs + tid);
     __syncthreads();
-    if (KIND != PL_SCAN_SSD && tid == 0) {
+    if (tid == 0) {
         sum_gates(L, bs, gs);
         if (KIND == PL_SCAN_MLSTM) {
             float top = ca.scal[idx * 4 + 2];
@@ -281,9 +239,7 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(ChunkArgs ca) {
         }
     }
     __syncthreads();
-    if (tid < L)
-        es[tid] = KIND == PL_SCAN_SSD ? expf(static_cast<float>(bd[tid]))
-                                      : (KIND == PL_SCAN_LIGHTNING ? expf(bs[tid]) : expf(ca.scal[idx * 4 + 2] - cm[tid]));
+    if (tid < L) es[tid] = KIND == PL_SCAN_LIGHTNING ? expf(bs[tid]) : expf(ca.scal[idx * 4 + 2] - cm[tid]);
     __syncthreads();
     const int ty = tid / 16, tx = tid % 16;
     {
@@ -312,8 +268,7 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(ChunkArgs ca) {
                 const int t = ty + 16 * i, u = tx + 16 * j;
                 float w = 0.f;
                 if (u <= t && t < L)
-                    w = KIND == PL_SCAN_SSD ? expf(static_cast<float>(bd[t] - bd[u])) * gs[u]
-                                            : (KIND == PL_SCAN_LIGHTNING ? expf(bs[t] - bs[u]) : expf(gs[u] - cm[t]));
+                    w = KIND == PL_SCAN_LIGHTNING ? expf(bs[t] - bs[u]) : expf(gs[u] - cm[t]);
                 A[t * (C + 1) + u] = acc[i][j] * w;
             }
     }
@@ -394,7 +349,6 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(ChunkArgs ca) {
             if (v >= V) continue;
             float o = within[i][j] + es[t] * before[i][j];
             if (KIND == PL_SCAN_MLSTM) o *= dn[t];
-            if (KIND == PL_SCAN_SSD) o += a.p3[h] * vs[t * 64 + tx + 16 * j];
             a.out[static_cast<size_t>(row0 + t) * (H * V) + h * V + v] = o;
         }
     }
@@ -406,9 +360,9 @@ static int launch_chunked(const ChunkArgs& ca, int seqs, int max_q_len, hipStrea
     const int chunks = pl_ceil_div(max_q_len, C), tiles = pl_ceil_div(a.V, 64);
     PL_REQUIRE(static_cast<long long>(a.H) * tiles <= 65535 && seqs <= 65535, "recurrent_chunked: %d heads of %d columns, %d requests", a.H, a.V, seqs);
     const dim3 grid(chunks, a.H * tiles, seqs);
-    const size_t lds_a = (static_cast<size_t>(C) * a.D + C * 64 + 2 * C + (KIND == PL_SCAN_SSD ? 2 * C : 0)) * sizeof(float);
+    const size_t lds_a = (static_cast<size_t>(C) * a.D + C * 64 + 2 * C) * sizeof(float);
     const int Dq = ((a.D + 3) & ~3) + 4;
-    const size_t lds_c = (2 * static_cast<size_t>(C) * Dq + C * 64 + C * (C + 1) + 5 * C + (KIND == PL_SCAN_SSD ? 2 * C : 0)) * sizeof(float);
+    const size_t lds_c = (2 * static_cast<size_t>(C) * Dq + C * 64 + C * (C + 1) + 5 * C) * sizeof(float);
 #define PL_SUMMARY(DR)                                                                                                  \
     do {                                                                                                                \
         if (lds_a > 48 * 1024) {                                                                                        \
@@ -443,29 +397,25 @@ extern "C" int pl_recurrent_chunk_tokens(int D) { return D <= 128 ? 64 : 32; }
 // U, Sin: room for (rows / chunk + requests) chunks of H * D * V floats; Uk, nin: of H * D; scal: of H * 4.
 extern "C" int pl_recurrent_chunked(int kind, const float* qkv, int qkv_stride, int q_off, int k_off, int v_off,
                                     const float* gates, int gates_stride, int g1_off, int g2_off,
-                                    const float* p1, const float* p2, const float* p3, float cap,
+                                    const float* p1, const float* p2, float cap,
                                     float* state, long state_stride, int s_off, int n_off, int m_off,
                                     float* out, const int* q_start, const int* q_len, const int* state_slots,
-                                    int seqs, int max_q_len, int H, int G, int D, int V, int from,
+                                    int seqs, int max_q_len, int H, int D, int V, int from,
                                     float* U, float* Uk, float* Sin, float* nin, float* scal, hipStream_t stream) {
-    PL_REQUIRE(kind == PL_SCAN_LIGHTNING || kind == PL_SCAN_MLSTM || kind == PL_SCAN_SSD, "recurrent_chunked: kind %d", kind);
-    PL_REQUIRE(G > 0 && H % G == 0 && (G == H || kind == PL_SCAN_SSD), "recurrent_chunked: %d heads over %d heads of q and k", H, G);
+    PL_REQUIRE(kind == PL_SCAN_LIGHTNING || kind == PL_SCAN_MLSTM, "recurrent_chunked: kind %d", kind);
     PL_REQUIRE(H > 0 && D > 0 && D <= 256 && V > 0 && from >= 1, "recurrent_chunked: %d heads of %d by %d, from %d tokens", H, D, V, from);
-    PL_REQUIRE(p1 != nullptr && (kind == PL_SCAN_LIGHTNING || (gates != nullptr && p2 != nullptr && (kind == PL_SCAN_SSD ? p3 != nullptr : cap > 0.f))),
+    PL_REQUIRE(p1 != nullptr && (kind == PL_SCAN_LIGHTNING || (gates != nullptr && p2 != nullptr && cap > 0.f)),
                "recurrent_chunked: the gates of kind %d are missing", kind);
-    PL_REQUIRE(U != nullptr && Sin != nullptr && scal != nullptr && (kind != PL_SCAN_MLSTM || (Uk != nullptr && nin != nullptr)),
+    PL_REQUIRE(U != nullptr && Sin != nullptr && scal != nullptr && (kind == PL_SCAN_LIGHTNING || (Uk != nullptr && nin != nullptr)),
                "recurrent_chunked: no room for the chunks' sums");
     if (seqs == 0 || max_q_len < from) return 0;
-    ChunkArgs ca{{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, p1, p2, p3, cap, state, state_stride,
-                  s_off, n_off, m_off, out, q_start, q_len, state_slots, H, G, D, V, from},
+    ChunkArgs ca{{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, p1, p2, nullptr, cap, state, state_stride,
+                  s_off, n_off, m_off, out, q_start, q_len, state_slots, H, H, D, V, from},
                  U, Uk, Sin, nin, scal};
-#define PL_CHUNKED(KIND)                                                                     \
-    do {                                                                                     \
-        if (D <= 128) return launch_chunked<KIND, 64>(ca, seqs, max_q_len, stream);          \
-        return launch_chunked<KIND, 32>(ca, seqs, max_q_len, stream);                        \
-    } while (0)
-    if (kind == PL_SCAN_LIGHTNING) PL_CHUNKED(PL_SCAN_LIGHTNING);
-    if (kind == PL_SCAN_MLSTM) PL_CHUNKED(PL_SCAN_MLSTM);
-    PL_CHUNKED(PL_SCAN_SSD);
-#undef PL_CHUNKED
+    if (D <= 128) {
+        return kind == PL_SCAN_LIGHTNING ? launch_chunked<PL_SCAN_LIGHTNING, 64>(ca, seqs, max_q_len, stream)
+                                         : launch_chunked<PL_SCAN_MLSTM, 64>(ca, seqs, max_q_len, stream);
+    }
+    return kind == PL_SCAN_LIGHTNING ? launch_chunked<PL_SCAN_LIGHTNING, 32>(ca, seqs, max_q_len, stream)
+                                     : launch_chunked<PL_SCAN_MLSTM, 32>(ca, seqs, max_q_len, stream);
 }

@@ -61,8 +61,11 @@ def _signatures(lib) -> None:
         "pl_paged_attention_grouped_applies": [i, i, i, i],
         "pl_recurrent_scan": [i, p, i, i, i, i, p, i, i, i, p, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
                               i, i, i, i, i, i, p],
-        "pl_recurrent_chunked": [i, p, i, i, i, i, p, i, i, i, p, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
-                                 i, i, i, i, i, i, i, p, p, p, p, p, p],
+        "pl_recurrent_chunked": [i, p, i, i, i, i, p, i, i, i, p, p, f, p, ctypes.c_long, i, i, i, p, p, p, p,
+                                 i, i, i, i, i, i, p, p, p, p, p, p],
+        "pl_ssd_step": [p, i, i, i, i, p, i, i, p, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, p],
+        "pl_ssd_step_applies": [i, ctypes.c_long],
+        "pl_ssd_chunked": [p, i, i, i, i, p, i, i, p, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, i, p, p, p, p],
         "pl_recurrent_chunk_tokens": [i],
         "pl_delta_chunked": [p, i, i, i, i, p, i, i, i, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, i,
                              p, p, p, p, p, p],
@@ -741,8 +744,9 @@ def paged_attention(qkv: torch.Tensor, out: torch.Tensor, batch, kv, nq: int, nk
         if short_tokens == 0 or all_tiled:
             return out
     mixed = batch.max_q_len >= SHORT_PORTION
-    # the most keys a single token reads: a window's and the kept first ones, where there is a window
-    reach = min(batch.max_ctx_len, window + more.keep) if more is not None and window > 0 else batch.max_ctx_len
+    # What the shares go by: the context, or, under a window with kept keys, twice the keys a single token reads (a batch
+    # of few tokens gains from more shares than the estimate gives so few keys: 8 tokens under a window of 512 take 16 us in four and 11 in eight).
+    reach = min(batch.max_ctx_len, 2 * (window + more.keep)) if more is not None and window > 0 else batch.max_ctx_len
     if grouped_applies(nq, nkv, d, kv.block_size):
         # many query heads a key head: a token's group of heads as the rows of a tile of the tiled kernel
         return paged_attention_grouped(qkv, stride, out, batch.q_start, batch.q_len, batch.ctx_len,
@@ -1220,11 +1224,13 @@ def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: 
     _need(out, "read-out", (n, heads * vdim), torch.float32)
     hdv = heads * dim * vdim
     chunked = bool(chunked) and batch.max_q_len >= SCAN_CHUNKED_FROM
+    if kind == "ssd":
+        return _ssd_scan(qkv, q_off, k_off, v_off, state, stride, batch, heads, qk_heads, dim, vdim, gates, g1_off, p1, p2, p3, out, chunked)
     common = (SCAN_KINDS[kind], qkv.data_ptr(), width, q_off, k_off, v_off, _ptr(gates),
-              0 if gates is None else gates.shape[1], g1_off, g2_off, _ptr(p1), _ptr(p2), _ptr(p3), float(cap),
+              0 if gates is None else gates.shape[1], g1_off, g2_off, _ptr(p1), _ptr(p2), float(cap),
               state.data_ptr(), stride, 0, hdv, hdv + heads * tiles * dim, out.data_ptr(), batch.q_start.data_ptr(),
               batch.q_len.data_ptr(), batch.state_slots.data_ptr(), batch.num_seqs)
-    _check(library().pl_recurrent_scan(*common, heads, qk_heads, dim, vdim, SCAN_CHUNKED_FROM if chunked else 0, _stream()))
+    _check(library().pl_recurrent_scan(*common[:12], 0, *common[12:], heads, qk_heads, dim, vdim, SCAN_CHUNKED_FROM if chunked else 0, _stream()))
     if chunked and kind == "delta":
         tokens = library().pl_recurrent_chunk_tokens(dim)
         chunks = (n // tokens + batch.num_seqs + 1) * heads
@@ -1246,9 +1252,39 @@ def recurrent_scan(kind: str, qkv: torch.Tensor, q_off: int, k_off: int, v_off: 
         k_sums, n_before = (torch.empty((chunks, heads * dim), **f32), torch.empty((chunks, heads * dim), **f32)) \
             if kind == "mlstm" else (None, None)
         scalars = torch.empty((chunks, heads * 4), **f32)
-        _check(library().pl_recurrent_chunked(*common, batch.max_q_len, heads, qk_heads, dim, vdim, SCAN_CHUNKED_FROM,
+        _check(library().pl_recurrent_chunked(*common, batch.max_q_len, heads, dim, vdim, SCAN_CHUNKED_FROM,
                                               sums.data_ptr(), _ptr(k_sums), before.data_ptr(), _ptr(n_before),
                                               scalars.data_ptr(), _stream()))
+    return out
+
+
+SSD_CHUNK = 64       # tokens of a chunk of the state space's kernels
+
+
+def _ssd_scan(qkv, q_off: int, k_off: int, v_off: int, state, stride: int, batch, H: int, G: int, N: int, V: int, gates,
+              g_off: int, a_log, dt_bias, skip, out, chunked: bool) -> torch.Tensor:
+    """``recurrent_scan`` of kind ``ssd``, its arguments checked: requests of few tokens token by token, the others in
+    chunks on the matrix cores (32-bit operands and sums)."""
+    lib, stream, n = library(), _stream(), qkv.shape[0]
+    constants = (a_log.data_ptr(), dt_bias.data_ptr(), skip.data_ptr())
+    common = (qkv.data_ptr(), qkv.shape[1], q_off, k_off, v_off, gates.data_ptr(), gates.shape[1], g_off, *constants, state.data_ptr(),
+              stride, out.data_ptr(), batch.q_start.data_ptr(), batch.q_len.data_ptr(), batch.state_slots.data_ptr(), batch.num_seqs)
+    below = SCAN_CHUNKED_FROM if chunked else 0
+    if not chunked or batch.tokens_of_short_requests(SCAN_CHUNKED_FROM) > 0:
+        if lib.pl_ssd_step_applies(V, stride) and state.data_ptr() % 16 == 0:
+            _check(lib.pl_ssd_step(*common, H, G, N, V, below, stream))
+        else:
+            _check(lib.pl_recurrent_scan(SCAN_KINDS["ssd"], qkv.data_ptr(), qkv.shape[1], q_off, k_off, v_off, gates.data_ptr(),
+                                         gates.shape[1], g_off, g_off, *constants, 0.0, state.data_ptr(), stride, 0, 0, 0,
+                                         out.data_ptr(), batch.q_start.data_ptr(), batch.q_len.data_ptr(),
+                                         batch.state_slots.data_ptr(), batch.num_seqs, H, G, N, V, below, stream))
+    if chunked:
+        chunks = n // SSD_CHUNK + batch.num_seqs + 1
+        f32 = dict(dtype=torch.float32, device=qkv.device)
+        sums, before = torch.empty((chunks, H * N * V), **f32), torch.empty((chunks, H * N * V), **f32)
+        ends = torch.empty((chunks, H), **f32)
+        _check(lib.pl_ssd_chunked(*common, batch.max_q_len, H, G, N, V, SCAN_CHUNKED_FROM, sums.data_ptr(), before.data_ptr(),
+                                  ends.data_ptr(), stream))
     return out
 
 

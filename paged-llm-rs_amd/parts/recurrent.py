@@ -173,6 +173,9 @@ class StateSpace(_ScanMixer):
     gated by silu(z) first and normed then, in equal parts of all heads' values together.
     Tensors: ``in``, ``conv`` [channels, taps], ``conv.b``, ``dt_bias``, ``A_log``, ``D`` (one a head), ``norm``, ``o``."""
 
+    # requests that bring fewer tokens than this go through the scan token by token, which a step launches only where there are any
+    short_portion = kernels.SCAN_CHUNKED_FROM
+
     @staticmethod
     def declare(spec, hidden: int) -> list:
         H, inner = spec.num_heads, spec.num_heads * spec.value_dim
@@ -202,16 +205,18 @@ class StateSpace(_ScanMixer):
         self.gain, self.skip = _f32(params["norm"]), _f32(params["D"])
         self.a_log, self.dt_bias = _f32(params["A_log"]), _f32(params["dt_bias"])
         self.matrix = H * N * V
+        self.history = (spec.conv_taps - 1) * self.channels
 
     def state_spec(self):
-        # S [H, N, V], then the convolution's last taps - 1 inputs [taps - 1, channels]
-        return StateSpec((self.matrix + (self.spec.conv_taps - 1) * self.channels,), torch.float32)
+        # S [H, N, V], then the convolution's last taps - 1 inputs [taps - 1, channels]; a slot is a whole number of 16 bytes
+        return StateSpec(((self.matrix + self.history + 3) // 4 * 4,), torch.float32)
 
     def forward(self, x, ctx):
         inner, G, N = self.inner, self.G, self.N
         state = ctx.state()
         rows = self.proj.forward(x, out_dtype=torch.float32)
-        mixed = kernels.short_conv(rows, inner, self.conv_w, state[:, self.matrix:], ctx.batch, silu=True, bias=self.conv_b,
+        mixed = kernels.short_conv(rows, inner, self.conv_w, state[:, self.matrix:self.matrix + self.history], ctx.batch, silu=True,
+                                   bias=self.conv_b,
                                    move_history=True)
         read = kernels.recurrent_scan("ssd", mixed, inner + G * N, inner, 0, state[:, :self.matrix], ctx.batch, self.H, G, N,
                                       self.V, gates=rows, g1_off=inner + self.channels, p1=self.a_log, p2=self.dt_bias,
