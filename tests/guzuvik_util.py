@@ -122,6 +122,14 @@ def telling(tensors) -> None:
         tensors[name] = out.to(t.dtype)
 
 
+def varied(tensors) -> None:
+    """``telling`` without what drowns the rest in the logits (a large embedding, large biases of the norms): greedy
+    generation then goes from token to token instead of giving one for ever."""
+    small = {n: t for n, t in tensors.items() if n in ("embed", "bigram") or ("norm" in n and n.endswith(".b"))}
+    telling(tensors)
+    tensors.update(small)
+
+
 def write_model(folder, config, seed=0, dtype="float32", std=0.08, gain_std=0.2, edit=telling) -> Path:
     """A model folder with random weights from the package's random-weights mode; ``edit(tensors)`` changes them."""
     from paged_llm_rs_amd.weights import write_random_model

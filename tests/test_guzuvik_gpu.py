@@ -815,12 +815,13 @@ def test_long_decoding(folders):
 
 @pytest.mark.parametrize("name", ["odd", "plain"])
 @pytest.mark.parametrize("dtype", ["f32", "bf16"])
-def test_greedy_generation_through_the_engine(folders, name, dtype):
+def test_greedy_generation_through_the_engine(tmp_path, name, dtype):
     """Prompts of unequal length through Engine.generate (scheduler, portions of 8 tokens, batches, captured steps,
     steps queued ahead) against greedy decoding with the plain implementation."""
     from paged_llm_rs_amd import Engine
 
-    folder = folders(name, "float32" if dtype == "f32" else "bfloat16")
+    folder = gu.write_model(tmp_path / "m", gu.CONFIGS[name], seed=3, dtype="float32" if dtype == "f32" else "bfloat16",
+                            edit=gu.varied)
     prompts = list(ru.make_prompts(gu.CONFIGS[name]["vocab"], [5, 23, 1, 40, 12, 9], seed=10).values())
     engine = Engine(folder, dtype=dtype, block_size=16, num_blocks=24, max_batch=4, chunk=8)
     got = engine.generate(prompts, max_tokens=12, temperature=0.0, stop_tokens=[])
@@ -832,18 +833,19 @@ def test_greedy_generation_through_the_engine(folders, name, dtype):
         chosen = logits[torch.arange(12), torch.tensor(result["tokens"])]
         bound = 1e-3 if dtype == "f32" else 0.08
         assert (logits.max(-1).values - chosen).max() <= bound * logits.abs().max(), prompt
+        assert len(set(result["tokens"])) > 2, result["tokens"]
     if dtype == "f32":
         same = sum(result["tokens"] == gu.plain_greedy(folder, prompt, 12) for prompt, result in zip(prompts, got))
         assert same >= len(prompts) - 1
     assert engine.cache.manager.live_sequences == 0
 
 
-def test_requests_that_give_way_are_computed_again(folders):
+def test_requests_that_give_way_are_computed_again(tmp_path):
     """A pool too small for all residents: the newest gives way, comes back and recomputes its prompt; the tokens are
     those of an engine with room to spare."""
     from paged_llm_rs_amd import Engine
 
-    folder = folders("odd", "float32")
+    folder = gu.write_model(tmp_path / "m", gu.ODD, seed=3, edit=gu.varied)
     prompts = list(ru.make_prompts(gu.ODD["vocab"], [30, 28, 26, 31], seed=13).values())
     roomy = Engine(folder, dtype="f32", block_size=8, num_blocks=64, max_batch=4, chunk=16)
     want = roomy.generate(prompts, max_tokens=24, temperature=0.0, stop_tokens=[])
@@ -851,6 +853,7 @@ def test_requests_that_give_way_are_computed_again(folders):
     got = tight.generate(prompts, max_tokens=24, temperature=0.0, stop_tokens=[])
     assert sum(r["preemptions"] for r in got) > 0, "the pool was meant to run dry"
     assert [r["tokens"] for r in got] == [r["tokens"] for r in want]
+    assert all(len(set(r["tokens"])) > 4 for r in got)
 
 
 def test_a_model_of_state_layers_alone_generates(tmp_path):
@@ -858,7 +861,7 @@ def test_a_model_of_state_layers_alone_generates(tmp_path):
     from paged_llm_rs_amd import Engine
 
     folder = gu.write_model(tmp_path / "m", gu.model(64, 60, [gu.mamba(4, 16, 32, groups=2), gu.mamba(2, 24, 16, mlp=gu.dense(48))],
-                                                     bigram=(50, 7, 3)), seed=5, std=0.2)
+                                                     bigram=(50, 7, 3)), seed=5, std=0.2, edit=gu.varied)
     prompts = list(ru.make_prompts(60, [5, 23, 1, 40, 12, 9], seed=10).values())
     engine = Engine(folder, dtype="f32", block_size=16, num_blocks=24, max_batch=3, chunk=8)
     got = engine.generate(prompts, max_tokens=8, temperature=0.0, stop_tokens=[])
