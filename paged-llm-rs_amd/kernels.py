@@ -1056,10 +1056,16 @@ def library_splits(rows: int, weight_rows: int, width: int) -> int:
     return 1
 
 
+def may_split_library(weight_rows: int, width: int) -> bool:
+    """Whether ``library_splits`` cuts products of this weight at some count of rows."""
+    return any(library_splits(rows, weight_rows, width) > 1 for rows in (STREAM_ROWS + 1, SPLIT_MAX_ROWS))
+
+
 def gemm_split_library(x: torch.Tensor, w: torch.Tensor, splits: int, out_dtype: torch.dtype = torch.bfloat16,
-                       add_into: torch.Tensor | None = None) -> torch.Tensor:
+                       add_into: torch.Tensor | None = None, turned: torch.Tensor | None = None) -> torch.Tensor:
     """y = x . w^T as ``splits`` products over stretches of K, run by the library as one batch, and their sum in
-    a fixed order: stored, or added into the 32-bit residual stream ``add_into`` (which is returned)."""
+    a fixed order: stored, or added into the 32-bit residual stream ``add_into`` (which is returned).  ``turned``: w^T as a
+    tensor of its own, [K, N], which the batch reads (made here where it is not given)."""
     _need(x, "matrix product input", None, torch.bfloat16)
     _need(w, "weight", None, torch.bfloat16)
     if x.dim() != 2 or w.dim() != 2 or w.shape[1] != x.shape[1]:
@@ -1069,8 +1075,10 @@ def gemm_split_library(x: torch.Tensor, w: torch.Tensor, splits: int, out_dtype:
     if splits < 2 or K % (8 * splits):
         raise TensorError(f"a width of {K} in {splits} stretches")
     part = K // splits
-    partial = torch.bmm(x.view(M, splits, part).transpose(0, 1), w.view(N, splits, part).permute(1, 2, 0),
-                        out_dtype=torch.float32)
+    if turned is None:
+        turned = w.t().contiguous()
+    _need(turned, "turned weight", (K, N), torch.bfloat16)
+    partial = torch.bmm(x.view(M, splits, part).transpose(0, 1), turned.view(splits, part, N), out_dtype=torch.float32)
     if add_into is not None:
         _need(add_into, "residual stream", (M, N), torch.float32)
         out, epilogue, out_f32 = add_into, 2, 1
@@ -1113,10 +1121,11 @@ def fused_norm_applies(rows_out: int, width: int, weight: torch.Tensor) -> bool:
 
 
 def linear_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype,
-                strips: torch.Tensor | None = None) -> torch.Tensor:
+                strips: torch.Tensor | None = None, turned: torch.Tensor | None = None) -> torch.Tensor:
     """y = x . w^T for bfloat16 operands with 32-bit accumulation: few rows stream the
     weights through the hand-written kernel, many rows go to the library's product.
-    ``strips``: the weights again as ``weights_in_strips`` lays them out, for the product that reads them so."""
+    ``strips``: the weights again as ``weights_in_strips`` lays them out, for the product that reads them so; ``turned``: w^T as
+    a tensor of its own, without which no product is cut into stretches."""
     _need(x, "matrix product input", None, torch.bfloat16)
     _need(w, "weight", None, torch.bfloat16)
     if out_dtype == torch.float32:
@@ -1133,8 +1142,8 @@ def linear_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype,
     if stream_wins(x.shape[0], w.shape[0], x.shape[1]):
         return gemm_stream(x, w, out_dtype)
     splits = library_splits(x.shape[0], w.shape[0], x.shape[1])
-    if splits > 1:
-        return gemm_split_library(x, w, splits, out_dtype)
+    if splits > 1 and turned is not None:
+        return gemm_split_library(x, w, splits, out_dtype, turned=turned)
     return torch.mm(x, w.t())
 
 
@@ -1442,13 +1451,20 @@ def weighted_sum_(x: torch.Tensor, a: float, y: torch.Tensor, b: float) -> torch
 
 # ---- attention layers with sinks, distance penalties, and pages that hold one small vector a token -------------
 
+def head_weights(w: torch.Tensor) -> torch.Tensor:
+    """The weights of a product a head, given as [heads, N, K] (a view will do), as ``gemm_heads`` takes them: [heads, N, K]
+    in 32-bit; in bfloat16 [heads, K, N], a tensor of its own (the library's batched product reads its right operand
+    as it lies in memory: turned views of it are not handed over)."""
+    return w.contiguous() if w.dtype == torch.float32 else w.transpose(1, 2).contiguous()
+
+
 def gemm_heads(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
-    """A product a head: out[t, h, :N] = x[t, h, :K] . w[h]^T, w [heads, N, K].  ``x`` [n, heads, >= K] and ``out``
+    """A product a head: out[t, h, :N] = x[t, h, :K] . W[h]^T with ``w = head_weights(W)``, W [heads, N, K].  ``x`` [n, heads, >= K] and ``out``
     [n, heads, >= N] may be views whose rows and heads lie further apart than their own sizes (the last axis
     contiguous); a view's values behind K or N are neither read nor written.  In 32-bit on the vector units
     (sums in ascending k: the true 32-bit path); in bfloat16 the library's batched product on the matrix cores."""
-    heads, N, K = w.shape
     _need(w, "weights a head")
+    heads, N, K = w.shape if w.dtype == torch.float32 else (w.shape[0], w.shape[2], w.shape[1])
     n = x.shape[0]
     if x.dim() != 3 or out.dim() != 3 or x.shape[1] != heads or out.shape[1] != heads or out.shape[0] != n:
         raise TensorError(f"a product a head of {tuple(x.shape)} with {tuple(w.shape)} into {tuple(out.shape)}")
@@ -1458,16 +1474,12 @@ def gemm_heads(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> torch.Ten
         raise TensorError("a product a head needs its operands on the GPU and of one type")
     if n == 0:
         return out
-    if w.dtype == torch.bfloat16 and n > GEMM_HEADS_PLAIN_ROWS:
-        torch.bmm(x.transpose(0, 1), w.transpose(1, 2), out=out.transpose(0, 1))
+    if w.dtype == torch.bfloat16:
+        torch.bmm(x.transpose(0, 1), w, out=out.transpose(0, 1))
         return out
     _check(library().pl_gemm_heads(x.data_ptr(), w.data_ptr(), out.data_ptr(), n, heads, N, K, x.stride(0), x.stride(1),
                                    out.stride(0), out.stride(1), _code(w, "weights a head"), 0, _stream()))
     return out
-
-
-# Up to this many rows a bfloat16 product a head runs on the vector units (one small launch); above, the library's.
-GEMM_HEADS_PLAIN_ROWS = 0
 
 
 def head_prepare(rows: torch.Tensor, off: int, batch, kv, q_out: torch.Tensor, H: int, G: int, D: int, V: int,

@@ -79,8 +79,8 @@ class LatentAttention:
             self.gain = None
         self.proj = Linear.fused(pieces)
         # U_h^T as the weights of a product a head, [H, R, D], and W_h, [H, V, R]
-        self.uk_t = params["uk"].view(H, D, R).transpose(1, 2).contiguous()
-        self.uv = params["uv"].view(H, V, R).contiguous()
+        self.uk_t = kernels.head_weights(params["uk"].view(H, D, R).transpose(1, 2))
+        self.uv = kernels.head_weights(params["uv"].view(H, V, R))
         self.sinks = head_sinks(spec.sink, H, params, device)
         # the rotation's angles: tables of cosines and sines where the spec bounds the positions, otherwise the
         # frequencies alone (rounded from 64-bit), and the kernel multiplies by the position in 32-bit

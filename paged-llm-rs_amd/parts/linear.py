@@ -16,6 +16,7 @@ class Linear:
     # Whether a bfloat16 weight is kept a second time in the order the product of few rows reads fastest
     # (``kernels.weights_in_strips``): the decoding steps then read that copy, everything else the weight as
     # stored.  It doubles the memory of the weights; ``load_model(..., strips=False)`` builds a model without.
+    # The same goes for w^T of the matrices that the library multiplies in stretches (``turned``).
     keep_strips = True
 
     def __init__(self, weight: torch.Tensor, bias: torch.Tensor | None = None):
@@ -24,6 +25,9 @@ class Linear:
         self.weight = weight.contiguous()
         self.strips = kernels.weights_in_strips(self.weight) if Linear.keep_strips else None
         self.out_features, self.in_features = weight.shape
+        # (w^T of the few large deep matrices whose library product is cut into stretches of its inner width)
+        self.turned = (self.weight.t().contiguous() if Linear.keep_strips and self.weight.dtype == torch.bfloat16
+                       and kernels.may_split_library(self.out_features, self.in_features) else None)
         if bias is not None and tuple(bias.shape) != (self.out_features,):
             raise TensorError(f"a bias of shape {tuple(bias.shape)} for {self.out_features} outputs")
         self.bias = None if bias is None else bias.contiguous()
@@ -96,14 +100,14 @@ class Linear:
             return kernels.gemm_stream(x, self.weight, out_dtype, swiglu=swiglu, activation=activation)
         if add_into is not None and not swiglu:
             splits = kernels.library_splits(x.shape[0], self.out_features, self.in_features)
-            if splits > 1:
-                kernels.gemm_split_library(x, self.weight, splits, add_into=add_into)
+            if splits > 1 and self.turned is not None:
+                kernels.gemm_split_library(x, self.weight, splits, add_into=add_into, turned=self.turned)
                 return None
         if swiglu:
             if kernels.tiled_swiglu_wins(x.shape[0], self.out_features // 2, self.in_features):
                 return kernels.gemm_tiled(x, self.weight, swiglu=True, activation=activation)
-            return kernels.swiglu(kernels.linear_bf16(x, self.weight, x.dtype, self.strips), activation=activation)
-        return kernels.linear_bf16(x, self.weight, out_dtype, self.strips)
+            return kernels.swiglu(kernels.linear_bf16(x, self.weight, x.dtype, self.strips, self.turned), activation=activation)
+        return kernels.linear_bf16(x, self.weight, out_dtype, self.strips, self.turned)
 
 
 def linears_of(part, seen=None, depth: int = 0):

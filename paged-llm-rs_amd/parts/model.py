@@ -203,11 +203,11 @@ class DecoderModel:
         return isinstance(self.embed_transform, EmbedTransforms)
 
     def matrix_bytes(self) -> tuple:
-        """(bytes of the weight matrices as stored, bytes of their second copies in strips)."""
+        """(bytes of the weight matrices as stored, bytes of their further copies: in strips, turned)."""
         stored = strips = 0
         tensors = set()
         for linear in linears_of(self):
-            for which, t in (("stored", linear.weight), ("strips", linear.strips)):
+            for which, t in (("stored", linear.weight), ("strips", linear.strips), ("turned", linear.turned)):
                 if t is None or t.data_ptr() in tensors:
                     continue
                 tensors.add(t.data_ptr())
