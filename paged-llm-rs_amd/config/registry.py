@@ -13,6 +13,7 @@ from .dimalix import DimalixConfig
 from .guzuvik import GuzuvikConfig
 from .lefavik import LefavikConfig
 from .mukenex import MukenexConfig
+from .nikonex import NikonexConfig
 from .papivik import PapivikConfig
 from .qwen3 import Qwen3Config, read_json
 
@@ -72,3 +73,4 @@ register_architecture("Lefavik", LefavikConfig, model_type="lefavik")
 register_architecture("Mukenex", MukenexConfig, model_type="mukenex")
 register_architecture("Dimalix", DimalixConfig, model_type="dimalix")
 register_architecture("Guzuvik", GuzuvikConfig, model_type="guzuvik")
+register_architecture("Nikonex", NikonexConfig, model_type="nikonex")

@@ -66,6 +66,7 @@ class LayerSpec:
     names: Optional[dict] = None            # other tensor-name parts for the block's members (norm1, mixer, norm2, feed_forward)
     stream_copies: Optional[int] = None     # for an arrangement over several copies of the stream: how many
     layer_scale: bool = False               # a sublayer's output times a gain a column before it joins the stream (``ls1``, ``ls2``)
+    residual_mult: float = 1.0              # what the sublayers' outputs are multiplied by before they join the stream (block ``parallel``)
 
 
 @dataclass(frozen=True)
@@ -119,6 +120,23 @@ class LinearAttentionSpec:
     head_dim: int = 0            # size of q and k a head
     value_dim: int = 0           # size of v a head
     decay: tuple = ()            # one a head
+    eps: float = 1e-6
+
+
+@dataclass(frozen=True)
+class RetentionSpec:
+    """Linear attention with one fixed decay a head and rotated queries and keys: S = decay S + k v^T, o = S^T q, where the
+    first ``rotary_dims`` values of every head of q and k turn in pairs (i, i + rotary_dims / 2) and k is multiplied by
+    ``key_scale`` behind that; every head's read-out divided by its root mean square (no gain), times silu(gate)."""
+    kind: str = "retention"
+    num_heads: int = 0
+    head_dim: int = 0            # size of q and k a head
+    value_dim: int = 0           # size of v a head
+    decay: tuple = ()            # one a head
+    rotary_dims: int = 0
+    rotary_base: float = 10000.0
+    rotary_ramp: Optional[tuple] = None     # as in ``LatentAttentionSpec``
+    key_scale: Optional[float] = None       # None = 1/sqrt(head_dim)
     eps: float = 1e-6
 
 
@@ -254,6 +272,11 @@ class LatentAttentionSpec:
     borrows: bool = False                   # no projection onto the small vector: the schedule names the layer whose pages are read
     # the rotation's frequencies rescaled by wavelength: (factor, low, high, original), see ``TiedAttentionSpec``
     rotary_scaling: Optional[tuple] = None
+    # ... or blended by a ramp over the pairs: (factor, original, fast, slow), see ``parts.rotary.ramped_frequencies``
+    rotary_ramp: Optional[tuple] = None
+    # Queries through a small vector of their own: x is projected onto ``q_rank`` values (``dq``), normed (``dq.norm``,
+    # ``norm_eps``) and projected onto the heads (``uq``).  None: one projection (``q``).
+    q_rank: Optional[int] = None
 
 
 # ---- several copies of the stream, experts chosen by a table ----------------------------------------
@@ -305,8 +328,11 @@ class RoutedExpertsSpec:
     chosen (``groups`` 1: no groups).  A chosen expert weighs its score (without the correction), divided, where
     ``normalised``, by the chosen scores' sum plus ``weight_eps``.  ``biased``: a tensor ``router.b`` is added to the logits.
     ``score`` "chosen_logits" instead of "softmax": the choice goes by the logits and the weights are the softmax over the chosen
-    logits alone.  ``activation`` "clamped" with its ``limit``: an expert is down(g sigmoid(1.702 g) (u + 1)) with
-    g = min(gate x, limit) and u = clamp(up x, -limit, limit)."""
+    logits alone.  ``score`` "sigmoid": a score is the sigmoid of its own logit.  ``activation`` "clamped" with its ``limit``: an
+    expert is down(g sigmoid(1.702 g) (u + 1)) with g = min(gate x, limit) and u = clamp(up x, -limit, limit).
+    ``gated`` False: an expert is down(act(up x)).  ``group_best`` members' choice scores are added up for a group's own score.
+    Weights are multiplied by ``weight_scale`` at the end.  ``shared_size``: beside the chosen ones every token uses one more expert
+    of the same form and of that size (``shared.*``), which counts sigmoid(``shared.sg`` x)."""
     kind: str = "routed_experts"
     experts: int = 0
     identity: int = 0
@@ -321,3 +347,7 @@ class RoutedExpertsSpec:
     weight_eps: float = 1e-20
     biased: bool = False
     limit: Optional[float] = None
+    gated: bool = True
+    group_best: int = 1
+    weight_scale: float = 1.0
+    shared_size: int = 0                    # 0: no shared expert

@@ -31,6 +31,7 @@ typedef float gt_f32x2 __attribute__((ext_vector_type(2)));
 #define GT_SWIGLU 1
 #define GT_ADD 2
 #define GT_STORE32 3       // y is 32-bit and takes the result as it is (grouped products only)
+#define GT_ACT 4           // y = act(result), bfloat16 (grouped products only)
 
 // Grouped: the rows are dealt to groups (experts), every group with a weight matrix of its own, one behind the
 // other in w.  A tile of 128 rows belongs to one group (`tile_group`, negative: a tile nobody uses); row r of
@@ -46,6 +47,10 @@ struct GtGroups {
     int splits;
     long long y_split_stride;
     float limit;               // of the clamped gate (PL_ACT_CLAMPED)
+    int x_pitch, y_pitch;      // elements between two rows of x and of y
+    // One group, `last` (-1: none), may have a matrix of other sizes: w_last, [N_last (2 N_last for SwiGLU), K_last].
+    int last, N_last, K_last;
+    const bf16_t* w_last;
 };
 
 // 16 bytes a lane from global memory straight into LDS (see attention_prefill.hip: assembly, so that
@@ -85,8 +90,16 @@ gemm_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, vo
     if constexpr (GROUPED) {
         const int group = groups.tile_group[m0 / GT_BM];
         if (group < 0) return;                       // (the whole workgroup)
-        w += static_cast<long long>(group) * groups.w_stride;
+        if (group == groups.last) {
+            w = groups.w_last;
+            N = groups.N_last;
+            K = groups.K_last;
+        } else {
+            w += static_cast<long long>(group) * groups.w_stride;
+        }
+        if (n0 >= N) return;                         // (this group has fewer columns than another)
     }
+    const int x_pitch = GROUPED ? groups.x_pitch : K, y_pitch = GROUPED ? groups.y_pitch : N;
 
     const int tid = threadIdx.x, lane = tid & 63;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -108,7 +121,7 @@ gemm_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, vo
             if constexpr (GROUPED) {
                 if (groups.gather != nullptr) grow = static_cast<size_t>(max(groups.gather[m0 + row], 0));
             }
-            from[i] = reinterpret_cast<const char*>(x) + (grow * K + piece * 8) * 2;
+            from[i] = reinterpret_cast<const char*>(x) + (grow * x_pitch + piece * 8) * 2;
         } else {
             // SwiGLU: rows 0..63 of the tile are gate rows n0.., rows 64..127 the up rows N + n0..
             // (grouped, the last tile of columns may reach past N: it reads the last row again)
@@ -249,6 +262,14 @@ gemm_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, vo
 #pragma unroll
                         for (int i = 0; i < 4; ++i) v[i] = acc[t][mb][4 * j + i];
                         *reinterpret_cast<gt_f32x4*>(at_row + col * 4) = v;
+                    } else if constexpr (EPI == GT_ACT) {
+                        float v[4];
+#pragma unroll
+                        for (int i = 0; i < 4; ++i) v[i] = pl_activate<false>(acc[t][mb][4 * j + i], act);
+                        uint2 packed;
+                        packed.x = gt_pack2(v[0], v[1]);
+                        packed.y = gt_pack2(v[2], v[3]);
+                        *reinterpret_cast<uint2*>(at_row + col * 2) = packed;
                     } else {
                         uint2 packed;
                         packed.x = gt_pack2(acc[t][mb][4 * j], acc[t][mb][4 * j + 1]);
@@ -270,7 +291,7 @@ gemm_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, vo
             if (n0 + (piece + 1) * (16 / OUT_BYTES) > N) continue;      // columns past the matrix
         }
         const gt_f32x4 got = *reinterpret_cast<const gt_f32x4*>(staged + r * PITCH + piece * 16);
-        char* out = static_cast<char*>(y_) + (static_cast<size_t>(row) * N + n0) * OUT_BYTES + piece * 16;
+        char* out = static_cast<char*>(y_) + (static_cast<size_t>(row) * y_pitch + n0) * OUT_BYTES + piece * 16;
         if constexpr (EPI == GT_ADD) {
             gt_f32x4 old = *reinterpret_cast<const gt_f32x4*>(out);
 #pragma unroll
@@ -306,7 +327,7 @@ static int gt_launch(const void* x, const void* w, void* y, int M, int N, int K,
     }
     gemm_tiled_kernel<EPI><<<static_cast<int>(total), 256, lds_bytes, stream>>>(
         static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(w), y, M, N, K, row_tiles, static_cast<int>(total), act,
-        GtGroups{nullptr, nullptr, 0, 1, 0, 0.f});
+        GtGroups{nullptr, nullptr, 0, 1, 0, 0.f, K, N, -1, 0, 0, nullptr});
     PL_CHECK_LAUNCH("gemm_tiled");
     return 0;
 }
@@ -315,7 +336,8 @@ template <int EPI>
 static int gt_launch_grouped(const void* x, const void* w, void* y, int row_tiles, int N, int K, int act, GtGroups groups,
                              int x_rows, hipStream_t stream) {
     constexpr int COLS = EPI == GT_SWIGLU ? GT_BN / 2 : GT_BN;
-    const long long total = static_cast<long long>(row_tiles) * pl_ceil_div(N, COLS);
+    const int columns = groups.last >= 0 && groups.N_last > N ? groups.N_last : N;
+    const long long total = static_cast<long long>(row_tiles) * pl_ceil_div(columns, COLS);
     PL_REQUIRE(total > 0 && total < (1ll << 30), "grouped tiled product: %lld workgroups", total);
     constexpr size_t out_bytes = gt_out_bytes<EPI>();
     constexpr size_t stage_bytes = static_cast<size_t>(GT_STAGES) * GT_STAGE_ELEMS * 2;
@@ -340,19 +362,30 @@ static int gt_launch_grouped(const void* x, const void* w, void* y, int row_tile
 // null, in place (x_rows >= row_tiles * 128).  w: bfloat16, group g's matrix at w + g * w_stride: [N, K], or
 // [2 N, K] with the gate rows first for epilogue 1.  y: [row_tiles * 128, N], bfloat16 for epilogues 0 and 1
 // (1: act(gate) * up), 32-bit for epilogue 3.  K a multiple of 32, N of 8 (of 64 for epilogue 1).
-// splits > 1 (epilogue 3 only): y has that many copies, [splits][row_tiles * 128, N], a stretch of K each.
+// Epilogue 4: y = act(result), bfloat16.  splits > 1 (epilogue 3 only): y has that many copies, [splits][row_tiles * 128, y_pitch], a stretch of K each.
+// x_pitch, y_pitch: elements between two rows (K and N, or more: multiples of 8).  last >= 0: that group's matrix is w_last, of N_last and K_last
+// in the places of N and K, under the same rules.
 extern "C" int pl_gemm_tiled_grouped(const void* x, const void* w, void* y, const int* tile_group, const int* gather,
                                      long long w_stride, int row_tiles, int x_rows, int N, int K, int epilogue, int act,
-                                     int splits, float limit, hipStream_t stream) {
+                                     int splits, float limit, int x_pitch, int y_pitch, int last, const void* w_last, int N_last,
+                                     int K_last, hipStream_t stream) {
+    PL_REQUIRE(last < 0 || (w_last != nullptr && N_last > 0 && K_last > 0 && K_last % GT_BK == 0 && N_last % 8 == 0 && splits <= K_last / GT_BK &&
+                            (epilogue != GT_SWIGLU || N_last % (GT_BN / 2) == 0)),
+               "grouped tiled product: a last group of %d columns, inner width %d, epilogue %d", N_last, K_last, epilogue);
+    PL_REQUIRE(x_pitch >= K && y_pitch >= N && x_pitch % 8 == 0 && y_pitch % 8 == 0 && (last < 0 || (x_pitch >= K_last && y_pitch >= N_last)),
+               "grouped tiled product: rows of %d and %d for an inner width of %d and %d columns", x_pitch, y_pitch, K, N);
+    PL_REQUIRE(epilogue != GT_ACT || act <= PL_ACT_RELU2, "grouped tiled product: activation code %d without a gate", act);
     PL_REQUIRE(splits >= 1 && splits <= K / GT_BK && (splits == 1 || epilogue == GT_STORE32),
                "grouped tiled product: %d stretches of an inner width of %d, epilogue %d", splits, K, epilogue);
     PL_REQUIRE(act >= PL_ACT_SILU && act <= PL_ACT_CLAMPED, "grouped tiled product: activation code %d", act);
     PL_REQUIRE(row_tiles > 0 && x_rows > 0 && N > 0 && K > 0 && K % GT_BK == 0 && N % 8 == 0 && (epilogue != GT_SWIGLU || N % (GT_BN / 2) == 0),
                "grouped tiled product: %d tiles of rows, %d columns, inner width %d, epilogue %d", row_tiles, N, K, epilogue);
     PL_REQUIRE(tile_group != nullptr && (gather != nullptr || x_rows >= row_tiles * GT_BM), "grouped tiled product: %d rows for %d tiles", x_rows, row_tiles);
-    const GtGroups groups{tile_group, gather, w_stride, splits, static_cast<long long>(row_tiles) * GT_BM * N, limit};
+    const GtGroups groups{tile_group, gather, w_stride, splits, static_cast<long long>(row_tiles) * GT_BM * y_pitch, limit, x_pitch, y_pitch,
+                          last, N_last, K_last, static_cast<const bf16_t*>(w_last)};
     if (epilogue == GT_SWIGLU) return gt_launch_grouped<GT_SWIGLU>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
     if (epilogue == GT_STORE32) return gt_launch_grouped<GT_STORE32>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
+    if (epilogue == GT_ACT) return gt_launch_grouped<GT_ACT>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
     if (epilogue == GT_STORE) return gt_launch_grouped<GT_STORE>(x, w, y, row_tiles, N, K, act, groups, x_rows, stream);
     PL_REQUIRE(false, "grouped tiled product: epilogue %d", epilogue);
     return 0;

@@ -301,11 +301,14 @@ struct LatentPrepareArgs {
     const float* rows;        // [n, stride]
     int stride;
     int q_off;                // H heads of [D | rot] from here
+    const float* kv_rows;     // [n, kv_stride] (the same rows, or another product's)
+    int kv_stride;
     int kv_off;               // [R | rot] from here (unused when nothing is written)
     const float* gain;        // [R]
     float eps;
     const float* cos;         // [positions, turned / 2]
     const float* sin;
+    float amplitude;          // what cosine and sine are multiplied by
     int turned, table_rows;   // the first `turned` values of a rotated part turn
     const int* positions;
     const int* seq_of;
@@ -343,7 +346,7 @@ __global__ __launch_bounds__(64) void latent_prepare_kernel(LatentPrepareArgs a)
         const int s = a.seq_of[t];
         const int page = a.block_table[static_cast<size_t>(s) * a.max_blocks + pos / a.block_size];
         if (page < 0) return;
-        const float* src = row + a.kv_off;
+        const float* src = a.kv_rows + static_cast<size_t>(t) * a.kv_stride + a.kv_off;
         T* out = static_cast<T*>(a.pool) + (static_cast<size_t>(page) * a.block_size + pos % a.block_size) * P;
         float ss = 0.f;
         for (int e = lane; e < R; e += 64) ss += src[e] * src[e];
@@ -366,6 +369,8 @@ __global__ __launch_bounds__(64) void latent_prepare_kernel(LatentPrepareArgs a)
                 } else {
                     sincosf(static_cast<float>(pos) * cs[i], &sn_i, &c);
                 }
+                c *= a.amplitude;
+                sn_i *= a.amplitude;
                 x = (e & 1) ? part[e] * c + part[e - 1] * sn_i : part[e] * c - part[e + 1] * sn_i;
             }
         }
@@ -373,8 +378,8 @@ __global__ __launch_bounds__(64) void latent_prepare_kernel(LatentPrepareArgs a)
     }
 }
 
-extern "C" int pl_latent_prepare(const float* rows, int stride, int q_off, int kv_off, const float* gain, float eps,
-                                 const float* cos, const float* sin, int turned, int table_rows, const int* positions,
+extern "C" int pl_latent_prepare(const float* rows, int stride, int q_off, const float* kv_rows, int kv_stride, int kv_off,
+                                 const float* gain, float eps, const float* cos, const float* sin, float amplitude, int turned, int table_rows, const int* positions,
                                  const int* seq_of, const int* block_table, int max_blocks, int block_size, int write_kv,
                                  void* q_plain, void* q_out, void* pool, int dtype, int n, int H, int D, int rot, int R,
                                  int P, hipStream_t stream) {
@@ -382,10 +387,10 @@ extern "C" int pl_latent_prepare(const float* rows, int stride, int q_off, int k
                "latent_prepare: rows %d, %d heads of %d + %d, vectors of %d in rows of %d", n, H, D, rot, R, P);
     PL_REQUIRE(turned >= 0 && turned % 2 == 0 && turned <= rot && (turned == 0 || (cos != nullptr && (sin == nullptr || table_rows > 0))),
                "latent_prepare: a rotation over %d of %d values", turned, rot);
-    PL_REQUIRE(block_size > 0 && max_blocks > 0 && stride >= q_off + H * (D + rot) && (!write_kv || (stride >= kv_off + R + rot && gain != nullptr && pool != nullptr)),
+    PL_REQUIRE(block_size > 0 && max_blocks > 0 && stride >= q_off + H * (D + rot) && (!write_kv || (kv_rows != nullptr && kv_stride >= kv_off + R + rot && gain != nullptr && pool != nullptr)),
                "latent_prepare: pages of %d, tables of %d, rows of %d values", block_size, max_blocks, stride);
     if (n == 0) return 0;
-    LatentPrepareArgs a{rows, stride, q_off, kv_off, gain, eps, cos, sin, turned, table_rows, positions, seq_of, block_table,
+    LatentPrepareArgs a{rows, stride, q_off, kv_rows, kv_stride, kv_off, gain, eps, cos, sin, amplitude, turned, table_rows, positions, seq_of, block_table,
                         max_blocks, block_size, write_kv, q_plain, q_out, pool, n, H, D, rot, R, P};
     const dim3 grid(n, H + 1);
     if (dtype == PL_DTYPE_F32) latent_prepare_kernel<float><<<grid, 64, 0, stream>>>(a);
@@ -441,5 +446,46 @@ extern "C" int pl_add_position_rows(float* x, const void* table, int dtype, cons
     else if (dtype == PL_DTYPE_BF16) add_position_rows_kernel<bf16_t><<<n, 256, 0, stream>>>(x, static_cast<const bf16_t*>(table), positions, width, table_rows);
     else PL_REQUIRE(false, "add_position_rows: dtype code %d", dtype);
     PL_CHECK_LAUNCH("add_position_rows");
+    return 0;
+}
+
+// A stretch of columns of 32-bit rows, normed: out[t, e] = x / sqrt(mean(x^2) + eps) * gain[e].  A workgroup a row; up to
+// eight values a thread stay in registers between the sum and the store.
+template <typename T>
+__global__ __launch_bounds__(256) void rows_norm_kernel(const float* __restrict__ rows, int stride, int off, const float* __restrict__ gain,
+                                                        int W, float eps, T* __restrict__ out) {
+    __shared__ float scratch[16];
+    const float* x = rows + static_cast<size_t>(blockIdx.x) * stride + off;
+    constexpr int KEEP = 8;
+    float kept[KEEP], g[KEEP];
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+        const int e = threadIdx.x + blockDim.x * k;
+        kept[k] = e < W ? x[e] : 0.f;
+        g[k] = e < W ? gain[e] : 0.f;
+        ss += kept[k] * kept[k];
+    }
+    for (int e = threadIdx.x + blockDim.x * KEEP; e < W; e += blockDim.x) ss += x[e] * x[e];
+    ss = block_sum(ss, scratch);
+    const float inv = 1.f / sqrtf(ss / static_cast<float>(W) + eps);
+    T* o = out + static_cast<size_t>(blockIdx.x) * W;
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k) {
+        const int e = threadIdx.x + blockDim.x * k;
+        if (e < W) o[e] = from_float<T>(kept[k] * inv * g[k]);
+    }
+    for (int e = threadIdx.x + blockDim.x * KEEP; e < W; e += blockDim.x) o[e] = from_float<T>(x[e] * inv * gain[e]);
+}
+
+extern "C" int pl_rows_norm(const float* rows, int stride, int off, const float* gain, int W, float eps, void* out, int dtype, int n,
+                            hipStream_t stream) {
+    PL_REQUIRE(n >= 0 && W > 0 && off >= 0 && stride >= off + W, "rows_norm: %d rows of %d, %d columns from %d", n, stride, W, off);
+    if (n == 0) return 0;
+    const int threads = W <= 512 ? 64 : 256;
+    if (dtype == PL_DTYPE_F32) rows_norm_kernel<float><<<n, threads, 0, stream>>>(rows, stride, off, gain, W, eps, static_cast<float*>(out));
+    else if (dtype == PL_DTYPE_BF16) rows_norm_kernel<bf16_t><<<n, threads, 0, stream>>>(rows, stride, off, gain, W, eps, static_cast<bf16_t*>(out));
+    else PL_REQUIRE(false, "rows_norm: dtype code %d", dtype);
+    PL_CHECK_LAUNCH("rows_norm");
     return 0;
 }

@@ -243,7 +243,17 @@ struct MoeArgs {
     const float* weight;
     int identity;
     float limit;           // of the clamped gate (PL_ACT_CLAMPED)
+    int plain;             // an expert is down(act(up x)): w_gu holds up rows alone, [E, F, W]
+    // An expert of another size that every row of a router's choice names last, as number `shared_at` (-1: there is none).
+    int shared_at, shared_F;
+    const void* shared_gu; // [2 shared_F, W], or [shared_F, W] where plain
+    const void* shared_down;  // [W, shared_F]
 };
+
+// The values of a row's pairs lie one behind the other in h: pair c from c F on, the shared expert's, the last, of another length.
+__host__ __device__ static inline int moe_row_values(const MoeArgs& a) {
+    return a.shared_at >= 0 ? (a.top - 1) * a.F + a.shared_F : a.top * a.F;
+}
 
 // The expert of pair (t, c), or -1: the router's choice, or the table's row of the token's id.
 __device__ __forceinline__ int moe_pair_expert(const MoeArgs& a, int t, int c) {
@@ -259,17 +269,22 @@ __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
     const int t = blockIdx.x / a.top, c = blockIdx.x % a.top;
     if (a.positions[t] < 0) return;
     const int e = moe_pair_expert(a, t, c);
-    if (e < 0 || e >= a.E) return;
-    const int W = a.W, F = a.F;
+    const bool shared = a.shared_at >= 0 && e == a.shared_at && c == a.top - 1;
+    if (!shared && (e < 0 || e >= a.E)) return;
+    const int W = a.W, F = shared ? a.shared_F : a.F;
     const T* x = static_cast<const T*>(a.x) + static_cast<size_t>(t) * W;
     for (int k = threadIdx.x; k < W; k += blockDim.x) moe_x[k] = to_float(x[k]);
     __syncthreads();
     const int lane = threadIdx.x % PL_WAVE, wave = threadIdx.x / PL_WAVE, waves = blockDim.x / PL_WAVE;
-    const T* gate = static_cast<const T*>(a.w_gu) + static_cast<size_t>(e) * 2 * F * W;
+    const T* gate = shared ? static_cast<const T*>(a.shared_gu) : static_cast<const T*>(a.w_gu) + static_cast<size_t>(e) * (a.plain ? 1 : 2) * F * W;
     const T* up = gate + static_cast<size_t>(F) * W;
-    T* h = static_cast<T*>(a.h) + (static_cast<size_t>(t) * a.top + c) * F;
+    T* h = static_cast<T*>(a.h) + static_cast<size_t>(t) * moe_row_values(a) + c * a.F;
     for (int f = blockIdx.y * waves + wave; f < F; f += gridDim.y * waves) {
         const float g = moe_dot<T>(gate + static_cast<size_t>(f) * W, moe_x, W, lane);
+        if (a.plain) {
+            if (lane == 0) h[f] = from_float<T>(pl_activate<true>(g, a.act));
+            continue;
+        }
         const float u = moe_dot<T>(up + static_cast<size_t>(f) * W, moe_x, W, lane);
         if (lane == 0) h[f] = from_float<T>(pl_gate_pair<true>(g, u, a.act, a.limit));
     }
@@ -277,7 +292,7 @@ __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
 
 template <typename T>
 __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
-    extern __shared__ float moe_h[];                  // [top, F]
+    extern __shared__ float moe_h[];                  // the row's values of h
     const int t = blockIdx.x;
     const int W = a.W, F = a.F, top = a.top;
     float* o = a.out + static_cast<size_t>(t) * W;
@@ -288,8 +303,9 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
         return;
     }
     const T* x = static_cast<const T*>(a.x) + static_cast<size_t>(t) * W;
-    const T* h = static_cast<const T*>(a.h) + static_cast<size_t>(t) * top * F;
-    for (int k = threadIdx.x; k < top * F; k += blockDim.x) moe_h[k] = to_float(h[k]);
+    const int values = moe_row_values(a);
+    const T* h = static_cast<const T*>(a.h) + static_cast<size_t>(t) * values;
+    for (int k = threadIdx.x; k < values; k += blockDim.x) moe_h[k] = to_float(h[k]);
     __syncthreads();
     const float share = 1.f / static_cast<float>(top);
     for (int w = blockIdx.y * waves + wave; w < W; w += gridDim.y * waves) {
@@ -297,6 +313,11 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
         for (int c = 0; c < top; ++c) {
             const int e = moe_pair_expert(a, t, c);
             const float counts = a.weight != nullptr ? a.weight[static_cast<size_t>(t) * top + c] : share;
+            if (a.shared_at >= 0 && e == a.shared_at && c == top - 1) {
+                const T* down = static_cast<const T*>(a.shared_down) + static_cast<size_t>(w) * a.shared_F;
+                sum += moe_dot<T>(down, moe_h + c * F, a.shared_F, lane) * counts;
+                continue;
+            }
             if (e >= a.E && e < a.E + a.identity) sum += to_float(x[w]) * counts;
             if (e < 0 || e >= a.E) continue;
             const T* down = static_cast<const T*>(a.w_down) + (static_cast<size_t>(e) * W + w) * F;
@@ -308,20 +329,34 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
 
 // out[t] (32-bit) = (1/top) sum over the experts e that table[id of t] names of down_e (act(gate_e x_t) * (up_e x_t)).
 // x [n, W], w_gu [E, 2 F, W], w_down [E, W, F] and the workspace h [n, top, F] in `dtype`; table [vocab, top].
-// With `choice` [n, top] (and `weight` [n, top]) a router has chosen instead of the table: see MoeArgs.
+// With `choice` [n, top] (and `weight` [n, top]) a router has chosen instead of the table: see MoeArgs, which also says what
+// `plain` and the shared expert are (h is then [n, moe_row_values]).
 extern "C" int pl_moe_rows(const void* x, const int* ids, const int* src, const int* fed, const int* positions,
                            const int* table, const void* w_gu, const void* w_down, void* h, float* out, int dtype,
                            int n, int W, int F, int E, int top, int vocab, int act, const int* choice, const float* weight,
-                           int identity, float limit, hipStream_t stream) {
-    PL_REQUIRE(n >= 0 && W > 0 && F > 0 && E > 0 && top > 0 && top <= E + identity && identity >= 0 && vocab > 0 && act >= 0 && act <= PL_ACT_CLAMPED,
+                           int identity, float limit, int plain, int shared_F, const void* shared_gu, const void* shared_down,
+                           hipStream_t stream) {
+    PL_REQUIRE(shared_F >= 0 && (shared_F == 0 || (choice != nullptr && shared_gu != nullptr && shared_down != nullptr)),
+               "moe_rows: a shared expert of %d needs its matrices and a router's choice", shared_F);
+    PL_REQUIRE(!plain || act <= PL_ACT_RELU2, "moe_rows: activation %d between two matrices", act);
+    PL_REQUIRE(n >= 0 && W > 0 && F > 0 && E > 0 && top > 0 && top <= E + identity + (shared_F > 0 ? 1 : 0) && identity >= 0 && vocab > 0 && act >= 0 && act <= PL_ACT_CLAMPED,
                "moe_rows: %d rows of %d, %d experts of %d, %d a row", n, W, E, F, top);
     PL_REQUIRE((choice != nullptr) != (table != nullptr) && (weight == nullptr || choice != nullptr),
                "moe_rows: the experts of a row are a table's or a router's");
     PL_REQUIRE((src == nullptr) == (fed == nullptr), "moe_rows: rows fed from the step before need both the rows and the tokens");
-    PL_REQUIRE(W <= 16384 && static_cast<long long>(top) * F <= 16384, "moe_rows: rows of %d, %d experts of %d a row", W, top, F);
+    const long long values = shared_F > 0 ? static_cast<long long>(top - 1) * F + shared_F : static_cast<long long>(top) * F;
+    PL_REQUIRE(W <= 16384 && values <= 40000, "moe_rows: rows of %d, %d experts of %d a row (and one of %d)", W, top, F, shared_F);
     PL_REQUIRE(static_cast<long long>(n) * top < (1ll << 31), "moe_rows: %d rows", n);
     if (n == 0) return 0;
-    MoeArgs a{x, ids, src, fed, positions, table, w_gu, w_down, h, out, n, W, F, E, top, vocab, act, choice, weight, identity, limit};
+    MoeArgs a{x, ids, src, fed, positions, table, w_gu, w_down, h, out, n, W, F, E, top, vocab, act, choice, weight, identity, limit,
+              plain, shared_F > 0 ? E + identity : -1, shared_F, shared_gu, shared_down};
+    const size_t h_bytes = static_cast<size_t>(values) * sizeof(float);
+    if (h_bytes > 48 * 1024) {
+        const void* kernel = dtype == PL_DTYPE_F32 ? reinterpret_cast<const void*>(&moe_down_kernel<float>)
+                                                   : reinterpret_cast<const void*>(&moe_down_kernel<bf16_t>);
+        const hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(h_bytes));
+        PL_REQUIRE(e == hipSuccess, "moe_rows: %zu bytes of LDS refused: %s", h_bytes, hipGetErrorString(e));
+    }
     // few rows: deal an expert's rows of weights to several workgroups, so that the chip has work
     const int cu = pl_compute_units();
     int up_parts = 1, down_parts = 1;
@@ -330,10 +365,10 @@ extern "C" int pl_moe_rows(const void* x, const int* ids, const int* src, const 
     const dim3 up_grid(n * top, up_parts), down_grid(n, down_parts);
     if (dtype == PL_DTYPE_F32) {
         moe_up_kernel<float><<<up_grid, 256, W * sizeof(float), stream>>>(a);
-        moe_down_kernel<float><<<down_grid, 256, static_cast<size_t>(top) * F * sizeof(float), stream>>>(a);
+        moe_down_kernel<float><<<down_grid, 256, h_bytes, stream>>>(a);
     } else if (dtype == PL_DTYPE_BF16) {
         moe_up_kernel<bf16_t><<<up_grid, 256, W * sizeof(float), stream>>>(a);
-        moe_down_kernel<bf16_t><<<down_grid, 256, static_cast<size_t>(top) * F * sizeof(float), stream>>>(a);
+        moe_down_kernel<bf16_t><<<down_grid, 256, h_bytes, stream>>>(a);
     } else {
         PL_REQUIRE(false, "moe_rows: dtype code %d", dtype);
     }
@@ -348,9 +383,10 @@ extern "C" int pl_moe_rows(const void* x, const int* ids, const int* src, const 
 // between the experts' stretches), slot_of[p] = slot (or -1 for a pair of a padding row),
 // tile_group[i] = the expert of tile i (or -1 behind the last).  Which of an expert's pairs gets which of
 // its slots is left to the order in which the threads arrive: nothing computed from a slot depends on it.
+// shared_at: the number under which a choice names the shared expert (-1: there is none); it is dealt to as expert E - 1.
 __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* ids, const int* src, const int* fed, const int* positions,
-                                                        const int* table, const int* choice, int n, int top, int E, int vocab, int tile,
-                                                        int tiles, int* gather, int* slot_of, int* tile_group) {
+                                                        const int* table, const int* choice, int n, int top, int E, int vocab, int shared_at,
+                                                        int tile, int tiles, int* gather, int* slot_of, int* tile_group) {
     extern __shared__ int moe_counts[];               // count [E], base [E], cursor [E]
     int* count = moe_counts;
     int* base = moe_counts + E;
@@ -364,7 +400,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* ids, const in
         if (positions[t] < 0) return -1;
         int e;
         if (choice != nullptr) {
-            e = choice[p];                            // (an identity expert, E or beyond, takes no slot)
+            e = choice[p];                            // (an identity expert, at the given experts' count or beyond, takes no slot)
+            if (shared_at >= 0) e = e == shared_at ? E - 1 : (e < E - 1 ? e : -1);
         } else {
             const int id = moe_token(ids, src, fed, t);
             if (id < 0 || id >= vocab) return -1;
@@ -402,14 +439,15 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* ids, const in
 
 // tiles: what the caller has room for, at least ceil(n * top / tile) + min(E, n * top).
 extern "C" int pl_moe_sort(const int* ids, const int* src, const int* fed, const int* positions, const int* table,
-                           const int* choice, int n, int top, int E, int vocab, int tile, int tiles, int* gather, int* slot_of,
+                           const int* choice, int n, int top, int E, int vocab, int shared_at, int tile, int tiles, int* gather, int* slot_of,
                            int* tile_group, hipStream_t stream) {
+    PL_REQUIRE(shared_at < 0 || (choice != nullptr && shared_at >= E - 1), "moe_sort: a shared expert chosen as number %d of %d", shared_at, E);
     PL_REQUIRE(n > 0 && top > 0 && E > 0 && E <= 4096 && vocab > 0 && tile > 0, "moe_sort: %d rows, %d of %d experts", n, top, E);
     PL_REQUIRE((choice != nullptr) != (table != nullptr), "moe_sort: the experts of a row are a table's or a router's");
     PL_REQUIRE(static_cast<long long>(n) * top < (1ll << 30) && tiles >= (n * top + tile - 1) / tile + (E < n * top ? E : n * top),
                "moe_sort: %d tiles of %d for %d rows with %d of %d experts", tiles, tile, n, top, E);
     PL_REQUIRE((src == nullptr) == (fed == nullptr), "moe_sort: rows fed from the step before need both the rows and the tokens");
-    moe_sort_kernel<<<1, 1024, 3 * E * sizeof(int), stream>>>(ids, src, fed, positions, table, choice, n, top, E, vocab, tile, tiles,
+    moe_sort_kernel<<<1, 1024, 3 * E * sizeof(int), stream>>>(ids, src, fed, positions, table, choice, n, top, E, vocab, shared_at, tile, tiles,
                                                                gather, slot_of, tile_group);
     PL_CHECK_LAUNCH("moe_sort");
     return 0;
@@ -525,13 +563,15 @@ __device__ __forceinline__ void router_dots(const T* __restrict__ w, const float
 
 // A workgroup a row; its first wave chooses.  z [n, stride] are the router's 32-bit logits over `total` outputs; `bias`
 // [total], where there is one, is added to them first.
-// `of_chosen`: the choice goes by the logits themselves and the weights are the softmax over the chosen logits alone
+// `scoring` 1: the choice goes by the logits themselves and the weights are the softmax over the chosen logits alone
 // (`correction`, `normalised` and `weight_eps` then do not enter).  Otherwise
-// s = softmax(z); the choice goes
-// by s + correction; outputs form `groups` equal groups of neighbours, a group counts by its largest choice score and
-// only members of the `kept` best groups can be chosen (the others count as minus infinity); the `top` largest are
+// s = softmax(z) (`scoring` 0) or the sigmoid of z, one by one (`scoring` 2); the choice goes
+// by s + correction; outputs form `groups` equal groups of neighbours, a group counts by its largest choice score (the sum of its two largest,
+// with group_best 2) and only members of the `kept` best groups can be chosen (the others count as minus infinity); the `top` largest are
 // chosen (the lower index among equals), in that order; a chosen output weighs s, divided, with `normalised`, by the
-// chosen ones' sum plus weight_eps.  Rows at position -1 choose nothing (-1, weight 0).
+// chosen ones' sum plus weight_eps, times `scale`.  Rows at position -1 choose nothing (-1, weight 0).
+// `shared`: one more output behind the `total`; a row names number `total` behind its `top` chosen ones, with that output's
+// sigmoid as its weight (the rows of `choice` and `weight` are one longer).
 // With `x` [n, W] and the router's matrix `w` [total, W] (both of type T) the workgroup works the logits out itself
 // first, all its waves at it, 32-bit sums of the products in an order that W alone fixes: for steps of few rows, where
 // a product's launch costs more than the product.  (The waves behind the first then walk through the choice with
@@ -542,7 +582,9 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
                                                             int kept, int normalised, float weight_eps, int* __restrict__ choice,
                                                             float* __restrict__ weight, const T* __restrict__ x,
                                                             const T* __restrict__ w, int W, const float* __restrict__ bias,
-                                                            int of_chosen) {
+                                                            int scoring, int group_best, float scale, int shared) {
+    const bool of_chosen = scoring == 1;
+    const int named = top + shared, outputs = total_all + shared;     // what a row names, and the router's rows
     extern __shared__ float router_lds[];             // score [total], choice score [total], group score [groups], kept or not [groups]
     float* score = router_lds;                        // (and behind them, where the logits are worked out here: logits [total], the row [W])
     float* pick = router_lds + total_all;
@@ -550,10 +592,10 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     float* stays = group + groups_all;
     const int t = blockIdx.x, lane = threadIdx.x % PL_WAVE, wave = threadIdx.x / PL_WAVE, waves = blockDim.x / PL_WAVE;
     const bool chooser = wave == 0;
-    int* chosen = choice + static_cast<size_t>(t) * top;
-    float* counts = weight + static_cast<size_t>(t) * top;
+    int* chosen = choice + static_cast<size_t>(t) * named;
+    float* counts = weight + static_cast<size_t>(t) * named;
     if (positions != nullptr && positions[t] < 0) {
-        for (int c = threadIdx.x; c < top; c += blockDim.x) {
+        for (int c = threadIdx.x; c < named; c += blockDim.x) {
             chosen[c] = -1;
             counts[c] = 0.f;
         }
@@ -562,15 +604,15 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     const float* row = z + static_cast<size_t>(t) * stride;
     if (x != nullptr) {
         float* logits = stays + groups_all;
-        float* xs = logits + total_all;
+        float* xs = logits + outputs;
         for (int k = threadIdx.x; k < W; k += blockDim.x) xs[k] = to_float(x[static_cast<size_t>(t) * W + k]);
         __syncthreads();
-        for (int e0 = wave; e0 < total_all; e0 += 4 * waves) {
+        for (int e0 = wave; e0 < outputs; e0 += 4 * waves) {
             float sums[4];
-            router_dots<T>(w, xs, W, lane, e0, waves, total_all, sums);
+            router_dots<T>(w, xs, W, lane, e0, waves, outputs, sums);
 #pragma unroll
             for (int j = 0; j < 4; ++j)
-                if (lane == 0 && e0 + j * waves < total_all) logits[e0 + j * waves] = sums[j];
+                if (lane == 0 && e0 + j * waves < outputs) logits[e0 + j * waves] = sums[j];
         }
         __syncthreads();
         row = logits;
@@ -584,7 +626,13 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
         pick[e] = v;
         largest = fmaxf(largest, v);
     }
-    if (!of_chosen) {
+    if (scoring == 2) {
+        for (int e = lane; e < total; e += PL_WAVE) {
+            const float s = 1.f / (1.f + expf(-score[e]));
+            score[e] = s;
+            pick[e] = correction != nullptr ? s + correction[e] : s;
+        }
+    } else if (!of_chosen) {
         largest = wave_max(largest);
         float sum = 0.f;
         for (int e = lane; e < total; e += PL_WAVE) {
@@ -603,9 +651,13 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     if (groups_all > 1) {
         const int size = total_all / groups_all;
         for (int g = lane; g < groups; g += PL_WAVE) {
-            float best = -INFINITY;
-            for (int e = g * size; e < (g + 1) * size; ++e) best = fmaxf(best, pick[e]);
-            group[g] = best;
+            float best = -INFINITY, second = -INFINITY;
+            for (int e = g * size; e < (g + 1) * size; ++e) {
+                const float s = pick[e];
+                second = fmaxf(second, fminf(best, s));
+                best = fmaxf(best, s);
+            }
+            group[g] = group_best == 2 && size > 1 ? best + second : best;
             stays[g] = 0.f;
         }
         __syncthreads();
@@ -655,19 +707,25 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
         __syncthreads();
     }
     if (of_chosen && chooser) {
-        for (int c = lane; c < top; c += PL_WAVE) counts[c] = counts[c] / chosen_sum;
-    } else if (normalised && chooser) {
-        for (int c = lane; c < top; c += PL_WAVE) counts[c] = counts[c] / (chosen_sum + weight_eps);
+        for (int c = lane; c < top; c += PL_WAVE) counts[c] = counts[c] / chosen_sum * scale;
+    } else if (chooser) {
+        for (int c = lane; c < top; c += PL_WAVE) counts[c] = (normalised ? counts[c] / (chosen_sum + weight_eps) : counts[c]) * scale;
+    }
+    if (shared && chooser && lane == 0) {
+        chosen[top] = total_all;
+        counts[top] = 1.f / (1.f + expf(-row[total_all]));
     }
 }
 
 // z [n, stride] holds the logits, or, where it is null, x [n, W] and w [total, W] of type `dtype` give them.
 extern "C" int pl_router_select(const float* z, int stride, const float* correction, const int* positions, int n, int total,
                                 int top, int groups, int kept, int normalised, float weight_eps, int* choice, float* weight,
-                                const void* x, const void* w, int W, int dtype, const float* bias, int of_chosen,
-                                hipStream_t stream) {
-    PL_REQUIRE(!of_chosen || correction == nullptr, "router_select: a correction of scores where the logits themselves choose");
-    PL_REQUIRE(n >= 0 && total > 0 && total <= 8192 && top > 0 && top <= total && (z == nullptr || stride >= total),
+                                const void* x, const void* w, int W, int dtype, const float* bias, int scoring, int group_best,
+                                float scale, int shared, hipStream_t stream) {
+    PL_REQUIRE(scoring >= 0 && scoring <= 2 && (group_best == 1 || group_best == 2) && (shared == 0 || shared == 1),
+               "router_select: scores of kind %d, groups by their best %d, %d shared experts", scoring, group_best, shared);
+    PL_REQUIRE(scoring != 1 || correction == nullptr, "router_select: a correction of scores where the logits themselves choose");
+    PL_REQUIRE(n >= 0 && total > 0 && total <= 8192 && top > 0 && top <= total && (z == nullptr || stride >= total + shared),
                "router_select: %d rows, %d of %d outputs in rows of %d", n, top, total, stride);
     PL_REQUIRE((z != nullptr) != (x != nullptr) && (x == nullptr || (w != nullptr && W > 0 && W <= 8192 && total <= 1024)),
                "router_select: logits, or rows of up to 8192 and a router of up to 1024 outputs to work them out from");
@@ -677,17 +735,17 @@ extern "C" int pl_router_select(const float* z, int stride, const float* correct
     size_t lds = 2 * (static_cast<size_t>(total) + groups) * sizeof(float);
     if (x == nullptr) {
         router_select_kernel<float><<<n, 64, lds, stream>>>(z, stride, correction, positions, total, top, groups, kept, normalised,
-                                                            weight_eps, choice, weight, nullptr, nullptr, 0, bias, of_chosen);
+                                                            weight_eps, choice, weight, nullptr, nullptr, 0, bias, scoring, group_best, scale, shared);
     } else {
-        lds += (static_cast<size_t>(total) + W) * sizeof(float);
+        lds += (static_cast<size_t>(total) + shared + W) * sizeof(float);
         if (dtype == PL_DTYPE_F32)
             router_select_kernel<float><<<n, 256, lds, stream>>>(nullptr, 0, correction, positions, total, top, groups, kept, normalised,
                                                                 weight_eps, choice, weight, static_cast<const float*>(x),
-                                                                static_cast<const float*>(w), W, bias, of_chosen);
+                                                                static_cast<const float*>(w), W, bias, scoring, group_best, scale, shared);
         else if (dtype == PL_DTYPE_BF16)
             router_select_kernel<bf16_t><<<n, 256, lds, stream>>>(nullptr, 0, correction, positions, total, top, groups, kept, normalised,
                                                                  weight_eps, choice, weight, static_cast<const bf16_t*>(x),
-                                                                 static_cast<const bf16_t*>(w), W, bias, of_chosen);
+                                                                 static_cast<const bf16_t*>(w), W, bias, scoring, group_best, scale, shared);
         else
             PL_REQUIRE(false, "router_select: dtype code %d", dtype);
     }

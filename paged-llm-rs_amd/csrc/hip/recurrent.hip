@@ -1,5 +1,5 @@
 // Mixers that carry a matrix of state from token to token instead of keys and values in pages:
-// linear attention with a fixed decay a head, the matrix memory with exponential gates, the gated
+// linear attention with a fixed decay a head (with and without silu on q, k and v), the matrix memory with exponential gates, the gated
 // delta rule, and the state space whose decay and step size a token brings itself (ssd: q, k and v are its
 // C, B and x; S = e^(-e^A_log dt) S + dt k v^T, o = S^T q + D v, dt = softplus(x1 + dt_bias)); the short causal convolution with its carried history; and the norm over groups of the
 // read-out, multiplied by a gate.  States, gates, decays and read-outs are 32-bit whatever the model's
@@ -65,7 +65,7 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
         m = slot_state[a.m_off + h * tiles + blockIdx.x];
     }
     float decay = 0.f, a_rate = 0.f, dt_bias = 0.f, bias_i = 0.f, bias_f = 0.f;
-    if (KIND == PL_SCAN_LIGHTNING) decay = a.p1[h];
+    if (KIND == PL_SCAN_LIGHTNING || KIND == PL_SCAN_RETENTION) decay = a.p1[h];
     if (KIND == PL_SCAN_DELTA || KIND == PL_SCAN_SSD) { a_rate = expf(a.p1[h]); dt_bias = a.p2[h]; }
     const float skip = KIND == PL_SCAN_SSD ? a.p3[h] : 0.f;
     if (KIND == PL_SCAN_MLSTM) { bias_i = a.p1[h]; bias_f = a.p2[h]; }
@@ -95,7 +95,7 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
             if (KIND == PL_SCAN_LIGHTNING) v = silu_f(v);
             vs[t * 64 + lane] = v;
         }
-        if (KIND != PL_SCAN_LIGHTNING && lane < count) {
+        if (KIND != PL_SCAN_LIGHTNING && KIND != PL_SCAN_RETENTION && lane < count) {
             const float* row = a.gates + static_cast<size_t>(start + c0 + lane) * a.gates_stride;
             const float x1 = row[a.g1_off + h], x2 = KIND == PL_SCAN_SSD ? 0.f : row[a.g2_off + h];
             if (KIND == PL_SCAN_SSD) {
@@ -133,7 +133,7 @@ __global__ __launch_bounds__(64) void scan_kernel(ScanArgs a) {
             const float* k = ks + t * Dp;
             const float v = vs[t * 64 + lane];
             float o = 0.f;
-            if (KIND == PL_SCAN_LIGHTNING) {
+            if (KIND == PL_SCAN_LIGHTNING || KIND == PL_SCAN_RETENTION) {
                 PL_ROWS_OF_S {
                         S[i] = decay * S[i] + k[i] * v;
                         o += S[i] * q[i];
@@ -214,14 +214,14 @@ extern "C" int pl_recurrent_scan(int kind, const float* qkv, int qkv_stride, int
                                  float* state, long state_stride, int s_off, int n_off, int m_off,
                                  float* out, const int* q_start, const int* q_len, const int* state_slots,
                                  int seqs, int H, int G, int D, int V, int below, hipStream_t stream) {
-    PL_REQUIRE(kind >= 0 && kind <= PL_SCAN_SSD, "recurrent_scan: kind %d", kind);
+    PL_REQUIRE(kind >= 0 && kind <= PL_SCAN_RETENTION, "recurrent_scan: kind %d", kind);
     PL_REQUIRE(kind != PL_SCAN_SSD || p3 != nullptr, "recurrent_scan: what v counts in its own read-out is missing");
     PL_REQUIRE(H > 0 && G > 0 && H % G == 0, "recurrent_scan: %d heads over %d heads of q and k", H, G);
     PL_REQUIRE(D > 0 && D <= 256 && V > 0, "recurrent_scan: a state of %d by %d a head (q and k up to 256)", D, V);
     PL_REQUIRE(seqs >= 0 && seqs <= 65535 && H <= 65535, "recurrent_scan: %d requests, %d heads", seqs, H);
-    PL_REQUIRE(kind == PL_SCAN_LIGHTNING || (gates != nullptr && p1 != nullptr && p2 != nullptr),
+    PL_REQUIRE(kind == PL_SCAN_LIGHTNING || kind == PL_SCAN_RETENTION || (gates != nullptr && p1 != nullptr && p2 != nullptr),
                "recurrent_scan: the gates of kind %d are missing", kind);
-    PL_REQUIRE(kind != PL_SCAN_LIGHTNING || p1 != nullptr, "recurrent_scan: the decays are missing");
+    PL_REQUIRE(p1 != nullptr, "recurrent_scan: the decays are missing");
     PL_REQUIRE(kind != PL_SCAN_MLSTM || cap > 0.f, "recurrent_scan: a gate cap of %g", cap);
     if (seqs == 0) return 0;
     ScanArgs a{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g1_off, g2_off, p1, p2, p3, cap,
@@ -229,6 +229,7 @@ extern "C" int pl_recurrent_scan(int kind, const float* qkv, int qkv_stride, int
     if (kind == PL_SCAN_LIGHTNING) return launch_scan<PL_SCAN_LIGHTNING>(a, seqs, stream);
     if (kind == PL_SCAN_MLSTM) return launch_scan<PL_SCAN_MLSTM>(a, seqs, stream);
     if (kind == PL_SCAN_SSD) return launch_scan<PL_SCAN_SSD>(a, seqs, stream);
+    if (kind == PL_SCAN_RETENTION) return launch_scan<PL_SCAN_RETENTION>(a, seqs, stream);
     return launch_scan<PL_SCAN_DELTA>(a, seqs, stream);
 }
 
@@ -416,7 +417,7 @@ extern "C" int pl_conv_history(const float* rows, int stride, int off, int C, in
 
 // ---------------------------------------------------------------------------
 // out[t, c] = x[t, c] / sqrt(mean over c's group of x^2 + eps) * gain[c mod gain_len] * act(gate[t, c])
-// Groups are runs of `group` columns (a head, or the whole row).  One wave a row and group.
+// (gain null: ones.)  Groups are runs of `group` columns (a head, or the whole row).  One wave a row and group.
 // act: 0 sigmoid, 1 silu, -1 no gate.  FIRST: the gate multiplies x before the statistic is taken, and not the result:
 //   u = x * act(gate);  out = u / sqrt(mean over the group of u^2 + eps) * gain
 // ---------------------------------------------------------------------------
@@ -454,13 +455,15 @@ __global__ __launch_bounds__(64) void gated_group_norm_kernel(const float* __res
     for (int k = 0; k < KEEP; ++k) {
         const int e = threadIdx.x + 64 * k;
         if (e < group) {
-            float y = kept[k] * inv * gain[(first + e) % gain_len];
+            float y = kept[k] * inv;
+            if (gain != nullptr) y *= gain[(first + e) % gain_len];
             if (!FIRST && act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
             o[e] = from_float<T>(y);
         }
     }
     for (int e = threadIdx.x + 64 * KEEP; e < group; e += 64) {
-        float y = value(e) * inv * gain[(first + e) % gain_len];
+        float y = value(e) * inv;
+        if (gain != nullptr) y *= gain[(first + e) % gain_len];
         if (!FIRST && act >= 0) y *= act == 0 ? sigmoid_f(g[e]) : silu_f(g[e]);
         o[e] = from_float<T>(y);
     }
@@ -477,7 +480,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
     const int t = blockIdx.x, first = blockIdx.y * group;
     const float* row = x + static_cast<size_t>(t) * width + first;
     const float* g = gate != nullptr ? gate + static_cast<size_t>(t) * gate_stride + gate_off + first : nullptr;
-    const float* gains = gain + (gain_len == width ? first : 0);     // (gain_len is the row's width or the group's)
+    const float* gains = gain != nullptr ? gain + (gain_len == width ? first : 0) : nullptr;     // (gain_len is the row's width or the group's)
     auto opened = [&](float gv) { return act == 0 ? sigmoid_f(gv) : silu_f(gv); };
     constexpr int KEEP = 8;
     float kept[KEEP], gates[KEEP], scale[KEEP];
@@ -487,7 +490,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
         const int e = threadIdx.x + 256 * k;
         kept[k] = e < group ? row[e] : 0.f;
         gates[k] = (e < group && act >= 0) ? g[e] : 0.f;
-        scale[k] = e < group ? gains[e] : 0.f;
+        scale[k] = e < group ? (gains != nullptr ? gains[e] : 1.f) : 0.f;
         if (FIRST && act >= 0) kept[k] *= opened(gates[k]);
         ss += kept[k] * kept[k];
     }
@@ -508,7 +511,8 @@ __global__ __launch_bounds__(256) void gated_group_norm_wide_kernel(const float*
         }
     }
     for (int e = threadIdx.x + 256 * KEEP; e < group; e += 256) {
-        float y = row[e] * inv * gains[e];
+        float y = row[e] * inv;
+        if (gains != nullptr) y *= gains[e];
         if (act >= 0) y *= opened(g[e]);
         o[e] = from_float<T>(y);
     }

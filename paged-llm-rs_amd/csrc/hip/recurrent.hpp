@@ -8,13 +8,14 @@
 #define PL_SCAN_MLSTM 1
 #define PL_SCAN_DELTA 2
 #define PL_SCAN_SSD 3
+#define PL_SCAN_RETENTION 4
 
 struct ScanArgs {
     const float* qkv;         // rows holding q, k and v (for the delta rule: already convolved and activated)
     int qkv_stride, q_off, k_off, v_off;
     const float* gates;       // rows holding the two pre-activations of the gates (mlstm: i, f; delta: beta, a); ssd: the step size's, from g1_off
     int gates_stride, g1_off, g2_off;
-    const float* p1;          // lightning: decay a head; mlstm: bias of i; delta, ssd: A_log
+    const float* p1;          // lightning, retention: decay a head; mlstm: bias of i; delta, ssd: A_log
     const float* p2;          // mlstm: bias of f; delta, ssd: dt_bias
     const float* p3;          // ssd: what a head's v counts in its own read-out
     float cap;                // mlstm: the cap of the gates' pre-activations

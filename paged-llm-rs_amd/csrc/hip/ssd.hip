@@ -3,6 +3,11 @@
 //     S_t = e^(-a dt_t) S_(t-1) + dt_t B_t x_t^T   (N x V),     y_t = S_t^T C_t + D x_t .
 // q, k and v of the scan's arguments are C, B and x; C and B have G heads, head h reads head h / (H / G).
 //
+// Linear attention with a fixed decay a head (kind retention) is the same recurrence with e^(-a dt) = decay, dt = 1 in front of
+// B x^T and no D: the chunked kernels serve it as FIXED instances (p1 holds the decays), retention_step is its kernel for few tokens.
+// Its q and k turn with their positions: retention_turn does that to a step's rows in front of the chunked kernels,
+// retention_step to what it reads.
+//
 // ssd_step: requests of few tokens, token by token, the state read and written once, 16 bytes a lane.
 //
 // ssd_chunked: requests of many tokens in chunks of 64.  With b_t the sum of -a dt over a chunk's tokens up to t,
@@ -117,6 +122,137 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(ScanArgs a) {
         if (owns && n0 + i < N) *reinterpret_cast<ssd_f32x4*>(Sg + static_cast<size_t>(n0 + i) * V + v0) = S[i];
 }
 
+// How q and k of a head turn: values i and i + dims / 2 by position * freq[i], cosine and sine times `amplitude`, i < dims / 2;
+// k times `k_scale` behind that.
+struct HalfTurn {
+    const float* freq;
+    const int* positions;
+    int dims;
+    float amplitude, k_scale;
+};
+
+// Pair i of q and k (values i and i + dims / 2), turned.
+struct TurnedPair {
+    float q0, q1, k0, k1;
+};
+__device__ __forceinline__ TurnedPair turn_pair(const float* q, const float* k, int i, int half, float cs, float sn, float k_scale) {
+    const float q0 = q[i], q1 = q[i + half], k0 = k[i], k1 = k[i + half];
+    return {q0 * cs - q1 * sn, q1 * cs + q0 * sn, (k0 * cs - k1 * sn) * k_scale, (k1 * cs + k0 * sn) * k_scale};
+}
+__device__ __forceinline__ void half_angle(const HalfTurn& turn, int position, int i, float& cs, float& sn) {
+    sincosf(static_cast<float>(position) * turn.freq[i], &sn, &cs);
+    cs *= turn.amplitude;
+    sn *= turn.amplitude;
+}
+
+// As ssd_step_kernel, a workgroup 64 columns of a head's state for one request; every token's q and k are turned into LDS first
+// (`turns`: they have not been turned yet).
+template <int R>
+__global__ __launch_bounds__(256) void retention_step_kernel(ScanArgs a, HalfTurn turn, int turns) {
+    __shared__ ssd_f32x4 part[4][16];
+    __shared__ __attribute__((aligned(16))) float qs[16 * R], ks[16 * R];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int h = blockIdx.y, s = blockIdx.z;
+    const int slot = a.state_slots[s];
+    const int count = a.q_len[s];
+    if (slot < 0 || count <= 0 || (a.below > 0 && count >= a.below)) return;
+    const int start = a.q_start[s];
+    const int N = a.D, V = a.V, H = a.H;
+    const int n0 = (4 * wave + (lane >> 4)) * R;
+    const int v0 = blockIdx.x * 64 + 4 * (lane & 15);
+    const bool owns = v0 < V;                                   // (V is a multiple of 4)
+    float* Sg = a.state + static_cast<size_t>(slot) * a.state_stride + a.s_off + static_cast<size_t>(h) * N * V;
+    ssd_f32x4 S[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i)
+        S[i] = (owns && n0 + i < N) ? *reinterpret_cast<const ssd_f32x4*>(Sg + static_cast<size_t>(n0 + i) * V + v0) : ssd_f32x4{0.f, 0.f, 0.f, 0.f};
+    const float keep = a.p1[h];
+    const int half = turns ? turn.dims / 2 : 0;
+    const float k_scale = turns ? turn.k_scale : 1.f;
+    for (int i = N + tid; i < 16 * R; i += 256) qs[i] = ks[i] = 0.f;
+    for (int t = 0; t < count; ++t) {
+        const float* row = a.qkv + static_cast<size_t>(start + t) * a.qkv_stride;
+        const float* kr = row + a.k_off + h * N;
+        const float* qr = row + a.q_off + h * N;
+        ssd_f32x4 v = {0.f, 0.f, 0.f, 0.f};
+        if (owns) {
+            const float* vr = row + a.v_off + h * V + v0;
+            v = ssd_f32x4{vr[0], vr[1], vr[2], vr[3]};
+        }
+        if (tid < half) {
+            float cs, sn;
+            half_angle(turn, turn.positions[start + t], tid, cs, sn);
+            const TurnedPair p = turn_pair(qr, kr, tid, half, cs, sn, k_scale);
+            qs[tid] = p.q0;
+            qs[tid + half] = p.q1;
+            ks[tid] = p.k0;
+            ks[tid + half] = p.k1;
+        } else if (tid + half < N) {
+            qs[tid + half] = qr[tid + half];
+            ks[tid + half] = kr[tid + half] * k_scale;
+        }
+        __syncthreads();
+        float k[R], q[R];
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+            k[i] = ks[n0 + i];
+            q[i] = qs[n0 + i];
+        }
+        ssd_f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < R; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                S[i][e] = keep * S[i][e] + k[i] * v[e];
+                o[e] += S[i][e] * q[i];
+            }
+#pragma unroll
+        for (int off = 16; off < 64; off <<= 1)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] += __shfl_xor(o[e], off, 64);
+        if (lane < 16) part[wave][lane] = o;
+        __syncthreads();
+        if (wave == 0 && lane < 16 && owns) {
+            ssd_f32x4 y = part[0][lane];
+#pragma unroll
+            for (int w = 1; w < 4; ++w)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[e] += part[w][lane][e];
+            *reinterpret_cast<ssd_f32x4*>(a.out + static_cast<size_t>(start + t) * (H * V) + h * V + v0) = y;
+        }
+        // (nobody writes `part` again before the next token's first barrier, which the first wave reaches behind its reads)
+    }
+#pragma unroll
+    for (int i = 0; i < R; ++i)
+        if (owns && n0 + i < N) *reinterpret_cast<ssd_f32x4*>(Sg + static_cast<size_t>(n0 + i) * V + v0) = S[i];
+}
+
+// A workgroup a token: q and k of every head, turned in place.
+__global__ __launch_bounds__(256) void retention_turn_kernel(float* __restrict__ rows, int stride, int q_off, int k_off, int H, int N, HalfTurn turn) {
+    __shared__ float cosine[128], sine[128];
+    const int t = blockIdx.x;
+    const int position = turn.positions[t];
+    if (position < 0) return;
+    const int half = turn.dims / 2, each = N - half;             // pairs, then the values that do not turn
+    for (int i = threadIdx.x; i < half; i += 256) half_angle(turn, position, i, cosine[i], sine[i]);
+    __syncthreads();
+    float* row = rows + static_cast<size_t>(t) * stride;
+    for (int e = threadIdx.x; e < H * each; e += 256) {
+        const int h = e / each, i = e - h * each;
+        float* q = row + q_off + h * N;
+        float* k = row + k_off + h * N;
+        if (i < half) {
+            const TurnedPair p = turn_pair(q, k, i, half, cosine[i], sine[i], turn.k_scale);
+            q[i] = p.q0;
+            q[i + half] = p.q1;
+            k[i] = p.k0;
+            k[i + half] = p.k1;
+        } else {
+            k[i + half] *= turn.k_scale;
+        }
+    }
+}
+
 // ---- many tokens -----------------------------------------------------------------------------------------
 
 struct SsdArgs {
@@ -132,8 +268,15 @@ __device__ __forceinline__ int ssd_chunk(const ScanArgs& a, int s, int c) { retu
 
 // By one wave, all its lanes: the running sums b (64-bit) and the step sizes of a chunk's L <= 64 tokens; the sum
 // over the chunk comes back.  Lanes past the chunk hold the last sum and a step of zero.
+template <bool FIXED>
 __device__ __forceinline__ double ssd_gates(const ScanArgs& a, int h, int row0, int L, int lane, double& b, float& dt) {
     dt = 0.f;
+    if (FIXED) {
+        const double each = log(static_cast<double>(a.p1[h]));
+        if (lane < L) dt = 1.f;
+        b = each * (min(lane, L - 1) + 1);
+        return each * L;
+    }
     if (lane < L) dt = softplus_f(a.gates[static_cast<size_t>(row0 + lane) * a.gates_stride + a.g1_off + h] + a.p2[h]);
     double sum = -static_cast<double>(expf(a.p1[h])) * static_cast<double>(dt);
 #pragma unroll
@@ -145,8 +288,11 @@ __device__ __forceinline__ double ssd_gates(const ScanArgs& a, int h, int row0, 
     return __shfl(sum, L - 1, 64);
 }
 
+// (FIXED: one decay a head, p1, and steps of one.)
+
 // summary: a wave a tile of 32 rows of N (and the tile four further on, where N has more than 128), 64 columns of V.
 // Both operands come straight from memory, a token a row: 128 bytes a half wave.
+template <bool FIXED>
 __global__ __launch_bounds__(256) void ssd_summary_kernel(SsdArgs sa) {
     const ScanArgs& a = sa.a;
     __shared__ float weight[SSD_CHUNK];
@@ -173,7 +319,7 @@ __global__ __launch_bounds__(256) void ssd_summary_kernel(SsdArgs sa) {
     if (wave == 0) {
         double b;
         float dt;
-        const double end = ssd_gates(a, h, row0, L, lane, b, dt);
+        const double end = ssd_gates<FIXED>(a, h, row0, L, lane, b, dt);
         weight[lane] = expf(static_cast<float>(end - b)) * dt;          // (zero past the chunk's tokens)
         if (vt == 0 && lane == 0) sa.ends[idx] = static_cast<float>(end);
     }
@@ -250,6 +396,7 @@ __global__ __launch_bounds__(256) void ssd_carry_kernel(SsdArgs sa) {
 // output: the read-outs of one chunk, head and tile of 64 columns.  Four waves; wave 2 ti + j owns the tokens 32 ti .. + 31 and, of the
 // scores, the earlier tokens 32 j .. + 31, of the read-outs, the columns 32 j .. + 31.
 // LDS: C [64][P], B [64][P] (behind the scores' barrier the weighted scores [64][68] lie in its place), b, step sizes.
+template <bool FIXED>
 __global__ __launch_bounds__(256, 2) void ssd_output_kernel(SsdArgs sa, int aligned) {
     const ScanArgs& a = sa.a;
     extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -320,7 +467,7 @@ __global__ __launch_bounds__(256, 2) void ssd_output_kernel(SsdArgs sa, int alig
     if (wave == 0) {
         double b;
         float dt;
-        ssd_gates(a, h, row0, L, lane, b, dt);
+        ssd_gates<FIXED>(a, h, row0, L, lane, b, dt);
         bd[lane] = b;
         dts[lane] = dt;
     }
@@ -390,13 +537,13 @@ __global__ __launch_bounds__(256, 2) void ssd_output_kernel(SsdArgs sa, int alig
             }
         }
     }
-    const float skip = a.p3[h];
+    const float skip = FIXED ? 0.f : a.p3[h];
     float* out = a.out + static_cast<size_t>(row0) * (H * V) + h * V;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
         const int t = 32 * ti + 8 * (r >> 2) + 4 * half + (r & 3);
         // (token t's own x is the one this lane holds in the same place of its half of the chunk)
-        if (t < L && v < V) out[static_cast<size_t>(t) * (H * V) + v] = y[r] + skip * (ti == 0 ? x[r] : x[16 + r]);
+        if (t < L && v < V) out[static_cast<size_t>(t) * (H * V) + v] = FIXED ? y[r] : y[r] + skip * (ti == 0 ? x[r] : x[16 + r]);
     }
 }
 
@@ -436,6 +583,26 @@ extern "C" int pl_ssd_step(const float* qkv, int qkv_stride, int q_off, int k_of
     return 0;
 }
 
+template <bool FIXED>
+static int launch_chunks(const SsdArgs& sa, int seqs, int max_q_len, hipStream_t stream) {
+    const ScanArgs& a = sa.a;
+    const int N = a.D, V = a.V, tiles = pl_ceil_div(V, 64);
+    const dim3 grid(pl_ceil_div(max_q_len, SSD_CHUNK), a.H * tiles, seqs);
+    ssd_summary_kernel<FIXED><<<grid, 256, 0, stream>>>(sa);
+    PL_CHECK_LAUNCH("ssd_chunked (summary)");
+    ssd_carry_kernel<<<dim3(pl_ceil_div(N * V, 256), a.H, seqs), 256, 0, stream>>>(sa);
+    PL_CHECK_LAUNCH("ssd_chunked (carry)");
+    const int P = ((N + 7) & ~7) + 4;
+    const size_t lds = (3 * SSD_CHUNK + SSD_CHUNK * static_cast<size_t>(P) + SSD_CHUNK * static_cast<size_t>(P > SSD_CHUNK + 4 ? P : SSD_CHUNK + 4)) * sizeof(float);
+    if (lds > 48 * 1024) {
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&ssd_output_kernel<FIXED>), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds));
+        PL_REQUIRE(e == hipSuccess, "ssd_chunked: %zu bytes of LDS refused: %s", lds, hipGetErrorString(e));
+    }
+    ssd_output_kernel<FIXED><<<grid, 256, lds, stream>>>(sa, ssd_aligned(a) ? 1 : 0);
+    PL_CHECK_LAUNCH("ssd_chunked (output)");
+    return 0;
+}
+
 // The requests that bring at least `from` tokens, in chunks of 64.  U, Sin: room for (rows / 64 + requests + 1) chunks of
 // H * N * V floats; ends: of H.
 extern "C" int pl_ssd_chunked(const float* qkv, int qkv_stride, int q_off, int k_off, int v_off, const float* gates, int gates_stride,
@@ -450,18 +617,55 @@ extern "C" int pl_ssd_chunked(const float* qkv, int qkv_stride, int q_off, int k
     if (seqs == 0 || max_q_len < from) return 0;
     const SsdArgs sa{{qkv, qkv_stride, q_off, k_off, v_off, gates, gates_stride, g_off, 0, a_log, dt_bias, skip, 0.f, state, state_stride,
                       0, 0, 0, out, q_start, q_len, state_slots, H, G, N, V, from}, U, Sin, ends};
-    const dim3 grid(pl_ceil_div(max_q_len, SSD_CHUNK), H * tiles, seqs);
-    ssd_summary_kernel<<<grid, 256, 0, stream>>>(sa);
-    PL_CHECK_LAUNCH("ssd_chunked (summary)");
-    ssd_carry_kernel<<<dim3(pl_ceil_div(N * V, 256), H, seqs), 256, 0, stream>>>(sa);
-    PL_CHECK_LAUNCH("ssd_chunked (carry)");
-    const int P = ((N + 7) & ~7) + 4;
-    const size_t lds = (3 * SSD_CHUNK + SSD_CHUNK * static_cast<size_t>(P) + SSD_CHUNK * static_cast<size_t>(P > SSD_CHUNK + 4 ? P : SSD_CHUNK + 4)) * sizeof(float);
-    if (lds > 48 * 1024) {
-        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&ssd_output_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds));
-        PL_REQUIRE(e == hipSuccess, "ssd_chunked: %zu bytes of LDS refused: %s", lds, hipGetErrorString(e));
-    }
-    ssd_output_kernel<<<grid, 256, lds, stream>>>(sa, ssd_aligned(sa.a) ? 1 : 0);
-    PL_CHECK_LAUNCH("ssd_chunked (output)");
+    return launch_chunks<false>(sa, seqs, max_q_len, stream);
+}
+
+// Retention: S = decay S + k v^T, o = S^T q, q and k turning with their positions (HalfTurn; freq null: not at all).
+// The rows of q and k in `rows` turn in place.
+extern "C" int pl_retention_turn(float* rows, int stride, int q_off, int k_off, int n, int H, int N, const float* freq, int dims,
+                                 float amplitude, float k_scale, const int* positions, hipStream_t stream) {
+    PL_REQUIRE(n >= 0 && H > 0 && N > 0 && N <= 256 && dims >= 0 && dims % 2 == 0 && dims <= N && (dims == 0 || freq != nullptr) && positions != nullptr,
+               "retention_turn: %d heads of %d values, %d of which turn", H, N, dims);
+    PL_REQUIRE(q_off >= 0 && k_off >= 0 && q_off + H * N <= stride && k_off + H * N <= stride, "retention_turn: q and k at %d and %d of rows of %d", q_off, k_off, stride);
+    if (n == 0) return 0;
+    retention_turn_kernel<<<n, 256, 0, stream>>>(rows, stride, q_off, k_off, H, N, HalfTurn{freq, positions, dims, amplitude, k_scale});
+    PL_CHECK_LAUNCH("retention_turn");
     return 0;
+}
+
+// The requests that bring fewer than `below` tokens (0: all), token by token.  turns: q and k of these rows have not been turned.
+extern "C" int pl_retention_step(const float* qkv, int qkv_stride, int q_off, int k_off, int v_off, const float* decay, const float* freq,
+                                 int dims, float amplitude, float k_scale, int turns, const int* positions, float* state, long state_stride,
+                                 float* out, const int* q_start, const int* q_len, const int* state_slots, int seqs, int H, int N, int V,
+                                 int below, hipStream_t stream) {
+    PL_REQUIRE(H > 0 && H <= 65535 && seqs >= 0 && seqs <= 65535, "retention_step: %d heads, %d requests", H, seqs);
+    PL_REQUIRE(N > 0 && N <= 256 && V > 0 && pl_ssd_step_applies(V, state_stride) && reinterpret_cast<uintptr_t>(state) % 16 == 0 &&
+               reinterpret_cast<uintptr_t>(out) % 16 == 0, "retention_step: a state of %d by %d a head, slots of %ld floats", N, V, state_stride);
+    PL_REQUIRE(decay != nullptr && positions != nullptr && dims >= 0 && dims % 2 == 0 && dims <= N && (dims == 0 || freq != nullptr),
+               "retention_step: %d of %d values turn", dims, N);
+    if (seqs == 0) return 0;
+    const ScanArgs a{qkv, qkv_stride, q_off, k_off, v_off, nullptr, 0, 0, 0, decay, nullptr, nullptr, 0.f, state, state_stride,
+                     0, 0, 0, out, q_start, q_len, state_slots, H, H, N, V, below};
+    const HalfTurn turn{freq, positions, dims, amplitude, k_scale};
+    const dim3 grid(pl_ceil_div(V, 64), H, seqs);
+    if (N <= 16) retention_step_kernel<1><<<grid, 256, 0, stream>>>(a, turn, turns);
+    else if (N <= 32) retention_step_kernel<2><<<grid, 256, 0, stream>>>(a, turn, turns);
+    else if (N <= 64) retention_step_kernel<4><<<grid, 256, 0, stream>>>(a, turn, turns);
+    else if (N <= 128) retention_step_kernel<8><<<grid, 256, 0, stream>>>(a, turn, turns);
+    else retention_step_kernel<16><<<grid, 256, 0, stream>>>(a, turn, turns);
+    PL_CHECK_LAUNCH("retention_step");
+    return 0;
+}
+
+// The requests that bring at least `from` tokens, in chunks of 64, q and k turned already; decays above zero.  Room as in pl_ssd_chunked.
+extern "C" int pl_retention_chunked(const float* qkv, int qkv_stride, int q_off, int k_off, int v_off, const float* decay, float* state,
+                                    long state_stride, float* out, const int* q_start, const int* q_len, const int* state_slots, int seqs,
+                                    int max_q_len, int H, int N, int V, int from, float* U, float* Sin, float* ends, hipStream_t stream) {
+    PL_REQUIRE(H > 0 && N > 0 && N <= 256 && V > 0 && from >= 1, "retention_chunked: %d heads of %d by %d, from %d tokens", H, N, V, from);
+    PL_REQUIRE(decay != nullptr && U != nullptr && Sin != nullptr && ends != nullptr, "retention_chunked: the decays or room for the chunks' sums are missing");
+    PL_REQUIRE(static_cast<long long>(H) * pl_ceil_div(V, 64) <= 65535 && seqs >= 0 && seqs <= 65535, "retention_chunked: %d heads of %d columns, %d requests", H, V, seqs);
+    if (seqs == 0 || max_q_len < from) return 0;
+    const SsdArgs sa{{qkv, qkv_stride, q_off, k_off, v_off, nullptr, 0, 0, 0, decay, nullptr, nullptr, 0.f, state, state_stride,
+                      0, 0, 0, out, q_start, q_len, state_slots, H, H, N, V, from}, U, Sin, ends};
+    return launch_chunks<true>(sa, seqs, max_q_len, stream);
 }

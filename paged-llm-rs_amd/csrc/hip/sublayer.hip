@@ -121,8 +121,8 @@ extern "C" int pl_weighted_sum(float* x, float a, const float* y, float b, long 
 // ---- a layer whose sublayers stand side by side -----------------------------------------------------------
 //
 // One pass over a row of the 32-bit stream, either half optional.  First the sums that are due,
-//   x <- x + ls1 * a + ls2 * b + more
-// (a, b: what the two sublayers of the layer before gave, 32-bit; ls1, ls2: a gain a column, or null for one; more: rows
+//   x <- x + mult * (ls1 * a + ls2 * b) + more
+// (a, b: what the two sublayers of the layer before gave, 32-bit; ls1, ls2: a gain a column, or null for one; mult: one number; more: rows
 // added as they are, e.g. what the model began with, before a stretch of layers runs again), written back to the stream.
 // Then the norms that read the updated row: out1 = x / sqrt(mean(x^2) + eps) * gain1 and out2 likewise with gain2,
 // rounded once into the model's type.  `rows` (with no sums due) names the rows to read.
@@ -140,6 +140,7 @@ struct ParallelStepArgs {
     void* out2;
     const int* rows;
     int W;
+    float mult;
 };
 
 template <int PER>
@@ -199,10 +200,10 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
             if (p.ls1 != nullptr) {
                 const Run<PER> g = load_run<PER>(p.ls1 + c);
 #pragma unroll
-                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * g.v[j];
+                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * g.v[j] * p.mult;
             } else {
 #pragma unroll
-                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j];
+                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * p.mult;
             }
         }
         if (p.b != nullptr) {
@@ -210,10 +211,10 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
             if (p.ls2 != nullptr) {
                 const Run<PER> g = load_run<PER>(p.ls2 + c);
 #pragma unroll
-                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * g.v[j];
+                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * g.v[j] * p.mult;
             } else {
 #pragma unroll
-                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j];
+                for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * p.mult;
             }
         }
         if (p.more != nullptr) {
@@ -249,14 +250,14 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
 
 extern "C" int pl_parallel_step(float* resid, const float* a, const float* ls1, const float* b, const float* ls2,
                                 const float* more, const float* gain1, const float* gain2, float eps, void* out1, void* out2,
-                                int dtype, const int* rows, int n, int W, hipStream_t stream) {
+                                int dtype, const int* rows, int n, int W, float mult, hipStream_t stream) {
     PL_REQUIRE(n >= 0 && W > 0, "parallel_step: rows %d, width %d", n, W);
     PL_REQUIRE(rows == nullptr || (a == nullptr && b == nullptr && more == nullptr), "parallel_step: a list of rows and sums into the stream");
     PL_REQUIRE((gain1 != nullptr || gain2 == nullptr) && (gain1 == nullptr || out1 != nullptr) && (gain2 == nullptr || out2 != nullptr),
                "parallel_step: a second norm without a first, or a norm without room for its rows");
     PL_REQUIRE(dtype == PL_DTYPE_F32 || dtype == PL_DTYPE_BF16, "parallel_step: dtype code %d", dtype);
     if (n == 0) return 0;
-    ParallelStepArgs p{resid, a, ls1, b, ls2, more, gain1, gain2, eps, out1, out2, rows, W};
+    ParallelStepArgs p{resid, a, ls1, b, ls2, more, gain1, gain2, eps, out1, out2, rows, W, mult};
     if (W % 4 == 0) {
         int threads = ((W / 4 + 63) / 64) * 64;
         threads = threads > 1024 ? 1024 : threads;

@@ -39,7 +39,8 @@ def _signatures(lib) -> None:
         "pl_gemm_heads": [p, p, p, i, i, i, i, i, ctypes.c_long, i, ctypes.c_long, i, i, p],
         "pl_head_prepare": [p, p, i, i, i, f, p, p, p, p, i, i, i, i, f, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, i,
                             p, i, p, f, p],
-        "pl_latent_prepare": [p, i, i, i, p, f, p, p, i, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, i, p],
+        "pl_latent_prepare": [p, i, i, p, i, i, p, f, p, p, f, i, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, i, p],
+        "pl_rows_norm": [p, i, i, p, i, f, p, i, i, p],
         "pl_head_gate": [p, i, p, i, i, p, i, i, i, i, p],
         "pl_add_position_rows": [p, p, i, p, i, i, i, p],
         "pl_paged_attention_prefill_tile": [i, i],
@@ -66,6 +67,9 @@ def _signatures(lib) -> None:
         "pl_ssd_step": [p, i, i, i, i, p, i, i, p, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, p],
         "pl_ssd_step_applies": [i, ctypes.c_long],
         "pl_ssd_chunked": [p, i, i, i, i, p, i, i, p, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, i, p, p, p, p],
+        "pl_retention_turn": [p, i, i, i, i, i, i, p, i, f, f, p, p],
+        "pl_retention_step": [p, i, i, i, i, p, p, i, f, f, i, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, p],
+        "pl_retention_chunked": [p, i, i, i, i, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, p, p, p, p],
         "pl_recurrent_chunk_tokens": [i],
         "pl_delta_chunked": [p, i, i, i, i, p, i, i, i, p, p, p, ctypes.c_long, p, p, p, p, i, i, i, i, i, i, i,
                              p, p, p, p, p, p],
@@ -82,13 +86,13 @@ def _signatures(lib) -> None:
         "pl_hc_step": [p, p, p, p, p, p, f, p, i, p, i, i, i, p],
         "pl_stream_copies": [p, p, i, i, i, p],
         "pl_softcap": [p, f, ctypes.c_long, p],
-        "pl_moe_rows": [p, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, p, p, i, f, p],
-        "pl_moe_sort": [p, p, p, p, p, p, i, i, i, i, i, i, p, p, p, p],
+        "pl_moe_rows": [p, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, p, p, i, f, i, i, p, p, p],
+        "pl_moe_sort": [p, p, p, p, p, p, i, i, i, i, i, i, i, p, p, p, p],
         "pl_moe_combine": [p, p, p, i, i, i, i, ctypes.c_longlong, p, p, p, i, i, p, p],
-        "pl_router_select": [p, i, p, p, i, i, i, i, i, i, f, p, p, p, p, i, i, p, i, p],
+        "pl_router_select": [p, i, p, p, i, i, i, i, i, i, f, p, p, p, p, i, i, p, i, i, f, i, p],
         "pl_wide_prepare": [p, p, i, i, i, f, p, p, p, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, p],
-        "pl_parallel_step": [p, p, p, p, p, p, p, p, f, p, p, i, p, i, i, p],
-        "pl_gemm_tiled_grouped": [p, p, p, p, p, ctypes.c_longlong, i, i, i, i, i, i, i, f, p],
+        "pl_parallel_step": [p, p, p, p, p, p, p, p, f, p, p, i, p, i, i, f, p],
+        "pl_gemm_tiled_grouped": [p, p, p, p, p, ctypes.c_longlong, i, i, i, i, i, i, i, f, i, i, i, p, i, i, p],
         "pl_sandwich_step": [p, p, p, p, f, p, p, f, p, i, p, i, i, i, p],
         "pl_bigram_add": [p, p, p, p, p, p, p, p, p, p, p, i, ctypes.c_longlong, ctypes.c_longlong, ctypes.c_longlong, i, i, p],
     }
@@ -1150,7 +1154,7 @@ def linear_bf16(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype,
 # ---------------------------------------------------------------------------
 # Mixers with a carried state, short convolutions, and the layer that normalises a sublayer's output
 
-SCAN_KINDS = {"lightning": 0, "mlstm": 1, "delta": 2, "ssd": 3}
+SCAN_KINDS = {"lightning": 0, "mlstm": 1, "delta": 2, "ssd": 3, "retention": 4}
 SCAN_MAX_DIM = 256
 # A request that brings at least this many tokens to a step goes through the chunked kernels, where its mixer has
 # them (64 tokens at once instead of one after the other); the others, single tokens among them, go token by token.
@@ -1297,6 +1301,65 @@ def _ssd_scan(qkv, q_off: int, k_off: int, v_off: int, state, stride: int, batch
     return out
 
 
+def retention_scan(rows: torch.Tensor, q_off: int, k_off: int, v_off: int, state: torch.Tensor, batch, heads: int, dim: int,
+                   vdim: int, decay: torch.Tensor, freq: torch.Tensor | None, amplitude: float, k_scale: float,
+                   chunked: bool = True) -> torch.Tensor:
+    """The read-out [rows, heads * vdim] (32-bit) of linear attention with a fixed decay a head, S = decay S + k v^T, o = S^T q, over
+    the tokens of a step from and into the requests' state slots.  ``rows`` (32-bit) hold q, k [heads, dim] and v [heads, vdim] from
+    their columns on; of every head of q and k the values i and i + len(freq) turn by position * ``freq``[i] (None: nothing turns),
+    cosine and sine times ``amplitude``, and k is multiplied by ``k_scale``.  q and k may be turned in place: the rows are
+    nobody else's.  ``chunked`` (decays above zero): requests of ``SCAN_CHUNKED_FROM`` tokens or more in chunks on the matrix
+    cores (32-bit operands and sums), the same sums in another order."""
+    n = rows.shape[0]
+    _need(rows, "rows of q, k and v", None, torch.float32)
+    width = rows.shape[1] if rows.dim() == 2 else -1
+    if not (0 <= q_off and q_off + heads * dim <= width and 0 <= k_off and k_off + heads * dim <= width
+            and 0 <= v_off and v_off + heads * vdim <= width):
+        raise TensorError(f"q, k, v at columns {q_off}, {k_off}, {v_off} of rows of shape {tuple(rows.shape)}")
+    if heads < 1 or not 1 <= dim <= SCAN_MAX_DIM or vdim < 1:
+        raise TensorError(f"a scan over {heads} heads of {dim} by {vdim}")
+    state, stride = _state_view(state, "the state")
+    if state.shape[1] != heads * dim * vdim:
+        raise TensorError(f"a state of {state.shape[1]} floats a slot, this mixer keeps {heads * dim * vdim}")
+    _step_rows(batch, n)
+    _need(decay, "decays", (heads,), torch.float32)
+    turned = 0
+    if freq is not None:
+        turned = 2 * freq.numel()
+        _need(freq, "rotation frequencies", (turned // 2,), torch.float32)
+        if turned > dim:
+            raise TensorError(f"a rotation over {turned} of {dim} values")
+    out = torch.empty((n, heads * vdim), dtype=torch.float32, device=rows.device)
+    if n == 0:
+        return out
+    lib, stream = library(), _stream()
+    chunked = bool(chunked) and batch.max_q_len >= SCAN_CHUNKED_FROM
+    by_token = not chunked or batch.tokens_of_short_requests(SCAN_CHUNKED_FROM) > 0
+    steps = lib.pl_ssd_step_applies(vdim, stride) and state.data_ptr() % 16 == 0
+    turn = (_ptr(freq), turned, float(amplitude), float(k_scale))
+    at = (rows.data_ptr(), width, q_off, k_off, v_off)
+    step = (batch.q_start.data_ptr(), batch.q_len.data_ptr(), batch.state_slots.data_ptr(), batch.num_seqs)
+    below = SCAN_CHUNKED_FROM if chunked else 0
+    # (a step of few tokens a request alone is turned by the kernel that walks them)
+    before = chunked or not steps
+    if before and (turned or k_scale != 1.0):
+        _check(lib.pl_retention_turn(rows.data_ptr(), width, q_off, k_off, n, heads, dim, *turn, batch.positions.data_ptr(), stream))
+    if by_token and steps:
+        _check(lib.pl_retention_step(*at, decay.data_ptr(), *turn, 0 if before else 1, batch.positions.data_ptr(), state.data_ptr(),
+                                     stride, out.data_ptr(), *step, heads, dim, vdim, below, stream))
+    elif by_token:
+        _check(lib.pl_recurrent_scan(SCAN_KINDS["retention"], *at, 0, 0, 0, 0, decay.data_ptr(), 0, 0, 0.0, state.data_ptr(), stride,
+                                     0, 0, 0, out.data_ptr(), *step, heads, heads, dim, vdim, below, stream))
+    if chunked:
+        chunks = n // SSD_CHUNK + batch.num_seqs + 1
+        f32 = dict(dtype=torch.float32, device=rows.device)
+        sums, before_chunks = torch.empty((chunks, heads * dim * vdim), **f32), torch.empty((chunks, heads * dim * vdim), **f32)
+        ends = torch.empty((chunks, heads), **f32)
+        _check(lib.pl_retention_chunked(*at, decay.data_ptr(), state.data_ptr(), stride, out.data_ptr(), *step, batch.max_q_len, heads,
+                                        dim, vdim, SCAN_CHUNKED_FROM, sums.data_ptr(), before_chunks.data_ptr(), ends.data_ptr(), stream))
+    return out
+
+
 def _conv_args(rows, off, weight, history, batch):
     n = rows.shape[0]
     _need(rows, "projected rows", None, torch.float32)
@@ -1349,17 +1412,20 @@ def conv_history(rows: torch.Tensor, off: int, weight: torch.Tensor, history: to
 GATES = {None: -1, "sigmoid": 0, "silu": 1}
 
 
-def gated_group_norm(x: torch.Tensor, group: int, gain: torch.Tensor, eps: float, out_dtype: torch.dtype,
+def gated_group_norm(x: torch.Tensor, group: int, gain: torch.Tensor | None, eps: float, out_dtype: torch.dtype,
                      gate: torch.Tensor | None = None, gate_off: int = 0, gate_act: str | None = None,
                      gate_first: bool = False) -> torch.Tensor:
     """x / sqrt(mean over each run of ``group`` columns of x^2 + eps) * gain * act(gate); ``gain`` has a value a
-    column or a value a column of a group; ``gate`` are the columns from ``gate_off`` of 32-bit rows.  ``gate_first``:
+    column or a value a column of a group, or is None for ones; ``gate`` are the columns from ``gate_off`` of 32-bit rows.  ``gate_first``:
     x * act(gate) takes the place of x, statistic included, and the result is not gated."""
     n, width = x.shape
     _need(x, "read-out", None, torch.float32)
-    _need(gain, "gain of the grouped norm", None, torch.float32)
-    if group < 1 or width % group or gain.numel() not in (group, width):
-        raise TensorError(f"rows of {width} in groups of {group} with {gain.numel()} gains")
+    gains = group
+    if gain is not None:
+        _need(gain, "gain of the grouped norm", None, torch.float32)
+        gains = gain.numel()
+    if group < 1 or width % group or gains not in (group, width):
+        raise TensorError(f"rows of {width} in groups of {group} with {gains} gains")
     if gate_act not in GATES or (gate_act is None) != (gate is None):
         raise TensorError(f"a gate through {gate_act!r}")
     if gate is not None:
@@ -1367,7 +1433,7 @@ def gated_group_norm(x: torch.Tensor, group: int, gain: torch.Tensor, eps: float
         if gate.dim() != 2 or gate.shape[0] != n or gate_off < 0 or gate_off + width > gate.shape[1]:
             raise TensorError(f"a gate at column {gate_off} of rows of shape {tuple(gate.shape)}")
     out = torch.empty((n, width), dtype=out_dtype, device=x.device)
-    _check(library().pl_gated_group_norm(x.data_ptr(), n, width, group, gain.data_ptr(), gain.numel(), float(eps),
+    _check(library().pl_gated_group_norm(x.data_ptr(), n, width, group, _ptr(gain), gains, float(eps),
                                          _ptr(gate), 0 if gate is None else gate.shape[1], gate_off, GATES[gate_act],
                                          1 if gate_first else 0, out.data_ptr(), _code(out, "normalised read-out"), _stream()))
     return out
@@ -1538,9 +1604,10 @@ def head_prepare(rows: torch.Tensor, off: int, batch, kv, q_out: torch.Tensor, H
 
 def latent_prepare(rows: torch.Tensor, q_off: int, kv_off: int, gain, eps: float, cos, sin, turned: int, batch, kv,
                    q_plain: torch.Tensor, q_out: torch.Tensor, H: int, D: int, rot: int, R: int, padded: int,
-                   write_kv: bool = True) -> None:
+                   write_kv: bool = True, kv_rows: torch.Tensor | None = None, amplitude: float = 1.0) -> None:
     """For a layer whose pages hold one small vector a token.  ``rows`` (32-bit): H query heads of [D | rot] from
-    column ``q_off``; the small vector's R values and the rotated key part's ``rot`` from ``kv_off``.  The
+    column ``q_off``; the small vector's R values and the rotated key part's ``rot`` from ``kv_off`` (of ``kv_rows``, where
+    they are the rows of another product).  Cosine and sine are multiplied by ``amplitude``.  The
     unrotated query parts go head-major into ``q_plain`` [H, n, D]; the rotated parts, turned, into values
     R .. R + rot of every head of ``q_out`` [n, H * padded] with zeros behind them; with ``write_kv`` the
     token's row of the pages becomes [norm(vector) * gain | turned key part | zeros]."""
@@ -1548,6 +1615,10 @@ def latent_prepare(rows: torch.Tensor, q_off: int, kv_off: int, gain, eps: float
     _need(rows, "projected rows", None, torch.float32)
     _need(q_out, "query buffer", (n, H * padded))
     _need(q_plain, "unrotated query parts", (H, n, D), q_out.dtype)
+    kv_rows = rows if kv_rows is None else kv_rows
+    _need(kv_rows, "projected rows of the keys", None, torch.float32)
+    if rows.dim() != 2 or kv_rows.dim() != 2 or kv_rows.shape[0] != n:
+        raise TensorError(f"projected rows of shape {tuple(rows.shape)} and, for the keys, {tuple(kv_rows.shape)}")
     pool = kv.k_pool
     _need(pool, "pages", None, q_out.dtype)
     if pool.dim() != 2 or pool.shape[1] != padded or pool.shape[0] % kv.block_size:
@@ -1565,11 +1636,23 @@ def latent_prepare(rows: torch.Tensor, q_off: int, kv_off: int, gain, eps: float
             raise TensorError(f"rotary tables have shape {tuple(cos.shape)}, expected [positions, {turned // 2}]")
         table_rows = cos.shape[0]
     _check(library().pl_latent_prepare(
-        rows.data_ptr(), rows.shape[1], int(q_off), int(kv_off), _ptr(gain) if write_kv else 0, float(eps),
-        _ptr(cos) if turned else 0, _ptr(sin) if turned else 0, int(turned), table_rows, batch.positions.data_ptr(),
+        rows.data_ptr(), rows.shape[1], int(q_off), kv_rows.data_ptr(), kv_rows.shape[1], int(kv_off), _ptr(gain) if write_kv else 0,
+        float(eps), _ptr(cos) if turned else 0, _ptr(sin) if turned else 0, float(amplitude), int(turned), table_rows, batch.positions.data_ptr(),
         batch.seq_of.data_ptr(), kv.block_table.data_ptr(), kv.block_table.shape[1], kv.block_size,
         1 if write_kv else 0, q_plain.data_ptr(), q_out.data_ptr(), pool.data_ptr(), _code(q_out, "query buffer"),
         n, H, D, rot, R, padded, _stream()))
+
+
+def rows_norm(rows: torch.Tensor, off: int, gain: torch.Tensor, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """x / sqrt(mean(x^2) + eps) * gain of the columns [off, off + len(gain)) of 32-bit rows, rounded once."""
+    _need(rows, "rows to norm", None, torch.float32)
+    _need(gain, "gain of the norm", None, torch.float32)
+    if rows.dim() != 2 or gain.dim() != 1 or not 0 <= off <= rows.shape[1] - gain.numel():
+        raise TensorError(f"a norm over {gain.numel()} columns from {off} of rows of shape {tuple(rows.shape)}")
+    out = torch.empty((rows.shape[0], gain.numel()), dtype=out_dtype, device=rows.device)
+    _check(library().pl_rows_norm(rows.data_ptr(), rows.shape[1], int(off), gain.data_ptr(), gain.numel(), float(eps),
+                                  out.data_ptr(), _code(out, "normed rows"), rows.shape[0], _stream()))
+    return out
 
 
 def head_gate_(x: torch.Tensor, rows: torch.Tensor, off: int, positions, H: int, V: int,
@@ -1665,54 +1748,72 @@ def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
     return x
 
 
-def _routed(n: int, E: int, choice, weight, identity: int) -> int:
+def _routed(n: int, E: int, choice, weight, identity: int, shared: int = 0) -> int:
     """Checks a router's choice for ``n`` rows ([n, top] int32, with weights [n, top] 32-bit) and gives ``top``."""
     _need(choice, "chosen experts", None, torch.int32)
-    if choice.dim() != 2 or choice.shape[0] != n or not 1 <= choice.shape[1] <= E + identity or identity < 0:
-        raise TensorError(f"chosen experts of shape {tuple(choice.shape)} for {n} rows and {E} + {identity} experts")
+    if choice.dim() != 2 or choice.shape[0] != n or not 1 <= choice.shape[1] <= E + identity + shared or identity < 0:
+        raise TensorError(f"chosen experts of shape {tuple(choice.shape)} for {n} rows and {E} + {identity} + {shared} experts")
     _need(weight, "weights of the chosen experts", tuple(choice.shape), torch.float32)
     return choice.shape[1]
 
 
+def _experts(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, gated: bool, shared, choice) -> tuple:
+    """(experts, their size, the shared expert's size or 0), every matrix checked."""
+    E, W = w_up.shape[0], x.shape[1]
+    halves = 2 if gated else 1
+    F = w_up.shape[1] // halves
+    _need(w_up, "gate and up weights of the experts" if gated else "up weights of the experts", (E, halves * F, W), x.dtype)
+    _need(w_down, "down weights of the experts", (E, W, F), x.dtype)
+    if shared is None:
+        return E, F, 0
+    if choice is None:
+        raise TensorError("a shared expert beside a table of experts")
+    size = shared[0].shape[0] // halves
+    _need(shared[0], "first matrix of the shared expert", (halves * size, W), x.dtype)
+    _need(shared[1], "down weights of the shared expert", (W, size), x.dtype)
+    return E, F, size
+
+
 def moe_rows(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: torch.Tensor,
-             activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None) -> torch.Tensor:
+             activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None,
+             gated: bool = True, shared: tuple | None = None) -> torch.Tensor:
     """Experts chosen by a table over token ids, a row at a time: 32-bit [n, W], row t the mean over the experts e
     that ``table[id of t]`` names of down_e (act(gate_e x_t) * (up_e x_t)).  ``w_gate_up`` [E, 2 F, W] (an expert's
     gate rows, then its up rows), ``w_down`` [E, W, F], of ``x``'s type; ``table`` [vocabulary, top] int32.  A row's
     id is the batch's, or the one an earlier step left on the device; padding rows give zeros.
     With ``choice`` and ``weight`` ([n, top]; no table) a router has chosen: pair (t, c) runs expert choice[t, c] and
     counts weight[t, c]; a choice of E .. E + ``identity`` - 1 is an identity expert, whose output is the row itself;
-    -1 is none.  ``activation`` "clamped" (with its ``limit``): see ``CLAMPED_GATE``."""
+    -1 is none.  ``activation`` "clamped" (with its ``limit``): see ``CLAMPED_GATE``.  ``gated`` False: an expert is
+    down_e (act(up_e x_t)), ``w_gate_up`` holding up rows alone, [E, F, W].  ``shared`` = (first matrix, down matrix) of an expert of
+    the same form and another size; every row's last choice names it, as number E + ``identity``."""
     n, W = x.shape
     _need(x, "rows")
-    E, F2, _ = w_gate_up.shape
-    F = F2 // 2
-    _need(w_gate_up, "gate and up weights of the experts", (E, 2 * F, W), x.dtype)
-    _need(w_down, "down weights of the experts", (E, W, F), x.dtype)
+    E, F, size = _experts(x, w_gate_up, w_down, gated, shared, choice)
     if choice is not None:
-        vocab, top = 1, _routed(n, E, choice, weight, identity)
+        vocab, top = 1, _routed(n, E, choice, weight, identity, 1 if size else 0)
     else:
         _need(table, "table of experts", None, torch.int32)
         vocab, top = table.shape
     act, bound = _gate_code(activation, limit)
     fed = getattr(batch, "fed_tokens", None)
     src = batch.token_src if fed is not None else None
-    h = torch.empty((n, top, F), dtype=x.dtype, device=x.device)
+    h = torch.empty((n, (top - 1) * F + (size or F)), dtype=x.dtype, device=x.device)
     out = torch.empty((n, W), dtype=torch.float32, device=x.device)
     _check(library().pl_moe_rows(x.data_ptr(), batch.token_ids.data_ptr(), _ptr(src), _ptr(fed),
                                  batch.positions.data_ptr(), _ptr(table), w_gate_up.data_ptr(), w_down.data_ptr(),
                                  h.data_ptr(), out.data_ptr(), _code(x, "rows"), n, W, F, E, top, vocab,
-                                 act, _ptr(choice), _ptr(weight), int(identity), bound, _stream()))
+                                 act, _ptr(choice), _ptr(weight), int(identity), bound, 0 if gated else 1, size,
+                                 shared[0].data_ptr() if size else 0, shared[1].data_ptr() if size else 0, _stream()))
     return out
 
 
 MOE_TILE = 128       # rows of a tile of the grouped product
 
 
-def moe_grouped_applies(x: torch.Tensor, width: int, ff: int) -> bool:
+def moe_grouped_applies(x: torch.Tensor, width: int, ff: int, gated: bool = True) -> bool:
     """Whether the experts of a step run as grouped products on the matrix cores: bfloat16, an inner width the
-    tiles take (a multiple of 32), an expert width that is a multiple of 64."""
-    return x.dtype == torch.bfloat16 and width % 32 == 0 and ff % 64 == 0
+    tiles take (a multiple of 32), an expert width that is a multiple of 64 (of 32 without a gate)."""
+    return x.dtype == torch.bfloat16 and width % 32 == 0 and ff % (64 if gated else 32) == 0
 
 
 def moe_down_splits(tiles: int, width: int, ff: int) -> int:
@@ -1726,20 +1827,19 @@ def moe_down_splits(tiles: int, width: int, ff: int) -> int:
 
 
 def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: torch.Tensor,
-                activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None) -> torch.Tensor:
+                activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None,
+                gated: bool = True, shared: tuple | None = None) -> torch.Tensor:
     """What ``moe_rows`` computes, with the step's (row, choice) pairs dealt to their experts first: an expert's
     pairs fill tiles of 128 rows, and two grouped products on the matrix cores (gate and up with the activation
     behind them; down with 32-bit sums out) read an expert's weights once a tile.  A last pass adds a row's
-    choices in their order, in 32-bit.  Nothing is read back by the host: the tiles are laid out for the most
+    choices in their order, in 32-bit.  A shared expert is one more group of the same products, with matrices of its own
+    size.  Nothing is read back by the host: the tiles are laid out for the most
     a step of so many rows can need."""
     n, W = x.shape
     _need(x, "rows", None, torch.bfloat16)
-    E, F2, _ = w_gate_up.shape
-    F = F2 // 2
-    _need(w_gate_up, "gate and up weights of the experts", (E, 2 * F, W), x.dtype)
-    _need(w_down, "down weights of the experts", (E, W, F), x.dtype)
+    E, F, size = _experts(x, w_gate_up, w_down, gated, shared, choice)
     if choice is not None:
-        vocab, top = 1, _routed(n, E, choice, weight, identity)
+        vocab, top = 1, _routed(n, E, choice, weight, identity, 1 if size else 0)
     else:
         _need(table, "table of experts", None, torch.int32)
         vocab, top = table.shape
@@ -1750,22 +1850,26 @@ def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: 
     fed = getattr(batch, "fed_tokens", None)
     src = batch.token_src if fed is not None else None
     pairs = n * top
+    dealt = E + (1 if size else 0)
     # every expert that has pairs may leave its last tile part empty
-    tiles = -(-pairs // MOE_TILE) + min(E, pairs)
+    tiles = -(-pairs // MOE_TILE) + min(dealt, pairs)
     slots = tiles * MOE_TILE
     lib, stream = library(), _stream()
     ints = torch.empty((slots + pairs + tiles,), dtype=torch.int32, device=x.device)
     gather, slot_of, tile_group = ints[:slots], ints[slots:slots + pairs], ints[slots + pairs:]
     _check(lib.pl_moe_sort(batch.token_ids.data_ptr(), _ptr(src), _ptr(fed), batch.positions.data_ptr(), _ptr(table),
-                           _ptr(choice), n, top, E, vocab, MOE_TILE, tiles, gather.data_ptr(), slot_of.data_ptr(),
-                           tile_group.data_ptr(), stream))
-    hidden = torch.empty((slots, F), dtype=torch.bfloat16, device=x.device)
+                           _ptr(choice), n, top, dealt, vocab, E + int(identity) if size else -1, MOE_TILE, tiles,
+                           gather.data_ptr(), slot_of.data_ptr(), tile_group.data_ptr(), stream))
+    longest = max(F, size)
+    last, shared_up, shared_down = (E, shared[0].data_ptr(), shared[1].data_ptr()) if size else (-1, 0, 0)
+    hidden = torch.empty((slots, longest), dtype=torch.bfloat16, device=x.device)
     _check(lib.pl_gemm_tiled_grouped(x.data_ptr(), w_gate_up.data_ptr(), hidden.data_ptr(), tile_group.data_ptr(),
-                                     gather.data_ptr(), 2 * F * W, tiles, n, F, W, 1, act, 1, bound, stream))
-    splits = moe_down_splits(tiles, W, F)
+                                     gather.data_ptr(), w_gate_up.stride(0), tiles, n, F, W, 1 if gated else 4, act, 1, bound,
+                                     W, longest, last, shared_up, size, W, stream))
+    splits = moe_down_splits(tiles, W, min(F, size) if size else F)
     y = torch.empty((splits, slots, W), dtype=torch.float32, device=x.device)
     _check(lib.pl_gemm_tiled_grouped(hidden.data_ptr(), w_down.data_ptr(), y.data_ptr(), tile_group.data_ptr(), 0,
-                                     W * F, tiles, slots, W, F, 3, 0, splits, 0.0, stream))
+                                     W * F, tiles, slots, W, F, 3, 0, splits, 0.0, longest, W, last, shared_down, W, size, stream))
     _check(lib.pl_moe_combine(y.data_ptr(), slot_of.data_ptr(), out.data_ptr(), n, top, W, splits, slots * W,
                               _ptr(weight), _ptr(choice), x.data_ptr(), _code(x, "rows"), E, batch.positions.data_ptr(), stream))
     return out
@@ -1775,6 +1879,7 @@ def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: 
 # of up to this many rows and routers of up to this many weights; beyond, a product of its own (the library's) is faster.
 ROUTER_FUSED_ROWS = 128
 ROUTER_FUSED_WEIGHTS = 1 << 18
+ROUTER_SCORES = {"softmax": 0, "chosen_logits": 1, "sigmoid": 2}
 
 
 def router_fuses(rows: int, total: int, width: int) -> bool:
@@ -1783,41 +1888,48 @@ def router_fuses(rows: int, total: int, width: int) -> bool:
 
 def router_select(logits, correction, positions, top: int, groups: int = 1, kept: int = 1,
                   normalised: bool = True, weight_eps: float = 1e-20, x=None, w=None, bias=None,
-                  of_chosen: bool = False):
+                  score: str = "softmax", group_best: int = 1, scale: float = 1.0, shared: bool = False):
     """A router's choice for every row of its 32-bit ``logits`` [n, outputs]: (chosen [n, top] int32, weights [n, top]
     32-bit).  Scores are the softmax over all outputs; the choice goes by score plus ``correction`` ([outputs] 32-bit, or
-    None); outputs form ``groups`` equal groups of neighbours, a group counts by its best choice score, and only members
+    None); outputs form ``groups`` equal groups of neighbours, a group counts by its best choice score (``group_best`` 2: by the
+    sum of its two best), and only members
     of the best ``kept`` groups can be chosen; the ``top`` largest are chosen, the lower index among equals; a chosen
-    output weighs its score, divided (``normalised``) by the chosen scores' sum plus ``weight_eps``.  Rows at
+    output weighs its score, divided (``normalised``) by the chosen scores' sum plus ``weight_eps``, times ``scale``.  Rows at
     position -1 choose nothing (-1).  With ``logits`` None the kernel works them out itself from the rows ``x`` [n, W]
     and the router's matrix ``w`` [outputs, W] (one type; 32-bit sums).  ``bias`` ([outputs] 32-bit) is added to the logits
-    first.  ``of_chosen``: the choice goes by the logits themselves and the weights are the softmax over the chosen
-    logits alone (no correction; ``normalised`` and ``weight_eps`` do not enter)."""
+    first.  ``score`` "sigmoid": a score is the sigmoid of its logit.  "chosen_logits": the choice goes by the logits themselves and
+    the weights are the softmax over the chosen logits alone (no correction; ``normalised`` and ``weight_eps`` do not enter).
+    ``shared``: the last output is no expert's, it gates one that every row uses: the row names ``top`` + 1, the last of them
+    number (outputs - 1) with the sigmoid of that output as its weight."""
+    if score not in ROUTER_SCORES:
+        raise TensorError(f"router scores of kind {score!r} ({', '.join(ROUTER_SCORES)})")
     if logits is not None:
         _need(logits, "router logits", None, torch.float32)
         if logits.dim() != 2:
             raise TensorError(f"router logits of shape {tuple(logits.shape)}")
-        n, total = logits.shape
+        n, outputs = logits.shape
         width, code, device = 0, F32, logits.device
     else:
         _need(x, "rows")
         _need(w, "router matrix", None, x.dtype)
         if x.dim() != 2 or w.dim() != 2 or w.shape[1] != x.shape[1]:
             raise TensorError(f"rows of shape {tuple(x.shape)} for a router of shape {tuple(w.shape)}")
-        (n, width), total, code, device = x.shape, w.shape[0], _code(x, "rows"), x.device
+        (n, width), outputs, code, device = x.shape, w.shape[0], _code(x, "rows"), x.device
+    one = 1 if shared else 0
+    total, named = outputs - one, int(top) + one
     if correction is not None:
         _need(correction, "correction of the choice", (total,), torch.float32)
     if bias is not None:
         _need(bias, "bias of the router", (total,), torch.float32)
     if positions is not None:
         _need(positions, "positions", (n,), torch.int32)
-    choice = torch.empty((n, top), dtype=torch.int32, device=device)
-    weight = torch.empty((n, top), dtype=torch.float32, device=device)
-    _check(library().pl_router_select(_ptr(logits), total, _ptr(correction), _ptr(positions), n, total, int(top),
+    choice = torch.empty((n, named), dtype=torch.int32, device=device)
+    weight = torch.empty((n, named), dtype=torch.float32, device=device)
+    _check(library().pl_router_select(_ptr(logits), outputs, _ptr(correction), _ptr(positions), n, total, int(top),
                                       int(groups), int(kept), 1 if normalised else 0, float(weight_eps),
                                       choice.data_ptr(), weight.data_ptr(), _ptr(x) if logits is None else 0,
                                       _ptr(w) if logits is None else 0, int(width), code, _ptr(bias),
-                                      1 if of_chosen else 0, _stream()))
+                                      ROUTER_SCORES[score], int(group_best), float(scale), one, _stream()))
     return choice, weight
 
 
@@ -1857,9 +1969,9 @@ def wide_prepare(rows: torch.Tensor, off: int, batch, kv, q_out: torch.Tensor, H
 
 
 def parallel_step(resid: torch.Tensor, a=None, ls1=None, b=None, ls2=None, more=None, gain1=None, gain2=None,
-                  eps: float = 0.0, out_dtype: torch.dtype = torch.float32, rows=None):
+                  eps: float = 0.0, out_dtype: torch.dtype = torch.float32, rows=None, mult: float = 1.0):
     """One pass over the rows of the 32-bit stream for a layer whose sublayers stand side by side, either half
-    optional.  Sums: resid += ls1 * a + ls2 * b + more (``a``, ``b``, ``more`` [n, W] 32-bit; ``ls1``, ``ls2`` [W] 32-bit
+    optional.  Sums: resid += mult * (ls1 * a + ls2 * b) + more (``a``, ``b``, ``more`` [n, W] 32-bit; ``ls1``, ``ls2`` [W] 32-bit
     or None for ones), in place.  Norms of the updated rows: rms-normed rows times ``gain1`` and, where given, times
     ``gain2`` (both [W] 32-bit), in ``out_dtype``; (rows1, rows2), each None where its gain is.  ``rows``: the rows to
     norm (then nothing is summed)."""
@@ -1885,7 +1997,7 @@ def parallel_step(resid: torch.Tensor, a=None, ls1=None, b=None, ls2=None, more=
         return None, None
     _check(library().pl_parallel_step(resid.data_ptr(), _ptr(a), _ptr(ls1), _ptr(b), _ptr(ls2), _ptr(more), _ptr(gain1),
                                       _ptr(gain2), float(eps), _ptr(out1), _ptr(out2), _CODES[out_dtype], _ptr(rows),
-                                      count, W, _stream()))
+                                      count, W, float(mult), _stream()))
     return out1, out2
 
 

@@ -434,20 +434,20 @@ register_block("hyper_connections", HyperConnectionBlock)
 
 
 class PendingSums:
-    """What a layer whose sublayers stand side by side has not added to the stream yet: its sublayers' 32-bit outputs
-    and their gains a column.  The layer behind adds them in the pass that norms its own rows."""
+    """What a layer whose sublayers stand side by side has not added to the stream yet: its sublayers' 32-bit outputs,
+    their gains a column and what both are multiplied by.  The layer behind adds them in the pass that norms its own rows."""
 
-    __slots__ = ("a", "ls1", "b", "ls2")
+    __slots__ = ("a", "ls1", "b", "ls2", "mult")
     filled = True            # (what a layer hands to the next is looked at only when it says it holds something)
 
-    def __init__(self, a, ls1, b, ls2):
-        self.a, self.ls1, self.b, self.ls2 = a, ls1, b, ls2
+    def __init__(self, a=None, ls1=None, b=None, ls2=None, mult: float = 1.0):
+        self.a, self.ls1, self.b, self.ls2, self.mult = a, ls1, b, ls2, mult
 
 
 class ParallelBlock:
     """The arrangement whose sublayers read the same stream through a norm each: with a = norm1(x) and b = norm2(x),
-    x <- x + ls1 * mixer(a) + ls2 * feed_forward(b).  ``LayerSpec.layer_scale`` says whether the gains a column ls1 and
-    ls2 exist (tensors ``ls1``, ``ls2``); without it the outputs are added as they are.  A layer whose spec has no
+    x <- x + m (ls1 * mixer(a) + ls2 * feed_forward(b)).  ``LayerSpec.layer_scale`` says whether the gains a column ls1 and
+    ls2 exist (tensors ``ls1``, ``ls2``); without it they are ones.  m is ``LayerSpec.residual_mult``.  A layer whose spec has no
     feed-forward adds the mixer's output only (``norm2`` and ``ls2``, if a checkpoint carries them, are not used).
 
     The stream and every sum into it are 32-bit; sublayers hand back 32-bit rows.  One kernel adds a layer's two outputs
@@ -493,6 +493,7 @@ class ParallelBlock:
             raise ConfigError(f"norm {layer.norm.kind!r} cannot run inside the pass over the stream of a layer whose "
                               "sublayers stand side by side (it needs a 32-bit gain and an eps, nothing else)")
         self.dtype, self.hidden = dtype, hidden
+        self.mult = float(getattr(layer, "residual_mult", 1.0))
         self.norm1 = norm(layer.norm, hidden, {"weight": params[n["norm1"]]}, dtype, device)
         self.norm1.takes_pending_sums = True       # (how the layer before learns that its sums can wait)
         self.mixer = lookup(MIXERS, layer.mixer.kind, "mixer")(
@@ -519,10 +520,10 @@ class ParallelBlock:
             kernels.residual_add(resid, delta)
         before = getattr(ctx, "handed", None)
         if not isinstance(before, PendingSums):
-            before = PendingSums(None, None, None, None)
+            before = PendingSums()
         eps = self.norm1.eps
         rows1, rows2 = kernels.parallel_step(
-            resid, a=before.a, ls1=before.ls1, b=before.b, ls2=before.ls2, more=getattr(ctx, "stream_addend", None),
+            resid, a=before.a, ls1=before.ls1, b=before.b, ls2=before.ls2, mult=before.mult, more=getattr(ctx, "stream_addend", None),
             gain1=self.norm1.gain32, gain2=self.norm2.gain32 if self.norm2 is not None else None, eps=eps,
             out_dtype=self.dtype)
         ctx.stream_addend = None
@@ -535,9 +536,9 @@ class ParallelBlock:
                 out = out.float()
         after = getattr(ctx, "norm_after", None)
         if ctx.trace is None and after is not None and getattr(after, "takes_pending_sums", False):
-            ctx.handed_out = PendingSums(mixed, self.ls1, out, self.ls2)
+            ctx.handed_out = PendingSums(mixed, self.ls1, out, self.ls2, self.mult)
         else:
-            kernels.parallel_step(resid, a=mixed, ls1=self.ls1, b=out, ls2=self.ls2)
+            kernels.parallel_step(resid, a=mixed, ls1=self.ls1, b=out, ls2=self.ls2, mult=self.mult)
         return None
 
 

@@ -9,7 +9,8 @@ part is carried into c's space once, q~_h = U_h^T q_h, and
 
 which is attention of H query heads over ONE key head whose keys are the pages' rows and whose values are the
 first kv_rank values of those same rows (``KVCacheSpec.values_in_keys``).  The softmax may have a learned
-sink a head, the read-out a gate a head (the sigmoid of a projection of the layer's input).  A layer built
+sink a head, the read-out a gate a head (the sigmoid of a projection of the layer's input).  Queries may go through a
+small normed vector of their own (``q_rank``): two projections with a norm between them.  A layer built
 with ``borrows`` has no projection onto c: the schedule names the layer whose pages it reads, with its own
 queries, U, W, sinks and gates.
 """
@@ -27,7 +28,7 @@ from ..errors import UnsupportedError
 from ..weights.loader import ParamDecl
 from .linear import Linear
 from .registry import register_mixer
-from .rotary import rotary_frequencies, rotary_tables
+from .rotary import rotary_tables, turning
 from .sink_attention import head_sinks
 
 
@@ -40,7 +41,11 @@ class LatentAttention:
     @staticmethod
     def declare(spec, hidden: int) -> list:
         H, D, rot, V, R = spec.num_heads, spec.head_dim, spec.rotary_dim, spec.value_dim, spec.kv_rank
-        decls = [ParamDecl("q", (H * (D + rot), hidden))]
+        if spec.q_rank is not None:
+            decls = [ParamDecl("dq", (spec.q_rank, hidden)), ParamDecl("dq.norm", (spec.q_rank,), "gain"),
+                     ParamDecl("uq", (H * (D + rot), spec.q_rank))]
+        else:
+            decls = [ParamDecl("q", (H * (D + rot), hidden))]
         if not spec.borrows:
             decls += [ParamDecl("dkv", (R + rot, hidden)), ParamDecl("dkv.norm", (R,), "gain")]
         decls += [ParamDecl("uk", (H * D, R)), ParamDecl("uv", (H * V, R))]
@@ -65,11 +70,16 @@ class LatentAttention:
         self.H, self.D, self.rot, self.V, self.R = H, D, rot, V, R
         self.scale = float(spec.scale) if spec.scale is not None else 1.0 / math.sqrt(D + rot)
         self.window = int(spec.window or 0)
-        # one product for everything the layer's input is projected onto: the row is [q | gates | c, key part]
-        pieces = [params["q"]]
+        # one product for everything the layer's input is projected onto: the row is [q | gates | c, key part], with the
+        # queries' small vector in the place of q where they have one
+        pieces = [params["q" if spec.q_rank is None else "dq"]]
+        self.q_gain = self.q_proj = None
+        if spec.q_rank is not None:
+            self.q_gain = params["dq.norm"].to(torch.float32).contiguous()
+            self.q_proj = Linear(params["uq"])
         self.gate_off = self.kv_off = 0
         if spec.gated:
-            self.gate_off = H * (D + rot)
+            self.gate_off = pieces[0].shape[0]
             pieces.append(params["g"])
         if not spec.borrows:
             self.kv_off = sum(p.shape[0] for p in pieces)
@@ -85,14 +95,15 @@ class LatentAttention:
         # the rotation's angles: tables of cosines and sines where the spec bounds the positions, otherwise the
         # frequencies alone (rounded from 64-bit), and the kernel multiplies by the position in 32-bit
         self.cos = self.sin = None
+        self.amplitude = 1.0
         if spec.rotary_turned and spec.max_positions:
-            if getattr(spec, "rotary_scaling", None) is not None:
+            if spec.rotary_scaling is not None or spec.rotary_ramp is not None:
                 raise UnsupportedError("rescaled rotation frequencies with tables of angles (max_positions = 0 works the angles out)")
             rotary = rotary_tables(PositionSpec("rotary_neighbours", spec.rotary_turned, float(spec.rotary_base),
                                                 int(spec.max_positions)), device, shared)
             self.cos, self.sin = rotary.cos, rotary.sin
         elif spec.rotary_turned:
-            self.cos = rotary_frequencies(spec.rotary_turned, spec.rotary_base, getattr(spec, "rotary_scaling", None), device)
+            self.cos, self.amplitude = turning(spec.rotary_turned, spec.rotary_base, spec.rotary_scaling, spec.rotary_ramp, device)
         self.o_proj = Linear(params["o"])
 
     def cache_spec(self):
@@ -110,9 +121,13 @@ class LatentAttention:
         n = rows.shape[0]
         q = torch.empty((n, H * P), dtype=self.dtype, device=rows.device)
         q_plain = torch.empty((H, n, D), dtype=self.dtype, device=rows.device)
-        kernels.latent_prepare(rows, 0, self.kv_off, self.gain, self.spec.norm_eps, self.cos, self.sin, self.spec.rotary_turned,
-                               batch, kv, q_plain, q, H, D, rot, R, P,
-                               write_kv=ctx.writes_cache and not self.spec.borrows)
+        queries = rows
+        if self.q_proj is not None:
+            queries = self.q_proj.forward(kernels.rows_norm(rows, 0, self.q_gain, self.spec.norm_eps, self.dtype),
+                                          out_dtype=torch.float32)
+        kernels.latent_prepare(queries, 0, self.kv_off, self.gain, self.spec.norm_eps, self.cos, self.sin, self.spec.rotary_turned,
+                               batch, kv, q_plain, q, H, D, rot, R, P, write_kv=ctx.writes_cache and not self.spec.borrows,
+                               kv_rows=rows, amplitude=self.amplitude)
         kernels.gemm_heads(q_plain.transpose(0, 1), self.uk_t, q.view(n, H, P)[:, :, :R])
         out = torch.empty((n, H * P), dtype=self.dtype, device=rows.device)
         kernels.sink_attention(q, out, batch, kv, H, 1, P, self.scale, self.window, sinks=self.sinks)

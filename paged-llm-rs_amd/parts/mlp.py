@@ -147,14 +147,15 @@ register_feed_forward("table_experts", TableExperts)
 
 
 class RoutedExperts:
-    """Small gated feed-forwards behind a router, with identity experts behind the real ones: a token's output is the
+    """Small feed-forwards behind a router, with identity experts behind the real ones: a token's output is the
     sum over its chosen e of weight_e * expert_e(x), where an identity expert's output is x itself.  The router's
     logits are one product with 32-bit sums out; scores, the correction for the choice, the groups, the choice and
     the weights are one kernel in 32-bit (``kernels.router_select``); the chosen pairs then run as the experts by table
-    do: dealt to their experts and multiplied as grouped products on the matrix cores, or a pair at a time.  Nothing
-    depends on the other rows of the step.  The result comes back in 32-bit.
-    Tensors: ``e<i>.gate``, ``e<i>.up`` [ff, width], ``e<i>.down`` [width, ff]; ``router`` [experts + identity, width];
-    ``router.b`` and ``correction`` [experts + identity], where the spec has them."""
+    do: dealt to their experts and multiplied as grouped products on the matrix cores, or a pair at a time.  A shared expert is one
+    more choice that every token makes: its gate is one more row of the router's product, its matrices one more group of the
+    experts' products.  Nothing depends on the other rows of the step.  The result comes back in 32-bit.
+    Tensors: ``e<i>.gate`` (where gated), ``e<i>.up`` [ff, width], ``e<i>.down`` [width, ff]; ``router`` [experts + identity, width];
+    ``router.b`` and ``correction`` [experts + identity], where the spec has them; ``shared.*`` likewise, ``shared.sg`` [1, width]."""
 
     # forward needs the step (padding rows choose nothing)
     takes_batch = True
@@ -162,30 +163,34 @@ class RoutedExperts:
 
     @staticmethod
     def declare(spec, hidden: int) -> list:
-        decls = []
-        for e in range(spec.experts):
-            decls += [ParamDecl(f"e{e}.gate", (spec.intermediate_size, hidden)),
-                      ParamDecl(f"e{e}.up", (spec.intermediate_size, hidden)),
-                      ParamDecl(f"e{e}.down", (hidden, spec.intermediate_size))]
+        def expert(name: str, size: int) -> list:
+            first = ["gate", "up"] if spec.gated else ["up"]
+            return [ParamDecl(f"{name}.{part}", (size, hidden)) for part in first] + [ParamDecl(f"{name}.down", (hidden, size))]
+
+        decls = [d for e in range(spec.experts) for d in expert(f"e{e}", spec.intermediate_size)]
         total = spec.experts + spec.identity
         decls.append(ParamDecl("router", (total, hidden), "router"))
         if spec.biased:
             decls.append(ParamDecl("router.b", (total,), "bias"))
         if spec.corrected:
             decls.append(ParamDecl("correction", (total,), "bias"))
+        if spec.shared_size:
+            decls += expert("shared", spec.shared_size) + [ParamDecl("shared.sg", (1, hidden))]
         return decls
 
     def __init__(self, spec, hidden: int, params: dict, dtype, device, shared: dict):
         if spec.activation == kernels.CLAMPED_GATE:
-            if spec.limit is None or not spec.limit > 0:
+            if spec.limit is None or not spec.limit > 0 or not spec.gated:
                 raise UnsupportedError(f"a clamped gate with a limit of {spec.limit}")
         elif spec.activation not in kernels.ACTIVATIONS or spec.limit is not None:
             raise UnsupportedError(f"activation {spec.activation!r} (limit {spec.limit}), the kernels know "
                                    f"{', '.join(sorted(kernels.ACTIVATIONS))} without a limit and {kernels.CLAMPED_GATE} with one")
-        if spec.score not in ("softmax", "chosen_logits"):
-            raise UnsupportedError(f"router scores of kind {spec.score!r} (softmax or chosen_logits)")
+        if spec.score not in kernels.ROUTER_SCORES:
+            raise UnsupportedError(f"router scores of kind {spec.score!r} ({', '.join(kernels.ROUTER_SCORES)})")
         if spec.score == "chosen_logits" and spec.corrected:
             raise UnsupportedError("a correction of the scores where the logits themselves choose")
+        if spec.group_best not in (1, 2):
+            raise UnsupportedError(f"groups that count by their best {spec.group_best} members (1 or 2)")
         E, total = spec.experts, spec.experts + spec.identity
         if E < 1 or spec.identity < 0 or not 1 <= spec.top <= total:
             raise UnsupportedError(f"{spec.top} of {E} + {spec.identity} experts a token")
@@ -194,16 +199,27 @@ class RoutedExperts:
             raise UnsupportedError(f"{total} router outputs in {spec.groups} groups of which {spec.groups_kept} are kept, "
                                    f"{spec.top} chosen")
         self.spec, self.activation = spec, spec.activation
-        # [E, 2 F, W]: an expert's gate rows, then its up rows; [E, W, F]
-        self.w_gate_up = torch.stack([torch.cat([params[f"e{e}.gate"], params[f"e{e}.up"]], 0) for e in range(E)]).contiguous()
+
+        def first(name: str):
+            """An expert's gate rows, then its up rows; without a gate its up rows."""
+            return torch.cat([params[f"{name}.gate"], params[f"{name}.up"]], 0) if spec.gated else params[f"{name}.up"]
+
+        # [E, 2 F, W] or [E, F, W]; [E, W, F]
+        self.w_first = torch.stack([first(f"e{e}") for e in range(E)]).contiguous()
         self.w_down = torch.stack([params[f"e{e}.down"] for e in range(E)]).contiguous()
-        self.router = Linear(params["router"])
+        self.shared_expert = None
+        gates = []
+        if spec.shared_size:
+            self.shared_expert = (first("shared").contiguous(), params["shared.down"].contiguous())
+            gates = [params["shared.sg"]]
+        self.router = Linear.fused([params["router"]] + gates)
         self.bias = params["router.b"].to(torch.float32).contiguous() if spec.biased else None
         self.correction = params["correction"].to(torch.float32).contiguous() if spec.corrected else None
 
     def forward(self, x, batch):
         spec = self.spec
-        how = dict(bias=self.bias, of_chosen=spec.score == "chosen_logits")
+        how = dict(bias=self.bias, score=spec.score, group_best=spec.group_best, scale=spec.weight_scale,
+                   shared=self.shared_expert is not None)
         if kernels.router_fuses(x.shape[0], self.router.out_features, x.shape[1]):
             # (few rows: the kernel that chooses works the logits out itself)
             logits, how["x"], how["w"] = None, x, self.router.weight
@@ -211,9 +227,11 @@ class RoutedExperts:
             logits = self.router.forward(x, out_dtype=torch.float32)
         choice, weight = kernels.router_select(logits, self.correction, batch.positions, spec.top, spec.groups,
                                                spec.groups_kept, spec.normalised, spec.weight_eps, **how)
-        run = kernels.moe_grouped if kernels.moe_grouped_applies(x, x.shape[1], spec.intermediate_size) else kernels.moe_rows
-        return run(x, batch, None, self.w_gate_up, self.w_down, self.activation, choice=choice, weight=weight,
-                   identity=spec.identity, limit=spec.limit)
+        dealt = all(kernels.moe_grouped_applies(x, x.shape[1], size, spec.gated)
+                    for size in (spec.intermediate_size, spec.shared_size) if size)
+        run = kernels.moe_grouped if dealt else kernels.moe_rows
+        return run(x, batch, None, self.w_first, self.w_down, self.activation, choice=choice, weight=weight,
+                   identity=spec.identity, limit=spec.limit, gated=spec.gated, shared=self.shared_expert)
 
 
 register_feed_forward("routed_experts", RoutedExperts)

@@ -1,5 +1,5 @@
 """Mixers that keep a matrix of state a head instead of keys and values in pages: linear attention with
-a fixed decay, the matrix memory with exponential gates (mLSTM), the gated delta rule, and the state space
+a fixed decay (``lightning_attention``, and ``retention`` with rotated q and k), the matrix memory with exponential gates (mLSTM), the gated delta rule, and the state space
 whose decay and step size come from the token (Mamba-2).
 
 All of them are one product for every projection of the layer's input (32-bit sums out), the scan over
@@ -19,6 +19,7 @@ from ..errors import ConfigError, UnsupportedError
 from ..weights.loader import ParamDecl
 from .linear import Linear
 from .registry import register_mixer
+from .rotary import turning
 
 
 def _f32(t: torch.Tensor) -> torch.Tensor:
@@ -226,7 +227,51 @@ class StateSpace(_ScanMixer):
         return self.o_proj.forward(normed, out_dtype=torch.float32)
 
 
+class Retention(_ScanMixer):
+    """Linear attention with a fixed decay a head and rotated queries and keys, no activations and no denominator; every head's read-out
+    divided by its root mean square, times silu(gate).  Tensors: ``q``, ``k``, ``v``, ``g``, ``o``."""
+
+    # requests that bring fewer tokens than this go token by token, which a step launches only where there are any
+    short_portion = kernels.SCAN_CHUNKED_FROM
+
+    @staticmethod
+    def declare(spec, hidden: int) -> list:
+        qk, v = spec.num_heads * spec.head_dim, spec.num_heads * spec.value_dim
+        return [ParamDecl("q", (qk, hidden)), ParamDecl("k", (qk, hidden)), ParamDecl("v", (v, hidden)),
+                ParamDecl("g", (v, hidden)), ParamDecl("o", (hidden, v))]
+
+    def __init__(self, spec, hidden: int, params: dict, dtype, device, shared: dict):
+        self._sizes(spec, "retention")
+        if len(spec.decay) != spec.num_heads:
+            raise ConfigError(f"{len(spec.decay)} decays for {spec.num_heads} heads")
+        if spec.rotary_dims % 2 or not 0 <= spec.rotary_dims <= spec.head_dim:
+            raise UnsupportedError(f"a rotation over {spec.rotary_dims} of {spec.head_dim} values")
+        self.spec, self.dtype = spec, dtype
+        self.H, self.D, self.V = spec.num_heads, spec.head_dim, spec.value_dim
+        self._fuse(params, ["q", "k", "v", "g"])
+        self.o_proj = Linear(params["o"])
+        self.decay = torch.tensor([float(d) for d in spec.decay], dtype=torch.float32, device=device)
+        # (in chunks a decay enters through its logarithm)
+        self.chunked = min(float(d) for d in spec.decay) > 0.0
+        self.freq, self.amplitude = None, 1.0
+        if spec.rotary_dims:
+            self.freq, self.amplitude = turning(spec.rotary_dims, spec.rotary_base, None, spec.rotary_ramp, device)
+        self.key_scale = float(spec.key_scale) if spec.key_scale is not None else self.D ** -0.5
+
+    def state_spec(self):
+        return StateSpec((self.H * self.D * self.V,), torch.float32)
+
+    def forward(self, x, ctx):
+        c = self.columns
+        rows = self.proj.forward(x, out_dtype=torch.float32)
+        read = kernels.retention_scan(rows, c["q"], c["k"], c["v"], ctx.state(), ctx.batch, self.H, self.D, self.V, self.decay,
+                                      self.freq, self.amplitude, self.key_scale, chunked=self.chunked)
+        normed = kernels.gated_group_norm(read, self.V, None, self.spec.eps, self.dtype, gate=rows, gate_off=c["g"], gate_act="silu")
+        return self.o_proj.forward(normed, out_dtype=torch.float32)
+
+
 register_mixer("lightning_attention", LightningAttention)
+register_mixer("retention", Retention)
 register_mixer("mlstm", Mlstm)
 register_mixer("gated_delta", GatedDelta)
 register_mixer("state_space", StateSpace)

@@ -71,3 +71,40 @@ def rotary_frequencies(dims: int, base: float, scaling=None, device=None) -> tor
         out.append(f)
     t = torch.tensor(out, dtype=torch.float64).to(torch.float32)
     return t.to(device) if device is not None else t
+
+
+def ramped_frequencies(dims: int, base: float, ramp: tuple, device=None):
+    """(frequencies, amplitude) of a rotation stretched over longer contexts pair by pair: ``ramp`` = (factor, original, fast,
+    slow).  Pair i of base^(-2i/dims) makes ``t`` turns over ``original`` positions at i = dims ln(original / (2 pi t)) / (2 ln base);
+    pairs up to the one of ``fast`` turns (rounded down) keep their frequency, pairs from the one of ``slow`` turns (rounded up) on
+    are divided by ``factor``, those between are blended in proportion.  Cosine and sine are multiplied by the
+    amplitude, 0.1 ln(factor) + 1.  Worked out in 64-bit, rounded once to 32-bit.  (YaRN.)"""
+    import math
+
+    if dims % 2 or dims <= 0:
+        raise UnsupportedError(f"a rotation over {dims} values, which do not pair")
+    factor, original, fast, slow = (float(v) for v in ramp)
+    if not (factor > 0 and original > 0 and fast > 0 and slow > 0 and base > 0) or base == 1.0:
+        raise UnsupportedError(f"a ramp of factor {factor}, original {original}, fast {fast}, slow {slow} over a base of {base}")
+
+    def pair_of(turns: float) -> float:
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    first = max(math.floor(pair_of(fast)), 0)
+    last = min(math.ceil(pair_of(slow)), dims - 1)
+    out = []
+    for i in range(dims // 2):
+        f = float(base) ** (-2.0 * i / dims)
+        share = min(max((i - first) / max(last - first, 0.001), 0.0), 1.0)
+        out.append(f / factor * share + f * (1.0 - share))
+    t = torch.tensor(out, dtype=torch.float64).to(torch.float32)
+    return (t.to(device) if device is not None else t), 0.1 * math.log(factor) + 1.0
+
+
+def turning(dims: int, base: float, scaling=None, ramp=None, device=None):
+    """(frequencies, amplitude) of a rotation without tables, rescaled in one of the two ways or not at all."""
+    if ramp is None:
+        return rotary_frequencies(dims, base, scaling, device), 1.0
+    if scaling is not None:
+        raise UnsupportedError("rotation frequencies rescaled by wavelength and by a ramp at once")
+    return ramped_frequencies(dims, base, ramp, device)

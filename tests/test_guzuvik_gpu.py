@@ -472,7 +472,7 @@ def test_a_router_of_chosen_logits(total, top):
     positions[17] = -1
     rows = [t for t in range(n) if t != 17]
     z = torch.randn((n, total), generator=g) * 40          # (far apart: a softmax over all of them would be next to nothing for most)
-    chosen, weight = kernels.router_select(dev(z), None, positions.cuda(), top, bias=dev(bias), of_chosen=True)
+    chosen, weight = kernels.router_select(dev(z), None, positions.cuda(), top, bias=dev(bias), score="chosen_logits")
     best, at = (z.float() + bias.float()).double().topk(top, -1)
     assert (chosen.cpu()[17] == -1).all() and (weight.cpu()[17] == 0).all()
     assert torch.equal(chosen.cpu()[rows].long(), at[rows])
@@ -480,7 +480,7 @@ def test_a_router_of_chosen_logits(total, top):
     for dtype in (torch.float32, torch.bfloat16):
         x, w = torch.randn((n, width), generator=g).to(dtype), (torch.randn((total, width), generator=g) * 0.3).to(dtype)
         z = x.double() @ w.double().T + bias.double()
-        chosen, weight = kernels.router_select(None, None, positions.cuda(), top, x=x.cuda(), w=w.cuda(), bias=dev(bias), of_chosen=True)
+        chosen, weight = kernels.router_select(None, None, positions.cuda(), top, x=x.cuda(), w=w.cuda(), bias=dev(bias), score="chosen_logits")
         best, at = z.topk(top, -1)
         same = [t for t in rows if torch.equal(chosen.cpu()[t].long(), at[t])]
         assert len(same) >= n - 3
