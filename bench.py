@@ -394,10 +394,32 @@ def guzuvik_config(width: int, ff: int, heads: int, layers: int, vocab: int) -> 
             "norm": {"eps": 1e-5}, "vocab": vocab, "width": width, "layers": [kinds[i % 3] for i in range(layers)]}
 
 
+# --only nikonex: the Nikonex design (layers whose mixer and feed-forward read the same stream through a norm each; windowed
+# attention over one small vector a token with queries through a small vector of their own and ramped rotation frequencies, and
+# two layers of retention, heads of 128 with values of 256; every layer with eight experts of half the dense width, two
+# matrices each, of which a sigmoid router chooses two out of the better two of four groups, and a shared expert of the same
+# width, so that a token multiplies as much as in the dense model) at the same sizes, beside Qwen3 dense, beside
+# Dimalix, the design whose layers are the nearest to these, and beside Guzuvik, whose chunked state space is the nearest to
+# retention.
+def nikonex_config(width: int, ff: int, heads: int, layers: int, vocab: int) -> dict:
+    experts = {"kind": "moe", "expert": {"ff": ff // 2}, "shared": {"ff": ff // 2},
+               "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 2}, "scale": 2.5}}
+    latent = {"type": "latent_attention", "mlp": experts,
+              "mixer": {"heads": heads, "dim": 64, "rot_dim": 64, "vdim": 128, "q_rank": width // 2, "kv_rank": 192,
+                        "scale": 128 ** -0.5, "mask": {"size": 512},
+                        "rot": {"dims": 64, "base": 10000.0,
+                                "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    retention = {"type": "retention", "mlp": experts,
+                 "mixer": {"heads": heads // 2, "dim": 128, "vdim": 256, "rot": {"dims": 128, "base": 10000.0},
+                           "decay": [1.0 - 2.0 ** (-5 - h) for h in range(heads // 2)]}}
+    return {"architecture": "Nikonex", "norm": {"eps": 1e-6}, "vocab": vocab, "width": width, "residual_mult": 0.5,
+            "layers": [(latent, retention, retention)[i % 3] for i in range(layers)]}
+
+
 DESIGNS = {"papivik": papivik_config, "lefavik": lefavik_config, "mukenex": mukenex_config, "dimalix": dimalix_config,
-           "guzuvik": guzuvik_config}
+           "guzuvik": guzuvik_config, "nikonex": nikonex_config}
 # the models a design is measured beside, after Qwen3 dense
-BESIDE = {"mukenex": ("lefavik",), "dimalix": ("mukenex",), "guzuvik": ("mukenex",)}
+BESIDE = {"mukenex": ("lefavik",), "dimalix": ("mukenex",), "guzuvik": ("mukenex",), "nikonex": ("dimalix", "guzuvik")}
 
 
 def papivik_table(torch, args, design: str = "papivik") -> int:
@@ -528,9 +550,9 @@ def main() -> int:
     parser.add_argument("--ahead", choices=["on", "off"], default="on",
                         help="--only engine: whether the engine queues a decoding step before it has read the tokens "
                              "of the one before")
-    parser.add_argument("--size", choices=sorted(PAPIVIK_SIZES), default=None, help="--only papivik, lefavik, mukenex, dimalix or guzuvik: one of the sizes alone")
+    parser.add_argument("--size", choices=sorted(PAPIVIK_SIZES), default=None, help="--only papivik, lefavik, mukenex, dimalix, guzuvik or nikonex: one of the sizes alone")
     parser.add_argument("--only", choices=["decode", "prefill", "engine", "mixed", "serving", "products", "papivik", "lefavik", "mukenex", "dimalix",
-                                           "guzuvik"], default=None,
+                                           "guzuvik", "nikonex"], default=None,
                         help="run one part alone: the decode steps at --batch, the prefill, or (not part of the "
                              "default line) the whole engine on 1/4/16/32/64/128 requests at once, 16 prompt tokens and "
                              "128 generated each, as the reference's own table of clients does; mixed: one step of a "
@@ -542,7 +564,8 @@ def main() -> int:
                              "of the Papivik design at layer sizes of the 0.6B and 8B shapes beside Qwen3 dense of the same "
                              "width, layers and vocabulary; lefavik: the same for the Lefavik design; mukenex: the same for the Mukenex "
                              "design, beside Lefavik too; dimalix: the same for the Dimalix design, beside Mukenex too; guzuvik: the "
-                             "same for the Guzuvik design, beside Mukenex too")
+                             "same for the Guzuvik design, beside Mukenex too; nikonex: the same for the Nikonex design, beside "
+                             "Dimalix and Guzuvik too")
     args = parser.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py measures one GPU; this engine has no multi-GPU path (N must be 1)")

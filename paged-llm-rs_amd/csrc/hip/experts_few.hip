@@ -1,0 +1,169 @@
+// The experts of a step of few rows (up to 64) that a router has dealt out, bfloat16 on the matrix cores: the experts' weights are
+// read once, whatever the rows, and what bounds the step is that reading.  Two launches, nothing sorted in front of them:
+//   up:   h[pair] = act(w_first x_row), or act(gate x) * (up x) where the experts are gated, bfloat16
+//   down: y[pair] = w_down h[pair], 32-bit sums
+// A workgroup of eight waves owns 32 rows of one expert's matrix (16 gate rows and their 16 up rows where gated).  It looks through the
+// step's choices for the pairs that are its expert's (none: it is done), cuts the inner width into a stretch a wave,
+// each wave multiplies its stretch of the weights, straight from memory in the matrix cores' layout, with its
+// stretch of the pairs' rows, and the waves' sums are added in order through LDS.  A pair's result does not depend on the
+// other pairs or on its place among them.
+//
+// D[16 x 16] += A[16 x 32] B[32 x 16], v_mfma_f32_16x16x32_bf16: lane l gives A[l % 16][8 (l / 16) ..+ 7] (a row of the weights) and
+// B[8 (l / 16) ..+ 7][l % 16] (a pair's row), and holds in register r D[4 (l / 16) + r][l % 16]: four neighbouring outputs of one pair.
+#include "experts.hpp"
+
+typedef __bf16 mf_bf16x8 __attribute__((ext_vector_type(8)));
+typedef float mf_f32x4 __attribute__((ext_vector_type(4)));
+
+#define MF_WAVES 8
+#define MF_ROWS 64            // rows of a step at most
+
+// One workgroup's products: up to 16 MT pairs.  `wa`, `wb`: this lane's rows of the two strips of 16 rows of the weights.
+template <int MT, int U>
+__device__ __forceinline__ void few_products(const bf16_t* wa, const bf16_t* wb, const bf16_t* const (&x)[MT], int first, int behind,
+                                             mf_f32x4 (&acc)[2][MT]) {
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int mt = 0; mt < MT; ++mt) acc[b][mt] = mf_f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = first; k0 < behind; k0 += U) {
+        mf_bf16x8 a[U][2], bx[U][MT];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const size_t at = static_cast<size_t>(min(k0 + u, behind - 1)) * 32;
+            a[u][0] = *reinterpret_cast<const mf_bf16x8*>(wa + at);
+            a[u][1] = *reinterpret_cast<const mf_bf16x8*>(wb + at);
+#pragma unroll
+            for (int mt = 0; mt < MT; ++mt) bx[u][mt] = *reinterpret_cast<const mf_bf16x8*>(x[mt] + at);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (k0 + u < behind) {                       // (the same for the whole wave)
+#pragma unroll
+                for (int b = 0; b < 2; ++b)
+#pragma unroll
+                    for (int mt = 0; mt < MT; ++mt)
+                        acc[b][mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u][b], bx[u][mt], acc[b][mt], 0, 0, 0);
+            }
+    }
+}
+
+template <bool DOWN, bool GATED, int MT>
+__device__ __forceinline__ void few_body(const MoeArgs& a, float* y, const bf16_t* w, int N, int K, int n0, const int* list, int pairs,
+                                         mf_f32x4* red) {
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c16 = lane & 15, g = lane >> 4;
+    const int values = moe_row_values(a);
+    constexpr bool PAIRED = GATED && !DOWN;
+    const int ra = min(n0 + c16, N - 1);
+    const int rb = PAIRED ? N + ra : min(n0 + 16 + c16, N - 1);
+    const bf16_t* x[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+        const int p = list[min(mt * 16 + c16, pairs - 1)];
+        const int t = p / a.top, c = p - t * a.top;
+        x[mt] = (DOWN ? static_cast<const bf16_t*>(a.h) + static_cast<size_t>(t) * values + c * a.F
+                      : static_cast<const bf16_t*>(a.x) + static_cast<size_t>(t) * a.W) + 8 * g;
+    }
+    const int chunks = K / 32;
+    mf_f32x4 acc[2][MT];
+    few_products<MT, (MT == 1 ? 8 : (MT == 2 ? 4 : 2))>(w + static_cast<size_t>(ra) * K + 8 * g, w + static_cast<size_t>(rb) * K + 8 * g, x,
+                                                       wave * chunks / MF_WAVES, (wave + 1) * chunks / MF_WAVES, acc);
+    // the waves' sums, one strip after the other: [wave][mt][lane]
+    mf_f32x4 sum[2];
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+        if (b == 1) __syncthreads();
+#pragma unroll
+        for (int mt = 0; mt < MT; ++mt) red[(wave * MT + mt) * 64 + lane] = acc[b][mt];
+        __syncthreads();
+        sum[b] = mf_f32x4{0.f, 0.f, 0.f, 0.f};
+        if (tid < MT * 64) {
+#pragma unroll
+            for (int v = 0; v < MF_WAVES; ++v) {
+                const mf_f32x4 part = red[v * MT * 64 + tid];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) sum[b][r] += part[r];
+            }
+        }
+    }
+    const int slot = (tid >> 6) * 16 + c16;
+    if (tid >= MT * 64 || slot >= pairs) return;
+    const int p = list[slot];
+    const int t = p / a.top, c = p - t * a.top;
+#pragma unroll
+    for (int b = 0; b < (PAIRED ? 1 : 2); ++b) {
+        const int col = n0 + 16 * b + 4 * g;
+        if (col >= N) continue;                          // (N is a multiple of 4)
+        if constexpr (DOWN) {
+            *reinterpret_cast<mf_f32x4*>(y + static_cast<size_t>(p) * a.W + col) = sum[b];
+        } else {
+            float v[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                v[r] = PAIRED ? pl_gate_pair<false>(sum[0][r], sum[1][r], a.act, a.limit) : pl_activate<false>(sum[b][r], a.act);
+            uint2 packed;
+            packed.x = bf16_bits_from_float(v[0]) | (static_cast<uint32_t>(bf16_bits_from_float(v[1])) << 16);
+            packed.y = bf16_bits_from_float(v[2]) | (static_cast<uint32_t>(bf16_bits_from_float(v[3])) << 16);
+            *reinterpret_cast<uint2*>(static_cast<bf16_t*>(a.h) + static_cast<size_t>(t) * values + c * a.F + col) = packed;
+        }
+    }
+}
+
+// blockIdx.y: the expert, a.E for the shared one.
+template <bool DOWN, bool GATED>
+__global__ __launch_bounds__(64 * MF_WAVES) void moe_few_kernel(MoeArgs a, float* y) {
+    __shared__ int list[MF_ROWS];
+    __shared__ int found;
+    extern __shared__ __attribute__((aligned(16))) mf_f32x4 few_red[];
+    const int group = blockIdx.y;
+    const bool shared = group == a.E;
+    const int number = shared ? a.shared_at : group;
+    const int F = shared ? a.shared_F : a.F;
+    const int K = DOWN ? F : a.W, N = DOWN ? a.W : F;
+    const int n0 = blockIdx.x * (GATED && !DOWN ? 16 : 32);
+    if (n0 >= N) return;
+    if (threadIdx.x == 0) found = 0;
+    __syncthreads();
+    for (int p = threadIdx.x; p < a.n * a.top; p += 64 * MF_WAVES) {
+        const int t = p / a.top;
+        if (a.choice[p] == number && (!shared || p - t * a.top == a.top - 1) && a.positions[t] >= 0) {
+            const int at = atomicAdd(&found, 1);
+            if (at < MF_ROWS) list[at] = p;              // (a row names an expert once: there are no more)
+        }
+    }
+    __syncthreads();
+    const int pairs = min(found, MF_ROWS);
+    if (pairs == 0) return;
+    const bf16_t* w;
+    if (DOWN) w = shared ? static_cast<const bf16_t*>(a.shared_down) : static_cast<const bf16_t*>(a.w_down) + static_cast<size_t>(group) * a.W * F;
+    else w = shared ? static_cast<const bf16_t*>(a.shared_gu) : static_cast<const bf16_t*>(a.w_gu) + static_cast<size_t>(group) * (GATED ? 2 : 1) * F * a.W;
+    if (pairs <= 16) few_body<DOWN, GATED, 1>(a, y, w, N, K, n0, list, pairs, few_red);
+    else if (pairs <= 32) few_body<DOWN, GATED, 2>(a, y, w, N, K, n0, list, pairs, few_red);
+    else few_body<DOWN, GATED, 4>(a, y, w, N, K, n0, list, pairs, few_red);
+}
+
+// x [n, W], the matrices and h [n, values of a row's pairs] bfloat16; y [n * top, W] 32-bit, a row a pair (a pair without an expert, and
+// of an identity expert, is not written).  choice [n, top]: a row names an expert at most once.  See MoeArgs for the rest.
+extern "C" int pl_moe_few(const void* x, const int* positions, const int* choice, const void* w_first, const void* w_down, void* h,
+                          float* y, int n, int W, int F, int E, int top, int act, int identity, float limit, int plain, int shared_F,
+                          const void* shared_first, const void* shared_down, hipStream_t stream) {
+    PL_REQUIRE(n >= 0 && n <= MF_ROWS && W > 0 && F > 0 && E > 0 && E < 65535 && top > 0 && identity >= 0 && top <= E + identity + (shared_F > 0 ? 1 : 0),
+               "moe_few: %d rows of %d, %d experts of %d, %d a row", n, W, E, F, top);
+    PL_REQUIRE(W % 32 == 0 && F % 32 == 0 && shared_F >= 0 && shared_F % 32 == 0, "moe_few: rows of %d, experts of %d and %d (multiples of 32)", W, F, shared_F);
+    PL_REQUIRE(act >= 0 && act <= (plain ? PL_ACT_RELU2 : PL_ACT_CLAMPED), "moe_few: activation code %d", act);
+    PL_REQUIRE(choice != nullptr && positions != nullptr && (shared_F == 0 || (shared_first != nullptr && shared_down != nullptr)),
+               "moe_few: a router's choice and the matrices of a shared expert");
+    if (n == 0) return 0;
+    const MoeArgs a{x, nullptr, nullptr, nullptr, positions, nullptr, w_first, w_down, h, nullptr, n, W, F, E, top, 1, act, choice, nullptr,
+                    identity, limit, plain, shared_F > 0 ? E + identity : -1, shared_F, shared_first, shared_down};
+    const int groups = E + (shared_F > 0 ? 1 : 0), widest = shared_F > F ? shared_F : F;
+    const size_t lds = static_cast<size_t>(MF_WAVES) * (n <= 16 ? 1 : (n <= 32 ? 2 : 4)) * 64 * sizeof(mf_f32x4);
+    if (plain) moe_few_kernel<false, false><<<dim3(pl_ceil_div(widest, 32), groups), 64 * MF_WAVES, lds, stream>>>(a, y);
+    else moe_few_kernel<false, true><<<dim3(pl_ceil_div(widest, 16), groups), 64 * MF_WAVES, lds, stream>>>(a, y);
+    PL_CHECK_LAUNCH("moe_few (up)");
+    moe_few_kernel<true, false><<<dim3(pl_ceil_div(W, 32), groups), 64 * MF_WAVES, lds, stream>>>(a, y);
+    PL_CHECK_LAUNCH("moe_few (down)");
+    return 0;
+}

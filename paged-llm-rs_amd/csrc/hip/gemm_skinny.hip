@@ -2,7 +2,7 @@
 // (those that start with a norm are in gemm_skinny_norm.hip: two files compile side by side).
 #include "gemm_skinny.hpp"
 
-int sk_launch_norm(int epilogue, int out_f32, const void* x, const void* w, void* y, const float* gain, float eps, const int* rows, int n, int N_out, int K, int act, int strips, hipStream_t stream);
+int sk_launch_norm(int epilogue, int out_f32, const void* x, const void* w, void* y, const float* gain, float eps, const int* rows, int n, int N_out, int K, int act, int strips, int x_stride, hipStream_t stream);
 
 static int sk_launch_plain(int epilogue, int out_f32, const void* x, const void* w, void* y, const float* gain,
                            float eps, const int* rows, int n, int N_out, int K, int act, const sk_extras_t& hand,
@@ -13,13 +13,16 @@ static int sk_launch_plain(int epilogue, int out_f32, const void* x, const void*
 // x: bfloat16 [n, K], or with a gain the 32-bit residual stream [*, K] whose rows rows[0..n) (or 0..n) are
 // normalised on the way in (the gain is 32-bit).  w: bfloat16 [N_out, K], or [2*N_out, K] with gate rows first for epilogue 1.
 // epilogue 0: y = result, bfloat16 or (out_f32) 32-bit.  1: y = act(gate) * up (act: PL_ACT_*).  2: y, 32-bit, += result.
+// x_stride (with a gain): elements between two rows of x (0: K), a multiple of 4.
 // strips: w holds the same weights in strips (gemm_skinny.hpp has the layout; pl_gemm_skinny_strips_apply says for
 // which products that is read).
 extern "C" int pl_gemm_skinny_strips_apply(int n, int N_out, int K) { return sk_strips_apply(n, N_out, K) ? 1 : 0; }
 
 extern "C" int pl_gemm_skinny(const void* x, const void* w, void* y, const float* gain, float eps,
                               const int* rows, int n, int N_out, int K, int epilogue, int out_f32, int act,
-                              int strips, hipStream_t stream) {
+                              int strips, int x_stride, hipStream_t stream) {
+    PL_REQUIRE(x_stride == 0 || (gain && x_stride >= K && x_stride % 4 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0),
+               "skinny product: rows %d apart for an inner width of %d", x_stride, K);
     PL_REQUIRE(n >= 0 && n <= 64, "skinny product: %d rows, it takes up to 64", n);
     PL_REQUIRE(N_out > 0 && K > 0 && K % 8 == 0, "skinny product: %d columns, inner width %d (a multiple of 8 is needed)", N_out, K);
     PL_REQUIRE(epilogue >= EPI_STORE && epilogue <= EPI_ADD, "skinny product: epilogue code %d", epilogue);
@@ -31,7 +34,7 @@ extern "C" int pl_gemm_skinny(const void* x, const void* w, void* y, const float
     if (n == 0) return 0;
     PL_REQUIRE(!strips || sk_strips_apply(n, N_out, K),
                "skinny product: %d rows, %d columns, width %d are not read from weights in strips", n, N_out, K);
-    if (gain) return sk_launch_norm(epilogue, out_f32, x, w, y, gain, eps, rows, n, N_out, K, act, strips ? 1 : 0, stream);
+    if (gain) return sk_launch_norm(epilogue, out_f32, x, w, y, gain, eps, rows, n, N_out, K, act, strips ? 1 : 0, x_stride, stream);
     sk_extras_t with{};
     with.strips = strips ? 1 : 0;
     return sk_launch_plain(epilogue, out_f32, x, w, y, gain, eps, rows, n, N_out, K, act, with, stream);

@@ -74,6 +74,8 @@ struct sk_extras_t {
     // the K steps a wave of the launch takes (ceil(steps / waves): the launch knows both, and a division by a number
     // the kernel learns only when it runs is some thirty instructions in front of its first loads); 0: not said
     int steps_a_wave;
+    // PRO_NORM: elements between two rows of the 32-bit rows that are read (0: K, a stream of its own)
+    int x_stride;
 };
 
 static inline sk_extras_t sk_with_steps(sk_extras_t extras, int K, int waves) {
@@ -169,7 +171,7 @@ gemm_skinny_kernel(const void* __restrict__ x_, const bf16_t* __restrict__ w, OU
         row_ok[m] = row < n;
         int src = row_ok[m] ? row : 0;
         if (PRO == PRO_NORM && rows) src = rows[src];
-        xrow[m] = static_cast<size_t>(src) * K;
+        xrow[m] = static_cast<size_t>(src) * (PRO == PRO_NORM && hand.x_stride > 0 ? hand.x_stride : K);
     }
 
     bf16x8 ax[MT][UNR];
@@ -569,7 +571,7 @@ gemm_skinny_rows_kernel(const void* __restrict__ x_, const bf16_t* __restrict__ 
     const bool row_ok = working && row < n;
     int src = row_ok ? row : 0;
     if (PRO == PRO_NORM && rows) src = rows[src];
-    const size_t xrow = static_cast<size_t>(src) * K;
+    const size_t xrow = static_cast<size_t>(src) * (PRO == PRO_NORM && hand.x_stride > 0 ? hand.x_stride : K);
     const bf16_t* xb = static_cast<const bf16_t*>(x_);
     const float* xf = static_cast<const float*>(x_);
     bf16x8 ax[PRO == PRO_BF16 ? STEPS : 1];

@@ -13,7 +13,7 @@
 // choice) pairs are dealt to their experts, every expert's pairs in tiles of 128 rows, so that an expert's
 // weights are read once a tile and multiplied on the matrix cores; a pair's result does not depend on which
 // other pairs share its tile.
-#include "common.hpp"
+#include "experts.hpp"
 
 #define HC_MAX_COPIES 8
 
@@ -193,16 +193,6 @@ extern "C" int pl_softcap(float* x, float cap, long count, hipStream_t stream) {
 
 // ---- experts by table, few rows -------------------------------------------------------------------------
 
-// The id of row t: its own, or the one an earlier kernel left on the device (as the embedding takes it).
-__device__ __forceinline__ int moe_token(const int* ids, const int* src, const int* fed, int t) {
-    int id = ids[t];
-    if (src != nullptr) {
-        const int from = src[t];
-        if (from >= 0) id = fed[from];
-    }
-    return id;
-}
-
 // A wave's dot product of a weight row with a row of 32-bit values in LDS; every lane gets the sum.
 // The order of the additions depends on K alone.
 template <typename T>
@@ -222,45 +212,6 @@ __device__ __forceinline__ float moe_dot(const T* __restrict__ w, const float* x
         for (int k = lane; k < K; k += 64) acc = fmaf(to_float(w[k]), xs[k], acc);
     }
     return wave_sum(acc);
-}
-
-struct MoeArgs {
-    const void* x;         // [n, W]
-    const int* ids;
-    const int* src;
-    const int* fed;
-    const int* positions;  // rows at position -1 are padding
-    const int* table;      // [vocab, top]
-    const void* w_gu;      // [E, 2 F, W]: an expert's gate rows, then its up rows
-    const void* w_down;    // [E, W, F]
-    void* h;               // [n, top, F]
-    float* out;            // [n, W]
-    int n, W, F, E, top, vocab, act;
-    // Where a router has chosen (null: the table decides and every choice counts 1/top): the expert of pair
-    // (t, c) is choice[t * top + c], -1 for none, E .. E + identity - 1 for an identity expert, whose output is the
-    // row itself; weight[t * top + c] is what the pair counts.
-    const int* choice;
-    const float* weight;
-    int identity;
-    float limit;           // of the clamped gate (PL_ACT_CLAMPED)
-    int plain;             // an expert is down(act(up x)): w_gu holds up rows alone, [E, F, W]
-    // An expert of another size that every row of a router's choice names last, as number `shared_at` (-1: there is none).
-    int shared_at, shared_F;
-    const void* shared_gu; // [2 shared_F, W], or [shared_F, W] where plain
-    const void* shared_down;  // [W, shared_F]
-};
-
-// The values of a row's pairs lie one behind the other in h: pair c from c F on, the shared expert's, the last, of another length.
-__host__ __device__ static inline int moe_row_values(const MoeArgs& a) {
-    return a.shared_at >= 0 ? (a.top - 1) * a.F + a.shared_F : a.top * a.F;
-}
-
-// The expert of pair (t, c), or -1: the router's choice, or the table's row of the token's id.
-__device__ __forceinline__ int moe_pair_expert(const MoeArgs& a, int t, int c) {
-    if (a.choice != nullptr) return a.choice[static_cast<size_t>(t) * a.top + c];
-    const int id = moe_token(a.ids, a.src, a.fed, t);
-    if (id < 0 || id >= a.vocab) return -1;
-    return a.table[static_cast<size_t>(id) * a.top + c];
 }
 
 template <typename T>
@@ -453,42 +404,29 @@ extern "C" int pl_moe_sort(const int* ids, const int* src, const int* fed, const
     return 0;
 }
 
-// out[t, :] = (1/top) sum over c of y[slot_of[t * top + c], :], the choices in their order; a pair without a slot adds nothing.
-// y may come in `splits` copies, `split_stride` floats apart, each a stretch of the product's inner width: a pair's
-// copies are added in their order.
-// With `weight` a pair counts weight[t * top + c] instead of 1/top, and a pair whose `choice` is E or beyond (an
+// out[t, :] = the row's pairs added up (ExpertSum); a pair without a slot whose choice is `identity_from` .. `identity_from` + identity - 1 (an
 // identity expert) adds the row of x itself (of type `x_dtype`) with its weight.
-__global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ slot_of,
-                                                          float* __restrict__ out, int top, int W, int splits, size_t split_stride,
-                                                          const float* __restrict__ weight, const int* __restrict__ choice,
-                                                          const void* __restrict__ x, int x_dtype, int E,
-                                                          const int* __restrict__ positions) {
-    const int t = blockIdx.x;
+__global__ __launch_bounds__(256) void moe_combine_kernel(ExpertSum s, float* __restrict__ out, int W, const void* __restrict__ x, int x_dtype,
+                                                          int identity_from, int identity, const int* __restrict__ positions) {
+    const int t = blockIdx.x, top = s.top;
     const float even = 1.f / static_cast<float>(top);
-    const bool padding = positions != nullptr && positions[t] < 0;        // (a row of padding has no identity expert either)
+    const bool padding = positions != nullptr && positions[t] < 0;        // (a row of padding has no expert, nor an identity expert)
     for (int w = threadIdx.x * 4; w < W; w += blockDim.x * 4) {
         float4 sum = {0.f, 0.f, 0.f, 0.f};
-        for (int c = 0; c < top; ++c) {
-            const int slot = slot_of[t * top + c];
-            const float share = weight != nullptr ? weight[t * top + c] : even;
-            if (slot < 0) {
-                if (choice != nullptr && !padding && choice[t * top + c] >= E) {
-                    const size_t at = static_cast<size_t>(t) * W + w;
-                    sum.x += load_as_float(x, x_dtype, at) * share;
-                    sum.y += load_as_float(x, x_dtype, at + 1) * share;
-                    sum.z += load_as_float(x, x_dtype, at + 2) * share;
-                    sum.w += load_as_float(x, x_dtype, at + 3) * share;
-                }
+        for (int c = 0; c < top && !padding; ++c) {
+            const int chosen = s.choice != nullptr ? s.choice[t * top + c] : -1;
+            const float share = s.weight != nullptr ? s.weight[t * top + c] : even;
+            if (chosen >= identity_from && chosen < identity_from + identity) {
+                const size_t at = static_cast<size_t>(t) * W + w;
+                sum.x += load_as_float(x, x_dtype, at) * share;
+                sum.y += load_as_float(x, x_dtype, at + 1) * share;
+                sum.z += load_as_float(x, x_dtype, at + 2) * share;
+                sum.w += load_as_float(x, x_dtype, at + 3) * share;
                 continue;
             }
-            float4 v = *reinterpret_cast<const float4*>(y + static_cast<size_t>(slot) * W + w);
-            for (int s = 1; s < splits; ++s) {
-                const float4 more = *reinterpret_cast<const float4*>(y + s * split_stride + static_cast<size_t>(slot) * W + w);
-                v.x += more.x;
-                v.y += more.y;
-                v.z += more.z;
-                v.w += more.w;
-            }
+            const int slot = expert_slot(s, t, c);
+            if (slot < 0) continue;
+            const float4 v = expert_output(s, slot, W, w);
             sum.x += v.x * share;
             sum.y += v.y * share;
             sum.z += v.z * share;
@@ -500,13 +438,14 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
 
 extern "C" int pl_moe_combine(const float* y, const int* slot_of, float* out, int n, int top, int W, int splits,
                               long long split_stride, const float* weight, const int* choice, const void* x, int x_dtype,
-                              int E, const int* positions, hipStream_t stream) {
+                              int identity_from, int identity, const int* positions, hipStream_t stream) {
     PL_REQUIRE(n >= 0 && top > 0 && W > 0 && W % 4 == 0 && splits >= 1, "moe_combine: %d rows of %d, %d a row, %d copies", n, W, top, splits);
-    PL_REQUIRE(choice == nullptr || (x != nullptr && (x_dtype == PL_DTYPE_F32 || x_dtype == PL_DTYPE_BF16)),
+    PL_REQUIRE(identity == 0 || (choice != nullptr && x != nullptr && (x_dtype == PL_DTYPE_F32 || x_dtype == PL_DTYPE_BF16)),
                "moe_combine: identity experts need the rows they hand through");
+    PL_REQUIRE(slot_of != nullptr || choice != nullptr, "moe_combine: pairs without slots are a router's");
     if (n == 0) return 0;
-    moe_combine_kernel<<<n, 256, 0, stream>>>(y, slot_of, out, top, W, splits, static_cast<size_t>(split_stride), weight, choice,
-                                              x, x_dtype, E, positions);
+    const ExpertSum s{y, slot_of, choice, weight, top, splits, static_cast<size_t>(split_stride)};
+    moe_combine_kernel<<<n, 256, 0, stream>>>(s, out, W, x, x_dtype, identity_from, identity, positions);
     PL_CHECK_LAUNCH("moe_combine");
     return 0;
 }
@@ -585,7 +524,7 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
                                                             int scoring, int group_best, float scale, int shared) {
     const bool of_chosen = scoring == 1;
     const int named = top + shared, outputs = total_all + shared;     // what a row names, and the router's rows
-    extern __shared__ float router_lds[];             // score [total], choice score [total], group score [groups], kept or not [groups]
+    extern __shared__ float router_lds[];             // score [total], choice score [total], group score [groups], kept or not [groups], places [2 top]
     float* score = router_lds;                        // (and behind them, where the logits are worked out here: logits [total], the row [W])
     float* pick = router_lds + total_all;
     float* group = pick + total_all;
@@ -603,7 +542,7 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
     }
     const float* row = z + static_cast<size_t>(t) * stride;
     if (x != nullptr) {
-        float* logits = stays + groups_all;
+        float* logits = stays + groups_all + 2 * top;
         float* xs = logits + outputs;
         for (int k = threadIdx.x; k < W; k += blockDim.x) xs[k] = to_float(x[static_cast<size_t>(t) * W + k]);
         __syncthreads();
@@ -662,7 +601,16 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
         }
         __syncthreads();
         // the best `kept` groups keep their members, the others' members leave
-        for (int k = 0; k < kept; ++k) {
+        if (groups_all <= PL_WAVE) {                  // (a group's place is the count of those before it: a lane a group)
+            if (lane < groups) {
+                const float mine = group[lane];
+                int before = 0;
+                for (int g = 0; g < groups; ++g) before += group[g] > mine || (group[g] == mine && g < lane);
+                if (before < kept) stays[lane] = 1.f;
+            }
+            __syncthreads();
+        }
+        for (int k = 0; k < kept && groups_all > PL_WAVE; ++k) {
             float v = -INFINITY;
             int at = 0x7fffffff;
             for (int g = lane; g < groups; g += PL_WAVE) {
@@ -679,6 +627,41 @@ __global__ __launch_bounds__(256) void router_select_kernel(const float* __restr
         for (int e = lane; e < total; e += PL_WAVE)
             if (stays[e / size] == 0.f) pick[e] = -INFINITY;
         __syncthreads();
+    }
+    if (total_all <= 4 * PL_WAVE) {
+        // An output's place is the count of those before it; the first `top` places are the chosen ones.
+        int* place_of = reinterpret_cast<int*>(stays + groups_all);
+        float* place_score = stays + groups_all + top;
+        for (int c = lane; c < top && chooser; c += PL_WAVE) {
+            place_of[c] = -1;
+            place_score[c] = 0.f;
+        }
+        __syncthreads();
+        for (int e = lane; e < total; e += PL_WAVE) {
+            const float mine = pick[e];
+            int before = 0;
+#pragma unroll 8
+            for (int o = 0; o < total; ++o) before += pick[o] > mine || (pick[o] == mine && o < e);
+            if (before < top) {
+                place_of[before] = e;
+                place_score[before] = score[e];
+            }
+        }
+        __syncthreads();
+        if (!chooser) return;                        // (no barrier follows)
+        float sum = 0.f;
+        const float first = place_score[0];
+        for (int c = 0; c < top; ++c) sum += of_chosen ? expf(place_score[c] - first) : place_score[c];
+        const float by = of_chosen ? sum : (normalised ? sum + weight_eps : 1.f);
+        for (int c = lane; c < top; c += PL_WAVE) {
+            chosen[c] = place_of[c];
+            counts[c] = (of_chosen ? expf(place_score[c] - first) : place_score[c]) / by * scale;
+        }
+        if (shared && lane == 0) {
+            chosen[top] = total_all;
+            counts[top] = 1.f / (1.f + expf(-row[total_all]));
+        }
+        return;
     }
     float chosen_sum = 0.f, first_logit = 0.f;
     for (int c = 0; c < top; ++c) {
@@ -732,7 +715,7 @@ extern "C" int pl_router_select(const float* z, int stride, const float* correct
     PL_REQUIRE(groups >= 1 && total % groups == 0 && kept >= 1 && kept <= groups && top <= kept * (total / groups),
                "router_select: %d outputs in %d groups of which %d are kept, %d chosen", total, groups, kept, top);
     if (n == 0) return 0;
-    size_t lds = 2 * (static_cast<size_t>(total) + groups) * sizeof(float);
+    size_t lds = 2 * (static_cast<size_t>(total) + groups + top) * sizeof(float);
     if (x == nullptr) {
         router_select_kernel<float><<<n, 64, lds, stream>>>(z, stride, correction, positions, total, top, groups, kept, normalised,
                                                             weight_eps, choice, weight, nullptr, nullptr, 0, bias, scoring, group_best, scale, shared);

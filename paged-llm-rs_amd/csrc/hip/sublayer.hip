@@ -2,7 +2,7 @@
 //   stream += rmsnorm(y) * gain     (with the updated rows again in the model's type, for the next part)
 // and small passes over rows: a scale, a change of type, an activation, a weighted sum of two branches.
 // The statistic, the gain and the sum into the stream are 32-bit.
-#include "common.hpp"
+#include "experts.hpp"
 
 template <typename T>
 __global__ void rmsnorm_onto_kernel(float* __restrict__ resid, const float* __restrict__ y,
@@ -141,6 +141,7 @@ struct ParallelStepArgs {
     const int* rows;
     int W;
     float mult;
+    ExpertSum experts;     // in the place of b: a row's pairs, to be added up here (W a multiple of 4)
 };
 
 template <int PER>
@@ -190,7 +191,7 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
     const size_t in_row = static_cast<size_t>(p.rows != nullptr ? p.rows[i] : i) * W;
     const size_t out_row = static_cast<size_t>(i) * W;
     float* x = p.resid + in_row;
-    const bool sums = p.a != nullptr || p.b != nullptr || p.more != nullptr;
+    const bool sums = p.a != nullptr || p.b != nullptr || p.more != nullptr || p.experts.y != nullptr;
     Run<PER> first;
     float ss = 0.f;
     for (int c = threadIdx.x * PER; c < W; c += blockDim.x * PER) {
@@ -216,6 +217,27 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
 #pragma unroll
                 for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * p.mult;
             }
+        }
+        if (PER == 4 && p.experts.y != nullptr) {
+            float4 sum = {0.f, 0.f, 0.f, 0.f};
+            for (int k = 0; k < p.experts.top; ++k) {
+                const int slot = expert_slot(p.experts, i, k);
+                if (slot < 0) continue;
+                const float share = p.experts.weight != nullptr ? p.experts.weight[i * p.experts.top + k] : 1.f / static_cast<float>(p.experts.top);
+                const float4 y = expert_output(p.experts, slot, W, c);
+                sum.x += y.x * share;
+                sum.y += y.y * share;
+                sum.z += y.z * share;
+                sum.w += y.w * share;
+            }
+            Run<PER> g;
+#pragma unroll
+            for (int j = 0; j < PER; ++j) g.v[j] = 1.f;
+            if (p.ls2 != nullptr) g = load_run<PER>(p.ls2 + c);
+            v.v[0] += sum.x * g.v[0] * p.mult;
+            v.v[1 % PER] += sum.y * g.v[1 % PER] * p.mult;
+            v.v[2 % PER] += sum.z * g.v[2 % PER] * p.mult;
+            v.v[3 % PER] += sum.w * g.v[3 % PER] * p.mult;
         }
         if (p.more != nullptr) {
             const Run<PER> y = load_run<PER>(p.more + in_row + c);
@@ -250,14 +272,18 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
 
 extern "C" int pl_parallel_step(float* resid, const float* a, const float* ls1, const float* b, const float* ls2,
                                 const float* more, const float* gain1, const float* gain2, float eps, void* out1, void* out2,
-                                int dtype, const int* rows, int n, int W, float mult, hipStream_t stream) {
+                                int dtype, const int* rows, int n, int W, float mult, const float* pairs, const int* slot_of,
+                                const int* choice, const float* weight, int top, int splits, long long split_stride, hipStream_t stream) {
+    PL_REQUIRE(pairs == nullptr || (b == nullptr && rows == nullptr && W % 4 == 0 && top > 0 && splits >= 1 && (slot_of != nullptr || choice != nullptr)),
+               "parallel_step: rows of %d with %d experts' outputs each, in %d stretches", W, top, splits);
     PL_REQUIRE(n >= 0 && W > 0, "parallel_step: rows %d, width %d", n, W);
     PL_REQUIRE(rows == nullptr || (a == nullptr && b == nullptr && more == nullptr), "parallel_step: a list of rows and sums into the stream");
     PL_REQUIRE((gain1 != nullptr || gain2 == nullptr) && (gain1 == nullptr || out1 != nullptr) && (gain2 == nullptr || out2 != nullptr),
                "parallel_step: a second norm without a first, or a norm without room for its rows");
     PL_REQUIRE(dtype == PL_DTYPE_F32 || dtype == PL_DTYPE_BF16, "parallel_step: dtype code %d", dtype);
     if (n == 0) return 0;
-    ParallelStepArgs p{resid, a, ls1, b, ls2, more, gain1, gain2, eps, out1, out2, rows, W, mult};
+    ParallelStepArgs p{resid, a, ls1, b, ls2, more, gain1, gain2, eps, out1, out2, rows, W, mult,
+                       ExpertSum{pairs, slot_of, choice, weight, top, splits, static_cast<size_t>(split_stride)}};
     if (W % 4 == 0) {
         int threads = ((W / 4 + 63) / 64) * 64;
         threads = threads > 1024 ? 1024 : threads;

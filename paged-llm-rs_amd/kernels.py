@@ -46,7 +46,7 @@ def _signatures(lib) -> None:
         "pl_paged_attention_prefill_tile": [i, i],
         "pl_argmax": [p, p, p, p, i, i, p],
         "pl_sample": [p, p, p, p, p, p, i, i, i, p],
-        "pl_gemm_skinny": [p, p, p, p, f, p, i, i, i, i, i, i, i, p],
+        "pl_gemm_skinny": [p, p, p, p, f, p, i, i, i, i, i, i, i, i, p],
         "pl_gemm_skinny_strips_apply": [i, i, i],
         "pl_gemm_skinny_hand": [p, p, p, i, i, i, i, i, i, p, i, f, p, p, p, i, p],
         "pl_gemm_skinny_hand_applies": [i, i, i, i, i],
@@ -88,10 +88,11 @@ def _signatures(lib) -> None:
         "pl_softcap": [p, f, ctypes.c_long, p],
         "pl_moe_rows": [p, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, p, p, i, f, i, i, p, p, p],
         "pl_moe_sort": [p, p, p, p, p, p, i, i, i, i, i, i, i, p, p, p, p],
-        "pl_moe_combine": [p, p, p, i, i, i, i, ctypes.c_longlong, p, p, p, i, i, p, p],
+        "pl_moe_combine": [p, p, p, i, i, i, i, ctypes.c_longlong, p, p, p, i, i, i, p, p],
+        "pl_moe_few": [p, p, p, p, p, p, p, i, i, i, i, i, i, i, f, i, i, p, p, p],
         "pl_router_select": [p, i, p, p, i, i, i, i, i, i, f, p, p, p, p, i, i, p, i, i, f, i, p],
         "pl_wide_prepare": [p, p, i, i, i, f, p, p, p, i, p, p, p, i, i, i, p, p, p, i, i, i, i, i, i, p],
-        "pl_parallel_step": [p, p, p, p, p, p, p, p, f, p, p, i, p, i, i, f, p],
+        "pl_parallel_step": [p, p, p, p, p, p, p, p, f, p, p, i, p, i, i, f, p, p, p, p, i, i, ctypes.c_longlong, p],
         "pl_gemm_tiled_grouped": [p, p, p, p, p, ctypes.c_longlong, i, i, i, i, i, i, i, f, i, i, i, p, i, i, p],
         "pl_sandwich_step": [p, p, p, p, f, p, p, f, p, i, p, i, i, i, p],
         "pl_bigram_add": [p, p, p, p, p, p, p, p, p, p, p, i, ctypes.c_longlong, ctypes.c_longlong, ctypes.c_longlong, i, i, p],
@@ -832,7 +833,7 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype = torch
                 norm_gain: torch.Tensor | None = None, eps: float = 0.0, rows: torch.Tensor | None = None,
                 add_into: torch.Tensor | None = None, activation: str = "silu",
                 handed: "HandedNorm | None" = None, hand: "HandedNorm | None" = None,
-                strips: torch.Tensor | None = None) -> torch.Tensor:
+                strips: torch.Tensor | None = None, columns: tuple | None = None) -> torch.Tensor:
     """y = x . w^T for up to 64 rows on the matrix cores, the bfloat16 weights streamed once.
 
     ``x`` is bfloat16 [n, K]; or, with ``norm_gain``, the 32-bit residual stream, whose rows
@@ -844,12 +845,20 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype = torch
     ``handed``: a norm that an earlier product left behind; its rows are the input (``x`` is not looked at)
     and its sums of squares scale the result.  ``hand`` (with ``add_into``): the norm that follows the
     stream is left behind in it.
+    ``columns`` = (first, count), with a norm and without a row list: the rows normalised are these columns of the 32-bit rows ``x``
+    (both multiples of 4).
     ``strips``: what ``weights_in_strips`` made of ``w``; read instead of ``w`` where ``strips_apply`` says so."""
     if handed is not None:
         if norm_gain is not None or not handed.filled:
             raise TensorError("a handed norm is the product's input by itself, once a product has written it")
         x = handed.x
     K = x.shape[1]
+    x_at, stride = x.data_ptr(), 0
+    if columns is not None:
+        first, K = columns
+        if norm_gain is None or rows is not None or first % 4 or x.shape[1] % 4 or not 0 <= first <= x.shape[1] - K:
+            raise TensorError(f"columns {columns} of rows of shape {tuple(x.shape)} for a product behind a norm")
+        x_at, stride = x_at + 4 * first, x.shape[1]
     if norm_gain is None:
         _need(x, "matrix product input", None, torch.bfloat16)
         n = x.shape[0]
@@ -900,8 +909,8 @@ def gemm_skinny(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype = torch
             hand.filled = True
         return out
     _check(library().pl_gemm_skinny(
-        x.data_ptr(), w.data_ptr(), out.data_ptr(), _ptr(norm_gain), float(eps), _ptr(rows), n, N_out, K,
-        epilogue, out_f32, activation_code(activation), in_strips, _stream()))
+        x_at, w.data_ptr(), out.data_ptr(), _ptr(norm_gain), float(eps), _ptr(rows), n, N_out, K,
+        epilogue, out_f32, activation_code(activation), in_strips, stride, _stream()))
     return out
 
 
@@ -1774,6 +1783,53 @@ def _experts(x: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, gated: b
     return E, F, size
 
 
+class ExpertSums:
+    """The 32-bit outputs of a step's (row, choice) pairs, not added up yet: ``y`` [splits, slots, W] (each copy a stretch of the product's
+    inner width), pair (t, c) in slot ``slot_of[t, c]`` or, without ``slot_of``, in its own.  ``total()`` adds them up a row;
+    ``parallel_step`` takes them as they are in the place of a sublayer's output (where ``W`` is a multiple of 4)."""
+
+    def __init__(self, y, slot_of, choice, weight, n: int, top: int, splits: int, x, first_identity: int, identity: int, positions):
+        self.y, self.slot_of, self.choice, self.weight = y, slot_of, choice, weight
+        self.n, self.top, self.splits, self.W = n, top, splits, y.shape[-1]
+        self.stride = y.stride(0) if splits > 1 else 0
+        self.x, self.first_identity, self.identity, self.positions = x, first_identity, identity, positions
+
+    def total(self) -> torch.Tensor:
+        out = torch.empty((self.n, self.W), dtype=torch.float32, device=self.y.device)
+        _check(library().pl_moe_combine(self.y.data_ptr(), _ptr(self.slot_of), out.data_ptr(), self.n, self.top, self.W, self.splits,
+                                        self.stride, _ptr(self.weight), _ptr(self.choice), self.x.data_ptr(), _code(self.x, "rows"),
+                                        self.first_identity, self.identity, self.positions.data_ptr(), _stream()))
+        return out
+
+    def as_they_are(self):
+        """Themselves where a pass can add them up, their total otherwise (identity experts hand rows through, which that pass does not)."""
+        return self if self.identity == 0 and self.W % 4 == 0 else self.total()
+
+
+MOE_FEW_ROWS = 64    # rows of a step up to which every expert's weights are read once by the kernels of few rows
+
+
+def moe_few_applies(x: torch.Tensor, width: int, ff: int) -> bool:
+    return x.dtype == torch.bfloat16 and 0 < x.shape[0] <= MOE_FEW_ROWS and width % 32 == 0 and ff % 32 == 0
+
+
+def moe_few(x: torch.Tensor, batch, w_gate_up: torch.Tensor, w_down: torch.Tensor, activation: str, choice, weight,
+            identity: int = 0, limit=None, gated: bool = True, shared: tuple | None = None) -> ExpertSums:
+    """What ``moe_grouped`` computes for a router's choice, for steps of up to ``MOE_FEW_ROWS`` rows: two launches, nothing sorted; an
+    expert's weights go from memory to the matrix cores once.  A row names an expert at most once."""
+    n, W = x.shape
+    _need(x, "rows", None, torch.bfloat16)
+    E, F, size = _experts(x, w_gate_up, w_down, gated, shared, choice)
+    top = _routed(n, E, choice, weight, identity, 1 if size else 0)
+    act, bound = _gate_code(activation, limit)
+    h = torch.empty((n, (top - 1) * F + (size or F)), dtype=x.dtype, device=x.device)
+    y = torch.empty((1, n * top, W), dtype=torch.float32, device=x.device)
+    _check(library().pl_moe_few(x.data_ptr(), batch.positions.data_ptr(), choice.data_ptr(), w_gate_up.data_ptr(), w_down.data_ptr(),
+                                h.data_ptr(), y.data_ptr(), n, W, F, E, top, act, int(identity), bound, 0 if gated else 1, size,
+                                shared[0].data_ptr() if size else 0, shared[1].data_ptr() if size else 0, _stream()))
+    return ExpertSums(y, None, choice, weight, n, top, 1, x, E, int(identity), batch.positions)
+
+
 def moe_rows(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: torch.Tensor,
              activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None,
              gated: bool = True, shared: tuple | None = None) -> torch.Tensor:
@@ -1828,13 +1884,13 @@ def moe_down_splits(tiles: int, width: int, ff: int) -> int:
 
 def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: torch.Tensor,
                 activation: str = "silu", choice=None, weight=None, identity: int = 0, limit=None,
-                gated: bool = True, shared: tuple | None = None) -> torch.Tensor:
+                gated: bool = True, shared: tuple | None = None, summed: bool = True):
     """What ``moe_rows`` computes, with the step's (row, choice) pairs dealt to their experts first: an expert's
     pairs fill tiles of 128 rows, and two grouped products on the matrix cores (gate and up with the activation
     behind them; down with 32-bit sums out) read an expert's weights once a tile.  A last pass adds a row's
     choices in their order, in 32-bit.  A shared expert is one more group of the same products, with matrices of its own
     size.  Nothing is read back by the host: the tiles are laid out for the most
-    a step of so many rows can need."""
+    a step of so many rows can need.  ``summed`` False: the pairs' outputs come back not added up (``ExpertSums``)."""
     n, W = x.shape
     _need(x, "rows", None, torch.bfloat16)
     E, F, size = _experts(x, w_gate_up, w_down, gated, shared, choice)
@@ -1844,9 +1900,8 @@ def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: 
         _need(table, "table of experts", None, torch.int32)
         vocab, top = table.shape
     act, bound = _gate_code(activation, limit)
-    out = torch.empty((n, W), dtype=torch.float32, device=x.device)
     if n == 0:
-        return out
+        return torch.empty((n, W), dtype=torch.float32, device=x.device)
     fed = getattr(batch, "fed_tokens", None)
     src = batch.token_src if fed is not None else None
     pairs = n * top
@@ -1870,9 +1925,8 @@ def moe_grouped(x: torch.Tensor, batch, table, w_gate_up: torch.Tensor, w_down: 
     y = torch.empty((splits, slots, W), dtype=torch.float32, device=x.device)
     _check(lib.pl_gemm_tiled_grouped(hidden.data_ptr(), w_down.data_ptr(), y.data_ptr(), tile_group.data_ptr(), 0,
                                      W * F, tiles, slots, W, F, 3, 0, splits, 0.0, longest, W, last, shared_down, W, size, stream))
-    _check(lib.pl_moe_combine(y.data_ptr(), slot_of.data_ptr(), out.data_ptr(), n, top, W, splits, slots * W,
-                              _ptr(weight), _ptr(choice), x.data_ptr(), _code(x, "rows"), E, batch.positions.data_ptr(), stream))
-    return out
+    sums = ExpertSums(y, slot_of, choice, weight, n, top, splits, x, E, int(identity), batch.positions)
+    return sums.total() if summed else sums
 
 
 # A router's logits are worked out inside the kernel that chooses (one wave a row, the router's matrix from L2) for steps
@@ -1972,20 +2026,25 @@ def parallel_step(resid: torch.Tensor, a=None, ls1=None, b=None, ls2=None, more=
                   eps: float = 0.0, out_dtype: torch.dtype = torch.float32, rows=None, mult: float = 1.0):
     """One pass over the rows of the 32-bit stream for a layer whose sublayers stand side by side, either half
     optional.  Sums: resid += mult * (ls1 * a + ls2 * b) + more (``a``, ``b``, ``more`` [n, W] 32-bit; ``ls1``, ``ls2`` [W] 32-bit
-    or None for ones), in place.  Norms of the updated rows: rms-normed rows times ``gain1`` and, where given, times
+    or None for ones), in place; ``b`` may be ``ExpertSums`` instead, which this pass adds up.  Norms of the updated rows: rms-normed rows times ``gain1`` and, where given, times
     ``gain2`` (both [W] 32-bit), in ``out_dtype``; (rows1, rows2), each None where its gain is.  ``rows``: the rows to
     norm (then nothing is summed)."""
     _need(resid, "residual stream", None, torch.float32)
     if resid.dim() != 2:
         raise TensorError(f"a stream of shape {tuple(resid.shape)}")
     n, W = resid.shape
+    pairs = None
+    if isinstance(b, ExpertSums):
+        pairs, b = b, None
+        if (pairs.n, pairs.W) != (n, W) or pairs.identity or W % 4 or rows is not None:
+            raise TensorError(f"experts' outputs of {pairs.n} rows of {pairs.W} for a stream of shape {tuple(resid.shape)}")
     for t, what in ((a, "first sublayer's output"), (b, "second sublayer's output"), (more, "rows to add")):
         if t is not None:
             _need(t, what, (n, W), torch.float32)
     for t, what in ((ls1, "first layer scale"), (ls2, "second layer scale"), (gain1, "first norm gain"), (gain2, "second norm gain")):
         if t is not None:
             _need(t, what, (W,), torch.float32)
-    if (ls1 is not None and a is None) or (ls2 is not None and b is None) or (gain2 is not None and gain1 is None):
+    if (ls1 is not None and a is None) or (ls2 is not None and b is None and pairs is None) or (gain2 is not None and gain1 is None):
         raise TensorError("a layer scale without its sublayer's output, or a second norm without a first")
     count = n
     if rows is not None:
@@ -1993,11 +2052,13 @@ def parallel_step(resid: torch.Tensor, a=None, ls1=None, b=None, ls2=None, more=
         count = rows.numel()
     out1 = torch.empty((count, W), dtype=out_dtype, device=resid.device) if gain1 is not None else None
     out2 = torch.empty((count, W), dtype=out_dtype, device=resid.device) if gain2 is not None else None
-    if a is None and b is None and more is None and gain1 is None:
+    if a is None and b is None and pairs is None and more is None and gain1 is None:
         return None, None
     _check(library().pl_parallel_step(resid.data_ptr(), _ptr(a), _ptr(ls1), _ptr(b), _ptr(ls2), _ptr(more), _ptr(gain1),
                                       _ptr(gain2), float(eps), _ptr(out1), _ptr(out2), _CODES[out_dtype], _ptr(rows),
-                                      count, W, float(mult), _stream()))
+                                      count, W, float(mult), *((pairs.y.data_ptr(), _ptr(pairs.slot_of), _ptr(pairs.choice), _ptr(pairs.weight),
+                                                                pairs.top, pairs.splits, pairs.stride) if pairs is not None
+                                                               else (0, 0, 0, 0, 0, 1, 0)), _stream()))
     return out1, out2
 
 

@@ -531,8 +531,11 @@ class ParallelBlock:
         out = None
         if self.feed_forward is not None:
             ffn = self.feed_forward
-            out = ffn.forward(rows2, batch=ctx.batch) if getattr(ffn, "takes_batch", False) else ffn.forward(rows2)
-            if out.dtype != torch.float32:
+            how = {"batch": ctx.batch} if getattr(ffn, "takes_batch", False) else {}
+            if getattr(ffn, "may_leave_sums", False):
+                how["summed"] = False                 # (the pass behind adds them up)
+            out = ffn.forward(rows2, **how)
+            if isinstance(out, torch.Tensor) and out.dtype != torch.float32:
                 out = out.float()
         after = getattr(ctx, "norm_after", None)
         if ctx.trace is None and after is not None and getattr(after, "takes_pending_sums", False):

@@ -112,6 +112,16 @@ class LatentAttention:
     def state_spec(self):
         return None
 
+    def _queries(self, rows):
+        """The queries out of their small vector: its norm is the first stage of the product of few rows, a kernel of its own otherwise."""
+        product, gain, eps = self.q_proj, self.q_gain, self.spec.norm_eps
+        width = product.in_features
+        if (kernels.fused_norm_applies(rows.shape[0], width, product.weight) and rows.shape[1] % 4 == 0
+                and product.out_features <= kernels.FUSED_NORM_MAX_COLUMNS):
+            return kernels.gemm_skinny(rows, product.weight, torch.float32, norm_gain=gain, eps=eps, strips=product.strips,
+                                       columns=(0, width))
+        return product.forward(kernels.rows_norm(rows, 0, gain, eps, self.dtype), out_dtype=torch.float32)
+
     def forward(self, x, ctx):
         """``x``: the normed rows, or a norm still to run.  The output comes back as 32-bit sums, or None where the output projection
         added them into ``ctx.residual`` itself."""
@@ -123,8 +133,7 @@ class LatentAttention:
         q_plain = torch.empty((H, n, D), dtype=self.dtype, device=rows.device)
         queries = rows
         if self.q_proj is not None:
-            queries = self.q_proj.forward(kernels.rows_norm(rows, 0, self.q_gain, self.spec.norm_eps, self.dtype),
-                                          out_dtype=torch.float32)
+            queries = self._queries(rows)
         kernels.latent_prepare(queries, 0, self.kv_off, self.gain, self.spec.norm_eps, self.cos, self.sin, self.spec.rotary_turned,
                                batch, kv, q_plain, q, H, D, rot, R, P, write_kv=ctx.writes_cache and not self.spec.borrows,
                                kv_rows=rows, amplitude=self.amplitude)

@@ -160,6 +160,8 @@ class RoutedExperts:
     # forward needs the step (padding rows choose nothing)
     takes_batch = True
     graph_safe = True
+    # ... and may hand back the pairs' outputs for the caller's next pass to add up (``summed=False``: ``kernels.ExpertSums``)
+    may_leave_sums = True
 
     @staticmethod
     def declare(spec, hidden: int) -> list:
@@ -216,7 +218,7 @@ class RoutedExperts:
         self.bias = params["router.b"].to(torch.float32).contiguous() if spec.biased else None
         self.correction = params["correction"].to(torch.float32).contiguous() if spec.corrected else None
 
-    def forward(self, x, batch):
+    def forward(self, x, batch, summed: bool = True):
         spec = self.spec
         how = dict(bias=self.bias, score=spec.score, group_best=spec.group_best, scale=spec.weight_scale,
                    shared=self.shared_expert is not None)
@@ -227,11 +229,15 @@ class RoutedExperts:
             logits = self.router.forward(x, out_dtype=torch.float32)
         choice, weight = kernels.router_select(logits, self.correction, batch.positions, spec.top, spec.groups,
                                                spec.groups_kept, spec.normalised, spec.weight_eps, **how)
-        dealt = all(kernels.moe_grouped_applies(x, x.shape[1], size, spec.gated)
-                    for size in (spec.intermediate_size, spec.shared_size) if size)
-        run = kernels.moe_grouped if dealt else kernels.moe_rows
-        return run(x, batch, None, self.w_first, self.w_down, self.activation, choice=choice, weight=weight,
-                   identity=spec.identity, limit=spec.limit, gated=spec.gated, shared=self.shared_expert)
+        sizes = [size for size in (spec.intermediate_size, spec.shared_size) if size]
+        how = dict(choice=choice, weight=weight, identity=spec.identity, limit=spec.limit, gated=spec.gated, shared=self.shared_expert)
+        if all(kernels.moe_few_applies(x, x.shape[1], size) for size in sizes):
+            sums = kernels.moe_few(x, batch, self.w_first, self.w_down, self.activation, **how)
+        elif all(kernels.moe_grouped_applies(x, x.shape[1], size, spec.gated) for size in sizes):
+            sums = kernels.moe_grouped(x, batch, None, self.w_first, self.w_down, self.activation, summed=False, **how)
+        else:
+            return kernels.moe_rows(x, batch, None, self.w_first, self.w_down, self.activation, **how)
+        return sums.total() if summed else sums.as_they_are()
 
 
 register_feed_forward("routed_experts", RoutedExperts)
