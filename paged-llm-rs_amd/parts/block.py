@@ -453,12 +453,15 @@ class ParallelBlock:
     The stream and every sum into it are 32-bit; sublayers hand back 32-bit rows.  One kernel adds a layer's two outputs
     into the stream and norms the next layer's two rows in the same pass (``kernels.parallel_step``): a layer that is
     followed by another of this arrangement leaves its sums to that layer's pass (``PendingSums``), so a layer is one
-    pass over the stream.  ``ctx.stream_addend`` (rows the decoder wants added to the stream before this run) joins
+    pass over the stream.  Behind that pass neither sublayer waits for the other: the feed-forward runs on a second stream beside the
+    mixer (``side_by_side``; a captured step keeps the two branches), and the pass behind the layer waits for both.  ``ctx.stream_addend`` (rows the decoder wants added to the stream before this run) joins
     that pass too.  Tensor names: the norms' gains under the norms' own names."""
 
     NAMES = {"norm1": "norm1", "mixer": "mix", "norm2": "norm2", "feed_forward": "mlp", "scale1": "ls1", "scale2": "ls2"}
     # the decoder may hand this block rows to add to the stream before it runs (``LayerContext.stream_addend``)
     takes_stream_addend = True
+    # the two sublayers on two streams (False: one behind the other; the same bits)
+    side_by_side = True
 
     @classmethod
     def names_of(cls, layer) -> dict:
@@ -492,7 +495,7 @@ class ParallelBlock:
         if not getattr(norm, "fuses_into_product", False):
             raise ConfigError(f"norm {layer.norm.kind!r} cannot run inside the pass over the stream of a layer whose "
                               "sublayers stand side by side (it needs a 32-bit gain and an eps, nothing else)")
-        self.dtype, self.hidden = dtype, hidden
+        self.dtype, self.hidden, self.shared = dtype, hidden, shared
         self.mult = float(getattr(layer, "residual_mult", 1.0))
         self.norm1 = norm(layer.norm, hidden, {"weight": params[n["norm1"]]}, dtype, device)
         self.norm1.takes_pending_sums = True       # (how the layer before learns that its sums can wait)
@@ -527,22 +530,42 @@ class ParallelBlock:
             gain1=self.norm1.gain32, gain2=self.norm2.gain32 if self.norm2 is not None else None, eps=eps,
             out_dtype=self.dtype)
         ctx.stream_addend = None
-        mixed = self.mixer.forward(rows1, ctx)
-        out = None
-        if self.feed_forward is not None:
-            ffn = self.feed_forward
-            how = {"batch": ctx.batch} if getattr(ffn, "takes_batch", False) else {}
-            if getattr(ffn, "may_leave_sums", False):
-                how["summed"] = False                 # (the pass behind adds them up)
-            out = ffn.forward(rows2, **how)
-            if isinstance(out, torch.Tensor) and out.dtype != torch.float32:
-                out = out.float()
+        side = None
+        if self.side_by_side and self.feed_forward is not None and ctx.trace is None:
+            side = self.shared.get("side_stream")
+            if side is None:
+                side = self.shared["side_stream"] = torch.cuda.Stream(resid.device)
+        if side is None:
+            mixed = self.mixer.forward(rows1, ctx)
+            out = self._fed_forward(rows2, ctx)
+        else:
+            # (What either branch allocates belongs to its own stream and is used again behind the join: ``rows2`` and the
+            # outputs are held until the pass behind this layer is queued, for which both streams wait.)
+            main = torch.cuda.current_stream(resid.device)
+            side.wait_stream(main)
+            try:
+                with torch.cuda.stream(side):
+                    out = self._fed_forward(rows2, ctx)
+                mixed = self.mixer.forward(rows1, ctx)
+            finally:
+                main.wait_stream(side)
         after = getattr(ctx, "norm_after", None)
         if ctx.trace is None and after is not None and getattr(after, "takes_pending_sums", False):
             ctx.handed_out = PendingSums(mixed, self.ls1, out, self.ls2, self.mult)
         else:
             kernels.parallel_step(resid, a=mixed, ls1=self.ls1, b=out, ls2=self.ls2, mult=self.mult)
         return None
+
+    def _fed_forward(self, rows, ctx):
+        """What the feed-forward gives, 32-bit: rows, or outputs of experts that the pass behind adds up."""
+        ffn = self.feed_forward
+        if ffn is None:
+            return None
+        how = {"batch": ctx.batch} if getattr(ffn, "takes_batch", False) else {}
+        if getattr(ffn, "may_leave_sums", False):
+            how["summed"] = False
+        out = ffn.forward(rows, **how)
+        return out.float() if isinstance(out, torch.Tensor) and out.dtype != torch.float32 else out
 
 
 register_block("parallel", ParallelBlock)
