@@ -157,7 +157,7 @@ __device__ __forceinline__ void few_body(const MoeArgs& a, float* y, const bf16_
 template <bool DOWN, bool GATED>
 __global__ __launch_bounds__(64 * MF_WAVES, 4) void moe_few_kernel(MoeArgs a, float* y, int speculate) {
     __shared__ int list[MF_ROWS];
-    __shared__ int found;
+    __shared__ int wave_found[MF_WAVES];
     extern __shared__ __attribute__((aligned(16))) mf_f32x4 few_red[];
     const int group = a.shared_at < 0 ? static_cast<int>(blockIdx.y) : (blockIdx.y == 0 ? a.E : static_cast<int>(blockIdx.y) - 1);
     const bool shared = group == a.E;
@@ -178,14 +178,27 @@ __global__ __launch_bounds__(64 * MF_WAVES, 4) void moe_few_kernel(MoeArgs a, fl
     FewEarly early;
     const bool ahead = speculate && (blockIdx.z == 0 || shared);
     if (ahead) few_ask_early(early, wa, wb, first, behind);
-    if (threadIdx.x == 0) found = 0;
-    __syncthreads();
-    for (int p = threadIdx.x; p < a.n * a.top; p += 64 * MF_WAVES) {
-        const int t = p / a.top;
-        if (a.choice[p] == number && (!shared || p - t * a.top == a.top - 1) && a.positions[t] >= 0) {
-            const int at = atomicAdd(&found, 1);
-            if (at < MF_ROWS) list[at] = p;              // (a row names an expert once: there are no more)
+    // The expert's pairs in ascending order (every workgroup of an expert has to see the same list: they take 32 pairs each).
+    int found = 0;
+    for (int p0 = 0; p0 < a.n * a.top; p0 += 64 * MF_WAVES) {
+        const int p = p0 + threadIdx.x;
+        bool mine = false;
+        if (p < a.n * a.top) {
+            const int t = p / a.top;
+            mine = a.choice[p] == number && (!shared || p - t * a.top == a.top - 1) && a.positions[t] >= 0;
         }
+        const unsigned long long mask = __ballot(mine);
+        if (p0 > 0) __syncthreads();
+        if (lane == 0) wave_found[wave] = __popcll(mask);
+        __syncthreads();
+        int at = found;
+#pragma unroll
+        for (int v = 0; v < MF_WAVES; ++v) {
+            at += v < wave ? wave_found[v] : 0;
+            found += wave_found[v];
+        }
+        at += __popcll(mask & ((1ull << lane) - 1ull));
+        if (mine && at < MF_ROWS) list[at] = p;          // (a row names an expert once: there are no more)
     }
     __syncthreads();
     // (an expert of more than 32 pairs has a workgroup for every 32 of them: registers for twice as many would leave the chip
