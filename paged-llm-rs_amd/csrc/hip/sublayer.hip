@@ -184,14 +184,15 @@ __device__ __forceinline__ void store_run(bf16_t* p, const Run<PER>& r) {
 
 // A workgroup a row; a thread takes runs of PER columns.  A thread's first run stays in registers between the two
 // halves (rows up to PER * blockDim columns are read once), further ones are read back from the stream.
-template <typename T, int PER>
+// EXPERTS: p.experts holds something (an instance of its own: the loads of a row's pairs take registers).
+template <typename T, int PER, bool EXPERTS>
 __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p) {
     __shared__ float scratch[16];
     const int i = blockIdx.x, W = p.W;
     const size_t in_row = static_cast<size_t>(p.rows != nullptr ? p.rows[i] : i) * W;
     const size_t out_row = static_cast<size_t>(i) * W;
     float* x = p.resid + in_row;
-    const bool sums = p.a != nullptr || p.b != nullptr || p.more != nullptr || p.experts.y != nullptr;
+    const bool sums = EXPERTS || p.a != nullptr || p.b != nullptr || p.more != nullptr;
     Run<PER> first;
     float ss = 0.f;
     for (int c = threadIdx.x * PER; c < W; c += blockDim.x * PER) {
@@ -218,17 +219,26 @@ __global__ __launch_bounds__(1024) void parallel_step_kernel(ParallelStepArgs p)
                 for (int j = 0; j < PER; ++j) v.v[j] += y.v[j] * p.mult;
             }
         }
-        if (PER == 4 && p.experts.y != nullptr) {
+        if constexpr (EXPERTS) {
             float4 sum = {0.f, 0.f, 0.f, 0.f};
-            for (int k = 0; k < p.experts.top; ++k) {
-                const int slot = expert_slot(p.experts, i, k);
-                if (slot < 0) continue;
-                const float share = p.experts.weight != nullptr ? p.experts.weight[i * p.experts.top + k] : 1.f / static_cast<float>(p.experts.top);
-                const float4 y = expert_output(p.experts, slot, W, c);
-                sum.x += y.x * share;
-                sum.y += y.y * share;
-                sum.z += y.z * share;
-                sum.w += y.w * share;
+            const int top = p.experts.top;
+            for (int k0 = 0; k0 < top; k0 += 4) {             // (four pairs' outputs on their way together)
+                float4 y[4];
+                int slot[4];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    slot[j] = k0 + j < top ? expert_slot(p.experts, i, k0 + j) : -1;
+                    y[j] = expert_output(p.experts, slot[j] < 0 ? 0 : slot[j], W, c);
+                }
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    if (slot[j] < 0) continue;
+                    const float share = p.experts.weight != nullptr ? p.experts.weight[i * top + k0 + j] : 1.f / static_cast<float>(top);
+                    sum.x += y[j].x * share;
+                    sum.y += y[j].y * share;
+                    sum.z += y[j].z * share;
+                    sum.w += y[j].w * share;
+                }
             }
             Run<PER> g;
 #pragma unroll
@@ -287,12 +297,17 @@ extern "C" int pl_parallel_step(float* resid, const float* a, const float* ls1, 
     if (W % 4 == 0) {
         int threads = ((W / 4 + 63) / 64) * 64;
         threads = threads > 1024 ? 1024 : threads;
-        if (dtype == PL_DTYPE_F32) parallel_step_kernel<float, 4><<<n, threads, 0, stream>>>(p);
-        else parallel_step_kernel<bf16_t, 4><<<n, threads, 0, stream>>>(p);
+        if (dtype == PL_DTYPE_F32) {
+            if (pairs != nullptr) parallel_step_kernel<float, 4, true><<<n, threads, 0, stream>>>(p);
+            else parallel_step_kernel<float, 4, false><<<n, threads, 0, stream>>>(p);
+        } else {
+            if (pairs != nullptr) parallel_step_kernel<bf16_t, 4, true><<<n, threads, 0, stream>>>(p);
+            else parallel_step_kernel<bf16_t, 4, false><<<n, threads, 0, stream>>>(p);
+        }
     } else {
         const int threads = W >= 1024 ? 256 : (W >= 256 ? 128 : 64);
-        if (dtype == PL_DTYPE_F32) parallel_step_kernel<float, 1><<<n, threads, 0, stream>>>(p);
-        else parallel_step_kernel<bf16_t, 1><<<n, threads, 0, stream>>>(p);
+        if (dtype == PL_DTYPE_F32) parallel_step_kernel<float, 1, false><<<n, threads, 0, stream>>>(p);
+        else parallel_step_kernel<bf16_t, 1, false><<<n, threads, 0, stream>>>(p);
     }
     PL_CHECK_LAUNCH("parallel_step");
     return 0;
